@@ -1,7 +1,7 @@
 """mdi_llm_amd — an MI355X-native model-distributed inference framework.
 
-A from-scratch rebuild of the capabilities of MDI-LLM (davmacario/MDI-LLM,
-surveyed in /root/repo/SURVEY.md): recurrent pipeline-parallel LLM inference
+A from-scratch rebuild of the capabilities of MDI-LLM (davmacario/MDI-LLM):
+recurrent pipeline-parallel LLM inference
 across the GPUs of one 8×MI355X node, with hand-written CDNA4 HIP kernels
 for the decode path, RCCL point-to-point activation passing over xGMI, and
 litGPT-compatible checkpoints/chunks, plus single-device generation, chat,

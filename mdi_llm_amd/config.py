@@ -674,7 +674,7 @@ for kind in ("", "-chat"):
     )
 
 
-# -- reference-parity registry completion (round 2): every remaining
+# -- reference-parity registry completion: every remaining
 # named config of the reference registry (same hyperparameters for
 # checkpoint compatibility; /root/reference/src/sub/config.py:180-1667)
 # -- stablelm ----------------------------------------------------

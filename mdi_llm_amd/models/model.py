@@ -16,7 +16,7 @@ Capability parity with the reference model (/root/reference/src/sub/model.py:
   modules per message (reference ``gptserver.py:975-978``).  A pooled cache
   is what lets the HIP decode path replay one hipGraph for every in-flight
   sample and keeps GQA caches at ``n_query_groups`` width (the reference
-  stores them expanded to ``n_head`` — SURVEY §5.7).
+  stores them expanded to ``n_head``).
 * Attention is computed with explicit matmul + softmax (library GEMMs) on
   the torch path — no Triton, no flash shims; the fused flash-decode lives
   in the HIP extension.

@@ -802,7 +802,7 @@ class DecodeEngine:
     # ------------------------------------------------------------------
     # envelope serve (pipelined secondary): slot comes from the message
     # header ON DEVICE, so the host never reads a header in the decode
-    # loop (the per-hop hdr.cpu() sync)
+    # loop (a per-hop hdr.cpu() would sync the device)
     # ------------------------------------------------------------------
     def ensure_env_graph(self) -> None:
         """Capture header-routed decode: route(hdr)->stage->blocks->advance.

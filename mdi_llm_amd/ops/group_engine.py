@@ -2,7 +2,7 @@
 per stage pass.
 
 Beyond-parity optimization over the reference's strict one-sample-per-
-message schedule (SURVEY §2.3): with B samples batched, each stage streams
+message schedule: with B samples batched, each stage streams
 its weights from HBM once per B tokens instead of once per token — decode
 is bandwidth-bound, so stage throughput scales nearly linearly with B until
 compute/latency limits.  The recurrent-pipeline principle is preserved at

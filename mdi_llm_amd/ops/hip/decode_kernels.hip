@@ -7,7 +7,7 @@
 // MLP, lm-head), RoPE + KV-cache append, and GQA flash-decode attention
 // (MFMA 16x16x32 bf16 QK^T with online softmax, split-S across workgroups).
 //
-// Design notes (per /opt/skills/guides/cdna_hip_programming.md):
+// Design notes:
 //  * wave = 64 lanes; all block sizes are multiples of 64.
 //  * bf16 global loads vectorized as int4 (16 B = 8 bf16 per lane).
 //  * decode GEMV streams weights once; x is staged in LDS per block.
@@ -503,8 +503,8 @@ __global__ void gemv_direct_kernel(bf16* __restrict__ out,
 // (+ bias / + residual), B in {16, 32, 64, 128}.
 //
 // The hipBLASLt skinny-M GEMMs run these shapes at ~68% of the weight-
-// stream roofline (round-1 measurement); this is the priced recipe from
-// the round-1 ROADMAP: X staged into LDS in BULK COALESCED chunks with
+// stream roofline (measured); this is the priced recipe from
+// the measurements: X staged into LDS in BULK COALESCED chunks with
 // register double-buffering (the naive per-fragment L2 X loads measured
 // 1.4-1.6 TB/s — latency-bound), W streamed non-temporally straight into
 // MFMA A-fragments.
@@ -3392,7 +3392,7 @@ static void attn_dispatch2(void* out, float* part_o, float* part_ml,
   // short/medium contexts: one block per (batch, kv_head), no global
   // partials, no combine kernel — the whole attention step is ONE launch.
   // MDI_ATTN_FORCE_SPLITS=1 forces the split-S + combine path instead
-  // (A/B knob: the round-2 split-S got block-cooperative staging and a
+  // (A/B knob: the later split-S got block-cooperative staging and a
   // parallel combine, so its short-S cost may have changed)
   static int force_splits = -1;
   if (force_splits < 0) {

@@ -559,7 +559,7 @@ class PipelineRuntime:
         env=True (requires n_samples): pipelined envelope serve — W
         pre-posted recv pairs, device-side header routing on the HIP
         engine, lagged stop detection; the host never blocks the GPU on a
-        header read (round-1 VERDICT item 2)."""
+        header read."""
         from ..utils.context_managers import catch_loop_errors
 
         assert not self.is_starter

@@ -8,12 +8,13 @@ Two-step build, fully controlled (no hipify, no JIT cache):
 
 Usage:  python setup.py build_ext --inplace
 The resulting mdi_llm_amd/_hip_ops*.so ships with the repo snapshot to the
-GPU box (it is git-ignored but NOT gpurun-ignored).
+GPU box (it is git-ignored).
 """
 
 import os
 import subprocess
 import sys
+from concurrent.futures import ThreadPoolExecutor
 from pathlib import Path
 
 from setuptools import setup
@@ -29,34 +30,41 @@ HIPCC = os.path.join(ROCM_HOME, "bin", "hipcc")
 OFFLOAD_ARCH = os.environ.get("PYTORCH_ROCM_ARCH", "gfx950").split(";")[0]
 
 KERNEL_SOURCES = ["decode_kernels.hip"]
+HEADERS = [HIP_DIR / "decode_kernels.h"]
+
+
+def compile_one(src: str) -> str:
+    src_path = HIP_DIR / src
+    obj_path = BUILD_DIR / (src_path.stem + ".o")
+    inputs = [src_path, Path(__file__), *HEADERS]
+    if not obj_path.exists() or any(
+        obj_path.stat().st_mtime < p.stat().st_mtime for p in inputs
+    ):
+        cmd = [
+            HIPCC,
+            f"--offload-arch={OFFLOAD_ARCH}",
+            "-O3",
+            "-std=c++17",
+            "-fPIC",
+            # the packed fp32 instructions are not reliable on this part
+            "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
+            "-c",
+            str(src_path),
+            "-o",
+            str(obj_path),
+        ]
+        print("[hipcc]", " ".join(cmd), flush=True)
+        subprocess.check_call(cmd)
+    return str(obj_path)
 
 
 def compile_hip_objects() -> list:
     BUILD_DIR.mkdir(parents=True, exist_ok=True)
-    objs = []
-    for src in KERNEL_SOURCES:
-        src_path = HIP_DIR / src
-        obj_path = BUILD_DIR / (src_path.stem + ".o")
-        if (
-            not obj_path.exists()
-            or obj_path.stat().st_mtime < src_path.stat().st_mtime
-            or obj_path.stat().st_mtime < (HIP_DIR / "decode_kernels.h").stat().st_mtime
-        ):
-            cmd = [
-                HIPCC,
-                f"--offload-arch={OFFLOAD_ARCH}",
-                "-O3",
-                "-std=c++17",
-                "-fPIC",
-                "-c",
-                str(src_path),
-                "-o",
-                str(obj_path),
-            ]
-            print("[hipcc]", " ".join(cmd), flush=True)
-            subprocess.check_call(cmd)
-        objs.append(str(obj_path))
-    return objs
+    with ThreadPoolExecutor(max_workers=8) as pool:
+        return list(pool.map(compile_one, KERNEL_SOURCES))
+
+
+HIP_OBJECTS = compile_hip_objects()
 
 
 def torch_lib_dir() -> str:
@@ -66,7 +74,9 @@ def torch_lib_dir() -> str:
 ext = CppExtension(
     name="mdi_llm_amd._hip_ops",
     sources=[str(HIP_DIR / "bindings.cpp")],
-    extra_objects=compile_hip_objects(),
+    extra_objects=HIP_OBJECTS,
+    # relink when an object changes, not only when the bindings do
+    depends=[*HIP_OBJECTS, *map(str, HEADERS)],
     include_dirs=[os.path.join(ROCM_HOME, "include")],
     library_dirs=[os.path.join(ROCM_HOME, "lib"), torch_lib_dir()],
     libraries=["amdhip64", "c10_hip", "torch_hip"],

@@ -1,6 +1,6 @@
 """Converter round trips (HF -> lit -> HF) for the neox/gpt2/phi families
-(VERDICT item 9; reference convert_lit_checkpoint.py:15-214) and the
-bounded-RAM streaming conversion (VERDICT item 5; reference streams via
+(reference convert_lit_checkpoint.py:15-214) and the
+bounded-RAM streaming conversion (reference streams via
 litgpt_utils.py:304-343 — here via IncrementalSaver)."""
 
 import json

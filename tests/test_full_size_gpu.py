@@ -1,4 +1,4 @@
-"""Full-size numerics on the GPU (VERDICT round-1 item 7): random-init
+"""Full-size numerics on the GPU: random-init
 Llama-3-8B, HIP engine vs the torch stage — per-step logits within bf16
 tolerance and 32-token greedy agreement.  Runs on one MI355X (two 16 GB
 bf16 copies fit easily in 288 GB)."""

@@ -118,8 +118,7 @@ def test_staged_forward_matches_full_model():
     ("TinyLlama-1.1B-Chat-v1.0", 3),
 ])
 def test_balanced_split_byte_balance(model, n_nodes):
-    """Analytic validation of the byte-balance objective (round-1 weak
-    #7): per-stage streamed bytes (blocks + the starter's lm_head) stay
+    """Analytic validation of the byte-balance objective: per-stage streamed bytes (blocks + the starter's lm_head) stay
     within ~1.3 per-layer quanta of each other — the best achievable at
     integer block granularity — so no stage is a >15% straggler on the
     bandwidth-bound decode."""

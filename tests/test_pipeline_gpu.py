@@ -5,7 +5,7 @@ device), each running the HIP DecodeEngine with hipGraph replays.
 Proves on-GPU what tests/test_pipeline_cpu.py proves on CPU: the pipelined
 generation (fused starter graph + ring hops + in-band stops) produces
 exactly the tokens of standalone generation, and the scheduled
-(headerless) bench path matches too.  the
+(headerless) bench path matches too.  The
 interaction of graph replays with ring recv ordering and per-slot
 send-buffer reuse, exercised on the GPU.
 
