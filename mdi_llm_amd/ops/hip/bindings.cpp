@@ -66,7 +66,7 @@ void gemv(torch::Tensor out, torch::Tensor W, torch::Tensor x,
           int64_t epilogue, c10::optional<torch::Tensor> norm_w,
           c10::optional<torch::Tensor> norm_b, int64_t norm_kind,
           double eps, int64_t rows, c10::optional<torch::Tensor> eidx,
-          int64_t estride) {
+          int64_t estride, double act_p, double act_q) {
   check_bf16(out, "out");
   check_bf16(W, "W");
   check_bf16(x, "x");
@@ -82,6 +82,7 @@ void gemv(torch::Tensor out, torch::Tensor W, torch::Tensor x,
     TORCH_CHECK(W.numel() == (int64_t)M * K, "W shape mismatch");
   }
   TORCH_CHECK(K % 8 == 0, "K must be a multiple of 8");
+  TORCH_CHECK(epilogue != 4 || norm_kind != 2, "xielu: no LayerNorm form");
   const void* bp = nullptr;
   const void* rp = nullptr;
   const void* nwp = nullptr;
@@ -107,7 +108,8 @@ void gemv(torch::Tensor out, torch::Tensor W, torch::Tensor x,
   }
   launch_gemv(out.data_ptr(), W.data_ptr(), x.data_ptr(), bp, rp, nwp, nbp,
               (float)eps, M, K, (int)epilogue, (int)norm_kind, (int)rows,
-              eip, (long long)estride, cur_stream());
+              eip, (long long)estride, (float)act_p, (float)act_q,
+              cur_stream());
 }
 
 void gemv_fp8(torch::Tensor out, torch::Tensor W, torch::Tensor wscale,
@@ -568,8 +570,11 @@ void add(torch::Tensor out, torch::Tensor a, torch::Tensor b) {
 
 }  // namespace
 
+void bind_hybrid(py::module_& m);  // hybrid_bindings.cpp
+
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.doc() = "mdi_llm_amd hand-written CDNA4 (gfx950) decode kernels";
+  bind_hybrid(m);
   m.def("rmsnorm", &rmsnorm, "RMSNorm (decode, bf16)");
   m.def("layernorm", &layernorm, "LayerNorm (decode, bf16)");
   m.def("gemv", &gemv, "decode GEMV out = W@norm?(x) (+bias)(+res)(act)",
@@ -578,7 +583,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         py::arg("norm_w") = c10::nullopt, py::arg("norm_b") = c10::nullopt,
         py::arg("norm_kind") = 0, py::arg("eps") = 1e-5,
         py::arg("rows") = 0, py::arg("eidx") = c10::nullopt,
-        py::arg("estride") = 0);
+        py::arg("estride") = 0, py::arg("act_p") = 0.0,
+        py::arg("act_q") = 0.0);
   m.def("gemv_fp8", &gemv_fp8,
         "decode GEMV with fp8(e4m3) weights + per-row scales",
         py::arg("out"), py::arg("W"), py::arg("wscale"), py::arg("x"),

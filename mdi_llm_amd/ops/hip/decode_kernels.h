@@ -12,7 +12,8 @@ void launch_rmsnorm(void* out, const void* x, const void* w, int n, float eps,
 void launch_layernorm(void* out, const void* x, const void* w, const void* b,
                       int n, float eps, hipStream_t stream);
 
-// epilogue: 0 none, 1 +res, 2 gelu(tanh), 3 silu
+// epilogue: 0 none, 1 +res, 2 gelu(tanh), 3 silu, 4 xielu(act_p, act_q)
+// (4 has no LayerNorm form)
 // norm_kind: 0 none, 1 fused RMSNorm on x, 2 fused LayerNorm on x
 // rows: output rows per wave (1/2/4); 0 = auto by M
 // eidx/estride (optional): W += eidx[0]*estride at replay time — selects
@@ -21,8 +22,8 @@ void launch_layernorm(void* out, const void* x, const void* w, const void* b,
 void launch_gemv(void* out, const void* W, const void* x, const void* bias,
                  const void* res, const void* norm_w, const void* norm_b,
                  float eps, int M, int K, int epilogue, int norm_kind,
-                 int rows, const int* eidx, long long estride,
-                 hipStream_t stream);
+                 int rows, const int* eidx, long long estride, float act_p,
+                 float act_q, hipStream_t stream);
 
 // fp8(e4m3)-weight variants: W is bytes, wscale fp32 per output row
 void launch_gemv_fp8(void* out, const void* W, const float* wscale,

@@ -232,11 +232,16 @@ __global__ void layernorm_kernel(bf16* __restrict__ out,
 // kernel + a global round-trip per call): after staging raw x, the block
 // reduces mean/meansq and rewrites LDS with the normalized+weighted value.
 // NORM: 0 none, 1 RMSNorm, 2 LayerNorm.
-// EPI:  0 none, 1 +residual, 2 gelu(tanh), 3 silu.
+// EPI:  0 none, 1 +residual, 2 gelu(tanh), 3 silu, 4 xielu(act_p, act_q).
 // ---------------------------------------------------------------------------
 DEVINL float gelu_tanh(float v) {
   float c = 0.7978845608028654f * (v + 0.044715f * v * v * v);
   return 0.5f * v * (1.f + tanhf(c));
+}
+
+// z/2 plus p z^2 above zero, (1/2 + q)(e^z - 1 - z) below
+DEVINL float xielu(float z, float p, float q) {
+  return 0.5f * z + (z > 0.f ? p * z * z : (0.5f + q) * (expm1f(z) - z));
 }
 
 // Stage x into LDS, optionally fusing the pre-norm.  Returns a uniform
@@ -419,7 +424,8 @@ __global__ void gemv_direct_kernel(bf16* __restrict__ out,
                                    const bf16* __restrict__ nw, float eps,
                                    int M, int K,
                                    const int* __restrict__ eidx,
-                                   long long estride) {
+                                   long long estride, float act_p,
+                                   float act_q) {
   static_assert(NORM == 0 || NORM == 1, "direct gemv: no LayerNorm");
   if (eidx != nullptr) W += (size_t)eidx[0] * (size_t)estride;
   const int tid = threadIdx.x;
@@ -492,6 +498,7 @@ __global__ void gemv_direct_kernel(bf16* __restrict__ out,
         if (EPI == 1 && res != nullptr) a += b2f(res[rw]);
         if (EPI == 2) a = gelu_tanh(a);
         if (EPI == 3) a = a / (1.f + expf(-a));
+        if (EPI == 4) a = xielu(a, act_p, act_q);
         out[rw] = f2b(a);
       }
     }
@@ -3186,8 +3193,8 @@ void launch_layernorm(void* out, const void* x, const void* w, const void* b,
 void launch_gemv(void* out, const void* W, const void* x, const void* bias,
                  const void* res, const void* norm_w, const void* norm_b,
                  float eps, int M, int K, int epilogue, int norm_kind,
-                 int rows, const int* eidx, long long estride,
-                 hipStream_t stream) {
+                 int rows, const int* eidx, long long estride, float act_p,
+                 float act_q, hipStream_t stream) {
   const int smem = K * sizeof(bf16);
   if (rows == 0) rows = M >= 32768 ? 4 : (M > 8192 ? 2 : 1);
   dim3 grid(gemv_grid(M, 4 * rows)), block(256);
@@ -3222,13 +3229,13 @@ void launch_gemv(void* out, const void* W, const void* x, const void* bias,
                          grid, block, 0, stream, (bf16*)out,                \
                          (const bf16*)W, (const bf16*)x, (const bf16*)bias, \
                          (const bf16*)res, (const bf16*)norm_w, eps, M, K,  \
-                         eidx, estride);                                    \
+                         eidx, estride, act_p, act_q);                      \
     else if (N != 2)                                                        \
       hipLaunchKernelGGL((gemv_direct_kernel<E, N == 2 ? 0 : N, R, 2>),     \
                          grid, block, 0, stream, (bf16*)out,                \
                          (const bf16*)W, (const bf16*)x, (const bf16*)bias, \
                          (const bf16*)res, (const bf16*)norm_w, eps, M, K,  \
-                         eidx, estride);                                    \
+                         eidx, estride, act_p, act_q);                      \
     else                                                                    \
       hipLaunchKernelGGL((gemv_kernel<E, N, R>), grid, block, smem, stream, \
                          (bf16*)out, (const bf16*)W, (const bf16*)x,        \
@@ -3255,6 +3262,8 @@ void launch_gemv(void* out, const void* W, const void* x, const void* bias,
     case 12: GEMV_CASE(3, 0); break;
     case 13: GEMV_CASE(3, 1); break;
     case 14: GEMV_CASE(3, 2); break;
+    case 16: GEMV_CASE(4, 0); break;
+    case 17: GEMV_CASE(4, 1); break;
     default: GEMV_CASE(0, 0);
   }
 #undef GEMV_CASE

@@ -29,8 +29,10 @@ ROCM_HOME = os.environ.get("ROCM_HOME", os.environ.get("ROCM_PATH", "/opt/rocm")
 HIPCC = os.path.join(ROCM_HOME, "bin", "hipcc")
 OFFLOAD_ARCH = os.environ.get("PYTORCH_ROCM_ARCH", "gfx950").split(";")[0]
 
-KERNEL_SOURCES = ["decode_kernels.hip"]
-HEADERS = [HIP_DIR / "decode_kernels.h"]
+KERNEL_SOURCES = ["decode_kernels.hip", "hybrid_kernels.hip",
+                  "paged_attn_bf16.hip", "paged_attn_f32.hip"]
+HEADERS = [HIP_DIR / h for h in ("decode_kernels.h", "hybrid_kernels.h",
+                                 "hybrid_common.h", "paged_attn.inc")]
 
 
 def compile_one(src: str) -> str:
@@ -73,7 +75,8 @@ def torch_lib_dir() -> str:
 
 ext = CppExtension(
     name="mdi_llm_amd._hip_ops",
-    sources=[str(HIP_DIR / "bindings.cpp")],
+    sources=[str(HIP_DIR / "bindings.cpp"),
+             str(HIP_DIR / "hybrid_bindings.cpp")],
     extra_objects=HIP_OBJECTS,
     # relink when an object changes, not only when the bindings do
     depends=[*HIP_OBJECTS, *map(str, HEADERS)],
