@@ -14,13 +14,15 @@ init RPC serializes configs, as the reference does via ``asdict``).
 from __future__ import annotations
 
 import copy
+import json
 from dataclasses import dataclass, field, asdict
 from pathlib import Path
 from typing import Any, Literal, Optional, Union
 
 import yaml
 
-__all__ = ["ModelConfig", "name_to_config", "configs"]
+__all__ = ["ModelConfig", "name_to_config", "configs",
+           "native_architectures", "is_native_checkpoint"]
 
 
 def find_multiple(n: int, k: int) -> int:
@@ -52,9 +54,8 @@ class ModelConfig:
     shared_attention_norm: bool = False
     norm_class_name: Literal["LayerNorm", "RMSNorm"] = "LayerNorm"
     norm_eps: float = 1e-5
-    mlp_class_name: Literal["GptNeoxMLP", "LLaMAMLP", "GemmaMLP", "LLaMAMoE"] = (
-        "GptNeoxMLP"
-    )
+    mlp_class_name: Literal["GptNeoxMLP", "LLaMAMLP", "GemmaMLP", "LLaMAMoE",
+                            "XieluMLP"] = "GptNeoxMLP"
     gelu_approximate: str = "none"
     intermediate_size: Optional[int] = None
     rope_condense_ratio: int = 1
@@ -65,8 +66,19 @@ class ModelConfig:
     scale_embeddings: bool = False
     # "rope" (default) or "learned" (GPT-2-style wpe table).
     pos_embedding: Literal["rope", "learned"] = "rope"
+    # -- stacks whose layers differ (models/hybrid.py) --
+    # one entry per layer: {"type": mixer, "mixer": {sizes and constants},
+    # "mlp": {"kind", "ff"} or None}; None means n_layer equal blocks
+    layers: Optional[list] = None
+    embedding_scale: float = 1.0
+    # RMS norm weights are stored as w with norm_offset + w applied
+    norm_offset: float = 0.0
+    # a second norm on each sublayer's output, before the residual add
+    post_norms: bool = False
 
     def __post_init__(self) -> None:
+        if self.layers is not None:
+            self._sizes_from_layers()
         if not self.name:
             self.name = self.hf_config.get("name", "")
         if self.head_size is None:
@@ -87,6 +99,51 @@ class ModelConfig:
                 )
             self.intermediate_size = 4 * self.n_embd
         self.rope_n_elem = int(self.rotary_percentage * self.head_size)
+
+    def _sizes_from_layers(self) -> None:
+        """Fill the uniform-stack fields from the layer list, so that code
+        which only sizes or splits a model need not know about it."""
+        first = self.layers[0]["mixer"]
+        self.n_layer = len(self.layers)
+        self.n_head = first["heads"]
+        self.n_query_groups = first.get("kv_heads", first["heads"])
+        self.head_size = first["dim"]
+        self.intermediate_size = max(
+            (l["mlp"]["ff"] for l in self.layers if l["mlp"]), default=0
+        )
+        self.rotary_percentage = 0.0
+        self.parallel_residual = False
+        self.bias = False
+
+    @property
+    def is_hybrid(self) -> bool:
+        return self.layers is not None
+
+    def residual_dtype(self, dtype):
+        """Type of the residual stream (and of what the ring carries) in a
+        model of the given dtype."""
+        import torch
+
+        return torch.float32 if self.is_hybrid else dtype
+
+    def layer_weights(self, i: int) -> int:
+        """Number of matrix weights of layer ``i``."""
+        E = self.n_embd
+        if self.layers is None:
+            mats = 2 if self.mlp_class_name == "GptNeoxMLP" else 3
+            return (E * self.qkv_dim + E * self.n_head * self.head_size
+                    + mats * E * self.intermediate_size)
+        layer = self.layers[i]
+        m = layer["mixer"]
+        if layer["type"] == "attention":
+            rows = (m["heads"] + m["kv_heads"]) * m["dim"] \
+                + m["kv_heads"] * m["vdim"]
+        else:
+            rows = m["heads"] * (2 * m["dim"] + m["vdim"])
+        rows += m["heads"] * m["vdim"]
+        if layer["mlp"]:
+            rows += 2 * layer["mlp"]["ff"]
+        return E * rows
 
     # -- derived sizes ----------------------------------------------------
     @property
@@ -128,9 +185,19 @@ class ModelConfig:
         cfg_file = path / "model_config.yaml"
         if cfg_file.is_file():
             return cls.from_file(cfg_file, **overrides)
+        if is_native_checkpoint(path):
+            raw = json.loads((path / "config.json").read_text())
+            return cls.from_native(raw, **overrides)
         if (conf_name := path.name) in name_to_config:
             return cls.from_name(conf_name, **overrides)
         raise FileNotFoundError(f"no model_config.yaml in {path} and {path.name!r} unknown")
+
+    @classmethod
+    def from_native(cls, raw: dict, **overrides: Any) -> "ModelConfig":
+        """From a parsed config.json that names its ``architecture``."""
+        conf = native_architectures[raw["architecture"]](raw)
+        conf.update(overrides)
+        return cls(**conf)
 
     @classmethod
     def from_dict(cls, d: dict) -> "ModelConfig":
@@ -145,6 +212,51 @@ class ModelConfig:
     def save(self, path: Union[str, Path]) -> None:
         with open(path, "w", encoding="utf-8") as fp:
             yaml.safe_dump(self.to_dict(), fp)
+
+
+########################################################################
+# Architectures with a config.json of their own
+########################################################################
+
+
+def _nerozen(raw: dict) -> dict:
+    """Nerozen: HGRN2 and biased-window attention layers in any order,
+    norms around each sublayer, xIELU feed-forwards."""
+    for layer in raw["layers"]:
+        if layer["type"] not in ("hgrn2", "attention"):
+            raise ValueError(f"Nerozen: unknown mixer {layer['type']!r}")
+        if layer["mlp"] is not None and layer["mlp"]["kind"] != "dense":
+            raise ValueError(
+                f"Nerozen: unknown feed-forward {layer['mlp']['kind']!r}")
+    return dict(
+        name="Nerozen",
+        # positions are unlimited; this only bounds what serving allots
+        block_size=32768,
+        vocab_size=raw["vocab"],
+        padded_vocab_size=raw["vocab"],
+        n_embd=raw["width"],
+        layers=copy.deepcopy(raw["layers"]),
+        embedding_scale=raw["embedding"]["scale"],
+        norm_class_name="RMSNorm",
+        norm_eps=raw["norm"]["eps"],
+        norm_offset=1.0,
+        post_norms=True,
+        mlp_class_name="XieluMLP",
+    )
+
+
+native_architectures = {"Nerozen": _nerozen}
+
+
+def is_native_checkpoint(path: Union[str, Path]) -> bool:
+    """A folder with config.json + model.safetensors whose config names an
+    architecture of this table (Hugging Face configs have ``architectures``)."""
+    path = Path(path)
+    if not ((path / "config.json").is_file()
+            and (path / "model.safetensors").is_file()):
+        return False
+    raw = json.loads((path / "config.json").read_text())
+    return raw.get("architecture") in native_architectures
 
 
 ########################################################################
@@ -2023,6 +2135,48 @@ configs.extend([
         n_embd=4096,
         rope_base=10000,
     ),
+])
+
+# -- Nerozen -----------------------------------------------------
+
+
+def _nerozen_named(name: str, n_layer: int, width: int, ff: int, vocab: int,
+                   hgrn2: dict, attention: dict, every: int,
+                   block_size: int) -> dict:
+    """A Nerozen stack with attention in every ``every``-th layer."""
+    layers = [
+        dict(type="attention" if i % every == every - 1 else "hgrn2",
+             mixer=dict(attention if i % every == every - 1 else hgrn2),
+             mlp=dict(kind="dense", ff=ff))
+        for i in range(n_layer)
+    ]
+    conf = _nerozen(dict(vocab=vocab, width=width, layers=layers,
+                         embedding=dict(scale=1.0), norm=dict(eps=1e-6)))
+    conf.update(name=name, block_size=block_size)
+    return conf
+
+
+def _nerozen_attention(heads: int, kv_heads: int, dim: int, size: int) -> dict:
+    return dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim,
+                scale=dim ** -0.5, bias_max=size,
+                mask=dict(size=size, keep_first=16))
+
+
+configs.extend([
+    _nerozen_named("nerozen-nano", 4, 128, 320, 384,
+                   dict(heads=4, dim=16, vdim=32),
+                   dict(heads=6, kv_heads=2, dim=32, vdim=32, scale=0.2,
+                        bias_max=100, mask=dict(size=72, keep_first=3)),
+                   every=2, block_size=1024),
+    # TinyLlama-1.1B and Llama-3-8B widths, one attention layer in four
+    _nerozen_named("nerozen-1b", 22, 2048, 6656, 32000,
+                   dict(heads=16, dim=128, vdim=128),
+                   _nerozen_attention(32, 4, 64, 1024), every=4,
+                   block_size=32768),
+    _nerozen_named("nerozen-8b", 32, 4096, 18432, 128256,
+                   dict(heads=32, dim=128, vdim=128),
+                   _nerozen_attention(32, 8, 128, 2048), every=4,
+                   block_size=32768),
 ])
 
 

@@ -1,0 +1,149 @@
+"""Sequence cache of hybrid stacks: paged K/V plus recurrent state slots.
+
+``model.KVCachePool`` gives every slot ``max_seq`` rows.  Here the K/V rows
+of all sequences share one pool of 64-token pages, taken as a sequence grows
+and given back when it ends, and each recurrent layer has one fixed-size
+state per slot.  One page table serves all attention layers of the stage:
+page ``p`` is row ``p`` of every layer's arena.
+
+Layout (what the kernels in ``paged_attn.inc`` and ``hybrid_kernels.hip``
+read): K pages ``[pages, kv_heads, 64, dpad]``, V pages transposed
+``[pages, kv_heads, vpad, 64]``, states ``[slots, heads, dim, vstride]`` in
+fp32.  Padding is zero and stays zero.  A state needs no clearing when its
+slot is taken again: kernels start from zero at position 0.
+"""
+
+from __future__ import annotations
+
+from typing import Dict, List, Optional, Sequence
+
+import torch
+
+__all__ = ["HybridCache", "CacheFull", "PAGE"]
+
+PAGE = 64
+
+
+class CacheFull(RuntimeError):
+    """No free slot, or not enough free pages."""
+
+
+def _pad_to(n: int, sizes: Sequence[int], what: str) -> int:
+    for s in sizes:
+        if n <= s:
+            return s
+    raise ValueError(f"{what} {n} is larger than {sizes[-1]}")
+
+
+class HybridCache:
+    """``n_tokens`` bounds the rows of all live sequences together, each
+    rounded up to whole pages.  One further slot with a page of its own (the
+    spare) absorbs the padding entries of fixed-size decode batches."""
+
+    fp8 = False
+
+    def __init__(self, mixers, n_slots: int, n_tokens: int,
+                 device: torch.device, dtype: torch.dtype) -> None:
+        self.n_slots = n_slots
+        self.n_pages = max(1, -(-n_tokens // PAGE))
+        self.spare = n_slots
+        self.device = device
+        self.dtype = dtype
+        self.k: Dict[int, torch.Tensor] = {}
+        self.v: Dict[int, torch.Tensor] = {}
+        self.state: Dict[int, torch.Tensor] = {}
+        for i, m in enumerate(mixers):
+            if m.kind == "attention":
+                dpad = _pad_to(m.dim, (32, 64, 128, 256), "attention dim")
+                vpad = _pad_to(m.vdim, (32, 64, 128, 256), "attention vdim")
+                P, G = self.n_pages + 1, m.kv_heads
+                self.k[i] = torch.zeros(P, G, PAGE, dpad, device=device,
+                                        dtype=dtype)
+                self.v[i] = torch.zeros(P, G, vpad, PAGE, device=device,
+                                        dtype=dtype)
+            else:
+                vstride = -(-m.vdim // 4) * 4
+                self.state[i] = torch.zeros(
+                    n_slots + 1, m.heads, m.dim, vstride, device=device,
+                    dtype=torch.float32)
+        # the spare slot's only page is the last one
+        self.table = torch.zeros(n_slots + 1, self.n_pages, device=device,
+                                 dtype=torch.int32)
+        self.table[self.spare] = self.n_pages
+        self._free_pages: List[int] = list(range(self.n_pages))[::-1]
+        self._free_slots: List[int] = list(range(n_slots))[::-1]
+        self._pages: List[Optional[List[int]]] = [None] * n_slots
+        self.length = [0] * n_slots
+
+    # -- slots ------------------------------------------------------------
+    @property
+    def free_slots(self) -> int:
+        return len(self._free_slots)
+
+    @property
+    def free_pages(self) -> int:
+        return len(self._free_pages)
+
+    @staticmethod
+    def pages_for(n_tokens: int) -> int:
+        return -(-n_tokens // PAGE)
+
+    def is_live(self, slot: int) -> bool:
+        return self._pages[slot] is not None
+
+    def admit(self, slot: Optional[int] = None) -> int:
+        """Start a sequence in a free slot (a given one, if asked)."""
+        if slot is None:
+            if not self._free_slots:
+                raise CacheFull("no free sequence slot")
+            slot = self._free_slots.pop()
+        else:
+            if self.is_live(slot):
+                raise ValueError(f"slot {slot} is in use")
+            self._free_slots.remove(slot)
+        self._pages[slot] = []
+        self.length[slot] = 0
+        return slot
+
+    def release(self, slot: int) -> None:
+        """End the slot's sequence; its pages can be used again."""
+        if not self.is_live(slot):
+            raise ValueError(f"slot {slot} is not in use")
+        self._free_pages.extend(reversed(self._pages[slot]))
+        self._pages[slot] = None
+        self.length[slot] = 0
+        self._free_slots.append(slot)
+
+    def reset(self, slot: Optional[int] = None) -> None:
+        for s in range(self.n_slots) if slot is None else (slot,):
+            if self.is_live(s):
+                self.release(s)
+
+    def missing_pages(self, slot: int, n_new: int) -> int:
+        return max(0, self.pages_for(self.length[slot] + n_new)
+                   - len(self._pages[slot]))
+
+    def extend(self, extra: Dict[int, int]) -> None:
+        """Make room for ``extra[slot]`` more tokens in each slot, all or
+        nothing, and count them as stored."""
+        need = {s: self.missing_pages(s, n) for s, n in extra.items()}
+        if sum(need.values()) > len(self._free_pages):
+            raise CacheFull(
+                f"{sum(need.values())} pages needed, "
+                f"{len(self._free_pages)} free")
+        rows, cols, pages = [], [], []
+        for s, n in need.items():
+            for _ in range(n):
+                page = self._free_pages.pop()
+                rows.append(s)
+                cols.append(len(self._pages[s]))
+                pages.append(page)
+                self._pages[s].append(page)
+            self.length[s] += extra[s]
+        if pages:
+            idx = torch.tensor([rows, cols, pages]).to(self.device)
+            self.table[idx[0], idx[1]] = idx[2].to(torch.int32)
+
+    def memory_bytes(self) -> int:
+        return sum(t.numel() * t.element_size()
+                   for d in (self.k, self.v, self.state) for t in d.values())

@@ -420,6 +420,10 @@ class GPT(nn.Module):
     def __init__(self, config: ModelConfig) -> None:
         super().__init__()
         assert config.padded_vocab_size is not None
+        if config.is_hybrid:
+            raise ValueError(
+                f"{config.name!r} is a hybrid stack: build it as pipeline "
+                "stages (models.stages), one stage for the whole model")
         self.config = config
         self.lm_head = nn.Linear(
             config.n_embd, config.padded_vocab_size, bias=config.lm_head_bias

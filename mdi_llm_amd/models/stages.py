@@ -23,6 +23,8 @@ import torch
 import torch.nn as nn
 
 from ..config import ModelConfig
+from .cache import HybridCache
+from .hybrid import HybridBlock, Scale
 from .model import Block, KVCachePool, build_rope_cache, norm_class
 
 __all__ = ["StageBase", "StarterStage", "SecondaryStage", "build_stage"]
@@ -31,13 +33,22 @@ __all__ = ["StageBase", "StarterStage", "SecondaryStage", "build_stage"]
 class StageBase(nn.Module):
     """Shared RoPE / KV-pool machinery for pipeline stages."""
 
-    def __init__(self, config: ModelConfig, n_local_layers: int) -> None:
+    def __init__(self, config: ModelConfig, n_local_layers: int,
+                 first_layer: int = 0) -> None:
         super().__init__()
         self.config = config
         self.n_local_layers = n_local_layers
+        self.first_layer = first_layer
         self.kv_pool: Optional[KVCachePool] = None
         self._max_seq_length = config.block_size
         self._build_rope()
+
+    def _make_blocks(self) -> nn.ModuleList:
+        cls = HybridBlock if self.config.is_hybrid else Block
+        return nn.ModuleList(
+            cls(self.config, self.first_layer + i)
+            for i in range(self.n_local_layers)
+        )
 
     # -- rope -------------------------------------------------------------
     def _build_rope(self) -> None:
@@ -87,11 +98,20 @@ class StageBase(nn.Module):
         n_slots: int,
         device: Optional[torch.device] = None,
         dtype: Optional[torch.dtype] = None,
+        n_tokens: Optional[int] = None,
     ) -> None:
+        """``n_tokens`` sizes the paged pool of a hybrid stack (all slots
+        together); other stacks hold ``max_seq_length`` rows per slot."""
         if device is None:
             device = next(self.parameters()).device
         if dtype is None:
             dtype = next(self.parameters()).dtype
+        if self.config.is_hybrid:
+            self.kv_pool = HybridCache(
+                [b.mixer for b in self.transformer.h], n_slots,
+                n_tokens or n_slots * self._max_seq_length,
+                device, dtype)
+            return
         self.kv_pool = KVCachePool(
             n_slots,
             self.n_local_layers,
@@ -124,8 +144,9 @@ class StarterStage(StageBase):
         super().__init__(config, n_local_layers)
         modules = dict(
             wte=nn.Embedding(config.padded_vocab_size, config.n_embd),
-            h=nn.ModuleList(Block(config, i) for i in range(n_local_layers)),
-            ln_f=norm_class(config)(config.n_embd),
+            h=self._make_blocks(),
+            ln_f=(Scale(config.n_embd) if config.is_hybrid
+                  else norm_class(config)(config.n_embd)),
         )
         if config.pos_embedding == "learned":
             modules["wpe"] = nn.Embedding(config.block_size, config.n_embd)
@@ -163,15 +184,10 @@ class StarterStage(StageBase):
 class SecondaryStage(StageBase):
     """A run of middle blocks (chunk ``model_secondary<i>.pth``)."""
 
-    def __init__(self, config: ModelConfig, n_local_layers: int) -> None:
-        super().__init__(config, n_local_layers)
-        self.transformer = nn.ModuleDict(
-            dict(
-                h=nn.ModuleList(
-                    Block(config, i) for i in range(n_local_layers)
-                )
-            )
-        )
+    def __init__(self, config: ModelConfig, n_local_layers: int,
+                 first_layer: int = 0) -> None:
+        super().__init__(config, n_local_layers, first_layer)
+        self.transformer = nn.ModuleDict(dict(h=self._make_blocks()))
 
     def forward(
         self, x: torch.Tensor, slot: int, input_pos: int
@@ -180,8 +196,11 @@ class SecondaryStage(StageBase):
 
 
 def build_stage(
-    config: ModelConfig, stage: int, n_local_layers: int
+    config: ModelConfig, stage: int, n_local_layers: int,
+    first_layer: int = 0,
 ) -> StageBase:
+    """``first_layer``: the model-wide index of the stage's first block
+    (only stacks whose layers differ look at it)."""
     if stage == 0:
         return StarterStage(config, n_local_layers)
-    return SecondaryStage(config, n_local_layers)
+    return SecondaryStage(config, n_local_layers, first_layer)

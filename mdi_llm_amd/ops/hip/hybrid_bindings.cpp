@@ -252,30 +252,14 @@ void paged_attn(torch::Tensor out, torch::Tensor q, torch::Tensor kpages,
               a.vpad);
 }
 
-void stage_batch(torch::Tensor slots, torch::Tensor pos_table,
-                 torch::Tensor token_table, torch::Tensor key_table,
-                 torch::Tensor pos, torch::Tensor tokens, torch::Tensor keys,
-                 int64_t spare) {
+void advance_batch(torch::Tensor slots, torch::Tensor sampled,
+                   torch::Tensor pos, torch::Tensor tokens, int64_t spare) {
   const int n = (int)slots.numel();
-  launch_stage_batch(i32_ptr(slots, n, "slots"),
-                     i32_ptr(pos_table, spare + 1, "pos_table"),
-                     i32_ptr(token_table, spare + 1, "token_table"),
-                     i32_ptr(key_table, spare + 1, "key_table"),
-                     const_cast<int*>(i32_ptr(pos, n, "pos")),
-                     const_cast<int*>(i32_ptr(tokens, n, "tokens")),
-                     const_cast<int*>(i32_ptr(keys, n, "keys")), (int)spare,
-                     n, cur_stream());
-}
-
-void advance_batch(torch::Tensor slots, torch::Tensor tokens,
-                   torch::Tensor pos_table, torch::Tensor token_table,
-                   int64_t spare) {
-  const int n = (int)slots.numel();
-  launch_advance_batch(
-      i32_ptr(slots, n, "slots"), i32_ptr(tokens, n, "tokens"),
-      const_cast<int*>(i32_ptr(pos_table, spare + 1, "pos_table")),
-      const_cast<int*>(i32_ptr(token_table, spare + 1, "token_table")),
-      (int)spare, n, cur_stream());
+  launch_advance_batch(i32_ptr(slots, n, "slots"),
+                       i32_ptr(sampled, n, "sampled"),
+                       const_cast<int*>(i32_ptr(pos, n, "pos")),
+                       const_cast<int*>(i32_ptr(tokens, n, "tokens")),
+                       (int)spare, n, cur_stream());
 }
 
 }  // namespace
@@ -314,6 +298,5 @@ void bind_hybrid(py::module_& m) {
         py::arg("max_len"), py::arg("window"), py::arg("keep_first"),
         py::arg("scale"), py::arg("splits"), py::arg("part_o") = none,
         py::arg("part_ml") = none);
-  m.def("stage_batch", &stage_batch, "decode staging from device tables");
   m.def("advance_batch", &advance_batch, "decode bookkeeping");
 }

@@ -84,13 +84,7 @@ struct PagedAttnArgs {
 int launch_paged_attn_bf16(const PagedAttnArgs& a, hipStream_t stream);
 int launch_paged_attn_f32(const PagedAttnArgs& a, hipStream_t stream);
 
-// decode staging: pos = pos_table[slot] (0 for the spare slot), token, key
-void launch_stage_batch(const int* slots, const int* pos_table,
-                        const int* token_table, const int* key_table,
-                        int* pos, int* tokens, int* keys, int spare, int n,
-                        hipStream_t stream);
-
-// token_table[slot] = token, pos_table[slot] += 1
-void launch_advance_batch(const int* slots, const int* tokens,
-                          int* pos_table, int* token_table, int spare, int n,
-                          hipStream_t stream);
+// Between the steps of an unchanged decode batch: tokens = sampled,
+// pos += 1; entries of the spare slot stay where they are.
+void launch_advance_batch(const int* slots, const int* sampled, int* pos,
+                          int* tokens, int spare, int n, hipStream_t stream);

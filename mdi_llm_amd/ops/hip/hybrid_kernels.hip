@@ -469,40 +469,20 @@ void launch_qk_norm_append(void* q_out, void* kpages, void* vpages,
 }
 
 // ---------------------------------------------------------------------------
-// decode bookkeeping on device tables (graph-replayable)
+// decode bookkeeping (graph-replayable)
 // ---------------------------------------------------------------------------
-__global__ void stage_batch_kernel(const int* slots, const int* pos_table,
-                                   const int* token_table,
-                                   const int* key_table, int* pos,
-                                   int* tokens, int* keys, int spare, int n) {
-  const int i = blockIdx.x * blockDim.x + threadIdx.x;
-  if (i >= n) return;
-  const int s = slots[i];
-  pos[i] = s == spare ? 0 : pos_table[s];
-  tokens[i] = token_table[s];
-  keys[i] = key_table[s];
-}
-
-__global__ void advance_batch_kernel(const int* slots, const int* tokens,
-                                     int* pos_table, int* token_table,
-                                     int spare, int n) {
+__global__ void advance_batch_kernel(const int* slots, const int* sampled,
+                                     int* pos, int* tokens, int spare,
+                                     int n) {
   const int i = blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= n || slots[i] == spare) return;
-  token_table[slots[i]] = tokens[i];
-  pos_table[slots[i]] += 1;
+  tokens[i] = sampled[i];
+  pos[i] += 1;
 }
 
-void launch_stage_batch(const int* slots, const int* pos_table,
-                        const int* token_table, const int* key_table,
-                        int* pos, int* tokens, int* keys, int spare, int n,
-                        hipStream_t stream) {
-  stage_batch_kernel<<<(n + 255) / 256, 256, 0, stream>>>(
-      slots, pos_table, token_table, key_table, pos, tokens, keys, spare, n);
-}
-
-void launch_advance_batch(const int* slots, const int* tokens,
-                          int* pos_table, int* token_table, int spare, int n,
+void launch_advance_batch(const int* slots, const int* sampled, int* pos,
+                          int* tokens, int spare, int n,
                           hipStream_t stream) {
   advance_batch_kernel<<<(n + 255) / 256, 256, 0, stream>>>(
-      slots, tokens, pos_table, token_table, spare, n);
+      slots, sampled, pos, tokens, spare, n);
 }

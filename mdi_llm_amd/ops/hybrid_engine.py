@@ -1,0 +1,522 @@
+"""Step engine of hybrid stacks (``ModelConfig.layers``): one ragged batch
+per step, portions of prompts beside single decoded tokens.
+
+Where ``DecodeEngine`` advances one sequence and ``GroupDecodeEngine`` a
+fixed group, every step here takes any mix of sequences: the rows of all
+entries lie flat in one activation matrix, so a projection is one matrix
+product for the whole step, and the kernels that look at neighbours in time
+(recurrence, attention) walk the entries as segments.  Steps in which every
+entry is one token are captured as hipGraphs per batch size.
+
+The residual stream, norms, gates, recurrent state and softmax are fp32; the
+weights, matrix products and cached K/V have the stage's dtype (bf16, or
+fp32 throughout).
+"""
+
+from __future__ import annotations
+
+import math
+from bisect import bisect_left
+from dataclasses import dataclass
+from fractions import Fraction
+from typing import Dict, List, Optional, Sequence, Tuple
+
+import torch
+import torch.nn.functional as F
+
+from ..config import ModelConfig
+from ..models.cache import PAGE, HybridCache
+from ..models.sampling import sample as sample_token
+from . import require_hip_ops
+from .engine import DecodeEngine
+
+__all__ = ["HybridEngine", "distance_bias"]
+
+
+def distance_bucket_starts(rows: int, far) -> List[int]:
+    """First distance of each bucket: one per distance below rows/2, then
+    geometric up to ``far``, compared exactly (no logarithms)."""
+    half = rows // 2
+    m = rows - half
+    starts = list(range(half))
+    span = range(half, math.ceil(far) + 1)
+    for k in range(m):
+        # smallest n with (n / half)^m >= (far / half)^k
+        bound = (Fraction(far) / half) ** k * half ** m
+        starts.append(span[bisect_left(span, bound, key=lambda n: n ** m)])
+    return starts
+
+
+def distance_bias(rel: torch.Tensor, far) -> torch.Tensor:
+    """[rows, heads] bucket table -> [heads, n] bias by distance in log2
+    units; distances past the end share the last entry."""
+    rows = rel.size(0)
+    if rows < 2 or far <= rows // 2:
+        raise ValueError("distance buckets: bias_max must exceed rows / 2")
+    starts = distance_bucket_starts(rows, far)
+    bucket = torch.zeros(starts[-1] + 1, dtype=torch.long)
+    for b, s in enumerate(starts):
+        bucket[s:] = b
+    per = rel.detach().double()[bucket.to(rel.device)].t()
+    return (per * math.log2(math.e)).float().contiguous()
+
+
+@dataclass
+class Batch:
+    """Device view of one step."""
+
+    n: int                   # rows
+    seg: torch.Tensor        # [4, entries]: start, len, slot, pos0
+    singles: int             # the first entries of seg are one token long
+    max_len: int
+    row_slot: torch.Tensor
+    row_pos: torch.Tensor
+    tokens: Optional[torch.Tensor]
+    max_ctx: int             # longest sequence, this step included
+
+
+class _LayerWeights:
+    """One layer's operands: matrices as they are, the rest in fp32."""
+
+    def __init__(self, block) -> None:
+        def f(t):
+            return None if t is None else t.detach().float().contiguous()
+
+        def w(norm):
+            return None if norm is None else f(norm.weight)
+
+        self.norm1, self.norm1b = w(block.norm_1), w(block.norm_1b)
+        self.norm2, self.norm2b = w(block.norm_2), w(block.norm_2b)
+        m = block.mixer
+        self.mixer = m
+        self.in_proj = m.in_proj.weight.detach()
+        self.proj = m.proj.weight.detach()
+        if m.kind == "hgrn2":
+            self.f_bias, self.lower = f(m.f_bias), f(m.lower)
+            self.norm = f(m.norm.weight)
+        else:
+            self.q_norm, self.k_norm = f(m.q_norm.weight), f(m.k_norm.weight)
+            self.bias = distance_bias(m.rel, m.bias_max)
+        self.mlp = block.mlp is not None
+        if self.mlp:
+            self.fc = block.mlp.fc.weight.detach()
+            self.down = block.mlp.proj.weight.detach()
+            self.act = tuple(F.softplus(block.mlp.act.detach().float())
+                             .tolist())
+
+
+class _DecodeStep:
+    """Static buffers and graphs of single-token steps of one batch size."""
+
+    def __init__(self, eng: "HybridEngine", size: int) -> None:
+        dev = eng.device
+        # start, len, slot, pos0 | token, sampling key
+        self.io = torch.zeros(6, size, dtype=torch.int32, device=dev)
+        self.load([], [], [], [], eng.cache.spare)
+        io = self.io
+        self.batch = Batch(size, io[:4], size, 1, io[2], io[3], io[4],
+                           eng.max_ctx)
+        self.sampled = torch.zeros(size, dtype=torch.int32, device=dev)
+        self.scratch = torch.zeros(520 * size, dtype=torch.int32, device=dev)
+        self.logits: Optional[torch.Tensor] = None
+        self.forward_graph = None
+        self.sample_graphs: dict = {}
+        self.slots: List[int] = []
+
+    def load(self, slots, pos, tokens, keys, spare: int) -> None:
+        size = self.io.size(1)
+        pad = [0] * (size - len(slots))
+        rows = [list(range(size)), [1] * size,
+                list(slots) + [spare] * len(pad), list(pos) + pad,
+                list(tokens) + pad, list(keys) + pad]
+        self.io.copy_(torch.tensor(rows, dtype=torch.int32))
+        self.slots = list(slots)
+
+
+class HybridEngine:
+    """Drives one stage (starter or secondary) of a hybrid stack."""
+
+    supports_hip_prefill = True
+
+    def __init__(self, stage, cache: HybridCache,
+                 use_graphs: bool = True) -> None:
+        self.config: ModelConfig = stage.config
+        self.stage = stage
+        self.cache = cache
+        p = next(stage.parameters())
+        self.device, self.dtype = p.device, p.dtype
+        if self.dtype not in (torch.bfloat16, torch.float32):
+            raise ValueError("hybrid stacks run in bfloat16 or float32")
+        self.hip = self.device.type == "cuda"
+        if self.hip:
+            self.ops = require_hip_ops()
+        else:
+            from . import hybrid_torch
+
+            self.ops = hybrid_torch
+        self.use_graphs = use_graphs and self.hip
+        self.is_starter = hasattr(stage, "lm_head")
+        self.layers = [_LayerWeights(b) for b in stage.transformer.h]
+        for lw in self.layers:
+            m = lw.mixer
+            if m.kind == "hgrn2" and (m.dim > 256 or m.vdim > 1024):
+                raise ValueError("hgrn2: dim <= 256 and vdim <= 1024")
+        # longest sequence that can occur
+        self.max_ctx = min(cache.n_pages * PAGE, stage.max_seq_length)
+        if self.is_starter:
+            self.wte = stage.transformer.wte.weight.detach()
+            self.final = stage.transformer.ln_f.weight.detach().float()
+            self.head = stage.lm_head.weight.detach()
+        self._steps: Dict[int, _DecodeStep] = {}
+        self._part: Optional[Tuple[torch.Tensor, torch.Tensor]] = None
+
+    # ------------------------------------------------------------------
+    # building blocks
+    # ------------------------------------------------------------------
+    def _norm_step(self, x, y=None, post_w=None, next_w=None, tokens=None):
+        """x <- embed(tokens) or x + post-norm(y); the next pre-norm."""
+        xn = None
+        if next_w is not None:
+            xn = torch.empty(x.shape, dtype=self.dtype, device=self.device)
+        self.ops.residual_norm(
+            x, y=y, post_w=post_w, xn=xn, next_w=next_w, tokens=tokens,
+            table=None if tokens is None else self.wte,
+            scale=self.config.embedding_scale,
+            offset=self.config.norm_offset, eps=self.config.norm_eps)
+        return xn
+
+    def _linear(self, x: torch.Tensor, w: torch.Tensor, act=None):
+        M, K = w.shape
+        if (x.size(0) == 1 and self.hip and self.dtype == torch.bfloat16
+                and K % 8 == 0):
+            out = torch.empty(1, M, dtype=self.dtype, device=self.device)
+            p, q = act or (0.0, 0.0)
+            self.ops.gemv(out, w, x, None, None, 4 if act else 0,
+                          rows=DecodeEngine._rows(M, K), act_p=p, act_q=q)
+            return out
+        out = F.linear(x, w)
+        if act is not None:
+            self.ops.xielu(out, *act)
+        return out
+
+    def _hgrn2(self, i: int, lw: _LayerWeights, b: Batch, xn: torch.Tensor):
+        m, eps = lw.mixer, self.config.norm_eps
+        proj = self._linear(xn, lw.in_proj)
+        y = torch.empty(b.n, m.heads * m.vdim, dtype=self.dtype,
+                        device=self.device)
+        state = self.cache.state[i]
+        if b.singles:
+            self.ops.hgrn2_step(y, proj, state, lw.f_bias, lw.lower, lw.norm,
+                                b.seg[:, :b.singles], eps)
+        if b.singles < b.seg.size(1):
+            o = torch.empty(y.shape, dtype=torch.float32, device=self.device)
+            self.ops.hgrn2_scan(y, o, proj, state, lw.f_bias, lw.lower,
+                                lw.norm, b.seg[:, b.singles:], b.max_len, eps)
+        return self._linear(y, lw.proj)
+
+    def _splits(self, m, n_seg: int, max_ctx: int) -> int:
+        """Blocks that share the keys of one (sequence, kv head): enough of
+        them to fill the chip, none with less than two tiles a wave."""
+        tiles = min(-(-max_ctx // 32),
+                    -(-m.window // 32) + -(-m.keep_first // 32) + 1)
+        want = -(-512 // (n_seg * m.kv_heads))
+        return max(1, min(want, -(-tiles // 8)))
+
+    def _attention(self, i: int, lw: _LayerWeights, b: Batch,
+                   xn: torch.Tensor):
+        m, eps, c = lw.mixer, self.config.norm_eps, self.cache
+        proj = self._linear(xn, lw.in_proj)
+        k, v = c.k[i], c.v[i]
+        q = torch.empty(b.n, m.heads, k.size(3), dtype=self.dtype,
+                        device=self.device)
+        self.ops.qk_norm_append(q, k, v, proj, lw.q_norm, lw.k_norm,
+                                b.row_slot, b.row_pos, c.table, m.vdim, eps)
+        y = torch.empty(b.n, m.heads * m.vdim, dtype=self.dtype,
+                        device=self.device)
+
+        def attend(seg, max_len, splits, part=(None, None)):
+            self.ops.paged_attn(y, q, k, v, lw.bias, c.table, seg, max_len,
+                                m.window, m.keep_first, m.scale, splits,
+                                *part)
+
+        if b.singles:
+            splits = self._splits(m, b.singles, b.max_ctx)
+            part = (None, None)
+            if splits > 1:
+                cells = b.singles * m.heads * splits
+                part = (torch.empty(cells * v.size(2), dtype=torch.float32,
+                                    device=self.device),
+                        torch.empty(cells * 2, dtype=torch.float32,
+                                    device=self.device))
+            attend(b.seg[:, :b.singles], 1, splits, part)
+        if b.singles < b.seg.size(1):
+            attend(b.seg[:, b.singles:], b.max_len, 0)
+        return self._linear(y, lw.proj)
+
+    def _run(self, b: Batch, x: Optional[torch.Tensor], final: bool,
+             layers_out: Optional[list] = None):
+        """All local layers.  Returns (x, final-normed rows or None)."""
+        norms = [lw.norm1 for lw in self.layers[1:]]
+        norms.append(self.final if final else None)
+        first = self.layers[0].norm1 if self.layers else norms[0]
+        if x is None:
+            x = torch.empty(b.n, self.config.n_embd, dtype=torch.float32,
+                            device=self.device)
+            xn = self._norm_step(x, next_w=first, tokens=b.tokens)
+        else:
+            xn = self._norm_step(x, next_w=first)
+        for i, (lw, after) in enumerate(zip(self.layers, norms)):
+            mix = self._hgrn2 if lw.mixer.kind == "hgrn2" else \
+                self._attention
+            y = mix(i, lw, b, xn)
+            if lw.mlp:
+                xn = self._norm_step(x, y, lw.norm1b, lw.norm2)
+                y = self._linear(self._linear(xn, lw.fc, lw.act), lw.down)
+                xn = self._norm_step(x, y, lw.norm2b, after)
+            else:
+                xn = self._norm_step(x, y, lw.norm1b, after)
+            if layers_out is not None:
+                layers_out.append(x.clone())
+        return x, xn
+
+    # ------------------------------------------------------------------
+    # batches
+    # ------------------------------------------------------------------
+    def _batch(self, entries: Sequence[Tuple[int, int]],
+               tokens: Optional[Sequence[int]]) -> Tuple[Batch, List[int]]:
+        """entries: (slot, rows).  Takes the cache rows and returns the
+        device batch and each entry's first row."""
+        c = self.cache
+        if len({s for s, _ in entries}) != len(entries):
+            raise ValueError("a sequence can be in a step only once")
+        for slot, n in entries:
+            if n < 1:
+                raise ValueError("an entry needs at least one token")
+            if c.length[slot] + n > self.max_ctx:
+                raise ValueError(
+                    f"sequence of {c.length[slot] + n} tokens, at most "
+                    f"{self.max_ctx} fit")
+        pos0 = [c.length[slot] for slot, _ in entries]
+        c.extend({slot: n for slot, n in entries})
+        starts, at = [], 0
+        for _, n in entries:
+            starts.append(at)
+            at += n
+        order = sorted(range(len(entries)), key=lambda e: entries[e][1] > 1)
+        seg = [[starts[e] for e in order], [entries[e][1] for e in order],
+               [entries[e][0] for e in order], [pos0[e] for e in order]]
+        row_slot = [s for s, n in entries for _ in range(n)]
+        row_pos = [p + t for p, (_, n) in zip(pos0, entries)
+                   for t in range(n)]
+        flat = torch.tensor(row_slot + row_pos + sum(seg, [])
+                            + list(tokens or ()), dtype=torch.int32)
+        flat = flat.to(self.device)
+        S = len(entries)
+        b = Batch(
+            n=at,
+            seg=flat[2 * at:2 * at + 4 * S].view(4, S),
+            singles=sum(n == 1 for _, n in entries),
+            max_len=max(n for _, n in entries),
+            row_slot=flat[:at], row_pos=flat[at:2 * at],
+            tokens=flat[2 * at + 4 * S:] if tokens is not None else None,
+            max_ctx=max(p + n for p, (_, n) in zip(pos0, entries)),
+        )
+        return b, starts
+
+    def _check_tokens(self, tokens) -> None:
+        V = self.wte.size(0)
+        if tokens and not (0 <= min(tokens) and max(tokens) < V):
+            raise ValueError(f"token ids must be in [0, {V})")
+
+    # ------------------------------------------------------------------
+    # public steps
+    # ------------------------------------------------------------------
+    @torch.inference_mode()
+    def step(self, entries: Sequence[Tuple[int, Sequence[int]]],
+             want: Optional[Sequence[Sequence[int]]] = None,
+             layers_out: Optional[list] = None) -> Optional[torch.Tensor]:
+        """Run the given tokens of each entry's sequence; ``want[e]`` are the
+        places among entry ``e``'s tokens whose logits are returned (default:
+        the last), in order, as [wanted, vocab]; None if none is wanted."""
+        if want is None:
+            want = [[len(t) - 1] for _, t in entries]
+        tokens = [int(t) for _, ts in entries for t in ts]
+        self._check_tokens(tokens)
+        if (self.use_graphs and layers_out is None
+                and all(len(t) == 1 for _, t in entries)):
+            logits = self.decode([s for s, _ in entries], tokens)
+            rows = [e for e, w in enumerate(want) for _ in w]
+            if not rows:
+                return None
+            return logits if rows == list(range(len(entries))) \
+                else logits[rows]
+        b, starts = self._batch([(s, len(t)) for s, t in entries], tokens)
+        rows = [s + k for s, w in zip(starts, want) for k in w]
+        _, xn = self._run(b, None, bool(rows), layers_out)
+        if not rows:
+            return None
+        if rows != list(range(b.n)):
+            xn = xn[torch.tensor(rows, device=self.device)]
+        return self._linear(xn, self.head)
+
+    @torch.inference_mode()
+    def hidden(self, slot: int, tokens: Optional[Sequence[int]] = None,
+               x: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """Pipeline stages: one sequence's tokens (starter) or residual rows
+        (secondary) -> residual rows after the local layers, fp32."""
+        if tokens is not None:
+            self._check_tokens(tokens)
+        else:
+            x = x.reshape(-1, self.config.n_embd).float().clone()
+        n = len(tokens) if x is None else x.size(0)
+        b, _ = self._batch([(slot, n)], tokens)
+        return self._run(b, x, False)[0]
+
+    @torch.inference_mode()
+    def logits(self, x: torch.Tensor) -> torch.Tensor:
+        """Residual rows -> logits."""
+        x = x.reshape(-1, self.config.n_embd).float().contiguous()
+        return self._linear(self._norm_step(x, next_w=self.final), self.head)
+
+    # ------------------------------------------------------------------
+    # single-token steps (hipGraph per batch size)
+    # ------------------------------------------------------------------
+    def _decode_step(self, n: int) -> _DecodeStep:
+        size = 1
+        while size < n:
+            size *= 2
+        st = self._steps.get(size)
+        if st is not None:
+            return st
+        st = _DecodeStep(self, size)
+
+        def forward():
+            _, xn = self._run(st.batch, None, True)
+            return self._linear(xn, self.head)
+
+        if self.use_graphs:
+            # warm-up and capture run on the spare slot only
+            s = torch.cuda.Stream()
+            s.wait_stream(torch.cuda.current_stream())
+            with torch.cuda.stream(s):
+                forward()
+            torch.cuda.current_stream().wait_stream(s)
+            g = torch.cuda.CUDAGraph()
+            with torch.cuda.graph(g):
+                st.logits = forward()
+            st.forward_graph = g
+        else:
+            st.forward_graph = None
+        st.forward = forward
+        self._steps[size] = st
+        return st
+
+    @torch.inference_mode()
+    def decode(self, slots: Sequence[int],
+               tokens: Optional[Sequence[int]] = None,
+               keys: Optional[Sequence[int]] = None) -> torch.Tensor:
+        """One token for each slot; logits [len(slots), vocab], valid until
+        the next call.  Without ``tokens`` the step continues from what
+        ``sample_decoded`` drew for the same slots, on the device."""
+        c = self.cache
+        slots = list(slots)
+        for s in slots:
+            if c.length[s] + 1 > self.max_ctx:
+                raise ValueError(f"at most {self.max_ctx} tokens fit")
+        st = self._decode_step(len(slots))
+        if tokens is None:
+            if st.slots != slots:
+                raise ValueError("the batch changed: pass its tokens")
+            c.extend({s: 1 for s in slots})
+        else:
+            if len(set(slots)) != len(slots):
+                raise ValueError("a sequence can be in a step only once")
+            pos = [c.length[s] for s in slots]
+            c.extend({s: 1 for s in slots})
+            st.load(slots, pos, [int(t) for t in tokens], keys or slots,
+                    c.spare)
+        if st.forward_graph is not None:
+            st.forward_graph.replay()
+        else:
+            st.logits = st.forward()
+        self._last = st
+        return st.logits[:len(slots)]
+
+    @torch.inference_mode()
+    def sample_decoded(self, temperature: float, top_k, seed: int,
+                       top_p: float = 1.0) -> torch.Tensor:
+        """Draw from the logits of the last ``decode`` on the device (bf16
+        stages) and make the drawn tokens its next input; int32 tokens."""
+        st = self._last
+        key = (float(temperature), int(top_k or 0), int(seed), float(top_p))
+
+        def draw():
+            self._hip_sample(st.sampled, st.logits, st.scratch, key,
+                             st.io[3], st.io[5], 1)
+            self.ops.advance_batch(st.io[2], st.sampled, st.io[3], st.io[4],
+                                   self.cache.spare)
+
+        if not self.use_graphs:
+            draw()
+        else:
+            g = st.sample_graphs.get(key)
+            if g is None:
+                torch.cuda.synchronize()
+                g = torch.cuda.CUDAGraph()
+                with torch.cuda.graph(g):
+                    draw()
+                st.sample_graphs[key] = g
+            g.replay()
+        return st.sampled[:len(st.slots)]
+
+    @property
+    def samples_on_device(self) -> bool:
+        return self.hip and self.dtype == torch.bfloat16
+
+    def _hip_sample(self, out, logits, scratch, key, pos, keys,
+                    pos_bias: int) -> None:
+        t, k, seed, p = key
+        self.ops.sample(out, logits, scratch, t, k, t > 0.0,
+                        seed & 0x7FFFFFFF, pos, keys, logits.size(0), p,
+                        pos_bias=pos_bias)
+
+    @torch.inference_mode()
+    def sample(self, logits: torch.Tensor, temperature: float, top_k, seed,
+               top_p: float, pos: Sequence[int], keys: Sequence[int],
+               generators=None) -> List[int]:
+        """Draw one token per row.  On the device the draw is keyed by
+        (seed, key, position of the drawn token), so it does not depend on
+        the schedule; elsewhere each row has a torch generator."""
+        if self.samples_on_device:
+            n = logits.size(0)
+            pk = torch.tensor([list(pos), list(keys)], dtype=torch.int32)
+            pk = pk.to(self.device)
+            out = torch.zeros(n, dtype=torch.int32, device=self.device)
+            scratch = torch.zeros(520 * n, dtype=torch.int32,
+                                  device=self.device)
+            self._hip_sample(out, logits.contiguous(), scratch,
+                             (float(temperature), int(top_k or 0),
+                              int(seed or 0), float(top_p)), pk[0], pk[1], 0)
+            return out.tolist()
+        return [int(sample_token(
+            row, temperature=temperature, top_k=top_k, top_p=top_p,
+            generator=generators[i] if generators else None))
+            for i, row in enumerate(logits)]
+
+    # ------------------------------------------------------------------
+    # what chat and the runners share with DecodeEngine
+    # ------------------------------------------------------------------
+    def prefill_prompt(self, tokens: torch.Tensor, slot: int,
+                       pos0: int = 0) -> torch.Tensor:
+        c = self.cache
+        if pos0 == 0:
+            if c.is_live(slot):
+                c.release(slot)
+            c.admit(slot)
+        if c.length[slot] != pos0:
+            raise ValueError(
+                f"slot {slot} holds {c.length[slot]} tokens, not {pos0}")
+        return self.hidden(slot, tokens=tokens.reshape(-1).tolist())
+
+    def set_slot_pos(self, slot: int, pos: int) -> None:
+        """Positions live in the cache; nothing to stage."""

@@ -153,7 +153,8 @@ class MDIRuntime:
         client = ControlClient()
         # envelope (pipelined) serve: device-side header routing on GPU
         # secondaries, no per-hop host syncs; MDI_ENV_SERVE=0/1 overrides
-        env_serve = self.device.type == "cuda"
+        # (hybrid stages route on the host: headered protocol)
+        env_serve = self.device.type == "cuda" and not config.is_hybrid
         if os.environ.get("MDI_ENV_SERVE"):
             env_serve = os.environ["MDI_ENV_SERVE"] not in ("0", "false")
         for r in range(1, self.world):
@@ -165,6 +166,7 @@ class MDIRuntime:
                 "model_config": config.to_dict(),
                 "n_nodes": self.world,
                 "n_local_layers": split[r],
+                "first_layer": sum(split[:r]),
                 "n_samples": n_samples,
                 "max_seq_length": seq_len,
                 "master_addr": self.topology.master_addr,
@@ -225,7 +227,8 @@ class MDIRuntime:
         )
         if self.world > 1:
             self.comm = RingComm(config.n_embd, seq_len, self.device,
-                                 n_samples, dtype=self.dtype)
+                                 n_samples,
+                                 dtype=config.residual_dtype(self.dtype))
         self.runtime = PipelineRuntime(self.runner, 0, self.world, self.comm,
                                        self.device)
 
@@ -287,7 +290,8 @@ class MDIRuntime:
                                 world_size=msg["world"],
                                 timeout=timedelta(seconds=600))
 
-        self.stage = build_stage(config, self.rank, n_local)
+        self.stage = build_stage(config, self.rank, n_local,
+                                 msg.get("first_layer", 0))
         hint = Path(msg["chunk_path"]) if msg.get("chunk_path") else None
         if self.chunk_path and self.chunk_path.is_file():
             self.stage.load_state_dict(
@@ -314,7 +318,7 @@ class MDIRuntime:
                                   self.device,
                                   expected_s=msg.get("expected_s"))
         self.comm = RingComm(config.n_embd, seq_len, self.device, n_samples,
-                             dtype=self.dtype)
+                             dtype=config.residual_dtype(self.dtype))
         self.runtime = PipelineRuntime(self.runner, msg["rank"],
                                        msg["world"], self.comm, self.device)
         self._log(f"serving (env={env_serve})")

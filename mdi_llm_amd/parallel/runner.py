@@ -14,13 +14,15 @@ import torch
 from ..config import ModelConfig
 from ..models.stages import StarterStage
 
-__all__ = ["TorchRunner", "HipRunner", "make_runner"]
+__all__ = ["TorchRunner", "HipRunner", "HybridRunner", "make_runner"]
 
 
 class TorchRunner:
     """Pure-PyTorch execution of a stage (CPU hosts, unsupported models)."""
 
     backend = "torch"
+    fused = False     # per-slot step graphs (DecodeEngine)
+    batched = False   # ragged batch steps (HybridEngine)
 
     def __init__(self, stage, n_slots: int) -> None:
         self.stage = stage
@@ -72,6 +74,7 @@ class HipRunner(TorchRunner):
     """HIP DecodeEngine for T=1 steps; torch stage forward for prefill."""
 
     backend = "hip"
+    fused = True
 
     def __init__(self, stage, n_slots: int, n_chunks: int = 16,
                  use_graphs: bool = True,
@@ -129,13 +132,70 @@ class HipRunner(TorchRunner):
         return self.engine.tail(x_last)
 
 
+class HybridRunner:
+    """Stages of hybrid stacks: every role is a step of ``HybridEngine``
+    (HIP kernels on a GPU; the torch operations on a CPU host)."""
+
+    fused = False
+    batched = True
+
+    def __init__(self, stage, n_slots: int, use_graphs: bool = True,
+                 n_tokens: "int | None" = None) -> None:
+        from ..ops.hybrid_engine import HybridEngine
+
+        self.stage = stage
+        self.config: ModelConfig = stage.config
+        self.is_starter = isinstance(stage, StarterStage)
+        if stage.kv_pool is None:
+            stage.set_kv_cache(n_slots, n_tokens=n_tokens)
+        self.cache = stage.kv_pool
+        self.engine = HybridEngine(stage, self.cache, use_graphs=use_graphs)
+        self.backend = "hip" if self.engine.hip else "torch"
+        self.pos = [0] * n_slots
+
+    def reset(self) -> None:
+        self.cache.reset()
+        self.pos = [0] * len(self.pos)
+
+    def _run(self, slot: int, fresh: bool, **what) -> torch.Tensor:
+        if fresh and self.cache.is_live(slot):
+            self.cache.release(slot)
+        if not self.cache.is_live(slot):
+            self.cache.admit(slot)
+        x = self.engine.hidden(slot, **what)
+        self.pos[slot] = self.cache.length[slot]
+        return x
+
+    def prefill_head(self, tokens: torch.Tensor, slot: int) -> torch.Tensor:
+        return self._run(slot, True, tokens=tokens.reshape(-1).tolist())
+
+    def prefill_mid(self, x: torch.Tensor, slot: int) -> torch.Tensor:
+        return self._run(slot, True, x=x)
+
+    def decode_head(self, token: torch.Tensor, slot: int) -> torch.Tensor:
+        return self._run(slot, False, tokens=[int(token)]).view(-1)
+
+    def decode_mid(self, x: torch.Tensor, slot: int) -> torch.Tensor:
+        return self._run(slot, False, x=x).view(-1)
+
+    def tail(self, x_last: torch.Tensor) -> torch.Tensor:
+        return self.engine.logits(x_last).view(-1)
+
+
 def make_runner(stage, n_slots: int, device: torch.device,
                 n_chunks: int = 16, use_graphs: bool = True,
                 force_torch: bool = False,
-                expected_s: "int | None" = None):
+                expected_s: "int | None" = None,
+                n_tokens: "int | None" = None):
     """Pick the HIP runner on GPU when the config is supported; fail loudly
     if a GPU is present but the extension is missing (no silent eager
-    fallback for supported configs)."""
+    fallback for supported configs).  ``n_tokens``: pool size of a hybrid
+    stack's cache, all sequences together."""
+    if stage.config.is_hybrid:
+        if force_torch and device.type == "cuda":
+            raise ValueError("hybrid stacks have no torch path on a GPU")
+        return HybridRunner(stage, n_slots, use_graphs=use_graphs,
+                            n_tokens=n_tokens)
     if force_torch or device.type != "cuda":
         return TorchRunner(stage, n_slots)
     from ..ops.engine import engine_supported

@@ -93,7 +93,12 @@ class PipelineRuntime:
         env = env and self.world > 1
         n_samples = len(prompts)
         runner = self.runner
-        if (self.world == 1 and getattr(runner, "backend", "") == "hip"
+        if self.world == 1 and getattr(runner, "batched", False):
+            return self._generate_batched(
+                prompts, max_new_tokens, sampling, stop_tokens,
+                token_callback,
+            )
+        if (self.world == 1 and self._fused(runner)
                 and runner.engine.use_graphs and sampling.top_p >= 1.0):
             return self._generate_standalone_fused(
                 prompts, max_new_tokens, sampling, stop_tokens,
@@ -104,7 +109,7 @@ class PipelineRuntime:
         # graphs must be captured BEFORE prefill (capture wipes caches)
         fused = (
             self.world > 1
-            and getattr(runner, "backend", "") == "hip"
+            and self._fused(runner)
             and runner.engine.use_graphs
             and sampling.top_p >= 1.0
         )
@@ -287,7 +292,40 @@ class PipelineRuntime:
     def _needs_clone(self) -> bool:
         # HIP runner returns a view of the engine's x buffer; standalone
         # loopback must snapshot it (the ring path copies into send bufs).
-        return getattr(self.runner, "backend", "") == "hip"
+        return self._fused(self.runner)
+
+    @staticmethod
+    def _fused(runner) -> bool:
+        """Does the runner have DecodeEngine's per-slot step graphs?"""
+        return getattr(runner, "fused", False)
+
+    def _generate_batched(
+        self, prompts, max_new_tokens, sampling: SamplingParams,
+        stop_tokens, token_callback,
+    ) -> GenerationResult:
+        """Standalone generation by ragged batch steps: prompts enter in
+        portions beside the sequences that already decode."""
+        from .scheduler import BatchScheduler
+
+        runner = self.runner
+        runner.reset()
+        res = GenerationResult()
+        sched = BatchScheduler(runner, sampling, stop_tokens)
+        for p in prompts:
+            sched.add(list(map(int, p.tolist())), max_new_tokens)
+        t_start = time.perf_counter()
+        while not sched.idle:
+            for rid, tok in sched.step():
+                res.total_new_tokens += 1
+                res.tok_time.append((res.total_new_tokens,
+                                     time.perf_counter() - t_start))
+                if token_callback is not None:
+                    token_callback(rid, tok)
+        res.gen_time = time.perf_counter() - t_start
+        res.sequences = [torch.tensor(r.prompt + r.output,
+                                      dtype=torch.int64)
+                         for r in sched.requests]
+        return res
 
     @staticmethod
     def _generators(sampling: SamplingParams, n: int, device):
@@ -330,7 +368,7 @@ class PipelineRuntime:
         """Capture the fused step graphs BEFORE prefill (capture warm-up
         scribbles on the KV pool, so it must precede cache filling)."""
         r = self.runner
-        if (self.is_starter and getattr(r, "backend", "") == "hip"
+        if (self.is_starter and self._fused(r)
                 and sampling.top_p >= 1.0 and r.engine.use_graphs):
             lanes = self._lane_count(n_samples) if self.world == 1 else 1
             r.engine.ensure_fused_graphs(
@@ -378,7 +416,7 @@ class PipelineRuntime:
         if gens is None:
             gens = self._generators(sampling, n, self.device)
         fused = (
-            getattr(runner, "backend", "") == "hip"
+            self._fused(runner)
             and sampling.top_p >= 1.0
             and runner.engine.use_graphs
         )
@@ -528,7 +566,7 @@ class PipelineRuntime:
 
     def _draw(self, logits, sampling: SamplingParams, gen):
         r = self.runner
-        if getattr(r, "backend", "") == "hip":
+        if self._fused(r):
             # fused on-GPU sampler (radix top-k + mass-radix top-p +
             # gumbel), no host sync.  Clone: sample_out is a single device
             # scalar reused by every draw — callers keep per-sample tokens
@@ -575,7 +613,7 @@ class PipelineRuntime:
         """Envelope serve: classic prefill phase, then the pipelined
         decode loop."""
         runner = self.runner
-        hip = getattr(runner, "backend", "") == "hip"
+        hip = self._fused(runner)
         if hip:
             # graph capture scribbles the KV pool: do it BEFORE prefill
             runner.engine.ensure_env_graph()

@@ -18,7 +18,7 @@ from typing import Optional, Tuple, Union
 
 import torch
 
-from ..config import ModelConfig
+from ..config import ModelConfig, is_native_checkpoint
 
 __all__ = [
     "load_from_pt",
@@ -26,6 +26,7 @@ __all__ = [
     "save_checkpoint",
     "init_from_state_dict",
     "get_checkpoint_files",
+    "has_weights",
 ]
 
 PathLike = Union[str, Path]
@@ -34,6 +35,12 @@ PathLike = Union[str, Path]
 def get_checkpoint_files(ckpt_dir: PathLike) -> Tuple[Path, Path]:
     ckpt_dir = Path(ckpt_dir)
     return ckpt_dir / "model_config.yaml", ckpt_dir / "lit_model.pth"
+
+
+def has_weights(ckpt_dir: PathLike) -> bool:
+    """True when ``load_from_pt`` can read the folder as it is."""
+    return get_checkpoint_files(ckpt_dir)[1].is_file() \
+        or is_native_checkpoint(ckpt_dir)
 
 
 def load_state_dict_lazy(path: PathLike) -> dict:
@@ -57,6 +64,13 @@ def load_from_pt(
     cfg_file, model_file = get_checkpoint_files(ckpt_dir)
     if config is None:
         config = ModelConfig.from_checkpoint(ckpt_dir)
+    if not model_file.is_file() and is_native_checkpoint(ckpt_dir):
+        from safetensors import safe_open
+
+        from ..models.hybrid import native_state_dict
+
+        with safe_open(Path(ckpt_dir) / "model.safetensors", "pt") as f:
+            return config, native_state_dict(config, f.get_tensor)
     if not model_file.is_file():
         raise FileNotFoundError(f"{model_file} not found")
     sd = load_state_dict_lazy(model_file)

@@ -116,11 +116,11 @@ def balanced_split(config, n_nodes: int, sampler_bytes: int = 150_000_000,
     """
     if n_nodes == 1:
         return [config.n_layer]
-    E, I, V = config.n_embd, config.intermediate_size, config.padded_vocab_size
-    hs, nh, ng = config.head_size, config.n_head, config.n_query_groups
-    layer_b = (E * (nh + 2 * ng) * hs + E * nh * hs + 3 * E * I) * dtype_bytes
-    if config.mlp_class_name == "GptNeoxMLP":
-        layer_b = (E * (nh + 2 * ng) * hs + E * nh * hs + 2 * E * I) * dtype_bytes
+    E, V = config.n_embd, config.padded_vocab_size
+    # layers of a hybrid stack differ; their mean sizes the starter's share
+    layer_b = dtype_bytes * sum(
+        config.layer_weights(i) for i in range(config.n_layer)
+    ) // config.n_layer
     starter_extra = V * E * dtype_bytes + sampler_bytes
     extra_layers = starter_extra / max(layer_b, 1)
     # starter share: solve x + extra = (n_layer - x) / (n_nodes - 1) balance

@@ -16,12 +16,16 @@ sys.path.insert(0, str(SCRIPT_DIR))
 
 
 def main(args):
-    from mdi_llm_amd.utils.checkpoint import get_checkpoint_files, load_from_pt
+    from mdi_llm_amd.utils.checkpoint import (
+        get_checkpoint_files,
+        has_weights,
+        load_from_pt,
+    )
     from mdi_llm_amd.utils.partition import split_and_store
 
     ckpt = args.ckpt
     cfg_file, model_file = get_checkpoint_files(ckpt)
-    if not model_file.is_file():
+    if not has_weights(ckpt):
         if ckpt.is_dir() and any(ckpt.glob("*.safetensors")) or \
                 (ckpt / "pytorch_model.bin").is_file() or \
                 any(ckpt.glob("*.bin.index.json")) or \

@@ -36,13 +36,12 @@ def main(args):
         model_name_to_prompt_style,
     )
     from mdi_llm_amd.tokenizer import Tokenizer
-    from mdi_llm_amd.utils.checkpoint import get_checkpoint_files, load_from_pt
+    from mdi_llm_amd.utils.checkpoint import has_weights, load_from_pt
     from mdi_llm_amd.utils.plots import tok_time_csv_name, write_tok_time_csv
 
     torch.manual_seed(args.seed)
     ckpt = args.ckpt
-    cfg_file, model_file = get_checkpoint_files(ckpt)
-    if not model_file.is_file():
+    if not has_weights(ckpt):
         # auto-convert an HF checkpoint dir (reference sample.py:66-76)
         from mdi_llm_amd.utils.convert_hf import convert_hf_checkpoint
 
