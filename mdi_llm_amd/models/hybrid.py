@@ -60,8 +60,9 @@ class BiasedAttention(nn.Module):
         self.dim, self.vdim = spec["dim"], spec["vdim"]
         self.scale = float(spec["scale"])
         self.bias_max = spec["bias_max"]
-        self.window = int(spec["mask"]["size"])
-        self.keep_first = int(spec["mask"]["keep_first"])
+        mask = spec.get("mask") or {}
+        self.window = int(mask.get("size", 1 << 30))
+        self.keep_first = int(mask.get("keep_first", 0))
         self.in_proj = nn.Linear(
             width,
             (self.heads + self.kv_heads) * self.dim

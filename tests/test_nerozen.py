@@ -1,0 +1,295 @@
+"""Nerozen through the framework's engine, cache and scheduler against the
+plain implementation in ``nerozen_oracle``: on a CPU host over the torch
+operations, on a GPU over the HIP kernels."""
+
+import random
+
+import pytest
+import torch
+
+import nerozen_oracle as oracle
+from nerozen_models import (MODELS, deviation, make_runner, tokens, weights)
+
+CPU = pytest.param("cpu", torch.float32, 2e-5, id="cpu-f32")
+GPU32 = pytest.param("cuda", torch.float32, 5e-5, id="gpu-f32",
+                     marks=pytest.mark.gpu)
+GPU16 = pytest.param("cuda", torch.bfloat16, 0.06, id="gpu-bf16",
+                     marks=pytest.mark.gpu)
+everywhere = pytest.mark.parametrize("device,dtype,tol", [CPU, GPU32, GPU16])
+
+_cache = {}
+
+
+def model(name, seed=0):
+    if (name, seed) not in _cache:
+        cfg, rows = MODELS[name]
+        _cache[name, seed] = (cfg, weights(cfg, rows, seed))
+    return _cache[name, seed]
+
+
+def expected(name, toks):
+    key = (name, tuple(toks))
+    if key not in _cache:
+        cfg, w = model(name)
+        _cache[key] = oracle.forward(cfg, w, toks)
+    return _cache[key]
+
+
+def run_portions(runner, toks, portions, slot=None):
+    """All logits of one sequence cut into the given portions (the last one
+    repeats)."""
+    c = runner.cache
+    slot = c.admit() if slot is None else slot
+    at, out, portions = 0, [], list(portions)
+    while at < len(toks):
+        n = portions.pop(0) if len(portions) > 1 else portions[0]
+        part = toks[at:at + n]
+        out.append(runner.engine.step([(slot, part)],
+                                      [range(len(part))]).float().clone())
+        at += n
+    c.release(slot)
+    return torch.cat(out)
+
+
+@everywhere
+@pytest.mark.parametrize("name", list(MODELS))
+def test_prompt(name, device, dtype, tol):
+    cfg, w = model(name)
+    r = make_runner(cfg, w, device, dtype)
+    for n in (1, 2, 17, 150):
+        toks = tokens(cfg, 150)[:n]
+        got = run_portions(r, toks, [n])
+        assert deviation(got, expected(name, tokens(cfg, 150))[:n]) < tol
+    assert r.cache.free_pages == r.cache.n_pages
+
+
+@everywhere
+def test_residual_stream_after_every_layer(device, dtype, tol):
+    cfg, w = model("mixed")
+    toks = tokens(cfg, 21)
+    want, got = [], []
+    oracle.forward(cfg, w, toks, want)
+    r = make_runner(cfg, w, device, dtype)
+    r.engine.step([(r.cache.admit(), toks)], layers_out=got)
+    assert len(got) == len(want)
+    for g, x in zip(got, want):
+        assert g.dtype == torch.float32
+        assert deviation(g, x) < tol
+
+
+@everywhere
+@pytest.mark.parametrize("name", ["mixed", "narrow", "odd", "wide"])
+def test_portions_and_decoding(name, device, dtype, tol):
+    """Cuts down to two tokens and one, across page (64) and window edges."""
+    cfg, w = model(name)
+    toks = tokens(cfg, 150)
+    want = expected(name, toks)
+    r = make_runner(cfg, w, device, dtype)
+    for portions in ([2], [1], [63, 2, 1, 1, 64], [3, 61, 5, 1, 7],
+                     [149, 1], [31, 33, 16, 17]):
+        assert deviation(run_portions(r, toks, portions), want) < tol, portions
+
+
+@everywhere
+def test_long_decoding(device, dtype, tol):
+    """Most of the sequence decoded, far past every window and the table."""
+    cfg, w = model("mixed")
+    toks = tokens(cfg, 400)
+    got = run_portions(make_runner(cfg, w, device, dtype), toks, [5, 1])
+    assert deviation(got, expected("mixed", toks)) < tol
+
+
+@everywhere
+@pytest.mark.parametrize("name", ["mixed", "narrow"])
+def test_unequal_batches(name, device, dtype, tol):
+    """Portions beside single tokens; slots and pages taken over by later
+    requests; a pool that only just holds the live ones."""
+    cfg, w = model(name)
+    lengths = [150, 1, 97, 40, 64, 129, 66, 2]
+    seqs = [tokens(cfg, n, seed=i) for i, n in enumerate(lengths)]
+    r = make_runner(cfg, w, device, dtype, n_slots=4, n_tokens=600)
+    rng = random.Random(5)
+    waiting, live = list(range(len(seqs))), {}
+    got = [[] for _ in seqs]
+    taken = set()
+    while waiting or live:
+        while waiting and len(live) < 4:
+            i = waiting.pop(0)
+            live[i] = (r.cache.admit(), 0)
+            taken.add(live[i][0])
+        step = [i for i in live if rng.random() < 0.8] or list(live)
+        rng.shuffle(step)
+        entries = []
+        for i in step:
+            slot, at = live[i]
+            n = rng.choice([1, 1, 2, 9, 33, 70])
+            entries.append((slot, seqs[i][at:at + n]))
+        out = r.engine.step(entries, [range(len(t)) for _, t in entries])
+        out = out.float().clone()
+        at0 = 0
+        for i, (slot, t) in zip(step, entries):
+            got[i].append(out[at0:at0 + len(t)])
+            at0 += len(t)
+            at = live[i][1] + len(t)
+            live[i] = (slot, at)
+            if at == len(seqs[i]):
+                r.cache.release(slot)
+                del live[i]
+    assert len(taken) < len(seqs)  # slots were used again
+    for i, s in enumerate(seqs):
+        assert deviation(torch.cat(got[i]), expected(name, s)) < tol, i
+    assert r.cache.free_pages == r.cache.n_pages
+
+
+@everywhere
+def test_a_reused_slot_starts_clean(device, dtype, tol):
+    """The same slot and pages, with another sequence and no clearing."""
+    cfg, w = model("mixed")
+    r = make_runner(cfg, w, device, dtype, n_slots=1, n_tokens=192)
+    for seed, n in ((1, 190), (2, 64), (3, 65), (4, 3), (5, 130)):
+        toks = tokens(cfg, n, seed)
+        for cut in ([n], [1]):
+            got = run_portions(r, toks, cut)
+            assert deviation(got, expected("mixed", toks)) < tol
+
+
+@everywhere
+def test_wanted_rows(device, dtype, tol):
+    cfg, w = model("mixed")
+    a, b = tokens(cfg, 30), tokens(cfg, 9, 1)
+    r = make_runner(cfg, w, device, dtype)
+    sa, sb = r.cache.admit(), r.cache.admit()
+    got = r.engine.step([(sa, a), (sb, b)], [[29, 0], [4]])
+    want = torch.stack([expected("mixed", a)[29], expected("mixed", a)[0],
+                        expected("mixed", b)[4]])
+    assert deviation(got.float(), want) < tol
+    assert r.engine.step([(sa, a[:2]), (sb, b[:1])], [[], []]) is None
+    assert r.cache.length[sa] == 32 and r.cache.length[sb] == 10
+
+
+def greedy_agrees(name, prompt, out, slack):
+    """Each token is the oracle's choice, or within ``slack`` of it."""
+    logits = expected(name, prompt + out)
+    for k, tok in enumerate(out):
+        row = logits[len(prompt) - 1 + k]
+        if float(row.max() - row[tok]) > slack:
+            return False
+    return True
+
+
+@everywhere
+def test_greedy_generation(device, dtype, tol):
+    """The runtime's entry point and scheduler, more requests than slots and
+    a pool that makes them wait."""
+    from mdi_llm_amd.parallel.runtime import PipelineRuntime, SamplingParams
+
+    cfg, w = model("mixed")
+    prompts = [tokens(cfg, n, 20 + n) for n in (3, 100, 1, 64, 31, 7)]
+    r = make_runner(cfg, w, device, dtype, n_slots=3, n_tokens=384)
+    rt = PipelineRuntime(r, device=torch.device(device))
+    seen = []
+    res = rt.generate([torch.tensor(p) for p in prompts], 20,
+                      SamplingParams(temperature=0.0),
+                      token_callback=lambda i, t: seen.append((i, t)))
+    assert len(seen) == res.total_new_tokens == 20 * len(prompts)
+    for i, (p, seq) in enumerate(zip(prompts, res.sequences)):
+        seq = seq.tolist()
+        assert seq[:len(p)] == p and len(seq) == len(p) + 20
+        assert [t for j, t in seen if j == i] == seq[len(p):]
+        assert greedy_agrees("mixed", p, seq[len(p):], 4 * tol), i
+    assert r.cache.free_pages == r.cache.n_pages
+    # and once more over used pages: same tokens
+    again = rt.generate([torch.tensor(p) for p in prompts], 20,
+                        SamplingParams(temperature=0.0))
+    if dtype == torch.float32:
+        assert [s.tolist() for s in again.sequences] == \
+            [s.tolist() for s in res.sequences]
+
+
+@everywhere
+def test_small_prefill_budget(device, dtype, tol):
+    """Prompts cut by the scheduler's step budget, stop sequences."""
+    from mdi_llm_amd.parallel.runtime import SamplingParams
+    from mdi_llm_amd.parallel.scheduler import BatchScheduler
+
+    cfg, w = model("mixed")
+    r = make_runner(cfg, w, device, dtype, n_slots=3)
+    s = BatchScheduler(r, SamplingParams(temperature=0.0), budget=10)
+    prompts = [tokens(cfg, n, 40 + n) for n in (45, 4, 23, 80)]
+    reqs = [s.add(p, 9) for p in prompts]
+    while not s.idle:
+        s.step()
+    for p, q in zip(prompts, reqs):
+        assert len(q.output) == 9
+        assert greedy_agrees("mixed", p, q.output, 4 * tol)
+    stop = reqs[0].output[3:5]
+    s = BatchScheduler(r, SamplingParams(temperature=0.0), [stop])
+    q = s.add(prompts[0], 9)
+    while not s.idle:
+        s.step()
+    assert q.output[-2:] == stop and len(q.output) <= 5
+
+
+@everywhere
+def test_runner_roles_match_steps(device, dtype, tol):
+    """The calls of the pipeline runtime: head, middle, tail."""
+    cfg, w = model("mixed")
+    toks = tokens(cfg, 40)
+    r = make_runner(cfg, w, device, dtype)
+    want = expected("mixed", toks)
+    for _ in range(2):  # the second prefill takes the slot over
+        x = r.prefill_head(torch.tensor(toks[:30]), 2)
+        assert x.shape == (30, cfg["width"]) and x.dtype == torch.float32
+        got = [r.tail(x[-1])]
+        for t in toks[30:]:
+            got.append(r.tail(r.decode_head(torch.tensor([t]), 2)))
+        assert r.pos[2] == 40
+        assert deviation(torch.stack(got).float(), want[29:]) < tol
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("n", [1, 3, 4])
+def test_decode_graph_replays(n):
+    """Replays between other work of the program, each against the eager
+    step of the same tokens."""
+    cfg, w = model("mixed")
+    r = make_runner(cfg, w, "cuda", torch.bfloat16)
+    e = make_runner(cfg, w, "cuda", torch.bfloat16)
+    e.engine.use_graphs = False
+    prompts = [tokens(cfg, 60 + i, i) for i in range(n)]
+    for q in (r, e):
+        for p in prompts:
+            q.engine.step([(q.cache.admit(), p)])
+    slots = list(range(3, 3 - n, -1)) if n == 4 else list(range(n))
+    slots = sorted(s for s in range(4) if r.cache.is_live(s))
+    for k in range(12):
+        toks = [tokens(cfg, 12, 50 + i)[k] for i in range(n)]
+        got = r.engine.decode(slots, toks).float().clone()
+        want = e.engine.step([(s, [t]) for s, t in zip(slots, toks)])
+        assert deviation(got, want.float()) < 1e-6, k
+        torch.randn(1000, device="cuda").sum().item()
+        if k % 4 == 3:
+            torch.cuda.synchronize()
+
+
+@pytest.mark.gpu
+def test_sampled_tokens_do_not_depend_on_the_schedule():
+    """Device draws are keyed by request and position: the same request
+    alone and among others, chained on the device and fed from the host."""
+    from mdi_llm_amd.parallel.runtime import PipelineRuntime, SamplingParams
+
+    cfg, w = model("mixed")
+    prompts = [torch.tensor(tokens(cfg, n, n)) for n in (12, 70, 5)]
+    sp = SamplingParams(temperature=0.7, top_k=20, seed=11)
+
+    def run(n_slots):
+        r = make_runner(cfg, w, "cuda", torch.bfloat16, n_slots=n_slots)
+        res = PipelineRuntime(r, device=torch.device("cuda")).generate(
+            prompts, 12, sp)
+        return [s.tolist() for s in res.sequences]
+
+    one, three = run(1), run(3)
+    # batch sizes round differently; a draw flips only at a near tie
+    same = sum(a == b for x, y in zip(one, three) for a, b in zip(x, y))
+    assert same >= 0.8 * sum(map(len, one))
+    assert run(3) == three
