@@ -46,6 +46,11 @@ def parse_args():
                     help="KV-cache dtype (fp8 = e4m3 per-row-scaled cache; "
                          "NOT the headline config — reported in dtype)")
     ap.add_argument("--no-graphs", action="store_true")
+    ap.add_argument("--hybrid", nargs="*", default=None,
+                    choices=["nerozen-1b", "nerozen-8b"], metavar="MODEL",
+                    help="instead of the headline workload: prefill and "
+                         "decode throughput of these hybrid stacks (default "
+                         "all) beside the existing model of equal size")
     return ap.parse_args()
 
 
@@ -53,8 +58,24 @@ def log(msg):
     print(f"[bench] {msg}", file=sys.stderr, flush=True)
 
 
+def bench_hybrid(names):
+    from mdi_llm_amd.utils.compare_bench import PAIRS, compare
+
+    for name in names or list(PAIRS):
+        print(json.dumps({
+            "metric": "hybrid_throughput", "unit": "tokens/s", "n_gpus": 1,
+            "dtype": "bf16", "data": "synthetic",
+            "config": {"prompt_len": 4096, "decode_context": 128,
+                       "batch": 32},
+            "models": compare(name),
+        }), flush=True)
+
+
 def main():
     args = parse_args()
+    if args.hybrid is not None:
+        bench_hybrid(args.hybrid)
+        return
     if args.weights == "fp8":
         os.environ["MDI_WEIGHT_DTYPE"] = "fp8"
     if args.kv == "fp8":

@@ -134,20 +134,26 @@ void hgrn2_step(torch::Tensor out, torch::Tensor proj, torch::Tensor state,
                     (float)eps, r.f32, cur_stream());
 }
 
-void hgrn2_scan(torch::Tensor out, torch::Tensor o, torch::Tensor proj,
-                torch::Tensor state, torch::Tensor f_bias,
-                torch::Tensor lower, torch::Tensor norm_w, torch::Tensor seg,
-                int64_t max_len, double eps) {
+void hgrn2_scan(torch::Tensor out, torch::Tensor proj, torch::Tensor state,
+                torch::Tensor f_bias, torch::Tensor lower,
+                torch::Tensor norm_w, torch::Tensor seg, int64_t max_len,
+                double eps) {
   const Recurrent r =
       recurrent(proj, state, f_bias, lower, norm_w.numel());
   check_like(out, r.f32, "out");
   TORCH_CHECK(out.numel() == proj.size(0) * r.heads * r.vdim, "out size");
-  float* op = const_cast<float*>(f32_ptr(o, out.numel(), "o"));
+  TORCH_CHECK(r.dim <= 256 && r.vdim <= 1024, "hgrn2_scan: sizes");
+  TORCH_CHECK(max_len > 0 && max_len <= proj.size(0), "max_len");
   const SegView sv = seg_view(seg);
-  const int rc =
-      launch_hgrn2_scan(op, proj.data_ptr(), r.state, r.f_bias, r.lower, sv,
-                        r.heads, r.dim, r.vdim, r.vstride, r.f32,
-                        cur_stream());
+  const auto fp = proj.options().dtype(torch::kFloat32);
+  torch::Tensor o = torch::empty({out.numel()}, fp);
+  torch::Tensor work = torch::empty(
+      {hgrn2_work_floats((int)proj.size(0), sv.n, r.heads, r.dim)}, fp);
+  float* op = o.data_ptr<float>();
+  const int rc = launch_hgrn2_scan(
+      op, work.data_ptr<float>(), proj.data_ptr(), r.state, r.f_bias,
+      r.lower, sv, (int)max_len, r.heads, r.dim, r.vdim, r.vstride, r.f32,
+      cur_stream());
   TORCH_CHECK(rc == 0, "hgrn2_scan: unsupported dim ", r.dim);
   launch_head_norm(out.data_ptr(), op, f32_ptr(norm_w, r.vdim, "norm_w"), sv,
                    (int)max_len, r.heads, r.vdim, (float)eps, r.f32,
@@ -282,8 +288,7 @@ void bind_hybrid(py::module_& m) {
         py::arg("f_bias"), py::arg("lower"), py::arg("norm_w"),
         py::arg("seg"), py::arg("eps"));
   m.def("hgrn2_scan", &hgrn2_scan, "HGRN2 over token segments",
-        py::arg("out"), py::arg("o"), py::arg("proj"), py::arg("state"),
-        py::arg("f_bias"), py::arg("lower"), py::arg("norm_w"),
+        py::arg("out"), py::arg("proj"), py::arg("state"), py::arg("f_bias"), py::arg("lower"), py::arg("norm_w"),
         py::arg("seg"), py::arg("max_len"), py::arg("eps"));
   m.def("qk_norm_append", &qk_norm_append,
         "per-head q/k RMS norms + paged cache append", py::arg("q_out"),

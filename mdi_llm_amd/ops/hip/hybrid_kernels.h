@@ -39,12 +39,14 @@ void launch_hgrn2_step(void* out, const void* proj, float* state,
                        int vdim, int vstride, float eps, int f32,
                        hipStream_t stream);
 
-// HGRN2 over longer segments; o is the raw read-out [rows, H*E] float.
+// HGRN2 over longer segments, which must be in the order of their rows; o is
+// the raw read-out [rows, H*E] float, work holds hgrn2_work_floats(...).
 // Returns -1 when dim has no instantiation.
-int launch_hgrn2_scan(float* o, const void* proj, float* state,
+long long hgrn2_work_floats(int rows, int segments, int heads, int dim);
+int launch_hgrn2_scan(float* o, float* work, const void* proj, float* state,
                       const float* f_bias, const float* lower, SegView seg,
-                      int heads, int dim, int vdim, int vstride, int f32,
-                      hipStream_t stream);
+                      int max_len, int heads, int dim, int vdim, int vstride,
+                      int f32, hipStream_t stream);
 
 // out[row] = rms(o[row]) * w per head, for the rows of the segments
 void launch_head_norm(void* out, const float* o, const float* w, SegView seg,

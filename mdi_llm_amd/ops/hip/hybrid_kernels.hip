@@ -166,24 +166,24 @@ void launch_xielu(void* z, long long n, float p, float q, int f32,
 // accesses along vdim), so the block holds all of the head's output and can
 // norm it before it leaves.
 // ---------------------------------------------------------------------------
-template <typename T>
-__global__ __launch_bounds__(256) void hgrn2_step_kernel(
+template <typename T, int NT>
+__global__ __launch_bounds__(NT) void hgrn2_step_kernel(
     T* __restrict__ out, const T* __restrict__ proj,
     float* __restrict__ state, const float* __restrict__ f_bias,
     const float* __restrict__ lower, const float* __restrict__ norm_w,
     SegView seg, int heads, int dim, int vdim, int vstride, float eps) {
   extern __shared__ float sm[];
-  __shared__ float red[4];
+  __shared__ float red[NT / 64];
   const int tid = threadIdx.x, h = blockIdx.x, s = blockIdx.y;
   const int nq = vstride / 4;                 // float4 columns
-  const int lanes = nq < 256 ? nq : 256;      // threads along the columns
-  const int groups = 256 / lanes;             // row groups
+  const int lanes = nq < NT ? nq : NT;      // threads along the columns
+  const int groups = NT / lanes;             // row groups
   float* qs = sm;                             // [dim]
   float* fs = qs + dim;                       // [dim]
   float* part = fs + dim;                     // [groups][vstride]
   const size_t row = seg.start[s];
   const T* pr = proj + row * (size_t)(heads * (2 * dim + vdim));
-  for (int d = tid; d < dim; d += 256) {
+  for (int d = tid; d < dim; d += NT) {
     const int c = h * dim + d;
     const float qv = to_f(pr[c]);
     qs[d] = qv * sigmoid(qv);
@@ -223,7 +223,7 @@ __global__ __launch_bounds__(256) void hgrn2_step_kernel(
   }
   __syncthreads();
   float ss = 0.f;
-  for (int c = tid; c < vdim; c += 256) {
+  for (int c = tid; c < vdim; c += NT) {
     float o = 0.f;
     for (int k = 0; k < groups; ++k) o += part[k * vstride + c];
     part[c] = o;  // only this thread reads column c
@@ -232,11 +232,28 @@ __global__ __launch_bounds__(256) void hgrn2_step_kernel(
   ss = wave_sum(ss);
   if ((tid & 63) == 0) red[tid >> 6] = ss;
   __syncthreads();
-  const float r =
-      1.f / sqrtf((red[0] + red[1] + red[2] + red[3]) / vdim + eps);
+  ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < NT / 64; ++k) ss += red[k];
+  const float r = 1.f / sqrtf(ss / vdim + eps);
   T* o_row = out + row * (size_t)(heads * vdim) + h * vdim;
-  for (int c = tid; c < vdim; c += 256)
+  for (int c = tid; c < vdim; c += NT)
     o_row[c] = from_f<T>(part[c] * r * norm_w[c]);
+}
+
+template <typename T, int NT>
+static void hgrn2_step_t(void* out, const void* proj, float* state,
+                         const float* f_bias, const float* lower,
+                         const float* norm_w, SegView seg, int heads, int dim,
+                         int vdim, int vstride, float eps,
+                         hipStream_t stream) {
+  const int nq = vstride / 4;
+  const int lanes = nq < NT ? nq : NT;
+  const size_t smem =
+      (2 * (size_t)dim + (size_t)(NT / lanes) * vstride) * sizeof(float);
+  hgrn2_step_kernel<T, NT><<<dim3(heads, seg.n), NT, smem, stream>>>(
+      (T*)out, (const T*)proj, state, f_bias, lower, norm_w, seg, heads, dim,
+      vdim, vstride, eps);
 }
 
 void launch_hgrn2_step(void* out, const void* proj, float* state,
@@ -244,208 +261,439 @@ void launch_hgrn2_step(void* out, const void* proj, float* state,
                        const float* norm_w, SegView seg, int heads, int dim,
                        int vdim, int vstride, float eps, int f32,
                        hipStream_t stream) {
-  const int nq = vstride / 4;
-  const int lanes = nq < 256 ? nq : 256;
-  const size_t smem =
-      (2 * (size_t)dim + (size_t)(256 / lanes) * vstride) * sizeof(float);
-  dim3 grid(heads, seg.n);
-  if (f32)
-    hgrn2_step_kernel<float><<<grid, 256, smem, stream>>>(
-        (float*)out, (const float*)proj, state, f_bias, lower, norm_w, seg,
-        heads, dim, vdim, vstride, eps);
-  else
-    hgrn2_step_kernel<bf16><<<grid, 256, smem, stream>>>(
-        (bf16*)out, (const bf16*)proj, state, f_bias, lower, norm_w, seg,
-        heads, dim, vdim, vstride, eps);
+  // few blocks with a large state each: more waves to keep loads in flight
+  const bool wide = dim * vstride >= 8192 && heads * seg.n <= 512;
+#define STEP(T, NT)                                                       \
+  hgrn2_step_t<T, NT>(out, proj, state, f_bias, lower, norm_w, seg,       \
+                      heads, dim, vdim, vstride, eps, stream)
+  if (f32) {
+    if (wide) STEP(float, 1024);
+    else STEP(float, 256);
+  } else {
+    if (wide) STEP(bf16, 1024);
+    else STEP(bf16, 256);
+  }
+#undef STEP
 }
 
 // ---------------------------------------------------------------------------
-// HGRN2 over longer segments.  The columns of the state never mix, so a
-// block keeps a [dim, 16] slice of one head in registers for the whole
-// segment: 16 lanes of a DPP row share a column, R rows each.  Tokens are
-// staged in LDS (gates computed once per block) TB at a time.
+// HGRN2 over longer segments, in chunks of 16 tokens.  With S the state at
+// the chunk's start, per channel
+//     R_t = f_first .. f_t          (decay from the start to t)
+//     U_s = f_(s+1) .. f_last       (decay from s to the end)
+// the chunk is three small matrix products,
+//     o_t = (q_t R_t)^T S + sum_(s<=t) P[t][s] v_s
+//     S  <- (f_first .. f_last) S + sum_s (U_s (1 - f_s)) v_s^T
+// with P[t][s] = sum_d q_t (1 - f_s) f_(s+1) .. f_t.  All decays are plain
+// products of gates, so every factor is at most 1 and nothing is divided
+// by; an underflow is a token that is forgotten.  Everything is float and
+// the products run on the float MFMA.
+//
+// The first kernel makes the factors of every (chunk, head) in parallel;
+// the second walks a segment's chunks with a [dim, 16] slice of the state
+// per block, held as MFMA accumulators split over the block's four waves by
+// rows.  An accumulator tile is at the same time the right operand of
+// (q R)^T S once the contraction index is permuted to its layout.
+//
+// Workspace of one (chunk, head), DP = dim padded to 64, 128 or 256:
+//   qr [16][DP] | uk [DP][16] | decay [DP] | P [16][16]
+// Segment s has its chunks from start[s] / 16 + s on, which cannot overlap
+// as long as the segments are in the order of their rows.
 // ---------------------------------------------------------------------------
-template <typename T, int R>
-__global__ __launch_bounds__(256) void hgrn2_scan_kernel(
-    float* __restrict__ o, const T* __restrict__ proj,
-    float* __restrict__ state, const float* __restrict__ f_bias,
-    const float* __restrict__ lower, SegView seg, int heads, int dim,
-    int vdim, int vstride) {
-  constexpr int DP = 16 * R, TB = 16;
-  __shared__ __attribute__((aligned(16))) float fs[TB][DP];
-  __shared__ __attribute__((aligned(16))) float qs[TB][DP];
-  __shared__ float vs[TB][16], os[TB][17];
-  const int tid = threadIdx.x, h = blockIdx.y, s = blockIdx.z;
-  const int c0 = blockIdx.x * 16;
-  const int rl = tid & 15, cl = tid >> 4, col = c0 + cl;
-  const int len = seg.len[s];
+using f32x4 = __attribute__((__vector_size__(16))) float;
+
+template <int DP>
+struct ChunkWork {
+  static constexpr int QR = 0, UK = 16 * DP, DECAY = 32 * DP,
+                       P = 33 * DP, SIZE = 33 * DP + 256;
+};
+
+template <typename T, int DP>
+__global__ __launch_bounds__(256) void hgrn2_factors_kernel(
+    float* __restrict__ work, const T* __restrict__ proj,
+    const float* __restrict__ f_bias, const float* __restrict__ lower,
+    SegView seg, int heads, int dim, int vdim) {
+  using W = ChunkWork<DP>;
+  constexpr int CH = DP / 16;
+  const int s = blockIdx.z, h = blockIdx.y, t0 = blockIdx.x * 16;
+  const int tn = min(16, seg.len[s] - t0);
+  if (tn <= 0) return;
+  __shared__ __attribute__((aligned(16))) float fs[16][DP];
+  __shared__ __attribute__((aligned(16))) float qs[16][DP];
+  const int tid = threadIdx.x;
+  const size_t row0 = (size_t)seg.start[s] + t0;
+  const size_t ld = (size_t)heads * (2 * dim + vdim);
+  float* w = work + (((size_t)seg.start[s] / 16 + s + blockIdx.x) * heads +
+                     h) * W::SIZE;
+  for (int i = tid; i < 16 * DP; i += 256) {
+    const int t = i / DP, d = i % DP;
+    float f = 1.f, q = 0.f;  // past the end: nothing decays or is written
+    if (d >= dim) {
+      f = 0.f;
+    } else if (t < tn) {
+      const T* pr = proj + (row0 + t) * ld + h * dim + d;
+      const int c = h * dim + d;
+      const float qv = to_f(pr[0]), l = lower[c];
+      q = qv * sigmoid(qv);
+      f = l + (1.f - l) * sigmoid(to_f(pr[heads * dim]) + f_bias[c]);
+    }
+    fs[t][d] = f;
+    qs[t][d] = q;
+  }
+  __syncthreads();
+  for (int i = tid; i < 2 * DP; i += 256) {
+    const int d = i % DP;
+    if (i < DP) {
+      float r = 1.f;
+#pragma unroll
+      for (int t = 0; t < 16; ++t) {
+        r *= fs[t][d];
+        w[W::QR + t * DP + d] = qs[t][d] * r;
+      }
+    } else {
+      float u = 1.f;
+      Pack<float, 4> k[4];
+#pragma unroll
+      for (int t = 15; t >= 0; --t) {
+        const float f = fs[t][d];
+        k[t / 4].v[t % 4] = d < dim ? u * (1.f - f) : 0.f;
+        u *= f;
+      }
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        *reinterpret_cast<Pack<float, 4>*>(w + W::UK + d * 16 + j * 4) = k[j];
+      w[W::DECAY + d] = u;
+    }
+  }
+  // P: thread (s', channels CH*dc ..) carries (1 - f_s') f .. f along t
+  const int sp = tid >> 4, dc = tid & 15;
+  float k[CH];
+#pragma unroll
+  for (int c = 0; c < CH; ++c) k[c] = 0.f;
+#pragma unroll 4
+  for (int t = 0; t < 16; ++t) {
+    float acc = 0.f;
+#pragma unroll
+    for (int c = 0; c < CH; ++c) {
+      const float f = fs[t][dc * CH + c];
+      k[c] = t == sp ? 1.f - f : k[c] * f;
+      acc += qs[t][dc * CH + c] * k[c];  // q is 0 in padding channels
+    }
+    acc = row16_sum(acc);
+    if (dc == 0) w[W::P + t * 16 + sp] = acc;
+  }
+}
+
+template <typename T, int TPW>
+__global__ __launch_bounds__(256) void hgrn2_chunks_kernel(
+    float* __restrict__ o, const float* __restrict__ work,
+    const T* __restrict__ proj, float* __restrict__ state, SegView seg,
+    int heads, int dim, int vdim, int vstride) {
+  constexpr int DP = 64 * TPW;
+  using W = ChunkWork<DP>;
+  __shared__ float red[2][4][16][17];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int c = lane & 15, quad = lane >> 4;
+  const int s = blockIdx.z, h = blockIdx.y, c0 = blockIdx.x * 16;
+  const int col = c0 + c, d0 = wave * TPW * 16;
+  const int len = seg.len[s], n = (len + 15) / 16;
   const size_t row0 = seg.start[s];
-  const int ld = heads * (2 * dim + vdim);
+  const size_t ld = (size_t)heads * (2 * dim + vdim);
+  const float* w = work + ((row0 / 16 + s) * heads + h) * W::SIZE;
+  const size_t wstep = (size_t)heads * W::SIZE;
+  const T* vp = proj + row0 * ld + 2 * heads * dim + h * vdim + col;
   float* S = state +
-             ((size_t)seg.slot[s] * heads + h) * (size_t)dim * vstride;
-  const bool live = col < vstride;
-  float st[R];
+             ((size_t)seg.slot[s] * heads + h) * (size_t)dim * vstride + col;
+  const bool keep = col < vstride && seg.pos0[s] != 0;
+
+  f32x4 st[TPW];
 #pragma unroll
-  for (int r = 0; r < R; ++r) {
-    const int d = rl * R + r;
-    st[r] = (live && d < dim && seg.pos0[s] != 0)
-                ? S[(size_t)d * vstride + col] : 0.f;
-  }
-  for (int t0 = 0; t0 < len; t0 += TB) {
-    const int tn = min(TB, len - t0);
-    for (int i = tid; i < TB * DP; i += 256) {
-      const int t = i / DP, d = i % DP;
-      float f = 0.f, q = 0.f;
-      if (t < tn && d < dim) {
-        const T* pr = proj + (row0 + t0 + t) * (size_t)ld;
-        const int c = h * dim + d;
-        const float qv = to_f(pr[c]), l = lower[c];
-        q = qv * sigmoid(qv);
-        f = l + (1.f - l) *
-                    sigmoid(to_f(pr[heads * dim + c]) + f_bias[c]);
-      }
-      fs[t][d] = f;
-      qs[t][d] = q;
+  for (int k = 0; k < TPW; ++k)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int d = d0 + k * 16 + quad * 4 + i;
+      st[k][i] = keep && d < dim ? S[(size_t)d * vstride] : 0.f;
     }
+
+  struct Operands {
+    f32x4 qr[TPW], uk[TPW], decay[TPW];
+    float p, v[4], vw;
+  } cur, nxt;
+  auto load = [&](Operands& a, int ch) {
+    const float* wc = w + ch * wstep;
+#pragma unroll
+    for (int k = 0; k < TPW; ++k) {
+      a.qr[k] = *reinterpret_cast<const f32x4*>(
+          wc + W::QR + c * DP + d0 + k * 16 + quad * 4);
+      a.uk[k] = *reinterpret_cast<const f32x4*>(
+          wc + W::UK + (d0 + k * 16 + c) * 16 + quad * 4);
+      a.decay[k] = *reinterpret_cast<const f32x4*>(
+          wc + W::DECAY + d0 + k * 16 + quad * 4);
+    }
+    a.p = wc[W::P + c * 16 + quad * 4 + wave];
+    auto value = [&](int t) {
+      return col < vdim && t < len ? to_f(vp[(size_t)t * ld]) : 0.f;
+    };
+#pragma unroll
+    for (int i = 0; i < 4; ++i) a.v[i] = value(ch * 16 + quad * 4 + i);
+    a.vw = value(ch * 16 + quad * 4 + wave);
+  };
+  load(cur, 0);
+  for (int ch = 0; ch < n; ++ch) {
+    if (ch + 1 < n) load(nxt, ch + 1);
+    // two accumulators: half the dependent chain
+    f32x4 a0{0.f, 0.f, 0.f, 0.f}, a1 = a0;
+    a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.p, cur.vw, a0, 0, 0, 0);
+#pragma unroll
+    for (int k = 0; k < TPW; ++k) {
+      a1 = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.qr[k][0], st[k][0], a1, 0, 0, 0);
+      a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.qr[k][1], st[k][1], a0, 0, 0, 0);
+      a1 = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.qr[k][2], st[k][2], a1, 0, 0, 0);
+      a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.qr[k][3], st[k][3], a0, 0, 0, 0);
+    }
+#pragma unroll
+    for (int k = 0; k < TPW; ++k) st[k] *= cur.decay[k];
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int k = 0; k < TPW; ++k)
+        st[k] = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.uk[k][i], cur.v[i],
+                                                     st[k], 0, 0, 0);
+    a0 += a1;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) red[ch & 1][wave][quad * 4 + i][c] = a0[i];
+    __syncthreads();  // one per chunk: the other half is written next
     {
-      const int t = tid >> 4, c = c0 + (tid & 15);
-      float v = 0.f;
-      if (t < tn && c < vdim)
-        v = to_f(proj[(row0 + t0 + t) * (size_t)ld + 2 * heads * dim +
-                      h * vdim + c]);
-      vs[t][tid & 15] = v;
-    }
-    __syncthreads();
-    for (int t = 0; t < tn; ++t) {
-      const float v = vs[t][cl];
-      float acc = 0.f;
+      const int t = tid >> 4, e = tid & 15, tt = ch * 16 + t;
+      if (tt < len && c0 + e < vdim) {
+        float v = 0.f;
 #pragma unroll
-      for (int r = 0; r < R; ++r) {
-        const float f = fs[t][rl * R + r];
-        // rows past dim hold f = q = 0: their state stays out of the sum
-        st[r] = f * st[r] + (1.f - f) * v;
-        acc += qs[t][rl * R + r] * st[r];
+        for (int k = 0; k < 4; ++k) v += red[ch & 1][k][t][e];
+        o[(row0 + tt) * (size_t)(heads * vdim) + h * vdim + c0 + e] = v;
       }
-      acc = row16_sum(acc);
-      if (rl == 0) os[t][cl] = acc;
     }
-    __syncthreads();
-    {
-      const int t = tid >> 4, c = c0 + (tid & 15);
-      if (t < tn && c < vdim)
-        o[(row0 + t0 + t) * (size_t)(heads * vdim) + h * vdim + c] =
-            os[t][tid & 15];
-    }
+    cur = nxt;
   }
-  if (live) {
+  if (col < vstride) {
 #pragma unroll
-    for (int r = 0; r < R; ++r) {
-      const int d = rl * R + r;
-      if (d < dim) S[(size_t)d * vstride + col] = st[r];
-    }
+    for (int k = 0; k < TPW; ++k)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int d = d0 + k * 16 + quad * 4 + i;
+        if (d < dim) S[(size_t)d * vstride] = st[k][i];
+      }
   }
+}
+
+static int chunk_dpad(int dim) {
+  return dim <= 64 ? 64 : dim <= 128 ? 128 : dim <= 256 ? 256 : 0;
+}
+
+long long hgrn2_work_floats(int rows, int segments, int heads, int dim) {
+  const long long chunks = rows / 16 + segments + 1;
+  return chunks * heads * (33 * chunk_dpad(dim) + 256);
+}
+
+template <typename T, int TPW>
+static void hgrn2_scan_sized(float* o, float* work, const void* proj,
+                             float* state, const float* f_bias,
+                             const float* lower, SegView seg, int max_len,
+                             int heads, int dim, int vdim, int vstride,
+                             hipStream_t stream) {
+  hgrn2_factors_kernel<T, 64 * TPW>
+      <<<dim3((max_len + 15) / 16, heads, seg.n), 256, 0, stream>>>(
+          work, (const T*)proj, f_bias, lower, seg, heads, dim, vdim);
+  hgrn2_chunks_kernel<T, TPW>
+      <<<dim3((vdim + 15) / 16, heads, seg.n), 256, 0, stream>>>(
+          o, work, (const T*)proj, state, seg, heads, dim, vdim, vstride);
 }
 
 template <typename T>
-static int hgrn2_scan_t(float* o, const void* proj, float* state,
-                        const float* f_bias, const float* lower, SegView seg,
+static int hgrn2_scan_t(float* o, float* work, const void* proj,
+                        float* state, const float* f_bias,
+                        const float* lower, SegView seg, int max_len,
                         int heads, int dim, int vdim, int vstride,
                         hipStream_t stream) {
-  dim3 grid((vdim + 15) / 16, heads, seg.n);
-#define SCAN(R)                                                          \
-  hgrn2_scan_kernel<T, R><<<grid, 256, 0, stream>>>(                     \
-      o, (const T*)proj, state, f_bias, lower, seg, heads, dim, vdim,    \
-      vstride)
-  if (dim <= 16) SCAN(1);
-  else if (dim <= 32) SCAN(2);
-  else if (dim <= 64) SCAN(4);
-  else if (dim <= 128) SCAN(8);
-  else if (dim <= 256) SCAN(16);
-  else return -1;
+#define SCAN(TPW)                                                          \
+  hgrn2_scan_sized<T, TPW>(o, work, proj, state, f_bias, lower, seg,       \
+                           max_len, heads, dim, vdim, vstride, stream)
+  switch (chunk_dpad(dim)) {
+    case 64: SCAN(1); return 0;
+    case 128: SCAN(2); return 0;
+    case 256: SCAN(4); return 0;
+  }
 #undef SCAN
-  return 0;
+  return -1;
 }
 
-int launch_hgrn2_scan(float* o, const void* proj, float* state,
+int launch_hgrn2_scan(float* o, float* work, const void* proj, float* state,
                       const float* f_bias, const float* lower, SegView seg,
-                      int heads, int dim, int vdim, int vstride, int f32,
-                      hipStream_t stream) {
-  return f32 ? hgrn2_scan_t<float>(o, proj, state, f_bias, lower, seg, heads,
-                                   dim, vdim, vstride, stream)
-             : hgrn2_scan_t<bf16>(o, proj, state, f_bias, lower, seg, heads,
-                                  dim, vdim, vstride, stream);
+                      int max_len, int heads, int dim, int vdim, int vstride,
+                      int f32, hipStream_t stream) {
+  return f32 ? hgrn2_scan_t<float>(o, work, proj, state, f_bias, lower, seg,
+                                   max_len, heads, dim, vdim, vstride, stream)
+             : hgrn2_scan_t<bf16>(o, work, proj, state, f_bias, lower, seg,
+                                  max_len, heads, dim, vdim, vstride, stream);
 }
 
-template <typename T>
+// one wave per (row, head); V columns per access, up to 4 accesses kept
+template <typename T, int V>
 __global__ __launch_bounds__(256) void head_norm_kernel(
     T* __restrict__ out, const float* __restrict__ o,
     const float* __restrict__ w, SegView seg, int heads, int vdim,
     float eps) {
-  const int s = blockIdx.z, t = blockIdx.x;
-  if (t >= seg.len[s]) return;
-  const int lane = threadIdx.x & 63;
-  for (int h = blockIdx.y * 4 + (threadIdx.x >> 6); h < heads;
-       h += gridDim.y * 4) {
-    const size_t base =
-        ((size_t)seg.start[s] + t) * heads * vdim + (size_t)h * vdim;
-    float ss = 0.f;
-    for (int c = lane; c < vdim; c += 64) ss += o[base + c] * o[base + c];
-    const float r = 1.f / sqrtf(wave_sum(ss) / vdim + eps);
-    for (int c = lane; c < vdim; c += 64)
-      out[base + c] = from_f<T>(o[base + c] * r * w[c]);
+  constexpr int KEEP = 16 / V;
+  const int s = blockIdx.z, lane = threadIdx.x & 63;
+  const long long i =
+      ((long long)blockIdx.x * 256 + threadIdx.x) >> 6;  // (row, head)
+  if (i >= (long long)seg.len[s] * heads) return;
+  const size_t base = ((size_t)seg.start[s] * heads + i) * vdim;
+  Pack<float, V> a[KEEP];
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < KEEP; ++k) {
+    const int c = (k * 64 + lane) * V;
+    if (c >= vdim) break;
+    a[k] = *reinterpret_cast<const Pack<float, V>*>(o + base + c);
+#pragma unroll
+    for (int j = 0; j < V; ++j) ss += a[k].v[j] * a[k].v[j];
   }
+  const float r = 1.f / sqrtf(wave_sum(ss) / vdim + eps);
+#pragma unroll
+  for (int k = 0; k < KEEP; ++k) {
+    const int c = (k * 64 + lane) * V;
+    if (c >= vdim) break;
+    Pack<T, V> b;
+#pragma unroll
+    for (int j = 0; j < V; ++j) b.v[j] = from_f<T>(a[k].v[j] * r * w[c + j]);
+    *reinterpret_cast<Pack<T, V>*>(out + base + c) = b;
+  }
+}
+
+template <typename T>
+static void head_norm_t(void* out, const float* o, const float* w,
+                        SegView seg, int max_len, int heads, int vdim,
+                        float eps, hipStream_t stream) {
+  dim3 grid((unsigned)(((long long)max_len * heads + 3) / 4), 1, seg.n);
+  if (vdim % 2 == 0)
+    head_norm_kernel<T, 2><<<grid, 256, 0, stream>>>((T*)out, o, w, seg,
+                                                     heads, vdim, eps);
+  else
+    head_norm_kernel<T, 1><<<grid, 256, 0, stream>>>((T*)out, o, w, seg,
+                                                     heads, vdim, eps);
 }
 
 void launch_head_norm(void* out, const float* o, const float* w, SegView seg,
                       int max_len, int heads, int vdim, float eps, int f32,
                       hipStream_t stream) {
-  dim3 grid(max_len, (heads + 3) / 4, seg.n);
   if (f32)
-    head_norm_kernel<float><<<grid, 256, 0, stream>>>((float*)out, o, w, seg,
-                                                      heads, vdim, eps);
+    head_norm_t<float>(out, o, w, seg, max_len, heads, vdim, eps, stream);
   else
-    head_norm_kernel<bf16><<<grid, 256, 0, stream>>>((bf16*)out, o, w, seg,
-                                                     heads, vdim, eps);
+    head_norm_t<bf16>(out, o, w, seg, max_len, heads, vdim, eps, stream);
 }
 
 // ---------------------------------------------------------------------------
-// q/k head norms + cache append: one wave per (row, head of q, k or v)
+// q/k head norms + cache append.  q and k: a group of L lanes per (row,
+// head), V channels per lane.  v: pages are transposed, so a wave takes 64
+// consecutive rows by V columns and writes along the rows.
 // ---------------------------------------------------------------------------
-template <typename T>
+template <typename T, int V, int L>
 __global__ __launch_bounds__(256) void qk_norm_append_kernel(
-    T* __restrict__ q_out, T* __restrict__ kpages, T* __restrict__ vpages,
+    T* __restrict__ q_out, T* __restrict__ kpages,
     const T* __restrict__ proj, const float* __restrict__ q_w,
     const float* __restrict__ k_w, const int* __restrict__ row_slot,
     const int* __restrict__ row_pos, const int* __restrict__ table,
-    int table_stride, int heads, int kv_heads, int dim, int vdim, int dpad,
-    int vpad, float eps) {
-  const int hd = blockIdx.y * 4 + (threadIdx.x >> 6);
-  if (hd >= heads + 2 * kv_heads) return;
-  const int lane = threadIdx.x & 63;
-  const size_t row = blockIdx.x;
-  const T* pr = proj + row * (size_t)((heads + kv_heads) * dim +
-                                      kv_heads * vdim);
+    int table_stride, int n, int heads, int kv_heads, int dim, int vdim,
+    int dpad, float eps) {
+  constexpr int PER = 256 / L;  // (row, head) pairs per block
+  using P = Pack<T, V>;
+  const int hk = heads + kv_heads;
+  const long long i = (long long)blockIdx.x * PER + threadIdx.x / L;
+  if (i >= (long long)n * hk) return;
+  const int lane = threadIdx.x % L;
+  const size_t row = i / hk;
+  const int hd = (int)(i - row * hk);
+  const bool is_q = hd < heads;
+  const T* src = proj + row * (size_t)(hk * dim + kv_heads * vdim) +
+                 (size_t)hd * dim;
+  const float* w = is_q ? q_w : k_w;
+  T* dst;
+  if (is_q) {
+    dst = q_out + (row * heads + hd) * (size_t)dpad;
+  } else {
+    const int pos = row_pos[row];
+    const size_t page =
+        table[(size_t)row_slot[row] * table_stride + (pos >> 6)];
+    dst = kpages + ((page * kv_heads + (hd - heads)) * 64 + (pos & 63)) *
+                       (size_t)dpad;
+  }
+  // dpad <= 256: at most 256 / (V * L) accesses per lane
+  constexpr int KEEP = 256 / (V * L);
+  P a[KEEP];
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < KEEP; ++k) {
+    const int d = (k * L + lane) * V;
+    if (d >= dim) break;
+    a[k] = *reinterpret_cast<const P*>(src + d);
+#pragma unroll
+    for (int j = 0; j < V; ++j) ss += to_f(a[k].v[j]) * to_f(a[k].v[j]);
+  }
+#pragma unroll
+  for (int off = L / 2; off > 0; off >>= 1) ss += __shfl_xor(ss, off, 64);
+  const float r = 1.f / sqrtf(ss / dim + eps);
+#pragma unroll
+  for (int k = 0; k < KEEP; ++k) {
+    const int d = (k * L + lane) * V;
+    if (d >= dpad) break;
+    P b;
+#pragma unroll
+    for (int j = 0; j < V; ++j)
+      b.v[j] = from_f<T>(d < dim ? to_f(a[k].v[j]) * r * w[d + j] : 0.f);
+    *reinterpret_cast<P*>(dst + d) = b;
+  }
+}
+
+template <typename T, int V>
+__global__ __launch_bounds__(256) void v_append_kernel(
+    T* __restrict__ vpages, const T* __restrict__ proj,
+    const int* __restrict__ row_slot, const int* __restrict__ row_pos,
+    const int* __restrict__ table, int table_stride, int n, int heads,
+    int kv_heads, int dim, int vdim, int vpad) {
+  const int chunks = kv_heads * (vdim / V);
+  const int ch = blockIdx.y * 4 + (threadIdx.x >> 6);
+  const size_t row = (size_t)blockIdx.x * 64 + (threadIdx.x & 63);
+  if (ch >= chunks || row >= n) return;
+  const int g = ch / (vdim / V), c = (ch % (vdim / V)) * V;
+  const size_t qk = (size_t)(heads + kv_heads) * dim;
+  const Pack<T, V> a = *reinterpret_cast<const Pack<T, V>*>(
+      proj + row * (qk + kv_heads * vdim) + qk + (size_t)g * vdim + c);
   const int pos = row_pos[row];
   const size_t page =
       table[(size_t)row_slot[row] * table_stride + (pos >> 6)];
-  if (hd >= heads + kv_heads) {
-    const int g = hd - heads - kv_heads;
-    const T* v = pr + (size_t)(heads + kv_heads) * dim + g * vdim;
-    T* dst = vpages + (page * kv_heads + g) * (size_t)vpad * 64 + (pos & 63);
-    for (int c = lane; c < vdim; c += 64) dst[(size_t)c * 64] = v[c];
-    return;
-  }
-  const T* src = pr + (size_t)hd * dim;
-  float ss = 0.f;
-  for (int d = lane; d < dim; d += 64) ss += to_f(src[d]) * to_f(src[d]);
-  const float r = 1.f / sqrtf(wave_sum(ss) / dim + eps);
-  const bool is_q = hd < heads;
-  const float* w = is_q ? q_w : k_w;
-  T* dst = is_q ? q_out + (row * heads + hd) * (size_t)dpad
-                : kpages + ((page * kv_heads + (hd - heads)) * 64 +
-                            (pos & 63)) * (size_t)dpad;
-  for (int d = lane; d < dpad; d += 64)
-    dst[d] = from_f<T>(d < dim ? to_f(src[d]) * r * w[d] : 0.f);
+  T* dst = vpages + ((page * kv_heads + g) * (size_t)vpad + c) * 64 +
+           (pos & 63);
+#pragma unroll
+  for (int j = 0; j < V; ++j) dst[(size_t)j * 64] = a.v[j];
+}
+
+template <typename T, int V, int L>
+static void append_t(void* q_out, void* kpages, void* vpages,
+                     const void* proj, const float* q_w, const float* k_w,
+                     const int* row_slot, const int* row_pos,
+                     const int* table, int table_stride, int n, int heads,
+                     int kv_heads, int dim, int vdim, int dpad, int vpad,
+                     float eps, hipStream_t stream) {
+  const long long pairs = (long long)n * (heads + kv_heads);
+  qk_norm_append_kernel<T, V, L>
+      <<<(unsigned)((pairs + 256 / L - 1) / (256 / L)), 256, 0, stream>>>(
+          (T*)q_out, (T*)kpages, (const T*)proj, q_w, k_w, row_slot, row_pos,
+          table, table_stride, n, heads, kv_heads, dim, vdim, dpad, eps);
+  const int chunks = kv_heads * (vdim / V);
+  v_append_kernel<T, V>
+      <<<dim3((n + 63) / 64, (chunks + 3) / 4), 256, 0, stream>>>(
+          (T*)vpages, (const T*)proj, row_slot, row_pos, table, table_stride,
+          n, heads, kv_heads, dim, vdim, vpad);
 }
 
 void launch_qk_norm_append(void* q_out, void* kpages, void* vpages,
@@ -455,17 +703,18 @@ void launch_qk_norm_append(void* q_out, void* kpages, void* vpages,
                            int table_stride, int n, int heads, int kv_heads,
                            int dim, int vdim, int dpad, int vpad, float eps,
                            int f32, hipStream_t stream) {
-  dim3 grid(n, (heads + 2 * kv_heads + 3) / 4);
-  if (f32)
-    qk_norm_append_kernel<float><<<grid, 256, 0, stream>>>(
-        (float*)q_out, (float*)kpages, (float*)vpages, (const float*)proj,
-        q_w, k_w, row_slot, row_pos, table, table_stride, heads, kv_heads,
-        dim, vdim, dpad, vpad, eps);
-  else
-    qk_norm_append_kernel<bf16><<<grid, 256, 0, stream>>>(
-        (bf16*)q_out, (bf16*)kpages, (bf16*)vpages, (const bf16*)proj, q_w,
-        k_w, row_slot, row_pos, table, table_stride, heads, kv_heads, dim,
-        vdim, dpad, vpad, eps);
+#define APPEND(T, V, L)                                                     \
+  append_t<T, V, L>(q_out, kpages, vpages, proj, q_w, k_w, row_slot,        \
+                    row_pos, table, table_stride, n, heads, kv_heads, dim,  \
+                    vdim, dpad, vpad, eps, stream)
+  if (f32) {
+    if (dim % 4 == 0 && vdim % 4 == 0) APPEND(float, 4, 16);
+    else APPEND(float, 1, 64);
+  } else {
+    if (dim % 8 == 0 && vdim % 8 == 0) APPEND(bf16, 8, 16);
+    else APPEND(bf16, 1, 64);
+  }
+#undef APPEND
 }
 
 // ---------------------------------------------------------------------------

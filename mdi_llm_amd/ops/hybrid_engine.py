@@ -209,8 +209,7 @@ class HybridEngine:
             self.ops.hgrn2_step(y, proj, state, lw.f_bias, lw.lower, lw.norm,
                                 b.seg[:, :b.singles], eps)
         if b.singles < b.seg.size(1):
-            o = torch.empty(y.shape, dtype=torch.float32, device=self.device)
-            self.ops.hgrn2_scan(y, o, proj, state, lw.f_bias, lw.lower,
+            self.ops.hgrn2_scan(y, proj, state, lw.f_bias, lw.lower,
                                 lw.norm, b.seg[:, b.singles:], b.max_len, eps)
         return self._linear(y, lw.proj)
 
@@ -220,7 +219,7 @@ class HybridEngine:
         tiles = min(-(-max_ctx // 32),
                     -(-m.window // 32) + -(-m.keep_first // 32) + 1)
         want = -(-512 // (n_seg * m.kv_heads))
-        return max(1, min(want, -(-tiles // 8)))
+        return max(1, min(want, -(-tiles // 8), 256))
 
     def _attention(self, i: int, lw: _LayerWeights, b: Batch,
                    xn: torch.Tensor):
@@ -331,7 +330,7 @@ class HybridEngine:
     # ------------------------------------------------------------------
     # public steps
     # ------------------------------------------------------------------
-    @torch.inference_mode()
+    @torch.no_grad()
     def step(self, entries: Sequence[Tuple[int, Sequence[int]]],
              want: Optional[Sequence[Sequence[int]]] = None,
              layers_out: Optional[list] = None) -> Optional[torch.Tensor]:
@@ -359,7 +358,7 @@ class HybridEngine:
             xn = xn[torch.tensor(rows, device=self.device)]
         return self._linear(xn, self.head)
 
-    @torch.inference_mode()
+    @torch.no_grad()
     def hidden(self, slot: int, tokens: Optional[Sequence[int]] = None,
                x: Optional[torch.Tensor] = None) -> torch.Tensor:
         """Pipeline stages: one sequence's tokens (starter) or residual rows
@@ -372,7 +371,7 @@ class HybridEngine:
         b, _ = self._batch([(slot, n)], tokens)
         return self._run(b, x, False)[0]
 
-    @torch.inference_mode()
+    @torch.no_grad()
     def logits(self, x: torch.Tensor) -> torch.Tensor:
         """Residual rows -> logits."""
         x = x.reshape(-1, self.config.n_embd).float().contiguous()
@@ -411,7 +410,7 @@ class HybridEngine:
         self._steps[size] = st
         return st
 
-    @torch.inference_mode()
+    @torch.no_grad()
     def decode(self, slots: Sequence[int],
                tokens: Optional[Sequence[int]] = None,
                keys: Optional[Sequence[int]] = None) -> torch.Tensor:
@@ -442,7 +441,7 @@ class HybridEngine:
         self._last = st
         return st.logits[:len(slots)]
 
-    @torch.inference_mode()
+    @torch.no_grad()
     def sample_decoded(self, temperature: float, top_k, seed: int,
                        top_p: float = 1.0) -> torch.Tensor:
         """Draw from the logits of the last ``decode`` on the device (bf16
@@ -480,7 +479,7 @@ class HybridEngine:
                         seed & 0x7FFFFFFF, pos, keys, logits.size(0), p,
                         pos_bias=pos_bias)
 
-    @torch.inference_mode()
+    @torch.no_grad()
     def sample(self, logits: torch.Tensor, temperature: float, top_k, seed,
                top_p: float, pos: Sequence[int], keys: Sequence[int],
                generators=None) -> List[int]:

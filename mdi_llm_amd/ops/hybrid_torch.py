@@ -39,8 +39,7 @@ def _segments(seg):
     return seg.t().tolist()  # rows of (start, len, slot, pos0)
 
 
-def hgrn2_scan(out, o, proj, state, f_bias, lower, norm_w, seg, max_len,
-               eps) -> None:
+def hgrn2_scan(out, proj, state, f_bias, lower, norm_w, seg, max_len, eps) -> None:
     _, H, D, _ = state.shape
     E = norm_w.numel()
     q, f, v = proj.float().split((H * D, H * D, H * E), dim=1)
@@ -58,7 +57,7 @@ def hgrn2_scan(out, o, proj, state, f_bias, lower, norm_w, seg, max_len,
 
 
 def hgrn2_step(out, proj, state, f_bias, lower, norm_w, seg, eps) -> None:
-    hgrn2_scan(out, None, proj, state, f_bias, lower, norm_w, seg, 1, eps)
+    hgrn2_scan(out, proj, state, f_bias, lower, norm_w, seg, 1, eps)
 
 
 def qk_norm_append(q_out, kpages, vpages, proj, q_w, k_w, row_slot, row_pos,

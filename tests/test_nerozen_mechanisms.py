@@ -146,8 +146,7 @@ def test_hgrn2_scan_and_step(H, D, E, device, dtype):
         if step:
             ops.hgrn2_step(y, flat, state, fb, lower, w, s, eps)
         else:
-            ops.hgrn2_scan(y, torch.empty(y.shape, device=device), flat,
-                           state, fb, lower, w, s, m, eps)
+            ops.hgrn2_scan(y, flat, state, fb, lower, w, s, m, eps)
         assert float(y[:2].abs().max()) == float(y[2 + m:].abs().max()) == 0
         got[seq][at:at + m] = y[2:2 + m]
 
@@ -178,8 +177,7 @@ def test_hgrn2_holds_a_far_token(device, dtype):
     first = oracle.rms(proj[0, 2 * D:].double().cpu(), 1e-5)
     state = torch.zeros(2, H, D, E, device=device)
     y = torch.zeros(n, E, dtype=dtype, device=device)
-    ops.hgrn2_scan(y, torch.empty(y.shape, device=device), proj, state, fb,
-                   lower, w, seg([(0, n, 0, 0)], device), n, 1e-5)
+    ops.hgrn2_scan(y, proj, state, fb, lower, w, seg([(0, n, 0, 0)], device), n, 1e-5)
     close(y[n - 1], first, dtype)
     ops.hgrn2_step(y, proj, state, fb, lower, w,
                    seg([(n - 1, 1, 0, n)], device), 1e-5)
