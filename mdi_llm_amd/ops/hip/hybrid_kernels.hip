@@ -392,19 +392,22 @@ __global__ __launch_bounds__(256) void hgrn2_chunks_kernel(
   constexpr int DP = 64 * TPW;
   using W = ChunkWork<DP>;
   __shared__ float red[2][4][16][17];
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int tid = threadIdx.x, lane = tid & 63;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int c = lane & 15, quad = lane >> 4;
-  const int s = blockIdx.z, h = blockIdx.y, c0 = blockIdx.x * 16;
+  // heads vary fastest: the column blocks of a head share an XCD's L2
+  const int s = blockIdx.z, h = blockIdx.x, c0 = blockIdx.y * 16;
   const int col = c0 + c, d0 = wave * TPW * 16;
   const int len = seg.len[s], n = (len + 15) / 16;
   const size_t row0 = seg.start[s];
   const size_t ld = (size_t)heads * (2 * dim + vdim);
   const float* w = work + ((row0 / 16 + s) * heads + h) * W::SIZE;
   const size_t wstep = (size_t)heads * W::SIZE;
-  const T* vp = proj + row0 * ld + 2 * heads * dim + h * vdim + col;
+  const T* vp = proj + row0 * ld + 2 * heads * dim + h * vdim +
+                min(col, vdim - 1);
   float* S = state +
              ((size_t)seg.slot[s] * heads + h) * (size_t)dim * vstride + col;
-  const bool keep = col < vstride && seg.pos0[s] != 0;
+  const bool keep = col < vdim && seg.pos0[s] != 0;
 
   f32x4 st[TPW];
 #pragma unroll
@@ -415,10 +418,14 @@ __global__ __launch_bounds__(256) void hgrn2_chunks_kernel(
       st[k][i] = keep && d < dim ? S[(size_t)d * vstride] : 0.f;
     }
 
+  // operands of the next chunks on their way (values stay unconverted, so
+  // that nothing waits for them early)
+  constexpr int AHEAD = TPW <= 2 ? 4 : 2;
   struct Operands {
     f32x4 qr[TPW], uk[TPW], decay[TPW];
-    float p, v[4], vw;
-  } cur, nxt;
+    float p;
+    T v[4], vw;
+  } ring[AHEAD];
   auto load = [&](Operands& a, int ch) {
     const float* wc = w + ch * wstep;
 #pragma unroll
@@ -431,50 +438,64 @@ __global__ __launch_bounds__(256) void hgrn2_chunks_kernel(
           wc + W::DECAY + d0 + k * 16 + quad * 4);
     }
     a.p = wc[W::P + c * 16 + quad * 4 + wave];
-    auto value = [&](int t) {
-      return col < vdim && t < len ? to_f(vp[(size_t)t * ld]) : 0.f;
-    };
+    // rows and columns past the end repeat the last: they meet zero factors
+    // or are not stored
+    auto value = [&](int t) { return vp[(size_t)min(t, len - 1) * ld]; };
 #pragma unroll
     for (int i = 0; i < 4; ++i) a.v[i] = value(ch * 16 + quad * 4 + i);
     a.vw = value(ch * 16 + quad * 4 + wave);
   };
-  load(cur, 0);
-  for (int ch = 0; ch < n; ++ch) {
-    if (ch + 1 < n) load(nxt, ch + 1);
+  auto chunk = [&](const Operands& a, int ch) {
     // two accumulators: half the dependent chain
     f32x4 a0{0.f, 0.f, 0.f, 0.f}, a1 = a0;
-    a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.p, cur.vw, a0, 0, 0, 0);
+    a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(a.p, to_f(a.vw), a0, 0, 0, 0);
 #pragma unroll
     for (int k = 0; k < TPW; ++k) {
-      a1 = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.qr[k][0], st[k][0], a1, 0, 0, 0);
-      a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.qr[k][1], st[k][1], a0, 0, 0, 0);
-      a1 = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.qr[k][2], st[k][2], a1, 0, 0, 0);
-      a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.qr[k][3], st[k][3], a0, 0, 0, 0);
+      a1 = __builtin_amdgcn_mfma_f32_16x16x4f32(a.qr[k][0], st[k][0], a1, 0, 0, 0);
+      a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(a.qr[k][1], st[k][1], a0, 0, 0, 0);
+      a1 = __builtin_amdgcn_mfma_f32_16x16x4f32(a.qr[k][2], st[k][2], a1, 0, 0, 0);
+      a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(a.qr[k][3], st[k][3], a0, 0, 0, 0);
     }
 #pragma unroll
-    for (int k = 0; k < TPW; ++k) st[k] *= cur.decay[k];
+    for (int k = 0; k < TPW; ++k) st[k] *= a.decay[k];
 #pragma unroll
     for (int i = 0; i < 4; ++i)
 #pragma unroll
       for (int k = 0; k < TPW; ++k)
-        st[k] = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.uk[k][i], cur.v[i],
+        st[k] = __builtin_amdgcn_mfma_f32_16x16x4f32(a.uk[k][i], to_f(a.v[i]),
                                                      st[k], 0, 0, 0);
     a0 += a1;
 #pragma unroll
     for (int i = 0; i < 4; ++i) red[ch & 1][wave][quad * 4 + i][c] = a0[i];
+  };
+  auto emit = [&](int ch) {
     __syncthreads();  // one per chunk: the other half is written next
-    {
-      const int t = tid >> 4, e = tid & 15, tt = ch * 16 + t;
-      if (tt < len && c0 + e < vdim) {
-        float v = 0.f;
+    const int t = tid >> 4, e = tid & 15, tt = ch * 16 + t;
+    if (tt < len && c0 + e < vdim) {
+      float v = 0.f;
 #pragma unroll
-        for (int k = 0; k < 4; ++k) v += red[ch & 1][k][t][e];
-        o[(row0 + tt) * (size_t)(heads * vdim) + h * vdim + c0 + e] = v;
-      }
+      for (int k = 0; k < 4; ++k) v += red[ch & 1][k][t][e];
+      o[(row0 + tt) * (size_t)(heads * vdim) + h * vdim + c0 + e] = v;
     }
-    cur = nxt;
+  };
+#pragma unroll
+  for (int r = 0; r < AHEAD; ++r) load(ring[r], min(r, n - 1));
+  int base = 0;
+  for (; base + AHEAD <= n; base += AHEAD) {
+#pragma unroll
+    for (int r = 0; r < AHEAD; ++r) {
+      chunk(ring[r], base + r);
+      load(ring[r], min(base + r + AHEAD, n - 1));
+      emit(base + r);
+    }
   }
-  if (col < vstride) {
+#pragma unroll
+  for (int r = 0; r < AHEAD - 1; ++r)
+    if (base + r < n) {
+      chunk(ring[r], base + r);
+      emit(base + r);
+    }
+  if (col < vdim) {
 #pragma unroll
     for (int k = 0; k < TPW; ++k)
 #pragma unroll
@@ -504,7 +525,7 @@ static void hgrn2_scan_sized(float* o, float* work, const void* proj,
       <<<dim3((max_len + 15) / 16, heads, seg.n), 256, 0, stream>>>(
           work, (const T*)proj, f_bias, lower, seg, heads, dim, vdim);
   hgrn2_chunks_kernel<T, TPW>
-      <<<dim3((vdim + 15) / 16, heads, seg.n), 256, 0, stream>>>(
+      <<<dim3(heads, (vdim + 15) / 16, seg.n), 256, 0, stream>>>(
           o, work, (const T*)proj, state, seg, heads, dim, vdim, vstride);
 }
 
