@@ -7,10 +7,11 @@ state per slot.  One page table serves all attention layers of the stage:
 page ``p`` is row ``p`` of every layer's arena.
 
 Layout (what the kernels in ``paged_attn.inc`` and ``hybrid_kernels.hip``
-read): K pages ``[pages, kv_heads, 64, dpad]``, V pages transposed
-``[pages, kv_heads, vpad, 64]``, states ``[slots, heads, dim, vstride]`` in
-fp32.  Padding is zero and stays zero.  A state needs no clearing when its
-slot is taken again: kernels start from zero at position 0.
+read): K pages ``[pages, kv_heads, 64 * dpad]`` and V pages ``[pages,
+kv_heads, 64 * vpad]`` in MFMA operand order (``k_index``, ``v_index``),
+states ``[slots, heads, dim, vstride]`` in fp32.  Nothing needs clearing when
+a page or slot is taken again: keys past a sequence's end are masked, and
+the recurrence starts from zero at position 0.
 """
 
 from __future__ import annotations
@@ -19,7 +20,7 @@ from typing import Dict, List, Optional, Sequence
 
 import torch
 
-__all__ = ["HybridCache", "CacheFull", "PAGE"]
+__all__ = ["HybridCache", "CacheFull", "PAGE", "k_index", "v_index"]
 
 PAGE = 64
 
@@ -33,6 +34,28 @@ def _pad_to(n: int, sizes: Sequence[int], what: str) -> int:
         if n <= s:
             return s
     raise ValueError(f"{what} {n} is larger than {sizes[-1]}")
+
+
+def _in_block(row: torch.Tensor, step: torch.Tensor) -> torch.Tensor:
+    """Place in a 16 x 32 block: lane (quad of steps, row) holds four steps
+    of either half."""
+    return ((step % 16 // 4) * 16 + row) * 8 + step // 16 * 4 + step % 4
+
+
+def k_index(dpad: int) -> torch.Tensor:
+    """[64 keys, dpad channels] -> place in a K page."""
+    key = torch.arange(PAGE).view(-1, 1)
+    d = torch.arange(dpad).view(1, -1)
+    return (key // 16 * (dpad // 32) + d // 32) * 512 \
+        + _in_block(key % 16, d % 32)
+
+
+def v_index(vpad: int) -> torch.Tensor:
+    """[64 keys, vpad columns] -> place in a V page."""
+    key = torch.arange(PAGE).view(-1, 1)
+    c = torch.arange(vpad).view(1, -1)
+    return (key // 32 * (vpad // 16) + c // 16) * 512 \
+        + _in_block(c % 16, key % 32)
 
 
 class HybridCache:
@@ -57,9 +80,9 @@ class HybridCache:
                 dpad = _pad_to(m.dim, (32, 64, 128, 256), "attention dim")
                 vpad = _pad_to(m.vdim, (32, 64, 128, 256), "attention vdim")
                 P, G = self.n_pages + 1, m.kv_heads
-                self.k[i] = torch.zeros(P, G, PAGE, dpad, device=device,
+                self.k[i] = torch.zeros(P, G, PAGE * dpad, device=device,
                                         dtype=dtype)
-                self.v[i] = torch.zeros(P, G, vpad, PAGE, device=device,
+                self.v[i] = torch.zeros(P, G, PAGE * vpad, device=device,
                                         dtype=dtype)
             else:
                 vstride = -(-m.vdim // 4) * 4

@@ -167,11 +167,11 @@ struct Pages {
 Pages pages(const torch::Tensor& k, const torch::Tensor& v, int f32) {
   check_like(k, f32, "kpages");
   check_like(v, f32, "vpages");
-  TORCH_CHECK(k.dim() == 4 && v.dim() == 4 && k.size(0) == v.size(0) &&
-                  k.size(1) == v.size(1) && k.size(2) == 64 &&
-                  v.size(3) == 64,
-              "pages: expected k [P, G, 64, dpad] and v [P, G, vpad, 64]");
-  return Pages{(int)k.size(1), (int)k.size(3), (int)v.size(2)};
+  TORCH_CHECK(k.dim() == 3 && v.dim() == 3 && k.size(0) == v.size(0) &&
+                  k.size(1) == v.size(1) && k.size(2) % (64 * 32) == 0 &&
+                  v.size(2) % (64 * 32) == 0,
+              "pages: expected k [P, G, 64 * dpad] and v [P, G, 64 * vpad]");
+  return Pages{(int)k.size(1), (int)k.size(2) / 64, (int)v.size(2) / 64};
 }
 
 void qk_norm_append(torch::Tensor q_out, torch::Tensor kpages,

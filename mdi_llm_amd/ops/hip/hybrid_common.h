@@ -40,4 +40,27 @@ DEVINL float row16_sum(float v) {
   return v;
 }
 
+// Order of one kv head's 64 keys in a page.  A page is made of 16 x 32 blocks
+// (K: keys x channels, V: columns x keys), each in the order in which a
+// wave's lanes hold it as an MFMA operand: lane (quad, row) has steps
+// quad*4 .. +3 of the first and of the second half of the 32.
+struct PageLayout {
+  static DEVINL int in_block(int row, int step) {
+    return ((((step & 15) >> 2) * 16 + row) << 3) + ((step >> 4) << 2) +
+           (step & 3);
+  }
+  static DEVINL int k_block(int key_tile, int chunk, int dpad) {
+    return (key_tile * (dpad >> 5) + chunk) << 9;
+  }
+  static DEVINL int v_block(int col_tile, int key_half, int vpad) {
+    return (key_half * (vpad >> 4) + col_tile) << 9;
+  }
+  static DEVINL int k(int key, int d, int dpad) {
+    return k_block(key >> 4, d >> 5, dpad) + in_block(key & 15, d & 31);
+  }
+  static DEVINL int v(int key, int col, int vpad) {
+    return v_block(col >> 4, key >> 5, vpad) + in_block(col & 15, key & 31);
+  }
+};
+
 DEVINL float sigmoid(float z) { return 1.f / (1.f + expf(-z)); }

@@ -54,8 +54,8 @@ void launch_head_norm(void* out, const float* o, const float* w, SegView seg,
                       hipStream_t stream);
 
 // Per-head q/k norms, q to a padded buffer, k and v into the paged cache.
-// proj [n, (H+G)*D + G*E] = q|k|v; k pages [P, G, 64, dpad],
-// v pages [P, G, vpad, 64].
+// proj [n, (H+G)*D + G*E] = q|k|v; k pages [P, G, 64 * dpad] and v pages
+// [P, G, 64 * vpad] in the order of PageLayout.
 void launch_qk_norm_append(void* q_out, void* kpages, void* vpages,
                            const void* proj, const float* q_w,
                            const float* k_w, const int* row_slot,

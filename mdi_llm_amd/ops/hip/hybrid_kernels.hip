@@ -615,8 +615,8 @@ void launch_head_norm(void* out, const float* o, const float* w, SegView seg,
 
 // ---------------------------------------------------------------------------
 // q/k head norms + cache append.  q and k: a group of L lanes per (row,
-// head), V channels per lane.  v: pages are transposed, so a wave takes 64
-// consecutive rows by V columns and writes along the rows.
+// head), V channels per lane.  v: pages run along the keys, so a wave takes
+// 64 consecutive rows by V columns.
 // ---------------------------------------------------------------------------
 template <typename T, int V, int L>
 __global__ __launch_bounds__(256) void qk_norm_append_kernel(
@@ -639,14 +639,15 @@ __global__ __launch_bounds__(256) void qk_norm_append_kernel(
                  (size_t)hd * dim;
   const float* w = is_q ? q_w : k_w;
   T* dst;
+  int key = 0;
   if (is_q) {
     dst = q_out + (row * heads + hd) * (size_t)dpad;
   } else {
     const int pos = row_pos[row];
     const size_t page =
         table[(size_t)row_slot[row] * table_stride + (pos >> 6)];
-    dst = kpages + ((page * kv_heads + (hd - heads)) * 64 + (pos & 63)) *
-                       (size_t)dpad;
+    key = pos & 63;
+    dst = kpages + (page * kv_heads + (hd - heads)) * (size_t)(64 * dpad);
   }
   // dpad <= 256: at most 256 / (V * L) accesses per lane
   constexpr int KEEP = 256 / (V * L);
@@ -671,7 +672,17 @@ __global__ __launch_bounds__(256) void qk_norm_append_kernel(
 #pragma unroll
     for (int j = 0; j < V; ++j)
       b.v[j] = from_f<T>(d < dim ? to_f(a[k].v[j]) * r * w[d + j] : 0.f);
-    *reinterpret_cast<P*>(dst + d) = b;
+    if (is_q) {
+      *reinterpret_cast<P*>(dst + d) = b;
+    } else {
+      // runs of four channels stay together in a page
+      constexpr int RUN = V < 4 ? V : 4;
+#pragma unroll
+      for (int j = 0; j < V; j += RUN)
+        *reinterpret_cast<Pack<T, RUN>*>(
+            dst + PageLayout::k(key, d + j, dpad)) =
+            *reinterpret_cast<const Pack<T, RUN>*>(b.v + j);
+    }
   }
 }
 
@@ -692,10 +703,10 @@ __global__ __launch_bounds__(256) void v_append_kernel(
   const int pos = row_pos[row];
   const size_t page =
       table[(size_t)row_slot[row] * table_stride + (pos >> 6)];
-  T* dst = vpages + ((page * kv_heads + g) * (size_t)vpad + c) * 64 +
-           (pos & 63);
+  T* dst = vpages + (page * kv_heads + g) * (size_t)(64 * vpad);
 #pragma unroll
-  for (int j = 0; j < V; ++j) dst[(size_t)j * 64] = a.v[j];
+  for (int j = 0; j < V; ++j)
+    dst[PageLayout::v(pos & 63, c + j, vpad)] = a.v[j];
 }
 
 template <typename T, int V, int L>

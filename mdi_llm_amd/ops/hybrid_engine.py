@@ -226,7 +226,7 @@ class HybridEngine:
         m, eps, c = lw.mixer, self.config.norm_eps, self.cache
         proj = self._linear(xn, lw.in_proj)
         k, v = c.k[i], c.v[i]
-        q = torch.empty(b.n, m.heads, k.size(3), dtype=self.dtype,
+        q = torch.empty(b.n, m.heads, k.size(2) // PAGE, dtype=self.dtype,
                         device=self.device)
         self.ops.qk_norm_append(q, k, v, proj, lw.q_norm, lw.k_norm,
                                 b.row_slot, b.row_pos, c.table, m.vdim, eps)
@@ -243,7 +243,7 @@ class HybridEngine:
             part = (None, None)
             if splits > 1:
                 cells = b.singles * m.heads * splits
-                part = (torch.empty(cells * v.size(2), dtype=torch.float32,
+                part = (torch.empty(cells * v.size(2) // PAGE, dtype=torch.float32,
                                     device=self.device),
                         torch.empty(cells * 2, dtype=torch.float32,
                                     device=self.device))

@@ -9,6 +9,8 @@ from __future__ import annotations
 
 import torch
 
+from ..models.cache import PAGE, k_index, v_index
+
 __all__ = ["residual_norm", "xielu", "hgrn2_step", "hgrn2_scan",
            "qk_norm_append", "paged_attn", "advance_batch"]
 
@@ -62,31 +64,34 @@ def hgrn2_step(out, proj, state, f_bias, lower, norm_w, seg, eps) -> None:
 
 def qk_norm_append(q_out, kpages, vpages, proj, q_w, k_w, row_slot, row_pos,
                    table, vdim, eps) -> None:
-    n, H = q_out.shape[:2]
-    G, P = kpages.shape[1:3]
+    n, H, dpad = q_out.shape
+    G = kpages.size(1)
     D = q_w.numel()
     q, k, v = proj.split((H * D, G * D, G * vdim), dim=1)
     q_out.zero_()
     q_out[..., :D] = (_rms(q.reshape(n, H, D), eps) * q_w).to(q_out.dtype)
     pos = row_pos.long()
-    page = table[row_slot.long(), pos // P].long()
-    kpages[page, :, pos % P, :D] = (
+    page = table[row_slot.long(), pos // PAGE].long().view(n, 1, 1)
+    head = torch.arange(G).view(1, G, 1)
+    at = k_index(dpad)[pos % PAGE, :D].view(n, 1, D)
+    kpages[page, head, at] = (
         _rms(k.reshape(n, G, D), eps) * k_w).to(kpages.dtype)
-    vpages[page, :, :vdim, pos % P] = v.reshape(n, G, vdim)
+    at = v_index(vpages.size(2) // PAGE)[pos % PAGE, :vdim].view(n, 1, vdim)
+    vpages[page, head, at] = v.reshape(n, G, vdim)
 
 
 def paged_attn(out, q, kpages, vpages, bias, table, seg, max_len, window,
                keep_first, scale, splits, part_o=None, part_ml=None) -> None:
     _, H, D = q.shape
-    G, P = kpages.shape[1:3]
+    G = kpages.size(1)
     E = out.size(1) // H
+    ki, vi = k_index(D), v_index(vpages.size(2) // PAGE)[:, :E]
     far = bias.size(1) - 1
     for start, n, slot, pos0 in _segments(seg):
         total = pos0 + n
-        pages = table[slot, : -(-total // P)].long()
-        k = kpages[pages].permute(1, 0, 2, 3).reshape(G, -1, D)[:, :total]
-        v = vpages[pages].permute(1, 0, 3, 2).reshape(
-            G, pages.numel() * P, -1)[:, :total, :E]
+        pages = table[slot, : -(-total // PAGE)].long()
+        k, v = (t[pages][:, :, at].transpose(0, 1).flatten(1, 2)[:, :total]
+                for t, at in ((kpages, ki), (vpages, vi)))
         k = k.float().repeat_interleave(H // G, 0)
         v = v.float().repeat_interleave(H // G, 0)
         i = torch.arange(pos0, total).view(-1, 1)

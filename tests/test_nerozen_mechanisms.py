@@ -204,12 +204,10 @@ class Paged:
         self.ops, self.device, self.dtype = ops_for(device), device, dtype
         self.H, self.G, self.D, self.E = H, G, D, E
         # what earlier owners of the pages left behind
-        self.k = rand(n_pages, G, PAGE, pad(D), seed=91, dtype=dtype,
+        self.k = rand(n_pages, G, PAGE * pad(D), seed=91, dtype=dtype,
                       device=device)
-        self.v = rand(n_pages, G, pad(E), PAGE, seed=92, dtype=dtype,
+        self.v = rand(n_pages, G, PAGE * pad(E), seed=92, dtype=dtype,
                       device=device)
-        self.k[..., D:] = 0
-        self.v[:, :, E:] = 0
         perm = torch.randperm(n_pages,
                               generator=torch.Generator().manual_seed(3))
         per = n_pages // slots
@@ -221,7 +219,7 @@ class Paged:
 
     def append(self, slot, pos0, proj):
         n = proj.size(0)
-        q = torch.empty(n, self.H, self.k.size(3), dtype=self.dtype,
+        q = torch.empty(n, self.H, self.k.size(2) // PAGE, dtype=self.dtype,
                         device=self.device)
         rs = torch.full((n,), slot, dtype=torch.int32, device=self.device)
         rp = torch.arange(pos0, pos0 + n, dtype=torch.int32,
@@ -236,7 +234,7 @@ class Paged:
         part = ()
         if splits > 1:
             cells = len(segs) * self.H * splits
-            part = (torch.full((cells * self.v.size(2),), math.nan,
+            part = (torch.full((cells * self.v.size(2) // PAGE,), math.nan,
                                device=self.device),
                     torch.full((cells * 2,), math.nan, device=self.device))
         self.ops.paged_attn(out, q, self.k, self.v, bias, self.table,
