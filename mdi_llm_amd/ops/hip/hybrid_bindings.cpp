@@ -76,7 +76,7 @@ void residual_norm(torch::Tensor x, Opt y, Opt post_w, Opt xn, Opt next_w,
     check_like(*table, f32, "table");
     TORCH_CHECK(table->dim() == 2 && table->size(1) == e, "table size");
   }
-  launch_residual_norm(
+  const int rc = launch_residual_norm(
       xp, y ? y->data_ptr() : nullptr,
       post_w ? f32_ptr(*post_w, e, "post_w") : nullptr,
       xn ? xn->data_ptr() : nullptr,
@@ -84,6 +84,7 @@ void residual_norm(torch::Tensor x, Opt y, Opt post_w, Opt xn, Opt next_w,
       tokens ? i32_ptr(*tokens, n, "tokens") : nullptr,
       table ? table->data_ptr() : nullptr, (float)scale, (float)offset,
       (float)eps, n, e, f32, cur_stream());
+  TORCH_CHECK(rc == 0, "residual_norm: row of ", e, " elements");
 }
 
 void xielu(torch::Tensor z, double p, double q) {

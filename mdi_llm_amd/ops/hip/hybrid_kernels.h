@@ -20,12 +20,12 @@ struct SegView {
 // Residual + norm step, one row per block.  x [n, e] float:
 //   tokens != null : x = scale * table[token]
 //   y != null      : x += post_w ? rms(y) * (offset + post_w) : y
-// then, if next_w, xn = rms(x) * (offset + next_w).
-void launch_residual_norm(float* x, const void* y, const float* post_w,
-                          void* xn, const float* next_w, const int* tokens,
-                          const void* table, float scale, float offset,
-                          float eps, int n, int e, int f32,
-                          hipStream_t stream);
+// then, if next_w, xn = rms(x) * (offset + next_w).  -1: e is too large.
+int launch_residual_norm(float* x, const void* y, const float* post_w,
+                         void* xn, const float* next_w, const int* tokens,
+                         const void* table, float scale, float offset,
+                         float eps, int n, int e, int f32,
+                         hipStream_t stream);
 
 // z <- xIELU(z), p and q already through softplus
 void launch_xielu(void* z, long long n, float p, float q, int f32,

@@ -5,119 +5,135 @@
 #include "hybrid_common.h"
 
 // ---------------------------------------------------------------------------
-// Residual + norms.  One 256-thread block per row; every thread only ever
-// touches its own elements of the row, so x can be re-read from cache
-// between the two reductions without a fence.
+// Residual + norms, one block of NT threads per row.  Every thread keeps its
+// KEEP accesses of V elements in registers, so a row is read once and all of
+// it is in flight before the first reduction.
 // ---------------------------------------------------------------------------
+template <int NT>
 DEVINL float block_sum(float v, float* red) {
   v = wave_sum(v);
   if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
   __syncthreads();
-  v = red[0] + red[1] + red[2] + red[3];
+  v = 0.f;
+#pragma unroll
+  for (int k = 0; k < NT / 64; ++k) v += red[k];
   __syncthreads();
   return v;
 }
 
-template <typename T, int V>
-__global__ __launch_bounds__(256) void residual_norm_kernel(
+template <typename T, int V, int NT, int KEEP>
+__global__ __launch_bounds__(NT) void residual_norm_kernel(
     float* __restrict__ x, const T* __restrict__ y,
     const float* __restrict__ post_w, T* __restrict__ xn,
     const float* __restrict__ next_w, const int* __restrict__ tokens,
     const T* __restrict__ table, float scale, float offset, float eps,
     int e) {
-  __shared__ float red[4];
+  __shared__ float red[NT / 64];
   const size_t row = blockIdx.x;
   x += row * e;
-  float ss = 0.f;
   using PT = Pack<T, V>;
   using PF = Pack<float, V>;
+  PF a[KEEP];
+  float ss = 0.f;
+#define EACH(i)                                                 \
+  _Pragma("unroll") for (int k = 0; k < KEEP; ++k)              \
+    if (const int i = (k * NT + threadIdx.x) * V; i < e)
   if (tokens != nullptr) {
     const T* t = table + (size_t)tokens[row] * e;
-    for (int i = threadIdx.x * V; i < e; i += 256 * V) {
-      PT a = *reinterpret_cast<const PT*>(t + i);
-      PF o;
+    EACH(i) {
+      const PT b = *reinterpret_cast<const PT*>(t + i);
 #pragma unroll
-      for (int j = 0; j < V; ++j) {
-        o.v[j] = to_f(a.v[j]) * scale;
-        ss += o.v[j] * o.v[j];
-      }
-      *reinterpret_cast<PF*>(x + i) = o;
-    }
-  } else if (y != nullptr) {
-    y += row * e;
-    float r = 1.f;
-    if (post_w != nullptr) {
-      float s = 0.f;
-      for (int i = threadIdx.x * V; i < e; i += 256 * V) {
-        PT a = *reinterpret_cast<const PT*>(y + i);
-#pragma unroll
-        for (int j = 0; j < V; ++j) s += to_f(a.v[j]) * to_f(a.v[j]);
-      }
-      r = 1.f / sqrtf(block_sum(s, red) / e + eps);
-    }
-    for (int i = threadIdx.x * V; i < e; i += 256 * V) {
-      PT a = *reinterpret_cast<const PT*>(y + i);
-      PF o = *reinterpret_cast<const PF*>(x + i);
-      if (post_w != nullptr) {
-        PF w = *reinterpret_cast<const PF*>(post_w + i);
-#pragma unroll
-        for (int j = 0; j < V; ++j)
-          o.v[j] += to_f(a.v[j]) * r * (offset + w.v[j]);
-      } else {
-#pragma unroll
-        for (int j = 0; j < V; ++j) o.v[j] += to_f(a.v[j]);
-      }
-#pragma unroll
-      for (int j = 0; j < V; ++j) ss += o.v[j] * o.v[j];
-      *reinterpret_cast<PF*>(x + i) = o;
+      for (int j = 0; j < V; ++j) a[k].v[j] = to_f(b.v[j]) * scale;
+      *reinterpret_cast<PF*>(x + i) = a[k];
     }
   } else {
-    for (int i = threadIdx.x * V; i < e; i += 256 * V) {
-      PF o = *reinterpret_cast<const PF*>(x + i);
+    EACH(i) a[k] = *reinterpret_cast<const PF*>(x + i);
+    if (y != nullptr) {
+      y += row * e;
+      PT b[KEEP];
+      EACH(i) b[k] = *reinterpret_cast<const PT*>(y + i);
+      if (post_w != nullptr) {
+        PF w[KEEP];
+        EACH(i) w[k] = *reinterpret_cast<const PF*>(post_w + i);
+        float s = 0.f;
+        EACH(i) {
 #pragma unroll
-      for (int j = 0; j < V; ++j) ss += o.v[j] * o.v[j];
+          for (int j = 0; j < V; ++j) s += to_f(b[k].v[j]) * to_f(b[k].v[j]);
+        }
+        const float r = 1.f / sqrtf(block_sum<NT>(s, red) / e + eps);
+        EACH(i) {
+#pragma unroll
+          for (int j = 0; j < V; ++j)
+            a[k].v[j] += to_f(b[k].v[j]) * r * (offset + w[k].v[j]);
+        }
+      } else {
+        EACH(i) {
+#pragma unroll
+          for (int j = 0; j < V; ++j) a[k].v[j] += to_f(b[k].v[j]);
+        }
+      }
+      EACH(i) *reinterpret_cast<PF*>(x + i) = a[k];
     }
   }
   if (next_w == nullptr) return;
-  const float r = 1.f / sqrtf(block_sum(ss, red) / e + eps);
+  PF w[KEEP];
+  EACH(i) {
+    w[k] = *reinterpret_cast<const PF*>(next_w + i);
+#pragma unroll
+    for (int j = 0; j < V; ++j) ss += a[k].v[j] * a[k].v[j];
+  }
+  const float r = 1.f / sqrtf(block_sum<NT>(ss, red) / e + eps);
   xn += row * e;
-  for (int i = threadIdx.x * V; i < e; i += 256 * V) {
-    PF a = *reinterpret_cast<const PF*>(x + i);
-    PF w = *reinterpret_cast<const PF*>(next_w + i);
+  EACH(i) {
     PT o;
 #pragma unroll
     for (int j = 0; j < V; ++j)
-      o.v[j] = from_f<T>(a.v[j] * r * (offset + w.v[j]));
+      o.v[j] = from_f<T>(a[k].v[j] * r * (offset + w[k].v[j]));
     *reinterpret_cast<PT*>(xn + i) = o;
   }
+#undef EACH
 }
 
 template <typename T>
-static void residual_norm_t(float* x, const void* y, const float* post_w,
-                            void* xn, const float* next_w, const int* tokens,
-                            const void* table, float scale, float offset,
-                            float eps, int n, int e, hipStream_t stream) {
-  if (e % 4 == 0)
-    residual_norm_kernel<T, 4><<<n, 256, 0, stream>>>(
-        x, (const T*)y, post_w, (T*)xn, next_w, tokens, (const T*)table,
-        scale, offset, eps, e);
-  else
-    residual_norm_kernel<T, 1><<<n, 256, 0, stream>>>(
-        x, (const T*)y, post_w, (T*)xn, next_w, tokens, (const T*)table,
-        scale, offset, eps, e);
+static int residual_norm_t(float* x, const void* y, const float* post_w,
+                           void* xn, const float* next_w, const int* tokens,
+                           const void* table, float scale, float offset,
+                           float eps, int n, int e, hipStream_t stream) {
+#define ROWS(V, NT, KEEP)                                                 \
+  residual_norm_kernel<T, V, NT, KEEP><<<n, NT, 0, stream>>>(             \
+      x, (const T*)y, post_w, (T*)xn, next_w, tokens, (const T*)table,    \
+      scale, offset, eps, e)
+  if (e % 4 != 0) {
+    if (e > 1024 * 16) return -1;
+    if (e <= 1024) ROWS(1, 256, 4);
+    else ROWS(1, 1024, 16);
+  } else if (n <= 256 && e >= 2048 && e <= 16384) {
+    if (e <= 4096) ROWS(4, 1024, 1);  // few rows: latency counts
+    else ROWS(4, 1024, 4);
+  } else if (e <= 1024) {
+    ROWS(4, 256, 1);
+  } else if (e <= 4096) {
+    ROWS(4, 256, 4);
+  } else if (e <= 8192) {
+    ROWS(4, 512, 4);
+  } else if (e <= 32768) {
+    ROWS(4, 1024, 8);
+  } else {
+    return -1;
+  }
+#undef ROWS
+  return 0;
 }
 
-void launch_residual_norm(float* x, const void* y, const float* post_w,
-                          void* xn, const float* next_w, const int* tokens,
-                          const void* table, float scale, float offset,
-                          float eps, int n, int e, int f32,
-                          hipStream_t stream) {
-  if (f32)
-    residual_norm_t<float>(x, y, post_w, xn, next_w, tokens, table, scale,
-                           offset, eps, n, e, stream);
-  else
-    residual_norm_t<bf16>(x, y, post_w, xn, next_w, tokens, table, scale,
-                          offset, eps, n, e, stream);
+int launch_residual_norm(float* x, const void* y, const float* post_w,
+                         void* xn, const float* next_w, const int* tokens,
+                         const void* table, float scale, float offset,
+                         float eps, int n, int e, int f32,
+                         hipStream_t stream) {
+  return f32 ? residual_norm_t<float>(x, y, post_w, xn, next_w, tokens, table,
+                                      scale, offset, eps, n, e, stream)
+             : residual_norm_t<bf16>(x, y, post_w, xn, next_w, tokens, table,
+                                     scale, offset, eps, n, e, stream);
 }
 
 // ---------------------------------------------------------------------------

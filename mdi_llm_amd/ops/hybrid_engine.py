@@ -28,7 +28,6 @@ from ..config import ModelConfig
 from ..models.cache import PAGE, HybridCache
 from ..models.sampling import sample as sample_token
 from . import require_hip_ops
-from .engine import DecodeEngine
 
 __all__ = ["HybridEngine", "distance_bias"]
 
@@ -192,7 +191,7 @@ class HybridEngine:
             out = torch.empty(1, M, dtype=self.dtype, device=self.device)
             p, q = act or (0.0, 0.0)
             self.ops.gemv(out, w, x, None, None, 4 if act else 0,
-                          rows=DecodeEngine._rows(M, K), act_p=p, act_q=q)
+                          rows=4 if M >= 65536 else 1, act_p=p, act_q=q)
             return out
         out = F.linear(x, w)
         if act is not None:

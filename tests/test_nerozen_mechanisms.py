@@ -51,7 +51,7 @@ def seg(rows, device):
 
 # ---------------------------------------------------------------------------
 @everywhere
-@pytest.mark.parametrize("e", [8, 27, 300, 1024, 5000])
+@pytest.mark.parametrize("e", [8, 27, 300, 1024, 1501, 4096, 5000, 9000])
 def test_residual_norm(e, device, dtype):
     ops, n, eps = ops_for(device), 5, 1e-5
     x = rand(n, e, seed=1, device=device) * 3
