@@ -259,6 +259,20 @@ void paged_attn(torch::Tensor out, torch::Tensor q, torch::Tensor kpages,
               a.vpad);
 }
 
+void skinny_gemm(torch::Tensor out, torch::Tensor w, torch::Tensor x,
+                 bool act, double act_p, double act_q) {
+  TORCH_CHECK(x.dim() == 2 && w.dim() == 2 && out.dim() == 2, "2-D operands");
+  const int n = (int)x.size(0), m = (int)w.size(0), k = (int)x.size(1);
+  for (const auto* t : {&out, &w, &x})
+    TORCH_CHECK(act_type(*t, "operand") == 0, "skinny_gemm: bf16 operands");
+  TORCH_CHECK(w.size(1) == k && out.size(0) == n && out.size(1) == m,
+              "skinny_gemm: sizes");
+  const int rc = launch_skinny_gemm(out.data_ptr(), w.data_ptr(),
+                                    x.data_ptr(), n, m, k, act ? 1 : 0,
+                                    (float)act_p, (float)act_q, cur_stream());
+  TORCH_CHECK(rc == 0, "skinny_gemm: unsupported n ", n, " or k ", k);
+}
+
 void advance_batch(torch::Tensor slots, torch::Tensor sampled,
                    torch::Tensor pos, torch::Tensor tokens, int64_t spare) {
   const int n = (int)slots.numel();
@@ -304,5 +318,8 @@ void bind_hybrid(py::module_& m) {
         py::arg("max_len"), py::arg("window"), py::arg("keep_first"),
         py::arg("scale"), py::arg("splits"), py::arg("part_o") = none,
         py::arg("part_ml") = none);
+  m.def("skinny_gemm", &skinny_gemm, "projection of up to 32 rows",
+        py::arg("out"), py::arg("w"), py::arg("x"), py::arg("act") = false,
+        py::arg("act_p") = 0.0, py::arg("act_q") = 0.0);
   m.def("advance_batch", &advance_batch, "decode bookkeeping");
 }

@@ -63,4 +63,9 @@ struct PageLayout {
   }
 };
 
+// z/2 plus p z^2 above zero, (1/2 + q)(e^z - 1 - z) below
+DEVINL float xielu(float z, float p, float q) {
+  return 0.5f * z + (z > 0.f ? p * z * z : (0.5f + q) * (expm1f(z) - z));
+}
+
 DEVINL float sigmoid(float z) { return 1.f / (1.f + expf(-z)); }

@@ -90,3 +90,9 @@ int launch_paged_attn_f32(const PagedAttnArgs& a, hipStream_t stream);
 // pos += 1; entries of the spare slot stay where they are.
 void launch_advance_batch(const int* slots, const int* sampled, int* pos,
                           int* tokens, int spare, int n, hipStream_t stream);
+
+// out[n, m] = x[n, :] . w[m, :] in bf16 for up to 32 rows of x, with xIELU
+// if act.  Returns -1 when n or k (a multiple of 64) does not fit.
+int launch_skinny_gemm(void* out, const void* w, const void* x, int n, int m,
+                       int k, int act, float act_p, float act_q,
+                       hipStream_t stream);

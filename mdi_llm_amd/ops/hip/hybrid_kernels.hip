@@ -139,10 +139,6 @@ int launch_residual_norm(float* x, const void* y, const float* post_w,
 // ---------------------------------------------------------------------------
 // xIELU on a whole GEMM output (single rows have it in the GEMV epilogue)
 // ---------------------------------------------------------------------------
-DEVINL float xielu(float z, float p, float q) {
-  return 0.5f * z + (z > 0.f ? p * z * z : (0.5f + q) * (expm1f(z) - z));
-}
-
 template <typename T, int V>
 __global__ __launch_bounds__(256) void xielu_kernel(T* __restrict__ z,
                                                     long long n, float p,

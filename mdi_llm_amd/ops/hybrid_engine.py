@@ -185,14 +185,20 @@ class HybridEngine:
         return xn
 
     def _linear(self, x: torch.Tensor, w: torch.Tensor, act=None):
-        M, K = w.shape
-        if (x.size(0) == 1 and self.hip and self.dtype == torch.bfloat16
-                and K % 8 == 0):
-            out = torch.empty(1, M, dtype=self.dtype, device=self.device)
+        (M, K), n = w.shape, x.size(0)
+        if self.hip and self.dtype == torch.bfloat16 and n <= 32:
+            # few rows: the weight stream decides.  Past 16 rows, and for
+            # the widest outputs, the library's kernels stream as well,
+            # except along a very long K.
             p, q = act or (0.0, 0.0)
-            self.ops.gemv(out, w, x, None, None, 4 if act else 0,
-                          rows=4 if M >= 65536 else 1, act_p=p, act_q=q)
-            return out
+            out = torch.empty(n, M, dtype=self.dtype, device=self.device)
+            if n == 1 and K % 8 == 0:
+                self.ops.gemv(out, w, x, None, None, 4 if act else 0,
+                              rows=4 if M >= 65536 else 1, act_p=p, act_q=q)
+                return out
+            if K % 64 == 0 and M < 65536 and (n <= 16 or K >= 16384):
+                self.ops.skinny_gemm(out, w, x, act is not None, p, q)
+                return out
         out = F.linear(x, w)
         if act is not None:
             self.ops.xielu(out, *act)

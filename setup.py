@@ -30,7 +30,8 @@ HIPCC = os.path.join(ROCM_HOME, "bin", "hipcc")
 OFFLOAD_ARCH = os.environ.get("PYTORCH_ROCM_ARCH", "gfx950").split(";")[0]
 
 KERNEL_SOURCES = ["decode_kernels.hip", "hybrid_kernels.hip",
-                  "paged_attn_bf16.hip", "paged_attn_f32.hip"]
+                  "paged_attn_bf16.hip", "paged_attn_f32.hip",
+                  "skinny_gemm.hip"]
 HEADERS = [HIP_DIR / h for h in ("decode_kernels.h", "hybrid_kernels.h",
                                  "hybrid_common.h", "paged_attn.inc")]
 

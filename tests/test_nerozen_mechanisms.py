@@ -348,3 +348,28 @@ def test_bias_counts_beside_the_score(device, dtype):
         o = P.attend(q, [(0, T, 0, 0)], bias, 1000, 0, scale, 0)
         want = P.oracle(proj, rel, far, 1000, 0, scale)
         close(o, want, dtype)
+
+
+# ---------------------------------------------------------------------------
+@pytest.mark.gpu
+@pytest.mark.parametrize("m,k", [(16, 64), (50, 192), (300, 4096),
+                                 (1000, 4160), (33, 20480)])
+@pytest.mark.parametrize("n", [1, 2, 5, 16, 17, 32])
+def test_few_row_projection(n, m, k):
+    """Odd output widths, K with and without whole unrolled stretches; the
+    activation in the epilogue; a row does not depend on its companions."""
+    ops = ops_for("cuda")
+    x = rand(n, k, seed=1, dtype=torch.bfloat16, device="cuda")
+    w = rand(m, k, seed=2, dtype=torch.bfloat16, device="cuda") * k ** -0.5
+    want = x.double().cpu() @ w.double().cpu().T
+    out = torch.full((n, m), math.nan, dtype=torch.bfloat16, device="cuda")
+    ops.skinny_gemm(out, w, x)
+    close(out, want, torch.bfloat16)
+    act = torch.tensor([0.2, -0.4], dtype=torch.float64)
+    p, q = torch.nn.functional.softplus(act).tolist()
+    ops.skinny_gemm(out, w, x, True, p, q)
+    close(out, oracle.xielu(want, act), torch.bfloat16)
+    one = torch.empty(1, m, dtype=torch.bfloat16, device="cuda")
+    ops.skinny_gemm(one, w, x[-1:].contiguous(), True, p, q)
+    if n <= 16:
+        assert torch.equal(one[0], out[-1])
