@@ -16,6 +16,8 @@ fp32 throughout).
 from __future__ import annotations
 
 import math
+import os
+import warnings
 from bisect import bisect_left
 from dataclasses import dataclass
 from fractions import Fraction
@@ -146,6 +148,11 @@ class HybridEngine:
         self.device, self.dtype = p.device, p.dtype
         if self.dtype not in (torch.bfloat16, torch.float32):
             raise ValueError("hybrid stacks run in bfloat16 or float32")
+        for var in ("MDI_WEIGHT_DTYPE", "MDI_KV_DTYPE"):
+            if os.environ.get(var, "bf16") != "bf16":
+                warnings.warn(f"{var}={os.environ[var]} ignored: hybrid "
+                              "stacks keep weights and K/V in the stage's "
+                              "dtype")
         self.hip = self.device.type == "cuda"
         if self.hip:
             self.ops = require_hip_ops()

@@ -168,7 +168,7 @@ def test_requests_that_never_fit_are_refused():
 
 
 # ---------------------------------------------------------------------------
-def _ring_worker(rank, world, tmp, port):
+def _ring_worker(rank, world, tmp, port, device):
     import torch.distributed as dist
 
     from mdi_llm_amd.models.stages import build_stage
@@ -184,15 +184,17 @@ def _ring_worker(rank, world, tmp, port):
     split = layer_split(cfg.n_layer, world)
     stage = build_stage(cfg, rank, split[rank], sum(split[:rank]))
     stage.load_state_dict(split_parameters(sd, world)[rank])
+    dev = torch.device(device)
+    stage = stage.to(device=dev, dtype=torch.float32)
     stage.max_seq_length = 256
     stage.eval()
-    cpu = torch.device("cpu")
     prompts = [torch.tensor(p) for p in torch.load(
         os.path.join(tmp, "prompts.pt"), weights_only=True)]
-    runner = make_runner(stage, len(prompts), cpu)
-    comm = RingComm(cfg.n_embd, stage.max_seq_length, cpu, len(prompts),
+    runner = make_runner(stage, len(prompts), dev)
+    comm = RingComm(cfg.n_embd, stage.max_seq_length, dev, len(prompts),
                     dtype=cfg.residual_dtype(torch.float32))
-    rt = PipelineRuntime(runner, rank=rank, world=world, comm=comm)
+    rt = PipelineRuntime(runner, rank=rank, world=world, comm=comm,
+                         device=dev)
     if rank == 0:
         res = rt.generate(prompts, 8, SamplingParams(temperature=0.0))
         torch.save([s.tolist() for s in res.sequences],
@@ -203,18 +205,22 @@ def _ring_worker(rank, world, tmp, port):
     dist.destroy_process_group()
 
 
+@device_param
 @pytest.mark.parametrize("world", [2, 3])
-def test_ring_pipeline_matches_standalone(world, tmp_path):
+def test_ring_pipeline_matches_standalone(world, device, tmp_path):
+    """Stages in processes of their own; on a GPU they share it, and the
+    activations go through host memory."""
     from mdi_llm_amd.parallel.runtime import PipelineRuntime, SamplingParams
 
     cfg, w = model()
     save(tmp_path, cfg, w)
     prompts = [tokens(cfg, n, n) for n in (70, 5, 33)]
     torch.save(prompts, tmp_path / "prompts.pt")
-    r = make_runner(cfg, w, "cpu", torch.float32)
-    ref = PipelineRuntime(r).generate([torch.tensor(p) for p in prompts], 8,
+    r = make_runner(cfg, w, device, torch.float32)
+    ref = PipelineRuntime(r, device=torch.device(device)).generate([torch.tensor(p) for p in prompts], 8,
                                       SamplingParams(temperature=0.0))
-    mp.spawn(_ring_worker, args=(world, str(tmp_path), 29930 + world),
+    mp.spawn(_ring_worker,
+             args=(world, str(tmp_path), 29930 + world, device),
              nprocs=world, join=True)
     got = torch.load(tmp_path / "out.pt", weights_only=True)
     assert got == [s.tolist() for s in ref.sequences]
