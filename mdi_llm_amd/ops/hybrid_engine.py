@@ -1,5 +1,5 @@
-"""Step engine of hybrid stacks (``ModelConfig.layers``): one ragged batch
-per step, portions of prompts beside single decoded tokens.
+"""Step engine of hybrid stacks (``ModelConfig.layers``): every step is one
+ragged batch, prompt pieces and decode tokens together.
 
 Where ``DecodeEngine`` advances one sequence and ``GroupDecodeEngine`` a
 fixed group, every step here takes any mix of sequences: the rows of all
@@ -120,7 +120,7 @@ class _DecodeStep:
         self.sampled = torch.zeros(size, dtype=torch.int32, device=dev)
         self.scratch = torch.zeros(520 * size, dtype=torch.int32, device=dev)
         self.logits: Optional[torch.Tensor] = None
-        self.forward_graph = None
+        self.forward = self.forward_graph = None
         self.sample_graphs: dict = {}
         self.slots: List[int] = []
 
@@ -174,7 +174,6 @@ class HybridEngine:
             self.final = stage.transformer.ln_f.weight.detach().float()
             self.head = stage.lm_head.weight.detach()
         self._steps: Dict[int, _DecodeStep] = {}
-        self._part: Optional[Tuple[torch.Tensor, torch.Tensor]] = None
 
     # ------------------------------------------------------------------
     # building blocks
@@ -416,8 +415,6 @@ class HybridEngine:
             with torch.cuda.graph(g):
                 st.logits = forward()
             st.forward_graph = g
-        else:
-            st.forward_graph = None
         st.forward = forward
         self._steps[size] = st
         return st

@@ -1,10 +1,9 @@
-"""Trace replay: feeds given token ids through a model step by step and
-writes logits.
+"""Replay of recorded token streams, for comparing logits across builds.
 
-Each input line is one engine step: the next tokens of any number of
-requests, run as one batch from the cache and state that earlier steps left.
-Nothing is sampled.  A step is ``HybridEngine.step``, which generation uses
-as well, over a ``HybridCache`` with a bounded page pool.
+The input is JSON lines, one engine step each: which requests take part, the
+ids they continue with, the places whose logits are kept (``want``), and the
+requests that end.  Steps go through ``HybridEngine.step``, as generation
+does, over a ``HybridCache`` whose pool the caller bounds; no token is drawn.
 """
 
 from __future__ import annotations
@@ -28,8 +27,8 @@ SLOTS = 4
 
 def load_runner(model_dir, dtype: torch.dtype, device: torch.device,
                 max_tokens: int):
-    """The checkpoint as a whole-model stage with a pool of ``max_tokens``
-    cache rows and ``SLOTS`` sequence slots."""
+    """The checkpoint as one whole-model stage, ``SLOTS`` sequences at a time
+    in ``max_tokens`` cache rows."""
     config, sd = load_from_pt(model_dir)
     if not config.is_hybrid:
         raise ValueError(

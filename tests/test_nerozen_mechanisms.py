@@ -119,7 +119,7 @@ def recurrence_oracle(proj, fb, lower, w, H, D, E, eps):
 
 
 @everywhere
-@pytest.mark.parametrize("H,D,E", [(2, 32, 64), (3, 16, 16), (1, 1, 3),
+@pytest.mark.parametrize("H,D,E", [(2, 32, 72), (3, 16, 16), (1, 1, 3),
                                    (2, 100, 30), (1, 256, 8), (2, 8, 130),
                                    (2, 64, 48), (2, 128, 128)])
 def test_hgrn2_scan_and_step(H, D, E, device, dtype):
