@@ -17,7 +17,7 @@ import copy
 import json
 from dataclasses import dataclass, field, asdict
 from pathlib import Path
-from typing import Any, Literal, Optional, Union
+from typing import Any, Dict, Literal, Optional, Union
 
 import yaml
 
@@ -55,7 +55,7 @@ class ModelConfig:
     norm_class_name: Literal["LayerNorm", "RMSNorm"] = "LayerNorm"
     norm_eps: float = 1e-5
     mlp_class_name: Literal["GptNeoxMLP", "LLaMAMLP", "GemmaMLP", "LLaMAMoE",
-                            "XieluMLP"] = "GptNeoxMLP"
+                            "XieluMLP", "GatedMLP"] = "GptNeoxMLP"
     gelu_approximate: str = "none"
     intermediate_size: Optional[int] = None
     rope_condense_ratio: int = 1
@@ -68,13 +68,15 @@ class ModelConfig:
     pos_embedding: Literal["rope", "learned"] = "rope"
     # -- stacks whose layers differ (models/hybrid.py) --
     # one entry per layer: {"type": mixer, "mixer": {sizes and constants},
-    # "mlp": {"kind", "ff"} or None}; None means n_layer equal blocks
+    # "mlp": {"kind", sizes} or None}; None means n_layer equal blocks
     layers: Optional[list] = None
     embedding_scale: float = 1.0
     # RMS norm weights are stored as w with norm_offset + w applied
     norm_offset: float = 0.0
     # a second norm on each sublayer's output, before the residual add
     post_norms: bool = False
+    # what a layer adds to the residual stream is multiplied by this
+    residual_mult: float = 1.0
 
     def __post_init__(self) -> None:
         if self.layers is not None:
@@ -109,10 +111,11 @@ class ModelConfig:
         self.n_query_groups = first.get("kv_heads", first["heads"])
         self.head_size = first["dim"]
         self.intermediate_size = max(
-            (l["mlp"]["ff"] for l in self.layers if l["mlp"]), default=0
+            (l["mlp"]["ff"] if l["mlp"]["kind"] == "dense"
+             else l["mlp"]["expert"]["ff"]
+             for l in self.layers if l["mlp"]), default=0
         )
         self.rotary_percentage = 0.0
-        self.parallel_residual = False
         self.bias = False
 
     @property
@@ -126,24 +129,55 @@ class ModelConfig:
 
         return torch.float32 if self.is_hybrid else dtype
 
-    def layer_weights(self, i: int) -> int:
-        """Number of matrix weights of layer ``i``."""
+    def shared_latents(self) -> Dict[int, int]:
+        """Layers whose cached latent other layers read (``kv_from``), with
+        the size of a row."""
+        rows = {}
+        for layer in self.layers or ():
+            src = layer["mixer"].get("kv_from")
+            if src is not None:
+                rows[src] = layer["mixer"]["kv_rank"]
+        return dict(sorted(rows.items()))
+
+    @property
+    def ring_width(self) -> int:
+        """Columns of the rows that pass between pipeline stages: the
+        residual stream, then the latents that a later stage may read."""
+        return self.n_embd + sum(self.shared_latents().values())
+
+    def layer_weights(self, i: int, active: bool = False) -> int:
+        """Number of matrix weights of layer ``i``; if ``active``, of those
+        that one token uses."""
         E = self.n_embd
         if self.layers is None:
             mats = 2 if self.mlp_class_name == "GptNeoxMLP" else 3
             return (E * self.qkv_dim + E * self.n_head * self.head_size
                     + mats * E * self.intermediate_size)
         layer = self.layers[i]
-        m = layer["mixer"]
-        if layer["type"] == "attention":
+        m, mlp = layer["mixer"], layer["mlp"]
+        inner = 0       # weights that do not touch the residual width
+        if layer["type"] == "latent_attention":
+            rows = m["q_rank"] + m["heads"]
+            if m.get("kv_from") is None:
+                rows += m["kv_rank"]
+            inner = m["heads"] * (m["q_rank"] * m["dim"]
+                                  + m["kv_rank"] * (m["dim"] + m["vdim"]))
+        elif layer["type"] == "attention":
             rows = (m["heads"] + m["kv_heads"]) * m["dim"] \
                 + m["kv_heads"] * m["vdim"]
         else:
             rows = m["heads"] * (2 * m["dim"] + m["vdim"])
         rows += m["heads"] * m["vdim"]
-        if layer["mlp"]:
-            rows += 2 * layer["mlp"]["ff"]
-        return E * rows
+        if mlp and mlp["kind"] == "moe":
+            router = mlp["router"]
+            used = router["top"] if active else router["experts"]
+            rows += router["experts"] + 3 * used * mlp["expert"]["ff"]
+            if mlp.get("shared"):
+                rows += 3 * mlp["shared"]["ff"]
+        elif mlp:
+            rows += (3 if self.mlp_class_name == "GatedMLP" else 2) \
+                * mlp["ff"]
+        return E * rows + inner
 
     # -- derived sizes ----------------------------------------------------
     @property
@@ -241,11 +275,54 @@ def _nerozen(raw: dict) -> dict:
         norm_eps=raw["norm"]["eps"],
         norm_offset=1.0,
         post_norms=True,
+        parallel_residual=False,
         mlp_class_name="XieluMLP",
     )
 
 
-native_architectures = {"Nerozen": _nerozen}
+def _resolorn(raw: dict) -> dict:
+    """Resolorn: windowed latent attention (own latent, or an earlier
+    layer's) beside a dense or routed gated feed-forward, one norm a layer;
+    learned positions."""
+    layers = copy.deepcopy(raw["layers"])
+    for i, layer in enumerate(layers):
+        m, mlp = layer["mixer"], layer["mlp"]
+        if layer["type"] != "latent_attention":
+            raise ValueError(f"Resolorn: unknown mixer {layer['type']!r}")
+        if mlp is not None and mlp["kind"] not in ("dense", "moe"):
+            raise ValueError(
+                f"Resolorn: unknown feed-forward {mlp['kind']!r}")
+        if mlp is not None and mlp["kind"] == "moe" and not (
+                1 <= mlp["router"]["top"] <= mlp["router"]["experts"]):
+            raise ValueError(f"Resolorn: layer {i} routes to "
+                             f"{mlp['router']['top']} of "
+                             f"{mlp['router']['experts']} experts")
+        src = m.get("kv_from")
+        if src is None:
+            continue
+        if not 0 <= src < i or layers[src]["mixer"].get("kv_from") is not None:
+            raise ValueError(f"Resolorn: layer {i} reads the latent of layer "
+                             f"{src}, which has none of its own before it")
+        if layers[src]["mixer"]["kv_rank"] != m["kv_rank"]:
+            raise ValueError(f"Resolorn: layers {i} and {src} share a latent "
+                             "of unequal size")
+    return dict(
+        name="Resolorn",
+        block_size=raw["max_positions"],
+        vocab_size=raw["vocab"],
+        padded_vocab_size=raw["vocab"],
+        n_embd=raw["width"],
+        layers=layers,
+        pos_embedding="learned",
+        norm_class_name="RMSNorm",
+        norm_eps=raw["norm"]["eps"],
+        parallel_residual=True,
+        residual_mult=raw["residual_mult"],
+        mlp_class_name="GatedMLP",
+    )
+
+
+native_architectures = {"Nerozen": _nerozen, "Resolorn": _resolorn}
 
 
 def is_native_checkpoint(path: Union[str, Path]) -> bool:

@@ -1,4 +1,5 @@
-"""Sequence cache of hybrid stacks: paged K/V plus recurrent state slots.
+"""Sequence cache of hybrid stacks: paged K/V and latents, and recurrent
+state slots.
 
 ``model.KVCachePool`` gives every slot ``max_seq`` rows.  Here the K/V rows
 of all sequences share one pool of 64-token pages, taken as a sequence grows
@@ -6,10 +7,12 @@ and given back when it ends, and each recurrent layer has one fixed-size
 state per slot.  One page table serves all attention layers of the stage:
 page ``p`` is row ``p`` of every layer's arena.
 
-Layout (what the kernels in ``paged_attn.inc`` and ``hybrid_kernels.hip``
-read): K pages ``[pages, kv_heads, 64 * dpad]`` and V pages ``[pages,
+Layout (what the kernels in ``paged_attn.inc``, ``row_attn.inc`` and
+``hybrid_kernels.hip`` read): K pages ``[pages, kv_heads, 64 * dpad]`` and V pages ``[pages,
 kv_heads, 64 * vpad]`` in MFMA operand order (``k_index``, ``v_index``),
-states ``[slots, heads, dim, vstride]`` in fp32.  Nothing needs clearing when
+latent pages ``[pages, 64, rpad]`` with one zero-padded row per token, states
+``[slots, heads, dim, vstride]`` in fp32.  Layers that read one latent share
+its pages (``latent`` is keyed by the layer that makes it).  Nothing needs clearing when
 a page or slot is taken again: keys past a sequence's end are masked, and
 the recurrence starts from zero at position 0.
 """
@@ -75,6 +78,7 @@ class HybridCache:
         self.k: Dict[int, torch.Tensor] = {}
         self.v: Dict[int, torch.Tensor] = {}
         self.state: Dict[int, torch.Tensor] = {}
+        self.latent: Dict[int, torch.Tensor] = {}
         for i, m in enumerate(mixers):
             if m.kind == "attention":
                 dpad = _pad_to(m.dim, (32, 64, 128, 256), "attention dim")
@@ -84,6 +88,13 @@ class HybridCache:
                                         dtype=dtype)
                 self.v[i] = torch.zeros(P, G, PAGE * vpad, device=device,
                                         dtype=dtype)
+            elif m.kind == "latent_attention":
+                if m.source not in self.latent:
+                    rpad = _pad_to(m.rank, (64, 128, 256, 512),
+                                   "latent size")
+                    self.latent[m.source] = torch.zeros(
+                        self.n_pages + 1, PAGE, rpad, device=device,
+                        dtype=dtype)
             else:
                 vstride = -(-m.vdim // 4) * 4
                 self.state[i] = torch.zeros(
@@ -169,4 +180,5 @@ class HybridCache:
 
     def memory_bytes(self) -> int:
         return sum(t.numel() * t.element_size()
-                   for d in (self.k, self.v, self.state) for t in d.values())
+                   for d in (self.k, self.v, self.state, self.latent)
+                   for t in d.values())

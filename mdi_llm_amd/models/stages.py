@@ -24,7 +24,7 @@ import torch.nn as nn
 
 from ..config import ModelConfig
 from .cache import HybridCache
-from .hybrid import HybridBlock, Scale
+from .hybrid import Scale, make_block
 from .model import Block, KVCachePool, build_rope_cache, norm_class
 
 __all__ = ["StageBase", "StarterStage", "SecondaryStage", "build_stage"]
@@ -44,7 +44,7 @@ class StageBase(nn.Module):
         self._build_rope()
 
     def _make_blocks(self) -> nn.ModuleList:
-        cls = HybridBlock if self.config.is_hybrid else Block
+        cls = make_block if self.config.is_hybrid else Block
         return nn.ModuleList(
             cls(self.config, self.first_layer + i)
             for i in range(self.n_local_layers)

@@ -53,9 +53,33 @@ SegView seg_view(const torch::Tensor& seg) {
   return SegView{p, p + st, p + 2 * st, p + 3 * st, (int)seg.size(1)};
 }
 
+// rows of a wider matrix: contiguous columns, any row stride
+struct Rows {
+  void* p;
+  int n, cols;
+  long long ld;
+};
+
+Rows rows_of(const torch::Tensor& t, int f32, const char* name) {
+  TORCH_CHECK(t.is_cuda() && t.dim() == 2 && t.size(0) > 0 && t.size(1) > 0 &&
+                  t.stride(1) == 1 && t.stride(0) >= t.size(1) &&
+                  t.scalar_type() ==
+                      (f32 ? torch::kFloat32 : torch::kBFloat16),
+              name, ": expected rows of the activation type on the GPU");
+  return Rows{t.data_ptr(), (int)t.size(0), (int)t.size(1), t.stride(0)};
+}
+
+int row_type(const torch::Tensor& t, const char* name) {
+  TORCH_CHECK(t.scalar_type() == torch::kBFloat16 ||
+                  t.scalar_type() == torch::kFloat32,
+              name, ": expected bf16 or float");
+  return t.scalar_type() == torch::kFloat32 ? 1 : 0;
+}
+
 void residual_norm(torch::Tensor x, Opt y, Opt post_w, Opt xn, Opt next_w,
                    Opt tokens, Opt table, double scale, double offset,
-                   double eps) {
+                   double eps, double mult, Opt pos_table, Opt row_pos,
+                   Opt routed, Opt routed_w) {
   TORCH_CHECK(x.dim() == 2 && x.size(0) > 0, "x must be [n, e]");
   const int n = (int)x.size(0), e = (int)x.size(1);
   float* xp = const_cast<float*>(f32_ptr(x, (int64_t)n * e, "x"));
@@ -76,14 +100,40 @@ void residual_norm(torch::Tensor x, Opt y, Opt post_w, Opt xn, Opt next_w,
     check_like(*table, f32, "table");
     TORCH_CHECK(table->dim() == 2 && table->size(1) == e, "table size");
   }
-  const int rc = launch_residual_norm(
-      xp, y ? y->data_ptr() : nullptr,
-      post_w ? f32_ptr(*post_w, e, "post_w") : nullptr,
-      xn ? xn->data_ptr() : nullptr,
-      next_w ? f32_ptr(*next_w, e, "next_w") : nullptr,
-      tokens ? i32_ptr(*tokens, n, "tokens") : nullptr,
-      table ? table->data_ptr() : nullptr, (float)scale, (float)offset,
-      (float)eps, n, e, f32, cur_stream());
+  TORCH_CHECK(!!pos_table == !!row_pos && (!pos_table || tokens) &&
+                  !!routed == !!routed_w && (!routed || y),
+              "residual_norm: bad combination of operands");
+  ResidualArgs a{};
+  if (pos_table) {
+    check_like(*pos_table, f32, "pos_table");
+    TORCH_CHECK(pos_table->dim() == 2 && pos_table->size(1) == e,
+                "pos_table size");
+    a.pos_table = pos_table->data_ptr();
+    a.row_pos = i32_ptr(*row_pos, n, "row_pos");
+  }
+  if (routed) {
+    check_like(*routed, f32, "routed");
+    TORCH_CHECK(routed->dim() == 3 && routed->size(0) == n &&
+                    routed->size(2) == e,
+                "routed must be [n, top, e]");
+    a.top = (int)routed->size(1);
+    a.routed = routed->data_ptr();
+    a.routed_w = f32_ptr(*routed_w, (int64_t)n * a.top, "routed_w");
+  }
+  a.x = xp;
+  a.y = y ? y->data_ptr() : nullptr;
+  a.post_w = post_w ? f32_ptr(*post_w, e, "post_w") : nullptr;
+  a.xn = xn ? xn->data_ptr() : nullptr;
+  a.next_w = next_w ? f32_ptr(*next_w, e, "next_w") : nullptr;
+  a.tokens = tokens ? i32_ptr(*tokens, n, "tokens") : nullptr;
+  a.table = table ? table->data_ptr() : nullptr;
+  a.scale = (float)scale;
+  a.offset = (float)offset;
+  a.eps = (float)eps;
+  a.mult = (float)mult;
+  a.n = n;
+  a.e = e;
+  const int rc = launch_residual_norm(a, f32, cur_stream());
   TORCH_CHECK(rc == 0, "residual_norm: row of ", e, " elements");
 }
 
@@ -259,6 +309,298 @@ void paged_attn(torch::Tensor out, torch::Tensor q, torch::Tensor kpages,
               a.vpad);
 }
 
+// latent pages [P, 64, rpad]
+int latent_pages(const torch::Tensor& pages, int f32) {
+  check_like(pages, f32, "pages");
+  TORCH_CHECK(pages.dim() == 3 && pages.size(1) == 64 &&
+                  pages.size(2) % 64 == 0,
+              "pages: expected [P, 64, rpad]");
+  return (int)pages.size(2);
+}
+
+void latent_norm_append(torch::Tensor pages, Opt kv, Opt kv_w,
+                        torch::Tensor row_slot, torch::Tensor row_pos,
+                        torch::Tensor table, double eps, Opt q_out, Opt q,
+                        Opt q_w) {
+  const int f32 = act_type(pages, "pages");
+  const int rpad = latent_pages(pages, f32);
+  TORCH_CHECK((kv || q) && !!q == !!q_out && !!q == !!q_w && (kv || !kv_w),
+              "latent_norm_append: bad combination of operands");
+  Rows k{}, r{};
+  int n = 0;
+  if (kv) {
+    k = rows_of(*kv, f32, "kv");
+    n = k.n;
+    TORCH_CHECK(k.cols <= rpad, "kv columns");
+  }
+  if (q) {
+    r = rows_of(*q, f32, "q");
+    TORCH_CHECK(!kv || r.n == n, "q and kv rows");
+    n = r.n;
+    check_like(*q_out, f32, "q_out");
+    TORCH_CHECK(q_out->numel() == (int64_t)n * r.cols, "q_out size");
+  }
+  TORCH_CHECK(table.dim() == 2, "table must be [slots, pages]");
+  launch_latent_norm_append(
+      q ? q_out->data_ptr() : nullptr, r.p,
+      q ? f32_ptr(*q_w, r.cols, "q_w") : nullptr, pages.data_ptr(), k.p,
+      kv_w ? f32_ptr(*kv_w, k.cols, "kv_w") : nullptr,
+      i32_ptr(row_slot, n, "row_slot"), i32_ptr(row_pos, n, "row_pos"),
+      i32_ptr(table, table.numel(), "table"), (int)table.size(1), n, r.cols,
+      r.ld, k.cols, k.ld, rpad, (float)eps, f32, cur_stream());
+}
+
+void latent_gather(torch::Tensor out, torch::Tensor pages,
+                   torch::Tensor table, torch::Tensor seg, int64_t max_len) {
+  const int f32 = act_type(pages, "pages");
+  const int rpad = latent_pages(pages, f32);
+  check_like(out, f32, "out");
+  TORCH_CHECK(out.dim() == 2 && out.size(1) <= rpad && max_len > 0 &&
+                  max_len <= out.size(0),
+              "latent_gather: out must be [rows, rank]");
+  TORCH_CHECK(table.dim() == 2, "table must be [slots, pages]");
+  launch_latent_gather(out.data_ptr(), pages.data_ptr(),
+                       i32_ptr(table, table.numel(), "table"),
+                       (int)table.size(1), seg_view(seg), (int)max_len,
+                       (int)out.size(1), rpad, f32, cur_stream());
+}
+
+void gated_act(torch::Tensor out, torch::Tensor gate, torch::Tensor up,
+               int64_t act) {
+  const int f32 = row_type(out, "out");
+  const Rows o = rows_of(out, f32, "out"), g = rows_of(gate, f32, "gate"),
+             u = rows_of(up, f32, "up");
+  TORCH_CHECK(o.n == g.n && o.n == u.n && o.cols == g.cols &&
+                  o.cols == u.cols && g.ld == u.ld && o.n < 65536,
+              "gated_act: sizes");
+  TORCH_CHECK(act == 0 || act == 1, "gated_act: act");
+  launch_gated_act(o.p, o.ld, g.p, u.p, g.ld, o.n, o.cols, (int)act, f32,
+                   cur_stream());
+}
+
+struct Parts {
+  float *o = nullptr, *ml = nullptr;
+};
+
+Parts parts(const Opt& part_o, const Opt& part_ml, int64_t cells, int k) {
+  TORCH_CHECK(part_o && part_ml, "split keys need scratch");
+  return Parts{
+      const_cast<float*>(f32_ptr(*part_o, cells * k, "part_o")),
+      const_cast<float*>(f32_ptr(*part_ml, cells * 2, "part_ml"))};
+}
+
+void head_proj(torch::Tensor out, Opt x, torch::Tensor w, Opt x_rows,
+               Opt out_rows, Opt gate, Opt part_o, Opt part_ml) {
+  const int f32 = act_type(w, "w");
+  const Rows o = rows_of(out, f32, "out");
+  HeadProjArgs a{};
+  TORCH_CHECK(w.dim() == 3 && w.size(2) % 32 == 0, "w must be [H, m, k]");
+  a.heads = (int)w.size(0);
+  a.m = (int)w.size(1);
+  a.k = (int)w.size(2);
+  TORCH_CHECK(o.cols == a.heads * a.m, "head_proj: out columns");
+  TORCH_CHECK(!!x != !!part_o, "head_proj: x or partial results");
+  if (x) {
+    const Rows r = rows_of(*x, f32, "x");
+    TORCH_CHECK(r.cols % a.heads == 0, "head_proj: x columns");
+    a.x = r.p;
+    a.x_ld = r.ld;
+    a.xk = r.cols / a.heads;
+    a.n = x_rows ? (int)x_rows->numel() : r.n;
+    TORCH_CHECK(a.xk <= a.k, "head_proj: x columns");
+    if (x_rows) a.x_rows = i32_ptr(*x_rows, a.n, "x_rows");
+  } else {
+    TORCH_CHECK(part_o->dim() == 4 && part_o->size(1) == a.heads &&
+                    part_o->size(3) == a.k && !x_rows,
+                "part_o must be [n, H, splits, k]");
+    a.n = (int)part_o->size(0);
+    a.splits = (int)part_o->size(2);
+    a.xk = a.k;
+    const Parts p = parts(part_o, part_ml,
+                          (int64_t)a.n * a.heads * a.splits, a.k);
+    a.part_o = p.o;
+    a.part_ml = p.ml;
+  }
+  if (out_rows) {
+    a.out_rows = i32_ptr(*out_rows, a.n, "out_rows");
+  } else {
+    TORCH_CHECK(o.n >= a.n, "head_proj: out rows");
+  }
+  if (gate) {
+    const Rows g = rows_of(*gate, f32, "gate");
+    TORCH_CHECK(g.n == o.n && g.cols == a.heads, "gate must be [n, H]");
+    a.gate = g.p;
+    a.gate_ld = g.ld;
+  }
+  a.out = o.p;
+  a.out_ld = o.ld;
+  a.w = w.data_ptr();
+  TORCH_CHECK(a.n > 0 && 16 * (a.k + 8) * (f32 ? 4 : 2) +
+                      16 * a.splits * 4 <= 65536,
+              "head_proj: sizes");
+  launch_head_proj(a, f32, cur_stream());
+}
+
+void latent_attn(Opt out, torch::Tensor q, torch::Tensor pages,
+                 torch::Tensor table, torch::Tensor seg, int64_t max_len,
+                 int64_t window, double scale, int64_t splits, Opt part_o,
+                 Opt part_ml) {
+  const int f32 = act_type(q, "q");
+  RowAttnArgs a{};
+  a.dim = a.vdim = latent_pages(pages, f32);
+  TORCH_CHECK(q.dim() == 3 && q.size(2) == a.dim, "q must be [n, H, rpad]");
+  a.heads = (int)q.size(1);
+  a.groups = 1;
+  a.q = q.data_ptr();
+  a.q_row = (int64_t)a.heads * a.dim;
+  a.k = a.v = pages.data_ptr();
+  TORCH_CHECK(table.dim() == 2, "table must be [slots, pages]");
+  a.table = i32_ptr(table, table.numel(), "table");
+  a.table_stride = (int)table.size(1);
+  a.seg = seg_view(seg);
+  a.max_len = (int)max_len;
+  a.splits = (int)splits;
+  a.window = (int)std::min<int64_t>(window, INT32_MAX / 2);
+  a.scale_log2 = (float)(scale * 1.4426950408889634);
+  a.vec = a.out_vec = 1;
+  TORCH_CHECK(window > 0 && max_len > 0 && max_len <= q.size(0) &&
+                  splits > 0 && splits <= 256,
+              "latent_attn: sizes");
+  if (splits > 1) {
+    TORCH_CHECK(part_o && part_o->dim() == 4 &&
+                    part_o->size(0) == q.size(0) &&
+                    part_o->size(2) == splits,
+                "part_o must be [n, H, splits, rpad]");
+    const Parts p = parts(part_o, part_ml, q.size(0) * a.heads * splits,
+                          a.dim);
+    a.part_o = p.o;
+    a.part_ml = p.ml;
+  } else {
+    TORCH_CHECK(out, "latent_attn: out");
+    check_like(*out, f32, "out");
+    TORCH_CHECK(out->numel() == q.numel(), "latent_attn: out size");
+    a.out = out->data_ptr();
+    a.out_row = a.q_row;
+  }
+  const int rc = f32 ? launch_latent_attn_f32(a, cur_stream())
+                     : launch_latent_attn_bf16(a, cur_stream());
+  TORCH_CHECK(rc == 0, "latent_attn: unsupported row size ", a.dim);
+}
+
+void head_attn(torch::Tensor out, torch::Tensor q, torch::Tensor kv,
+               torch::Tensor seg, torch::Tensor ctx_seg, int64_t max_len,
+               int64_t heads, int64_t dim, int64_t vdim, int64_t window,
+               double scale, Opt gate) {
+  const int f32 = row_type(q, "q");
+  const Rows o = rows_of(out, f32, "out"), r = rows_of(q, f32, "q"),
+             k = rows_of(kv, f32, "kv");
+  TORCH_CHECK(heads > 0 && r.cols == heads * dim && o.cols == heads * vdim &&
+                  k.cols == heads * (dim + vdim) && o.n == r.n,
+              "head_attn: columns");
+  RowAttnArgs a{};
+  a.heads = a.groups = (int)heads;
+  a.dim = (int)dim;
+  a.vdim = (int)vdim;
+  a.out = o.p;
+  a.out_row = o.ld;
+  a.q = r.p;
+  a.q_row = r.ld;
+  const int size = f32 ? 4 : 2, n = 16 / size;
+  a.k = k.p;
+  a.v = (char*)k.p + heads * dim * size;
+  a.kv_row = k.ld;
+  a.seg = seg_view(seg);
+  const SegView c = seg_view(ctx_seg);
+  TORCH_CHECK(c.n == a.seg.n, "head_attn: segments");
+  a.ctx_start = c.start;
+  a.ctx_first = c.pos0;
+  if (gate) {
+    const Rows g = rows_of(*gate, f32, "gate");
+    TORCH_CHECK(g.n == o.n && g.cols == heads, "gate must be [n, H]");
+    a.gate = g.p;
+    a.gate_row = g.ld;
+  }
+  TORCH_CHECK(window > 0 && max_len > 0 && max_len <= r.n, "head_attn: sizes");
+  a.window = (int)std::min<int64_t>(window, INT32_MAX / 2);
+  a.scale_log2 = (float)(scale * 1.4426950408889634);
+  a.splits = 1;
+  a.max_len = (int)max_len;
+  a.vec = dim % n == 0 && vdim % n == 0 && r.ld % n == 0 && k.ld % n == 0 &&
+          (size_t)r.p % 16 == 0 && (size_t)k.p % 16 == 0;
+  a.out_vec = vdim % 4 == 0 && o.ld % 4 == 0 && (size_t)o.p % (4 * size) == 0;
+  const int rc = f32 ? launch_head_attn_f32(a, cur_stream())
+                     : launch_head_attn_bf16(a, cur_stream());
+  TORCH_CHECK(rc == 0, "head_attn: unsupported sizes ", dim, ", ", vdim);
+}
+
+struct Experts {
+  MoePlan p;
+  int n, f32;
+};
+
+// the plan that moe_route made for n rows
+Experts experts_of(const torch::Tensor& w, const torch::Tensor& plan,
+                   int64_t pairs, int64_t top, int f32) {
+  TORCH_CHECK(top > 0 && pairs % top == 0 && pairs > 0, "expert rows");
+  const int n = (int)(pairs / top), e = (int)w.size(0);
+  const int* p = i32_ptr(plan, moe_plan_ints(n, (int)top, e), "plan");
+  return Experts{
+      moe_plan(const_cast<int*>(p), n, (int)top, e, f32 ? 0 : 1), n, f32};
+}
+
+torch::Tensor moe_route(torch::Tensor weight, torch::Tensor x,
+                        torch::Tensor router, int64_t top) {
+  const int f32 = act_type(x, "x");
+  check_like(router, f32, "router");
+  TORCH_CHECK(x.dim() == 2 && router.dim() == 2 &&
+                  router.size(1) == x.size(1),
+              "moe_route: sizes");
+  const int n = (int)x.size(0), e = (int)router.size(0);
+  TORCH_CHECK(n > 0 && e <= 256 && top >= 1 && top <= e && top <= 64,
+              "moe_route: at most 256 experts, 64 of them for a token");
+  float* wp = const_cast<float*>(f32_ptr(weight, n * top, "weight"));
+  torch::Tensor plan = torch::empty({moe_plan_ints(n, (int)top, e)},
+                                    x.options().dtype(torch::kInt32));
+  torch::Tensor z =
+      torch::empty({n, e}, x.options().dtype(torch::kFloat32));
+  launch_moe_route(wp, z.data_ptr<float>(), x.data_ptr(), router.data_ptr(),
+                   moe_plan(plan.data_ptr<int>(), n, (int)top, e,
+                            f32 ? 0 : 1),
+                   n, (int)x.size(1), f32, cur_stream());
+  return plan;
+}
+
+void moe_up(torch::Tensor mid, torch::Tensor x, torch::Tensor w,
+            torch::Tensor plan, int64_t act) {
+  const int f32 = act_type(x, "x");
+  check_like(mid, f32, "mid");
+  check_like(w, f32, "w");
+  TORCH_CHECK(x.dim() == 2 && mid.dim() == 2 && w.dim() == 3 &&
+                  w.size(1) == 2 * mid.size(1) && w.size(2) == x.size(1) &&
+                  mid.size(0) % x.size(0) == 0,
+              "moe_up: sizes");
+  TORCH_CHECK(act == 0 || act == 1, "moe_up: act");
+  const Experts e = experts_of(w, plan, mid.size(0),
+                               mid.size(0) / x.size(0), f32);
+  launch_moe_up(mid.data_ptr(), x.data_ptr(), w.data_ptr(), e.p,
+                (int)mid.size(1), (int)x.size(1), (int)act, f32,
+                cur_stream());
+}
+
+void moe_down(torch::Tensor out, torch::Tensor mid, torch::Tensor w,
+              torch::Tensor plan) {
+  const int f32 = act_type(mid, "mid");
+  check_like(out, f32, "out");
+  check_like(w, f32, "w");
+  TORCH_CHECK(out.dim() == 3 && mid.dim() == 2 && w.dim() == 3 &&
+                  w.size(1) == out.size(2) && w.size(2) == mid.size(1) &&
+                  mid.size(0) == out.size(0) * out.size(1),
+              "moe_down: sizes");
+  const Experts e = experts_of(w, plan, mid.size(0), out.size(1), f32);
+  launch_moe_down(out.data_ptr(), mid.data_ptr(), w.data_ptr(), e.p,
+                  (int)out.size(2), (int)mid.size(1), f32, cur_stream());
+}
+
 void skinny_gemm(torch::Tensor out, torch::Tensor w, torch::Tensor x,
                  bool act, double act_p, double act_q) {
   TORCH_CHECK(x.dim() == 2 && w.dim() == 2 && out.dim() == 2, "2-D operands");
@@ -293,7 +635,9 @@ void bind_hybrid(py::module_& m) {
         py::arg("xn") = none, py::arg("next_w") = none,
         py::arg("tokens") = none, py::arg("table") = none,
         py::arg("scale") = 1.0, py::arg("offset") = 0.0,
-        py::arg("eps") = 1e-6);
+        py::arg("eps") = 1e-6, py::arg("mult") = 1.0,
+        py::arg("pos_table") = none, py::arg("row_pos") = none,
+        py::arg("routed") = none, py::arg("routed_w") = none);
   m.def("xielu", &xielu, "in-place xIELU", py::arg("z"), py::arg("p"),
         py::arg("q"));
   m.def("hgrn2_step", &hgrn2_step,
@@ -318,6 +662,41 @@ void bind_hybrid(py::module_& m) {
         py::arg("max_len"), py::arg("window"), py::arg("keep_first"),
         py::arg("scale"), py::arg("splits"), py::arg("part_o") = none,
         py::arg("part_ml") = none);
+  m.def("latent_norm_append", &latent_norm_append,
+        "norms of the query and key/value latents + paged cache append",
+        py::arg("pages"), py::arg("kv"), py::arg("kv_w"),
+        py::arg("row_slot"), py::arg("row_pos"), py::arg("table"),
+        py::arg("eps"), py::arg("q_out") = none, py::arg("q") = none,
+        py::arg("q_w") = none);
+  m.def("latent_gather", &latent_gather, "cached latents as flat rows",
+        py::arg("out"), py::arg("pages"), py::arg("table"), py::arg("seg"),
+        py::arg("max_len"));
+  m.def("gated_act", &gated_act, "act(gate) * up", py::arg("out"),
+        py::arg("gate"), py::arg("up"), py::arg("act"));
+  m.def("head_proj", &head_proj, "per-head product of a few rows",
+        py::arg("out"), py::arg("x"), py::arg("w"), py::arg("x_rows") = none,
+        py::arg("out_rows") = none, py::arg("gate") = none,
+        py::arg("part_o") = none, py::arg("part_ml") = none);
+  m.def("latent_attn", &latent_attn,
+        "windowed attention of all heads over paged latents",
+        py::arg("out"), py::arg("q"), py::arg("pages"), py::arg("table"),
+        py::arg("seg"), py::arg("max_len"), py::arg("window"),
+        py::arg("scale"), py::arg("splits"), py::arg("part_o") = none,
+        py::arg("part_ml") = none);
+  m.def("head_attn", &head_attn,
+        "windowed attention per head over flat key/value rows, head gates",
+        py::arg("out"), py::arg("q"), py::arg("kv"), py::arg("seg"),
+        py::arg("ctx_seg"), py::arg("max_len"), py::arg("heads"),
+        py::arg("dim"), py::arg("vdim"), py::arg("window"), py::arg("scale"),
+        py::arg("gate") = none);
+  m.def("moe_route", &moe_route,
+        "float router, top experts, pairs ordered by expert",
+        py::arg("weight"), py::arg("x"), py::arg("router"), py::arg("top"));
+  m.def("moe_up", &moe_up, "experts' gate and up products + activation",
+        py::arg("mid"), py::arg("x"), py::arg("w"), py::arg("plan"),
+        py::arg("act"));
+  m.def("moe_down", &moe_down, "experts' down products", py::arg("out"),
+        py::arg("mid"), py::arg("w"), py::arg("plan"));
   m.def("skinny_gemm", &skinny_gemm, "projection of up to 32 rows",
         py::arg("out"), py::arg("w"), py::arg("x"), py::arg("act") = false,
         py::arg("act_p") = 0.0, py::arg("act_q") = 0.0);

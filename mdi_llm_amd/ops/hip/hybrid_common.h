@@ -69,3 +69,10 @@ DEVINL float xielu(float z, float p, float q) {
 }
 
 DEVINL float sigmoid(float z) { return 1.f / (1.f + expf(-z)); }
+
+DEVINL float gated(float gate, float up, int act) {
+  if (act == 0) return gate * sigmoid(gate) * up;
+  const float inner =
+      0.7978845608028654f * (gate + 0.044715f * gate * gate * gate);
+  return 0.5f * gate * (1.f + tanhf(inner)) * up;
+}

@@ -19,13 +19,29 @@ struct SegView {
 
 // Residual + norm step, one row per block.  x [n, e] float:
 //   tokens != null : x = scale * table[token]
-//   y != null      : x += post_w ? rms(y) * (offset + post_w) : y
-// then, if next_w, xn = rms(x) * (offset + next_w).  -1: e is too large.
-int launch_residual_norm(float* x, const void* y, const float* post_w,
-                         void* xn, const float* next_w, const int* tokens,
-                         const void* table, float scale, float offset,
-                         float eps, int n, int e, int f32,
-                         hipStream_t stream);
+//                    (+ pos_table[row_pos] if there is one)
+//   y != null      : x += mult * (post_w ? rms(y) * (offset + post_w) : y,
+//                    plus the weighted routed rows [n, top, e] if any)
+// then, if next_w, xn = rms(x) * (offset + next_w).
+struct ResidualArgs {
+  float* x;
+  const void* y;
+  const float* post_w;
+  void* xn;
+  const float* next_w;
+  const int* tokens;
+  const void* table;
+  const void* pos_table;
+  const int* row_pos;
+  const void* routed;
+  const float* routed_w;
+  int top;
+  float scale, offset, eps, mult;
+  int n, e;
+};
+
+// -1: e is too large
+int launch_residual_norm(const ResidualArgs& a, int f32, hipStream_t stream);
 
 // z <- xIELU(z), p and q already through softplus
 void launch_xielu(void* z, long long n, float p, float q, int f32,
@@ -85,6 +101,105 @@ struct PagedAttnArgs {
 // Returns -1 when (dpad, vpad) has no instantiation.
 int launch_paged_attn_bf16(const PagedAttnArgs& a, hipStream_t stream);
 int launch_paged_attn_f32(const PagedAttnArgs& a, hipStream_t stream);
+
+struct RowAttnArgs {
+  void* out;              // head h of row r at r * out_row + h * vdim
+  const void* q;          // head h of row r at r * q_row + h * dim
+  const void* k;          // latent: pages [P, 64, dim]; head: flat rows
+  const void* v;          // head: flat rows (kv_row apart, as k)
+  const int* table;       // latent: pages of a slot
+  const int* ctx_start;   // head: flat row of position ctx_first, by segment
+  const int* ctx_first;
+  const void* gate;       // head: sigmoid(gate[r * gate_row + h]) or null
+  float* part_o;          // latent, splits > 1: [rows, H, splits, dim]
+  float* part_ml;         // and [rows, H, splits, 2]
+  long long out_row, q_row, kv_row, gate_row;
+  SegView seg;
+  int table_stride;
+  int heads, groups;      // groups: 1 (latent) or heads
+  int dim, vdim;          // latent: the padded row, both
+  int window;
+  float scale_log2;
+  int splits, max_len;
+  int vec, out_vec;       // 16-byte loads and 4-element stores are aligned
+};
+
+// Return -1 when the sizes have no instantiation.
+int launch_latent_attn_bf16(const RowAttnArgs& a, hipStream_t stream);
+int launch_latent_attn_f32(const RowAttnArgs& a, hipStream_t stream);
+int launch_head_attn_bf16(const RowAttnArgs& a, hipStream_t stream);
+int launch_head_attn_f32(const RowAttnArgs& a, hipStream_t stream);
+
+// Norms of a row's two latents: q [n, q_rank] (rows q_ld apart) to q_out, kv
+// [n, rank] to its place in the pages [P, 64, rpad].  Either may be null;
+// kv_w null: kv is stored as it is.
+void launch_latent_norm_append(void* q_out, const void* q, const float* q_w,
+                               void* pages, const void* kv,
+                               const float* kv_w, const int* row_slot,
+                               const int* row_pos, const int* table,
+                               int table_stride, int n, int q_rank,
+                               long long q_ld, int rank, long long kv_ld,
+                               int rpad, float eps, int f32,
+                               hipStream_t stream);
+
+// out[start[s] + t, :rank] = the cached row of position pos0[s] + t
+void launch_latent_gather(void* out, const void* pages, const int* table,
+                          int table_stride, SegView seg, int max_len,
+                          int rank, int rpad, int f32, hipStream_t stream);
+
+// out = act(gate) * up over [n, cols] views; act 0 silu, 1 tanh-gelu
+void launch_gated_act(void* out, long long out_ld, const void* gate,
+                      const void* up, long long in_ld, int n, int cols,
+                      int act, int f32, hipStream_t stream);
+
+// Per-head product out[r, h*m ..] = w[h] x[r, h*xk ..] with w [H, m, k], k a
+// multiple of 32 and xk <= k.  x_rows / out_rows map the n rows (null: as
+// they are); gate is by output row.  part_o [n, H, splits, k] and part_ml, if
+// given, are merged to make x.
+struct HeadProjArgs {
+  void* out;
+  const void* x;
+  const void* w;
+  const int* x_rows;
+  const int* out_rows;
+  const void* gate;
+  const float* part_o;
+  const float* part_ml;
+  long long out_ld, x_ld, gate_ld;
+  int n, heads, m, k, xk, splits;
+};
+
+void launch_head_proj(const HeadProjArgs& a, int f32, hipStream_t stream);
+
+// Routing.  plan is one int buffer:
+//   chosen experts [n*top] | pairs ordered by expert [n*top] | number of
+//   tiles | tiles [max_tiles][3] = expert, first place in the order, rows
+// where pair p is choice p % top of row p / top and a tile is up to
+// tile_rows pairs of one expert.
+struct MoePlan {
+  int* chosen;
+  int* order;
+  int* n_tiles;
+  int* tiles;
+  int pairs, top, experts, tile_rows, max_tiles;
+};
+
+MoePlan moe_plan(int* buffer, int n, int top, int experts, int bf16_large);
+long long moe_plan_ints(int n, int top, int experts);
+
+// z [n, experts] = x router^T in float; weight [n, top] = softmax over the
+// top logits.
+void launch_moe_route(float* weight, float* z, const void* x,
+                      const void* router, MoePlan p, int n, int k, int f32,
+                      hipStream_t stream);
+
+// mid[pair] = act(gate x) * (up x), w [experts, 2 * ff, k]
+void launch_moe_up(void* mid, const void* x, const void* w, MoePlan p,
+                   int ff, int k, int act, int f32, hipStream_t stream);
+
+// out[pair] = w x, w [experts, m, ff], x [pairs, ff]
+void launch_moe_down(void* out, const void* mid, const void* w, MoePlan p,
+                     int m, int ff, int f32, hipStream_t stream);
 
 // Between the steps of an unchanged decode batch: tokens = sampled,
 // pos += 1; entries of the spare slot stay where they are.

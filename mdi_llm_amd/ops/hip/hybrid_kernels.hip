@@ -23,14 +23,13 @@ DEVINL float block_sum(float v, float* red) {
 
 template <typename T, int V, int NT, int KEEP>
 __global__ __launch_bounds__(NT) void residual_norm_kernel(
-    float* __restrict__ x, const T* __restrict__ y,
-    const float* __restrict__ post_w, T* __restrict__ xn,
-    const float* __restrict__ next_w, const int* __restrict__ tokens,
-    const T* __restrict__ table, float scale, float offset, float eps,
-    int e) {
+    ResidualArgs p) {
   __shared__ float red[NT / 64];
   const size_t row = blockIdx.x;
-  x += row * e;
+  const int e = p.e;
+  const float offset = p.offset, eps = p.eps;
+  float* __restrict__ x = p.x + row * e;
+  const T* __restrict__ y = (const T*)p.y;
   using PT = Pack<T, V>;
   using PF = Pack<float, V>;
   PF a[KEEP];
@@ -38,23 +37,31 @@ __global__ __launch_bounds__(NT) void residual_norm_kernel(
 #define EACH(i)                                                 \
   _Pragma("unroll") for (int k = 0; k < KEEP; ++k)              \
     if (const int i = (k * NT + threadIdx.x) * V; i < e)
-  if (tokens != nullptr) {
-    const T* t = table + (size_t)tokens[row] * e;
+  if (p.tokens != nullptr) {
+    const T* t = (const T*)p.table + (size_t)p.tokens[row] * e;
     EACH(i) {
       const PT b = *reinterpret_cast<const PT*>(t + i);
 #pragma unroll
-      for (int j = 0; j < V; ++j) a[k].v[j] = to_f(b.v[j]) * scale;
-      *reinterpret_cast<PF*>(x + i) = a[k];
+      for (int j = 0; j < V; ++j) a[k].v[j] = to_f(b.v[j]) * p.scale;
     }
+    if (p.pos_table != nullptr) {
+      const T* t = (const T*)p.pos_table + (size_t)p.row_pos[row] * e;
+      EACH(i) {
+        const PT b = *reinterpret_cast<const PT*>(t + i);
+#pragma unroll
+        for (int j = 0; j < V; ++j) a[k].v[j] += to_f(b.v[j]);
+      }
+    }
+    EACH(i) *reinterpret_cast<PF*>(x + i) = a[k];
   } else {
     EACH(i) a[k] = *reinterpret_cast<const PF*>(x + i);
     if (y != nullptr) {
       y += row * e;
       PT b[KEEP];
       EACH(i) b[k] = *reinterpret_cast<const PT*>(y + i);
-      if (post_w != nullptr) {
+      if (p.post_w != nullptr) {
         PF w[KEEP];
-        EACH(i) w[k] = *reinterpret_cast<const PF*>(post_w + i);
+        EACH(i) w[k] = *reinterpret_cast<const PF*>(p.post_w + i);
         float s = 0.f;
         EACH(i) {
 #pragma unroll
@@ -64,26 +71,36 @@ __global__ __launch_bounds__(NT) void residual_norm_kernel(
         EACH(i) {
 #pragma unroll
           for (int j = 0; j < V; ++j)
-            a[k].v[j] += to_f(b[k].v[j]) * r * (offset + w[k].v[j]);
+            a[k].v[j] +=
+                to_f(b[k].v[j]) * r * (offset + w[k].v[j]) * p.mult;
         }
       } else {
         EACH(i) {
 #pragma unroll
-          for (int j = 0; j < V; ++j) a[k].v[j] += to_f(b[k].v[j]);
+          for (int j = 0; j < V; ++j) a[k].v[j] += to_f(b[k].v[j]) * p.mult;
+        }
+      }
+      for (int r = 0; r < p.top; ++r) {
+        const float f = p.routed_w[row * p.top + r] * p.mult;
+        const T* z = (const T*)p.routed + (row * p.top + r) * e;
+        EACH(i) {
+          const PT v = *reinterpret_cast<const PT*>(z + i);
+#pragma unroll
+          for (int j = 0; j < V; ++j) a[k].v[j] += f * to_f(v.v[j]);
         }
       }
       EACH(i) *reinterpret_cast<PF*>(x + i) = a[k];
     }
   }
-  if (next_w == nullptr) return;
+  if (p.next_w == nullptr) return;
   PF w[KEEP];
   EACH(i) {
-    w[k] = *reinterpret_cast<const PF*>(next_w + i);
+    w[k] = *reinterpret_cast<const PF*>(p.next_w + i);
 #pragma unroll
     for (int j = 0; j < V; ++j) ss += a[k].v[j] * a[k].v[j];
   }
   const float r = 1.f / sqrtf(block_sum<NT>(ss, red) / e + eps);
-  xn += row * e;
+  T* __restrict__ xn = (T*)p.xn + row * e;
   EACH(i) {
     PT o;
 #pragma unroll
@@ -95,14 +112,10 @@ __global__ __launch_bounds__(NT) void residual_norm_kernel(
 }
 
 template <typename T>
-static int residual_norm_t(float* x, const void* y, const float* post_w,
-                           void* xn, const float* next_w, const int* tokens,
-                           const void* table, float scale, float offset,
-                           float eps, int n, int e, hipStream_t stream) {
-#define ROWS(V, NT, KEEP)                                                 \
-  residual_norm_kernel<T, V, NT, KEEP><<<n, NT, 0, stream>>>(             \
-      x, (const T*)y, post_w, (T*)xn, next_w, tokens, (const T*)table,    \
-      scale, offset, eps, e)
+static int residual_norm_t(const ResidualArgs& a, hipStream_t stream) {
+  const int n = a.n, e = a.e;
+#define ROWS(V, NT, KEEP) \
+  residual_norm_kernel<T, V, NT, KEEP><<<n, NT, 0, stream>>>(a)
   if (e % 4 != 0) {
     if (e > 1024 * 16) return -1;
     if (e <= 1024) ROWS(1, 256, 4);
@@ -125,15 +138,9 @@ static int residual_norm_t(float* x, const void* y, const float* post_w,
   return 0;
 }
 
-int launch_residual_norm(float* x, const void* y, const float* post_w,
-                         void* xn, const float* next_w, const int* tokens,
-                         const void* table, float scale, float offset,
-                         float eps, int n, int e, int f32,
-                         hipStream_t stream) {
-  return f32 ? residual_norm_t<float>(x, y, post_w, xn, next_w, tokens, table,
-                                      scale, offset, eps, n, e, stream)
-             : residual_norm_t<bf16>(x, y, post_w, xn, next_w, tokens, table,
-                                     scale, offset, eps, n, e, stream);
+int launch_residual_norm(const ResidualArgs& a, int f32, hipStream_t stream) {
+  return f32 ? residual_norm_t<float>(a, stream)
+             : residual_norm_t<bf16>(a, stream);
 }
 
 // ---------------------------------------------------------------------------

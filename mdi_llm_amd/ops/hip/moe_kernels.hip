@@ -1,0 +1,262 @@
+// Mixture of experts over a ragged batch (gfx950): float router, top
+// experts and their weights, the pairs (row, choice) ordered by expert, and
+// the experts' products over tiles of pairs of one expert.  Nothing comes
+// back to the host, so decode steps can be captured.
+
+#include "mfma_frag.h"
+
+namespace {
+
+constexpr int MAX_EXPERTS = 256;
+constexpr int FUSED_ROWS = 64;  // up to here one block chooses and orders
+
+// 8 contraction steps of a row of length k; vec: rows are 16-byte aligned
+template <typename T>
+DEVINL typename Frag<T>::Row load_steps(const T* row, int at, int k,
+                                        bool vec) {
+  using F = Frag<T>;
+  if (vec && at + 8 <= k) return F::load_frag(row + at);
+  typename F::Row r = F::zero();
+#pragma unroll
+  for (int j = 0; j < 8; ++j)
+    if (at + j < k) F::set(r, j, row[at + j]);
+  return r;
+}
+
+// out[row][m]: 16 x 16 tile of x w^T, the contraction split over NW waves in
+// stretches of 64 (a lane's 16 steps of a stretch are contiguous), NM weight
+// rows sets at once.  The sum is left in red[..][row][m] of every wave.
+template <typename T, int NW, int NM>
+DEVINL void tile_product(float (*red)[NM][16][17], const T* x,
+                         const T* const (&w)[NM], int k, bool vec) {
+  using F = Frag<T>;
+  const int lane = threadIdx.x & 63, c = lane & 15, quad = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  f32x4 acc[NM];
+#pragma unroll
+  for (int j = 0; j < NM; ++j) acc[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 2
+  for (int at = wave * 64; at < k; at += NW * 64) {
+    const int s = at + quad * 16;
+    const auto xa = load_steps<T>(x, s, k, vec);
+    const auto xb = load_steps<T>(x, s + 8, k, vec);
+#pragma unroll
+    for (int j = 0; j < NM; ++j) {
+      acc[j] = F::dot(load_steps<T>(w[j], s, k, vec), xa, acc[j]);
+      acc[j] = F::dot(load_steps<T>(w[j], s + 8, k, vec), xb, acc[j]);
+    }
+  }
+#pragma unroll
+  for (int j = 0; j < NM; ++j)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) red[wave][j][c][quad * 4 + i] = acc[j][i];
+  __syncthreads();
+}
+
+template <int NW, int NM>
+DEVINL float tile_sum(const float (*red)[NM][16][17], int j, int row, int m) {
+  float v = 0.f;
+#pragma unroll
+  for (int q = 0; q < NW; ++q) v += red[q][j][row][m];
+  return v;
+}
+
+// ---------------------------------------------------------------------------
+template <typename T, int NW>
+__global__ __launch_bounds__(NW * 64) void router_kernel(
+    float* __restrict__ z, const T* __restrict__ x, const T* __restrict__ w,
+    int n, int experts, int k, bool vec) {
+  __shared__ float red[NW][1][16][17];
+  const int c = threadIdx.x & 15, r0 = blockIdx.y * 16, e0 = blockIdx.x * 16;
+  const T* const wp[1] = {w + (size_t)min(e0 + c, experts - 1) * k};
+  tile_product<T, NW, 1>(red, x + (size_t)min(r0 + c, n - 1) * k, wp, k, vec);
+  for (int i = threadIdx.x; i < 256; i += NW * 64) {
+    const int row = i >> 4, e = i & 15;
+    if (r0 + row < n && e0 + e < experts)
+      z[(size_t)(r0 + row) * experts + e0 + e] =
+          tile_sum<NW, 1>(red, 0, row, e);
+  }
+}
+
+// One wave: the top logits of a row (lower index first among equals) and
+// their softmax.
+DEVINL void choose(float* weight, int* chosen, const float* z, int experts,
+                   int top, int lane) {
+  float v[MAX_EXPERTS / 64];
+#pragma unroll
+  for (int j = 0; j < MAX_EXPERTS / 64; ++j) {
+    const int e = j * 64 + lane;
+    v[j] = e < experts ? z[e] : -__builtin_huge_valf();
+  }
+  float zmax = 0.f, sum = 0.f, mine = 0.f;
+  for (int t = 0; t < top; ++t) {
+    float best = -__builtin_huge_valf();
+    int at = MAX_EXPERTS;
+#pragma unroll
+    for (int j = 0; j < MAX_EXPERTS / 64; ++j)
+      if (v[j] > best) {
+        best = v[j];
+        at = j * 64 + lane;
+      }
+#pragma unroll
+    for (int off = 32; off > 0; off >>= 1) {
+      const float ov = __shfl_xor(best, off, 64);
+      const int oa = __shfl_xor(at, off, 64);
+      if (ov > best || (ov == best && oa < at)) {
+        best = ov;
+        at = oa;
+      }
+    }
+    at = min(at, experts - 1);  // only if a logit is not a number
+    if (t == 0) zmax = best;
+    const float e = expf(best - zmax);
+    sum += e;
+    // a wave holds up to 64 choices, one per lane
+    if (lane == t) {
+      mine = e;
+      chosen[t] = at;
+    }
+#pragma unroll
+    for (int j = 0; j < MAX_EXPERTS / 64; ++j)
+      if (at == j * 64 + lane) v[j] = -__builtin_huge_valf();
+  }
+  if (lane < top) weight[lane] = mine / sum;
+}
+
+__global__ __launch_bounds__(256) void choose_kernel(
+    float* __restrict__ weight, const float* __restrict__ z, MoePlan p,
+    int n) {
+  const int row = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (row >= n) return;
+  choose(weight + (size_t)row * p.top, p.chosen + (size_t)row * p.top,
+         z + (size_t)row * p.experts, p.experts, p.top, threadIdx.x & 63);
+}
+
+// One block: the pairs ordered by expert, and the tiles.
+__global__ __launch_bounds__(1024) void order_kernel(
+    float* __restrict__ weight, const float* __restrict__ z, MoePlan p,
+    int n, bool choose_here) {
+  __shared__ int count[MAX_EXPERTS], next[MAX_EXPERTS];
+  const int tid = threadIdx.x;
+  if (choose_here)
+    for (int row = tid >> 6; row < n; row += 16)
+      choose(weight + row * p.top, p.chosen + row * p.top,
+             z + row * p.experts, p.experts, p.top, tid & 63);
+  if (tid < p.experts) count[tid] = 0;
+  __syncthreads();
+  // (the block's own global writes are visible to it after the barrier)
+  for (int i = tid; i < p.pairs; i += 1024) atomicAdd(&count[p.chosen[i]], 1);
+  __syncthreads();
+  if (tid < p.experts) {
+    int first = 0, tile = 0;
+    for (int e = 0; e < tid; ++e) {
+      first += count[e];
+      tile += (count[e] + p.tile_rows - 1) / p.tile_rows;
+    }
+    next[tid] = first;
+    for (int at = 0; at < count[tid]; at += p.tile_rows, ++tile) {
+      p.tiles[tile * 3] = tid;
+      p.tiles[tile * 3 + 1] = first + at;
+      p.tiles[tile * 3 + 2] = min(p.tile_rows, count[tid] - at);
+    }
+    if (tid == p.experts - 1) *p.n_tiles = tile;
+  }
+  __syncthreads();
+  for (int i = tid; i < p.pairs; i += 1024)
+    p.order[atomicAdd(&next[p.chosen[i]], 1)] = i;
+}
+
+// ---------------------------------------------------------------------------
+// Products of up to 16 pairs of one expert; the weights stream once.
+// ---------------------------------------------------------------------------
+template <typename T, int NW, bool UP>
+__global__ __launch_bounds__(NW * 64) void expert_rows_kernel(
+    T* __restrict__ out, const T* __restrict__ x, const T* __restrict__ w,
+    MoePlan p, int m, int k, int act, bool vec) {
+  constexpr int NM = UP ? 2 : 1;
+  __shared__ float red[NW][NM][16][17];
+  const int tile = blockIdx.y;
+  if (tile >= *p.n_tiles) return;
+  const int e = p.tiles[tile * 3], first = p.tiles[tile * 3 + 1];
+  const int rows = p.tiles[tile * 3 + 2];
+  const int c = threadIdx.x & 15, m0 = blockIdx.x * 16;
+  const int pair = p.order[first + min(c, rows - 1)];
+  const T* xp = x + (size_t)(UP ? pair / p.top : pair) * k;
+  const T* we = w + ((size_t)e * NM * m + min(m0 + c, m - 1)) * k;
+  const T* wp[NM];
+#pragma unroll
+  for (int j = 0; j < NM; ++j) wp[j] = we + (size_t)j * m * k;
+  tile_product<T, NW, NM>(red, xp, wp, k, vec);
+  for (int i = threadIdx.x; i < 256; i += NW * 64) {
+    const int row = i >> 4, j = i & 15;
+    if (row >= rows || m0 + j >= m) continue;
+    float v = tile_sum<NW, NM>(red, 0, row, j);
+    if (UP) v = gated(v, tile_sum<NW, NM>(red, NM - 1, row, j), act);
+    out[(size_t)p.order[first + row] * m + m0 + j] = from_f<T>(v);
+  }
+}
+
+template <typename T, bool UP>
+void expert_rows_t(void* out, const void* x, const void* w, MoePlan p, int m,
+                   int k, int act, hipStream_t stream) {
+  const dim3 grid((m + 15) / 16, p.max_tiles);
+  const bool vec = k % (16 / sizeof(T)) == 0;
+#define EXPERT(NW)                                                      \
+  expert_rows_kernel<T, NW, UP><<<grid, NW * 64, 0, stream>>>(          \
+      (T*)out, (const T*)x, (const T*)w, p, m, k, act, vec)
+  if (k >= 2048) EXPERT(16);
+  else EXPERT(4);
+#undef EXPERT
+}
+
+}  // namespace
+
+MoePlan moe_plan(int* buffer, int n, int top, int experts, int bf16_large) {
+  MoePlan p;
+  p.pairs = n * top;
+  p.top = top;
+  p.experts = experts;
+  p.tile_rows = 16;
+  (void)bf16_large;
+  // every expert's last tile may be short
+  const long long tiles = p.pairs / p.tile_rows + experts;
+  p.max_tiles = (int)(tiles < p.pairs ? tiles : p.pairs);
+  p.chosen = buffer;
+  p.order = p.chosen + p.pairs;
+  p.n_tiles = p.order + p.pairs;
+  p.tiles = p.n_tiles + 1;
+  return p;
+}
+
+long long moe_plan_ints(int n, int top, int experts) {
+  const long long pairs = (long long)n * top;
+  return 2 * pairs + 1 + 3 * (pairs / 16 + experts);
+}
+
+void launch_moe_route(float* weight, float* z, const void* x,
+                      const void* router, MoePlan p, int n, int k, int f32,
+                      hipStream_t stream) {
+  const dim3 grid((p.experts + 15) / 16, (n + 15) / 16);
+  if (f32)
+    router_kernel<float, 16><<<grid, 1024, 0, stream>>>(
+        z, (const float*)x, (const float*)router, n, p.experts, k,
+        k % 4 == 0);
+  else
+    router_kernel<bf16, 16><<<grid, 1024, 0, stream>>>(
+        z, (const bf16*)x, (const bf16*)router, n, p.experts, k, k % 8 == 0);
+  const bool fused = n <= FUSED_ROWS;
+  if (!fused) choose_kernel<<<(n + 3) / 4, 256, 0, stream>>>(weight, z, p, n);
+  order_kernel<<<1, 1024, 0, stream>>>(weight, z, p, n, fused);
+}
+
+void launch_moe_up(void* mid, const void* x, const void* w, MoePlan p,
+                   int ff, int k, int act, int f32, hipStream_t stream) {
+  if (f32) expert_rows_t<float, true>(mid, x, w, p, ff, k, act, stream);
+  else expert_rows_t<bf16, true>(mid, x, w, p, ff, k, act, stream);
+}
+
+void launch_moe_down(void* out, const void* mid, const void* w, MoePlan p,
+                     int m, int ff, int f32, hipStream_t stream) {
+  if (f32) expert_rows_t<float, false>(out, mid, w, p, m, ff, 0, stream);
+  else expert_rows_t<bf16, false>(out, mid, w, p, m, ff, 0, stream);
+}

@@ -19,7 +19,7 @@ import math
 import os
 import warnings
 from bisect import bisect_left
-from dataclasses import dataclass
+from dataclasses import dataclass, field
 from fractions import Fraction
 from typing import Dict, List, Optional, Sequence, Tuple
 
@@ -30,6 +30,7 @@ from ..config import ModelConfig
 from ..models.cache import PAGE, HybridCache
 from ..models.sampling import sample as sample_token
 from . import require_hip_ops
+from .latent_layer import LatentPlan, ParallelLayer, make_plan
 
 __all__ = ["HybridEngine", "distance_bias"]
 
@@ -74,6 +75,18 @@ class Batch:
     row_pos: torch.Tensor
     tokens: Optional[torch.Tensor]
     max_ctx: int             # longest sequence, this step included
+    # the columns of seg on the host; None: single tokens, known only there
+    entries: Optional[List[Tuple[int, int, int, int]]] = None
+    plans: dict = field(default_factory=dict)
+    contexts: dict = field(default_factory=dict)  # gathered latents
+
+    def latent_plan(self, m, device, form: Optional[str]) -> LatentPlan:
+        if self.entries is None:
+            return LatentPlan(seg=self.seg, n_rows=self.n)
+        key = (m.dim, m.vdim, m.rank, m.window)
+        if key not in self.plans:
+            self.plans[key] = make_plan(self.entries, self.n, m, device, form)
+        return self.plans[key]
 
 
 class _LayerWeights:
@@ -162,7 +175,12 @@ class HybridEngine:
             self.ops = hybrid_torch
         self.use_graphs = use_graphs and self.hip
         self.is_starter = hasattr(stage, "lm_head")
-        self.layers = [_LayerWeights(b) for b in stage.transformer.h]
+        self.parallel = self.config.parallel_residual
+        self.latent_form: Optional[str] = None  # "absorbed" or "expanded"
+        if self.parallel:
+            self.layers = [ParallelLayer(self, b) for b in stage.transformer.h]
+        else:
+            self.layers = [_LayerWeights(b) for b in stage.transformer.h]
         for lw in self.layers:
             m = lw.mixer
             if m.kind == "hgrn2" and (m.dim > 256 or m.vdim > 1024):
@@ -173,21 +191,44 @@ class HybridEngine:
             self.wte = stage.transformer.wte.weight.detach()
             self.final = stage.transformer.ln_f.weight.detach().float()
             self.head = stage.lm_head.weight.detach()
+            wpe = getattr(stage.transformer, "wpe", None)
+            self.wpe = None if wpe is None else wpe.weight.detach()
+        self._ring_columns(stage)
         self._steps: Dict[int, _DecodeStep] = {}
+
+    def _ring_columns(self, stage) -> None:
+        """Columns of the rows between stages that hold shared latents: those
+        that local layers read from an earlier stage, those made here."""
+        first = stage.first_layer
+        at, self.ring_in, self.ring_out = self.config.n_embd, {}, {}
+        for src, n in self.config.shared_latents().items():
+            cols = slice(at, at + n)
+            at += n
+            if first <= src < first + len(self.layers):
+                self.ring_out[src] = cols
+            elif src in self.cache.latent:
+                self.ring_in[src] = cols
 
     # ------------------------------------------------------------------
     # building blocks
     # ------------------------------------------------------------------
-    def _norm_step(self, x, y=None, post_w=None, next_w=None, tokens=None):
-        """x <- embed(tokens) or x + post-norm(y); the next pre-norm."""
-        xn = None
+    def _norm_step(self, x, y=None, post_w=None, next_w=None, tokens=None,
+                   row_pos=None, routed=None):
+        """x <- embed(tokens) or x + post-norm(y) (+ routed experts); the
+        next pre-norm."""
+        xn, extra = None, {}
+        if tokens is not None and self.wpe is not None:
+            extra.update(pos_table=self.wpe, row_pos=row_pos)
+        if routed is not None:
+            extra.update(routed=routed[0], routed_w=routed[1])
         if next_w is not None:
             xn = torch.empty(x.shape, dtype=self.dtype, device=self.device)
         self.ops.residual_norm(
             x, y=y, post_w=post_w, xn=xn, next_w=next_w, tokens=tokens,
             table=None if tokens is None else self.wte,
             scale=self.config.embedding_scale,
-            offset=self.config.norm_offset, eps=self.config.norm_eps)
+            offset=self.config.norm_offset, eps=self.config.norm_eps,
+            mult=self.config.residual_mult, **extra)
         return xn
 
     def _linear(self, x: torch.Tensor, w: torch.Tensor, act=None):
@@ -272,10 +313,17 @@ class HybridEngine:
         if x is None:
             x = torch.empty(b.n, self.config.n_embd, dtype=torch.float32,
                             device=self.device)
-            xn = self._norm_step(x, next_w=first, tokens=b.tokens)
+            xn = self._norm_step(x, next_w=first, tokens=b.tokens,
+                                 row_pos=b.row_pos)
         else:
             xn = self._norm_step(x, next_w=first)
         for i, (lw, after) in enumerate(zip(self.layers, norms)):
+            if self.parallel:
+                y, routed = lw.step(b, xn)
+                xn = self._norm_step(x, y, None, after, routed=routed)
+                if layers_out is not None:
+                    layers_out.append(x.clone())
+                continue
             mix = self._hgrn2 if lw.mixer.kind == "hgrn2" else \
                 self._attention
             y = mix(i, lw, b, xn)
@@ -313,8 +361,9 @@ class HybridEngine:
             starts.append(at)
             at += n
         order = sorted(range(len(entries)), key=lambda e: entries[e][1] > 1)
-        seg = [[starts[e] for e in order], [entries[e][1] for e in order],
-               [entries[e][0] for e in order], [pos0[e] for e in order]]
+        cols = [(starts[e], entries[e][1], entries[e][0], pos0[e])
+                for e in order]
+        seg = list(map(list, zip(*cols)))
         row_slot = [s for s, n in entries for _ in range(n)]
         row_pos = [p + t for p, (_, n) in zip(pos0, entries)
                    for t in range(n)]
@@ -330,6 +379,7 @@ class HybridEngine:
             row_slot=flat[:at], row_pos=flat[at:2 * at],
             tokens=flat[2 * at + 4 * S:] if tokens is not None else None,
             max_ctx=max(p + n for p, (_, n) in zip(pos0, entries)),
+            entries=cols,
         )
         return b, starts
 
@@ -372,20 +422,41 @@ class HybridEngine:
     @torch.no_grad()
     def hidden(self, slot: int, tokens: Optional[Sequence[int]] = None,
                x: Optional[torch.Tensor] = None) -> torch.Tensor:
-        """Pipeline stages: one sequence's tokens (starter) or residual rows
-        (secondary) -> residual rows after the local layers, fp32."""
+        """Pipeline stages: one sequence's tokens (starter) or the rows of
+        the stage before (secondary) -> rows after the local layers, fp32:
+        the residual stream, then the latents that later stages may read."""
+        rows = None
         if tokens is not None:
             self._check_tokens(tokens)
+            n = len(tokens)
         else:
-            x = x.reshape(-1, self.config.n_embd).float().clone()
-        n = len(tokens) if x is None else x.size(0)
+            rows = x.reshape(-1, self.config.ring_width).float()
+            n, x = rows.size(0), rows[:, :self.config.n_embd].clone()
         b, _ = self._batch([(slot, n)], tokens)
-        return self._run(b, x, False)[0]
+        for src, cols in self.ring_in.items():
+            self.ops.latent_norm_append(
+                self.cache.latent[src], rows[:, cols].to(self.dtype), None,
+                b.row_slot, b.row_pos, self.cache.table,
+                self.config.norm_eps)
+        x = self._run(b, x, False)[0]
+        if self.config.ring_width == self.config.n_embd:
+            return x
+        out = torch.zeros(n, self.config.ring_width, device=self.device) \
+            if rows is None else rows.clone()
+        out[:, :self.config.n_embd] = x
+        for src, cols in self.ring_out.items():
+            c = torch.empty(n, cols.stop - cols.start, dtype=self.dtype,
+                            device=self.device)
+            self.ops.latent_gather(c, self.cache.latent[src],
+                                   self.cache.table, b.seg, n)
+            out[:, cols] = c
+        return out
 
     @torch.no_grad()
     def logits(self, x: torch.Tensor) -> torch.Tensor:
-        """Residual rows -> logits."""
-        x = x.reshape(-1, self.config.n_embd).float().contiguous()
+        """Rows of the last stage -> logits."""
+        x = x.reshape(-1, self.config.ring_width)[:, :self.config.n_embd]
+        x = x.float().contiguous()
         return self._linear(self._norm_step(x, next_w=self.final), self.head)
 
     # ------------------------------------------------------------------

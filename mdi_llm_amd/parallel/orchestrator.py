@@ -226,7 +226,7 @@ class MDIRuntime:
             expected_s=min(seq_len, tokens_per_sample + 256),
         )
         if self.world > 1:
-            self.comm = RingComm(config.n_embd, seq_len, self.device,
+            self.comm = RingComm(config.ring_width, seq_len, self.device,
                                  n_samples,
                                  dtype=config.residual_dtype(self.dtype))
         self.runtime = PipelineRuntime(self.runner, 0, self.world, self.comm,
@@ -317,7 +317,7 @@ class MDIRuntime:
                                   n_samples + (1 if env_serve else 0),
                                   self.device,
                                   expected_s=msg.get("expected_s"))
-        self.comm = RingComm(config.n_embd, seq_len, self.device, n_samples,
+        self.comm = RingComm(config.ring_width, seq_len, self.device, n_samples,
                              dtype=config.residual_dtype(self.dtype))
         self.runtime = PipelineRuntime(self.runner, msg["rank"],
                                        msg["world"], self.comm, self.device)

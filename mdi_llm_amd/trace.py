@@ -36,7 +36,8 @@ def load_runner(model_dir, dtype: torch.dtype, device: torch.device,
     stage = StarterStage(config, config.n_layer)
     stage.load_state_dict(sd)
     stage = stage.to(device=device, dtype=dtype).eval()
-    config.block_size = max(config.block_size, max_tokens)
+    if config.pos_embedding != "learned":  # a table ends where it ends
+        config.block_size = max(config.block_size, max_tokens)
     stage.max_seq_length = config.block_size
     return make_runner(stage, SLOTS, device, n_tokens=max_tokens)
 

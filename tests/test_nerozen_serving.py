@@ -191,7 +191,7 @@ def _ring_worker(rank, world, tmp, port, device):
     prompts = [torch.tensor(p) for p in torch.load(
         os.path.join(tmp, "prompts.pt"), weights_only=True)]
     runner = make_runner(stage, len(prompts), dev)
-    comm = RingComm(cfg.n_embd, stage.max_seq_length, dev, len(prompts),
+    comm = RingComm(cfg.ring_width, stage.max_seq_length, dev, len(prompts),
                     dtype=cfg.residual_dtype(torch.float32))
     rt = PipelineRuntime(runner, rank=rank, world=world, comm=comm,
                          device=dev)
