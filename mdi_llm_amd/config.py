@@ -2257,4 +2257,51 @@ configs.extend([
 ])
 
 
+# -- Resolorn ----------------------------------------------------
+
+
+def _resolorn_named(name: str, n_layer: int, width: int, vocab: int,
+                    attention: dict, size: int, ff: int, experts: dict,
+                    block_size: int) -> dict:
+    """A Resolorn stack with experts in every second layer, which shares the
+    latent of the layer before."""
+    layers = []
+    for i in range(n_layer):
+        mixer = dict(attention, mask=dict(size=size),
+                     scale=attention["dim"] ** -0.5)
+        mlp = dict(kind="dense", ff=ff)
+        if i % 2:
+            mixer["kv_from"] = i - 1
+            mlp = dict(experts, kind="moe")
+        layers.append(dict(type="latent_attention", mixer=mixer, mlp=mlp))
+    conf = _resolorn(dict(vocab=vocab, width=width, layers=layers,
+                          norm=dict(eps=1e-6), residual_mult=1.0,
+                          max_positions=block_size))
+    conf.update(name=name)
+    return conf
+
+
+configs.extend([
+    _resolorn_named("resolorn-nano", 4, 128, 384,
+                    dict(heads=4, dim=32, vdim=48, q_rank=80, kv_rank=56),
+                    72, 320, dict(router=dict(experts=6, top=2),
+                                  expert=dict(ff=48), shared=dict(ff=72)),
+                    block_size=1024),
+    # TinyLlama-1.1B and Llama-3-8B widths and weights used per token
+    _resolorn_named("resolorn-1b", 22, 2048, 32000,
+                    dict(heads=32, dim=64, vdim=64, q_rank=768, kv_rank=256),
+                    1024, 5632, dict(router=dict(experts=32, top=6),
+                                     expert=dict(ff=704),
+                                     shared=dict(ff=1408)),
+                    block_size=32768),
+    _resolorn_named("resolorn-8b", 32, 4096, 128256,
+                    dict(heads=32, dim=128, vdim=128, q_rank=1536,
+                         kv_rank=512),
+                    2048, 14336, dict(router=dict(experts=32, top=6),
+                                      expert=dict(ff=2048),
+                                      shared=dict(ff=2048)),
+                    block_size=32768),
+])
+
+
 name_to_config: dict[str, dict] = {c["name"]: c for c in configs}

@@ -318,36 +318,77 @@ int latent_pages(const torch::Tensor& pages, int f32) {
   return (int)pages.size(2);
 }
 
+void set_act(BranchArgs& a, const torch::Tensor& out,
+             const torch::Tensor& gate, const torch::Tensor& up, int64_t act,
+             int f32) {
+  const Rows o = rows_of(out, f32, "act_out"), g = rows_of(gate, f32, "gate"),
+             u = rows_of(up, f32, "up");
+  TORCH_CHECK(o.n == g.n && o.n == u.n && o.cols == g.cols &&
+                  o.cols == u.cols && g.ld == u.ld,
+              "gated activation: sizes");
+  TORCH_CHECK(act == 0 || act == 1, "gated activation: act");
+  a.out = o.p;
+  a.out_ld = o.ld;
+  a.gate = g.p;
+  a.up = u.p;
+  a.in_ld = g.ld;
+  a.cols = o.cols;
+  a.act = (int)act;
+  a.n = o.n;
+}
+
 void latent_norm_append(torch::Tensor pages, Opt kv, Opt kv_w,
                         torch::Tensor row_slot, torch::Tensor row_pos,
                         torch::Tensor table, double eps, Opt q_out, Opt q,
-                        Opt q_w) {
+                        Opt q_w, Opt act_out, Opt gate, Opt up,
+                        int64_t act) {
   const int f32 = act_type(pages, "pages");
-  const int rpad = latent_pages(pages, f32);
-  TORCH_CHECK((kv || q) && !!q == !!q_out && !!q == !!q_w && (kv || !kv_w),
+  BranchArgs a{};
+  a.pages = pages.data_ptr();
+  a.rpad = latent_pages(pages, f32);
+  a.eps = (float)eps;
+  TORCH_CHECK((kv || q) && !!q == !!q_out && !!q == !!q_w && (kv || !kv_w) &&
+                  !!act_out == !!gate && !!act_out == !!up,
               "latent_norm_append: bad combination of operands");
-  Rows k{}, r{};
-  int n = 0;
+  if (act_out) set_act(a, *act_out, *gate, *up, act, f32);
+  auto same_rows = [&](const Rows& r) {
+    TORCH_CHECK(a.n == 0 || a.n == r.n, "latent_norm_append: rows");
+    a.n = r.n;
+  };
   if (kv) {
-    k = rows_of(*kv, f32, "kv");
-    n = k.n;
-    TORCH_CHECK(k.cols <= rpad, "kv columns");
+    const Rows r = rows_of(*kv, f32, "kv");
+    same_rows(r);
+    TORCH_CHECK(r.cols <= a.rpad, "kv columns");
+    a.kv = r.p;
+    a.kv_ld = r.ld;
+    a.rank = r.cols;
+    if (kv_w) a.kv_w = f32_ptr(*kv_w, r.cols, "kv_w");
   }
   if (q) {
-    r = rows_of(*q, f32, "q");
-    TORCH_CHECK(!kv || r.n == n, "q and kv rows");
-    n = r.n;
+    const Rows r = rows_of(*q, f32, "q");
+    same_rows(r);
     check_like(*q_out, f32, "q_out");
-    TORCH_CHECK(q_out->numel() == (int64_t)n * r.cols, "q_out size");
+    TORCH_CHECK(q_out->numel() == (int64_t)r.n * r.cols, "q_out size");
+    a.q = r.p;
+    a.q_ld = r.ld;
+    a.q_rank = r.cols;
+    a.q_out = q_out->data_ptr();
+    a.q_w = f32_ptr(*q_w, r.cols, "q_w");
   }
   TORCH_CHECK(table.dim() == 2, "table must be [slots, pages]");
-  launch_latent_norm_append(
-      q ? q_out->data_ptr() : nullptr, r.p,
-      q ? f32_ptr(*q_w, r.cols, "q_w") : nullptr, pages.data_ptr(), k.p,
-      kv_w ? f32_ptr(*kv_w, k.cols, "kv_w") : nullptr,
-      i32_ptr(row_slot, n, "row_slot"), i32_ptr(row_pos, n, "row_pos"),
-      i32_ptr(table, table.numel(), "table"), (int)table.size(1), n, r.cols,
-      r.ld, k.cols, k.ld, rpad, (float)eps, f32, cur_stream());
+  a.row_slot = i32_ptr(row_slot, a.n, "row_slot");
+  a.row_pos = i32_ptr(row_pos, a.n, "row_pos");
+  a.table = i32_ptr(table, table.numel(), "table");
+  a.table_stride = (int)table.size(1);
+  launch_branch(a, f32, cur_stream());
+}
+
+void gated_act(torch::Tensor out, torch::Tensor gate, torch::Tensor up,
+               int64_t act) {
+  const int f32 = row_type(out, "out");
+  BranchArgs a{};
+  set_act(a, out, gate, up, act, f32);
+  launch_branch(a, f32, cur_stream());
 }
 
 void latent_gather(torch::Tensor out, torch::Tensor pages,
@@ -363,19 +404,6 @@ void latent_gather(torch::Tensor out, torch::Tensor pages,
                        i32_ptr(table, table.numel(), "table"),
                        (int)table.size(1), seg_view(seg), (int)max_len,
                        (int)out.size(1), rpad, f32, cur_stream());
-}
-
-void gated_act(torch::Tensor out, torch::Tensor gate, torch::Tensor up,
-               int64_t act) {
-  const int f32 = row_type(out, "out");
-  const Rows o = rows_of(out, f32, "out"), g = rows_of(gate, f32, "gate"),
-             u = rows_of(up, f32, "up");
-  TORCH_CHECK(o.n == g.n && o.n == u.n && o.cols == g.cols &&
-                  o.cols == u.cols && g.ld == u.ld && o.n < 65536,
-              "gated_act: sizes");
-  TORCH_CHECK(act == 0 || act == 1, "gated_act: act");
-  launch_gated_act(o.p, o.ld, g.p, u.p, g.ld, o.n, o.cols, (int)act, f32,
-                   cur_stream());
 }
 
 struct Parts {
@@ -533,23 +561,26 @@ void head_attn(torch::Tensor out, torch::Tensor q, torch::Tensor kv,
   TORCH_CHECK(rc == 0, "head_attn: unsupported sizes ", dim, ", ", vdim);
 }
 
-struct Experts {
-  MoePlan p;
-  int n, f32;
-};
+void check_tile_rows(int64_t tile_rows, int f32, int64_t k) {
+  TORCH_CHECK(tile_rows == 16 || (tile_rows == 128 && !f32 && k % 64 == 0),
+              "expert tiles: 16 rows, or 128 in bf16 with k a multiple of 64");
+}
 
 // the plan that moe_route made for n rows
-Experts experts_of(const torch::Tensor& w, const torch::Tensor& plan,
-                   int64_t pairs, int64_t top, int f32) {
+MoePlan plan_of(const torch::Tensor& w, const torch::Tensor& plan,
+                int64_t pairs, int64_t top, int64_t tile_rows, int f32) {
   TORCH_CHECK(top > 0 && pairs % top == 0 && pairs > 0, "expert rows");
-  const int n = (int)(pairs / top), e = (int)w.size(0);
-  const int* p = i32_ptr(plan, moe_plan_ints(n, (int)top, e), "plan");
-  return Experts{
-      moe_plan(const_cast<int*>(p), n, (int)top, e, f32 ? 0 : 1), n, f32};
+  check_tile_rows(tile_rows, f32, w.size(2));
+  const int n = (int)(pairs / top), e = (int)w.size(0), t = (int)tile_rows;
+  const int64_t ints = moe_plan_ints(n, (int)top, e, t);
+  TORCH_CHECK(plan.numel() == ints, "plan of another shape");
+  return moe_plan(const_cast<int*>(i32_ptr(plan, ints, "plan")), n, (int)top,
+                  e, t);
 }
 
 torch::Tensor moe_route(torch::Tensor weight, torch::Tensor x,
-                        torch::Tensor router, int64_t top) {
+                        torch::Tensor router, int64_t top,
+                        int64_t tile_rows) {
   const int f32 = act_type(x, "x");
   check_like(router, f32, "router");
   TORCH_CHECK(x.dim() == 2 && router.dim() == 2 &&
@@ -559,19 +590,21 @@ torch::Tensor moe_route(torch::Tensor weight, torch::Tensor x,
   TORCH_CHECK(n > 0 && e <= 256 && top >= 1 && top <= e && top <= 64,
               "moe_route: at most 256 experts, 64 of them for a token");
   float* wp = const_cast<float*>(f32_ptr(weight, n * top, "weight"));
-  torch::Tensor plan = torch::empty({moe_plan_ints(n, (int)top, e)},
-                                    x.options().dtype(torch::kInt32));
+  check_tile_rows(tile_rows, f32, x.size(1));
+  torch::Tensor plan =
+      torch::empty({moe_plan_ints(n, (int)top, e, (int)tile_rows)},
+                   x.options().dtype(torch::kInt32));
   torch::Tensor z =
       torch::empty({n, e}, x.options().dtype(torch::kFloat32));
   launch_moe_route(wp, z.data_ptr<float>(), x.data_ptr(), router.data_ptr(),
                    moe_plan(plan.data_ptr<int>(), n, (int)top, e,
-                            f32 ? 0 : 1),
+                            (int)tile_rows),
                    n, (int)x.size(1), f32, cur_stream());
   return plan;
 }
 
 void moe_up(torch::Tensor mid, torch::Tensor x, torch::Tensor w,
-            torch::Tensor plan, int64_t act) {
+            torch::Tensor plan, int64_t act, int64_t tile_rows) {
   const int f32 = act_type(x, "x");
   check_like(mid, f32, "mid");
   check_like(w, f32, "w");
@@ -580,15 +613,21 @@ void moe_up(torch::Tensor mid, torch::Tensor x, torch::Tensor w,
                   mid.size(0) % x.size(0) == 0,
               "moe_up: sizes");
   TORCH_CHECK(act == 0 || act == 1, "moe_up: act");
-  const Experts e = experts_of(w, plan, mid.size(0),
-                               mid.size(0) / x.size(0), f32);
-  launch_moe_up(mid.data_ptr(), x.data_ptr(), w.data_ptr(), e.p,
+  // (the large tiles have 32-bit byte offsets)
+  TORCH_CHECK(tile_rows == 16 || (mid.size(1) % 4 == 0 &&
+                                  mid.size(1) >= 128 &&
+                                  x.numel() < (1LL << 30) &&
+                                  128 * x.size(1) < (1LL << 30)),
+              "moe_up: columns");
+  const MoePlan p = plan_of(w, plan, mid.size(0), mid.size(0) / x.size(0),
+                            tile_rows, f32);
+  launch_moe_up(mid.data_ptr(), x.data_ptr(), w.data_ptr(), p,
                 (int)mid.size(1), (int)x.size(1), (int)act, f32,
                 cur_stream());
 }
 
 void moe_down(torch::Tensor out, torch::Tensor mid, torch::Tensor w,
-              torch::Tensor plan) {
+              torch::Tensor plan, int64_t tile_rows) {
   const int f32 = act_type(mid, "mid");
   check_like(out, f32, "out");
   check_like(w, f32, "w");
@@ -596,8 +635,13 @@ void moe_down(torch::Tensor out, torch::Tensor mid, torch::Tensor w,
                   w.size(1) == out.size(2) && w.size(2) == mid.size(1) &&
                   mid.size(0) == out.size(0) * out.size(1),
               "moe_down: sizes");
-  const Experts e = experts_of(w, plan, mid.size(0), out.size(1), f32);
-  launch_moe_down(out.data_ptr(), mid.data_ptr(), w.data_ptr(), e.p,
+  TORCH_CHECK(tile_rows == 16 || (out.size(2) % 4 == 0 &&
+                                  out.size(2) >= 256 &&
+                                  mid.numel() < (1LL << 30)),
+              "moe_down: columns");
+  const MoePlan p =
+      plan_of(w, plan, mid.size(0), out.size(1), tile_rows, f32);
+  launch_moe_down(out.data_ptr(), mid.data_ptr(), w.data_ptr(), p,
                   (int)out.size(2), (int)mid.size(1), f32, cur_stream());
 }
 
@@ -663,11 +707,13 @@ void bind_hybrid(py::module_& m) {
         py::arg("scale"), py::arg("splits"), py::arg("part_o") = none,
         py::arg("part_ml") = none);
   m.def("latent_norm_append", &latent_norm_append,
-        "norms of the query and key/value latents + paged cache append",
+        "norms of the query and key/value latents + paged cache append, and "
+        "a gated activation in the same launch",
         py::arg("pages"), py::arg("kv"), py::arg("kv_w"),
         py::arg("row_slot"), py::arg("row_pos"), py::arg("table"),
         py::arg("eps"), py::arg("q_out") = none, py::arg("q") = none,
-        py::arg("q_w") = none);
+        py::arg("q_w") = none, py::arg("act_out") = none,
+        py::arg("gate") = none, py::arg("up") = none, py::arg("act") = 0);
   m.def("latent_gather", &latent_gather, "cached latents as flat rows",
         py::arg("out"), py::arg("pages"), py::arg("table"), py::arg("seg"),
         py::arg("max_len"));
@@ -691,12 +737,14 @@ void bind_hybrid(py::module_& m) {
         py::arg("gate") = none);
   m.def("moe_route", &moe_route,
         "float router, top experts, pairs ordered by expert",
-        py::arg("weight"), py::arg("x"), py::arg("router"), py::arg("top"));
+        py::arg("weight"), py::arg("x"), py::arg("router"), py::arg("top"),
+        py::arg("tile_rows") = 16);
   m.def("moe_up", &moe_up, "experts' gate and up products + activation",
         py::arg("mid"), py::arg("x"), py::arg("w"), py::arg("plan"),
-        py::arg("act"));
+        py::arg("act"), py::arg("tile_rows") = 16);
   m.def("moe_down", &moe_down, "experts' down products", py::arg("out"),
-        py::arg("mid"), py::arg("w"), py::arg("plan"));
+        py::arg("mid"), py::arg("w"), py::arg("plan"),
+        py::arg("tile_rows") = 16);
   m.def("skinny_gemm", &skinny_gemm, "projection of up to 32 rows",
         py::arg("out"), py::arg("w"), py::arg("x"), py::arg("act") = false,
         py::arg("act_p") = 0.0, py::arg("act_q") = 0.0);

@@ -40,6 +40,22 @@ DEVINL float row16_sum(float v) {
   return v;
 }
 
+// maximum over the wave, in every lane
+DEVINL float wave_max(float v) {
+#define ROR_MAX(n)                                                         \
+  v = fmaxf(v, __int_as_float(__builtin_amdgcn_update_dpp(                 \
+                   0, __float_as_int(v), 0x120 + n, 0xf, 0xf, false)))
+  ROR_MAX(8);
+  ROR_MAX(4);
+  ROR_MAX(2);
+  ROR_MAX(1);
+#undef ROR_MAX
+  auto lane = [&](int l) {
+    return __int_as_float(__builtin_amdgcn_readlane(__float_as_int(v), l));
+  };
+  return fmaxf(fmaxf(lane(0), lane(16)), fmaxf(lane(32), lane(48)));
+}
+
 // Order of one kv head's 64 keys in a page.  A page is made of 16 x 32 blocks
 // (K: keys x channels, V: columns x keys), each in the order in which a
 // wave's lanes hold it as an MFMA operand: lane (quad, row) has steps

@@ -130,27 +130,34 @@ int launch_latent_attn_f32(const RowAttnArgs& a, hipStream_t stream);
 int launch_head_attn_bf16(const RowAttnArgs& a, hipStream_t stream);
 int launch_head_attn_f32(const RowAttnArgs& a, hipStream_t stream);
 
-// Norms of a row's two latents: q [n, q_rank] (rows q_ld apart) to q_out, kv
-// [n, rank] to its place in the pages [P, 64, rpad].  Either may be null;
-// kv_w null: kv is stored as it is.
-void launch_latent_norm_append(void* q_out, const void* q, const float* q_w,
-                               void* pages, const void* kv,
-                               const float* kv_w, const int* row_slot,
-                               const int* row_pos, const int* table,
-                               int table_stride, int n, int q_rank,
-                               long long q_ld, int rank, long long kv_ld,
-                               int rpad, float eps, int f32,
-                               hipStream_t stream);
+// What follows the first product of a parallel block; any part may be absent
+// (null, with its sizes 0).  Norms of a row's two latents: q [n, q_rank] to
+// q_out, kv [n, rank] to its place in the pages [P, 64, rpad] (kv_w null: as
+// it is).  out = act(gate) * up over [n, cols]; act 0 silu, 1 tanh-gelu.
+struct BranchArgs {
+  void* q_out;
+  const void* q;
+  const float* q_w;
+  void* pages;
+  const void* kv;
+  const float* kv_w;
+  const int* row_slot;
+  const int* row_pos;
+  const int* table;
+  void* out;
+  const void* gate;
+  const void* up;
+  long long q_ld, kv_ld, in_ld, out_ld;
+  int n, table_stride, q_rank, rank, rpad, cols, act;
+  float eps;
+};
+
+void launch_branch(const BranchArgs& a, int f32, hipStream_t stream);
 
 // out[start[s] + t, :rank] = the cached row of position pos0[s] + t
 void launch_latent_gather(void* out, const void* pages, const int* table,
                           int table_stride, SegView seg, int max_len,
                           int rank, int rpad, int f32, hipStream_t stream);
-
-// out = act(gate) * up over [n, cols] views; act 0 silu, 1 tanh-gelu
-void launch_gated_act(void* out, long long out_ld, const void* gate,
-                      const void* up, long long in_ld, int n, int cols,
-                      int act, int f32, hipStream_t stream);
 
 // Per-head product out[r, h*m ..] = w[h] x[r, h*xk ..] with w [H, m, k], k a
 // multiple of 32 and xk <= k.  x_rows / out_rows map the n rows (null: as
@@ -173,19 +180,26 @@ void launch_head_proj(const HeadProjArgs& a, int f32, hipStream_t stream);
 
 // Routing.  plan is one int buffer:
 //   chosen experts [n*top] | pairs ordered by expert [n*top] | number of
-//   tiles | tiles [max_tiles][3] = expert, first place in the order, rows
+//   tiles | tiles
 // where pair p is choice p % top of row p / top and a tile is up to
 // tile_rows pairs of one expert.
+struct MoeTile {
+  int expert, first, rows;  // pairs order[first] .. order[first + rows - 1]
+  int tile0, n_tiles;       // the expert's tiles
+};
+
 struct MoePlan {
   int* chosen;
   int* order;
   int* n_tiles;
-  int* tiles;
+  MoeTile* tiles;
   int pairs, top, experts, tile_rows, max_tiles;
 };
 
-MoePlan moe_plan(int* buffer, int n, int top, int experts, int bf16_large);
-long long moe_plan_ints(int n, int top, int experts);
+// tile_rows: 16, or 128 (bf16, contractions multiples of 64, at least 128
+// expert and 256 model channels)
+MoePlan moe_plan(int* buffer, int n, int top, int experts, int tile_rows);
+long long moe_plan_ints(int n, int top, int experts, int tile_rows);
 
 // z [n, experts] = x router^T in float; weight [n, top] = softmax over the
 // top logits.

@@ -6,8 +6,9 @@
 namespace {
 
 // ---------------------------------------------------------------------------
-// Norms of a row's query and key/value latents; the latter goes to its place
-// in the cache.  One wave per (row, latent).
+// What follows the first product of a parallel block, in one launch: norms of
+// a row's query and key/value latents (the latter goes to its place in the
+// cache), one wave per (row, latent), and the gated activation.
 // ---------------------------------------------------------------------------
 template <typename T, int V>
 DEVINL void wave_norm(T* dst, const T* src, const float* w, int n, float eps,
@@ -34,26 +35,42 @@ DEVINL void wave_norm(T* dst, const T* src, const float* w, int n, float eps,
 }
 
 template <typename T, int V>
-__global__ __launch_bounds__(256) void latent_norm_append_kernel(
-    T* __restrict__ q_out, const T* __restrict__ q,
-    const float* __restrict__ q_w, T* __restrict__ pages,
-    const T* __restrict__ kv, const float* __restrict__ kv_w,
-    const int* __restrict__ row_slot, const int* __restrict__ row_pos,
-    const int* __restrict__ table, int table_stride, int n, int q_rank,
-    long long q_ld, int rank, long long kv_ld, int rpad, float eps) {
-  const int lane = threadIdx.x & 63;
-  const size_t row = (size_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (row >= n) return;
+DEVINL void act_row(const BranchArgs& a, size_t row, int i) {
+  using P = Pack<T, V>;
+  if (i >= a.cols) return;
+  const P g = *reinterpret_cast<const P*>((const T*)a.gate + row * a.in_ld + i);
+  const P u = *reinterpret_cast<const P*>((const T*)a.up + row * a.in_ld + i);
+  P o;
+#pragma unroll
+  for (int j = 0; j < V; ++j)
+    o.v[j] = from_f<T>(gated(to_f(g.v[j]), to_f(u.v[j]), a.act));
+  *reinterpret_cast<P*>((T*)a.out + row * a.out_ld + i) = o;
+}
+
+// blockIdx.y: 0 query latents, 1 key/value latents (four rows a block), then
+// the gated activation in blocks of 256 * AV columns of four rows
+template <typename T, int V, int AV>
+__global__ __launch_bounds__(256) void branch_kernel(BranchArgs a) {
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const size_t row = (size_t)blockIdx.x * 4 + wave;
   if (blockIdx.y == 0) {
-    if (q == nullptr) return;
-    wave_norm<T, V>(q_out + row * q_rank, q + row * q_ld, q_w, q_rank, eps,
+    if (row >= a.n || a.q == nullptr) return;
+    wave_norm<T, V>((T*)a.q_out + row * a.q_rank,
+                    (const T*)a.q + row * a.q_ld, a.q_w, a.q_rank, a.eps,
+                    lane);
+  } else if (blockIdx.y == 1) {
+    if (row >= a.n || a.kv == nullptr) return;
+    const int pos = a.row_pos[row];
+    const size_t page =
+        a.table[(size_t)a.row_slot[row] * a.table_stride + (pos >> 6)];
+    wave_norm<T, V>((T*)a.pages + (page * 64 + (pos & 63)) * a.rpad,
+                    (const T*)a.kv + row * a.kv_ld, a.kv_w, a.rank, a.eps,
                     lane);
   } else {
-    const int pos = row_pos[row];
-    const size_t page =
-        table[(size_t)row_slot[row] * table_stride + (pos >> 6)];
-    wave_norm<T, V>(pages + (page * 64 + (pos & 63)) * rpad, kv + row * kv_ld,
-                    kv_w, rank, eps, lane);
+    const int i = ((blockIdx.y - 2) * 256 + threadIdx.x) * AV;
+    for (int r = 0; r < 4; ++r)
+      if ((size_t)blockIdx.x * 4 + r < a.n)
+        act_row<T, AV>(a, (size_t)blockIdx.x * 4 + r, i);
   }
 }
 
@@ -76,24 +93,6 @@ __global__ __launch_bounds__(256) void latent_gather_kernel(
 }
 
 // ---------------------------------------------------------------------------
-template <typename T, int V>
-__global__ __launch_bounds__(256) void gated_act_kernel(
-    T* __restrict__ out, long long out_ld, const T* __restrict__ gate,
-    const T* __restrict__ up, long long in_ld, int cols, int act) {
-  using P = Pack<T, V>;
-  const size_t row = blockIdx.y;
-  const int i = (blockIdx.x * 256 + threadIdx.x) * V;
-  if (i >= cols) return;
-  const P a = *reinterpret_cast<const P*>(gate + row * in_ld + i);
-  const P b = *reinterpret_cast<const P*>(up + row * in_ld + i);
-  P o;
-#pragma unroll
-  for (int j = 0; j < V; ++j)
-    o.v[j] = from_f<T>(gated(to_f(a.v[j]), to_f(b.v[j]), act));
-  *reinterpret_cast<P*>(out + row * out_ld + i) = o;
-}
-
-// ---------------------------------------------------------------------------
 // Per-head products of a few rows.  A block has 16 rows of one head in LDS
 // (merged from the attention's partial results, if it has those) and its four
 // waves take 16 outputs each; the weights are the MFMA's A operand, straight
@@ -112,18 +111,37 @@ __global__ __launch_bounds__(256) void head_proj_kernel(HeadProjArgs a) {
   const int h = blockIdx.y, r0 = blockIdx.z * 16;
   const int ld = a.k + N;
   T* xs = reinterpret_cast<T*>(smem);
+  // the weights set out first: they need nothing of what follows
+  constexpr int PRE = sizeof(T) == 2 ? 16 : 8;
+  const int m0 = blockIdx.x * HEAD_COLS + wave * 16;
+  const T* wp = (const T*)a.w +
+                ((size_t)h * a.m + min(m0 + c, a.m - 1)) * a.k + quad * 8;
+  typename F::Row pre[PRE];
+#pragma unroll
+  for (int i = 0; i < PRE; ++i)
+    if (i * 32 < a.k) pre[i] = F::load_frag(wp + i * 32);
   if (PARTS) {
     float* we = reinterpret_cast<float*>(xs + 16 * ld);  // [16][splits]
+    // parts that saw keys come first; the others have no values
+    __shared__ int live[16];
     // 16 lanes per row
     const int row = tid >> 4, k = tid & 15;
     if (r0 + row < a.n) {
       const size_t cell = ((size_t)(r0 + row) * a.heads + h) * a.splits;
       const float* ml = a.part_ml + cell * 2;
       float mm = -__builtin_huge_valf();
-      for (int s = k; s < a.splits; s += 16) mm = fmaxf(mm, ml[s * 2]);
+      int used = 0;
+      for (int s = k; s < a.splits; s += 16) {
+        const float ms = ml[s * 2];
+        mm = fmaxf(mm, ms);
+        if (ms != -__builtin_huge_valf()) used = s + 1;
+      }
 #pragma unroll
-      for (int off = 8; off > 0; off >>= 1)
+      for (int off = 8; off > 0; off >>= 1) {
         mm = fmaxf(mm, __shfl_xor(mm, off, 64));
+        used = max(used, __shfl_xor(used, off, 64));
+      }
+      if (k == 0) live[row] = used;
       float sum = 0.f;
       for (int s = k; s < a.splits; s += 16)
         sum += __builtin_amdgcn_exp2f(ml[s * 2] - mm) * ml[s * 2 + 1];
@@ -141,7 +159,9 @@ __global__ __launch_bounds__(256) void head_proj_kernel(HeadProjArgs a) {
         const float* po =
             a.part_o +
             ((size_t)(r0 + row) * a.heads + h) * a.splits * a.k + k;
-        for (int s = 0; s < a.splits; ++s) {
+        const int used = live[row];
+#pragma unroll 8
+        for (int s = 0; s < used; ++s) {
           const float e = we[row * a.splits + s];
           const float4 v = *reinterpret_cast<const float4*>(
               po + (size_t)s * a.k);
@@ -178,14 +198,14 @@ __global__ __launch_bounds__(256) void head_proj_kernel(HeadProjArgs a) {
     }
   }
   __syncthreads();
-  const int m0 = blockIdx.x * HEAD_COLS + wave * 16;
   if (m0 >= a.m) return;
-  const T* wp = (const T*)a.w +
-                ((size_t)h * a.m + min(m0 + c, a.m - 1)) * a.k + quad * 8;
   const T* xp = xs + c * ld + quad * 8;
   f32x4 acc{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-  for (int k = 0; k < a.k; k += 32)
+#pragma unroll
+  for (int i = 0; i < PRE; ++i)
+    if (i * 32 < a.k)
+      acc = F::dot(pre[i], F::load_frag(xp + i * 32), acc);
+  for (int k = PRE * 32; k < a.k; k += 32)
     acc = F::dot(F::load_frag(wp + k), F::load_frag(xp + k), acc);
   if (r0 + c >= a.n) return;
   const size_t r = a.out_rows ? a.out_rows[r0 + c] : r0 + c;
@@ -219,32 +239,31 @@ void launch_head_proj(const HeadProjArgs& a, int f32, hipStream_t stream) {
   else head_proj_t<bf16>(a, stream);
 }
 
-void launch_latent_norm_append(void* q_out, const void* q, const float* q_w,
-                               void* pages, const void* kv,
-                               const float* kv_w, const int* row_slot,
-                               const int* row_pos, const int* table,
-                               int table_stride, int n, int q_rank,
-                               long long q_ld, int rank, long long kv_ld,
-                               int rpad, float eps, int f32,
-                               hipStream_t stream) {
-  const dim3 grid((n + 3) / 4, kv != nullptr ? 2 : 1);
-#define APPEND(T, V)                                                       \
-  latent_norm_append_kernel<T, V><<<grid, 256, 0, stream>>>(               \
-      (T*)q_out, (const T*)q, q_w, (T*)pages, (const T*)kv, kv_w,          \
-      row_slot, row_pos, table, table_stride, n, q_rank, q_ld, rank,       \
-      kv_ld, rpad, eps)
-  auto fits = [&](int v, size_t bytes) {
-    return q_rank % v == 0 && q_ld % v == 0 && rank % v == 0 &&
-           kv_ld % v == 0 && (size_t)q % bytes == 0 && (size_t)kv % bytes == 0;
+void launch_branch(const BranchArgs& a, int f32, hipStream_t stream) {
+  auto norms = [&](int v) {
+    return a.q_rank % v == 0 && a.q_ld % v == 0 && a.rank % v == 0 &&
+           a.kv_ld % v == 0 && ((size_t)a.q | (size_t)a.kv) % 16 == 0;
   };
+  auto acts = [&](int v) {
+    return a.cols % v == 0 && a.out_ld % v == 0 && a.in_ld % v == 0 &&
+           ((size_t)a.out | (size_t)a.gate | (size_t)a.up) % 16 == 0;
+  };
+#define BRANCH(T, V, AV)                                                   \
+  branch_kernel<T, V, AV>                                                  \
+      <<<dim3((a.n + 3) / 4, 2 + (a.cols + 256 * AV - 1) / (256 * AV)),    \
+         256, 0, stream>>>(a)
+#define BY_ALIGNMENT(T, V)                   \
+  if (norms(V) && acts(V)) BRANCH(T, V, V);  \
+  else if (norms(V)) BRANCH(T, V, 1);        \
+  else if (acts(V)) BRANCH(T, 1, V);         \
+  else BRANCH(T, 1, 1)
   if (f32) {
-    if (fits(4, 16)) APPEND(float, 4);
-    else APPEND(float, 1);
+    BY_ALIGNMENT(float, 4);
   } else {
-    if (fits(8, 16)) APPEND(bf16, 8);
-    else APPEND(bf16, 1);
+    BY_ALIGNMENT(bf16, 8);
   }
-#undef APPEND
+#undef BY_ALIGNMENT
+#undef BRANCH
 }
 
 void launch_latent_gather(void* out, const void* pages, const int* table,
@@ -262,25 +281,4 @@ void launch_latent_gather(void* out, const void* pages, const int* table,
     else GATHER(bf16, 1);
   }
 #undef GATHER
-}
-
-void launch_gated_act(void* out, long long out_ld, const void* gate,
-                      const void* up, long long in_ld, int n, int cols,
-                      int act, int f32, hipStream_t stream) {
-  auto fits = [&](int v) {
-    return cols % v == 0 && out_ld % v == 0 && in_ld % v == 0 &&
-           ((size_t)out | (size_t)gate | (size_t)up) % 16 == 0;
-  };
-#define ACT(T, V)                                                          \
-  gated_act_kernel<T, V>                                                   \
-      <<<dim3((cols + 256 * V - 1) / (256 * V), n), 256, 0, stream>>>(     \
-          (T*)out, out_ld, (const T*)gate, (const T*)up, in_ld, cols, act)
-  if (f32) {
-    if (fits(4)) ACT(float, 4);
-    else ACT(float, 1);
-  } else {
-    if (fits(8)) ACT(bf16, 8);
-    else ACT(bf16, 1);
-  }
-#undef ACT
 }

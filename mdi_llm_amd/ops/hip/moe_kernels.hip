@@ -30,13 +30,35 @@ template <typename T, int NW, int NM>
 DEVINL void tile_product(float (*red)[NM][16][17], const T* x,
                          const T* const (&w)[NM], int k, bool vec) {
   using F = Frag<T>;
+  constexpr int STRIDE = NW * 64, UNR = NM == 1 ? 4 : 2;
   const int lane = threadIdx.x & 63, c = lane & 15, quad = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   f32x4 acc[NM];
 #pragma unroll
   for (int j = 0; j < NM; ++j) acc[j] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 2
-  for (int at = wave * 64; at < k; at += NW * 64) {
+  int at = wave * 64;
+  // several stretches of the weight stream in flight
+  for (; vec && at + (UNR - 1) * STRIDE + 64 <= k; at += UNR * STRIDE) {
+    typename F::Row wa[UNR][NM], wb[UNR][NM];
+#pragma unroll
+    for (int u = 0; u < UNR; ++u)
+#pragma unroll
+      for (int j = 0; j < NM; ++j) {
+        wa[u][j] = F::load_frag(w[j] + at + u * STRIDE + quad * 16);
+        wb[u][j] = F::load_frag(w[j] + at + u * STRIDE + quad * 16 + 8);
+      }
+#pragma unroll
+    for (int u = 0; u < UNR; ++u) {
+      const auto xa = F::load_frag(x + at + u * STRIDE + quad * 16);
+      const auto xb = F::load_frag(x + at + u * STRIDE + quad * 16 + 8);
+#pragma unroll
+      for (int j = 0; j < NM; ++j) {
+        acc[j] = F::dot(wa[u][j], xa, acc[j]);
+        acc[j] = F::dot(wb[u][j], xb, acc[j]);
+      }
+    }
+  }
+  for (; at < k; at += STRIDE) {
     const int s = at + quad * 16;
     const auto xa = load_steps<T>(x, s, k, vec);
     const auto xb = load_steps<T>(x, s + 8, k, vec);
@@ -90,24 +112,16 @@ DEVINL void choose(float* weight, int* chosen, const float* z, int experts,
   }
   float zmax = 0.f, sum = 0.f, mine = 0.f;
   for (int t = 0; t < top; ++t) {
-    float best = -__builtin_huge_valf();
-    int at = MAX_EXPERTS;
+    float best = v[0];
 #pragma unroll
-    for (int j = 0; j < MAX_EXPERTS / 64; ++j)
-      if (v[j] > best) {
-        best = v[j];
-        at = j * 64 + lane;
-      }
+    for (int j = 1; j < MAX_EXPERTS / 64; ++j) best = fmaxf(best, v[j]);
+    best = wave_max(best);
+    int at = experts - 1;  // kept only if a logit is not a number
 #pragma unroll
-    for (int off = 32; off > 0; off >>= 1) {
-      const float ov = __shfl_xor(best, off, 64);
-      const int oa = __shfl_xor(at, off, 64);
-      if (ov > best || (ov == best && oa < at)) {
-        best = ov;
-        at = oa;
-      }
+    for (int j = MAX_EXPERTS / 64 - 1; j >= 0; --j) {
+      const unsigned long long hit = __ballot(v[j] == best);
+      if (hit != 0) at = min(j * 64 + __ffsll(hit) - 1, experts - 1);
     }
-    at = min(at, experts - 1);  // only if a logit is not a number
     if (t == 0) zmax = best;
     const float e = expf(best - zmax);
     sum += e;
@@ -148,17 +162,18 @@ __global__ __launch_bounds__(1024) void order_kernel(
   for (int i = tid; i < p.pairs; i += 1024) atomicAdd(&count[p.chosen[i]], 1);
   __syncthreads();
   if (tid < p.experts) {
+    const int shift = 31 - __clz(p.tile_rows);  // a power of two
     int first = 0, tile = 0;
     for (int e = 0; e < tid; ++e) {
       first += count[e];
-      tile += (count[e] + p.tile_rows - 1) / p.tile_rows;
+      tile += (count[e] + p.tile_rows - 1) >> shift;
     }
     next[tid] = first;
-    for (int at = 0; at < count[tid]; at += p.tile_rows, ++tile) {
-      p.tiles[tile * 3] = tid;
-      p.tiles[tile * 3 + 1] = first + at;
-      p.tiles[tile * 3 + 2] = min(p.tile_rows, count[tid] - at);
-    }
+    const int tile0 = tile, n_tiles = (count[tid] + p.tile_rows - 1) >> shift;
+    for (int at = 0; at < count[tid]; at += p.tile_rows, ++tile)
+      p.tiles[tile] = MoeTile{tid, first + at,
+                              min(p.tile_rows, count[tid] - at), tile0,
+                              n_tiles};
     if (tid == p.experts - 1) *p.n_tiles = tile;
   }
   __syncthreads();
@@ -177,8 +192,8 @@ __global__ __launch_bounds__(NW * 64) void expert_rows_kernel(
   __shared__ float red[NW][NM][16][17];
   const int tile = blockIdx.y;
   if (tile >= *p.n_tiles) return;
-  const int e = p.tiles[tile * 3], first = p.tiles[tile * 3 + 1];
-  const int rows = p.tiles[tile * 3 + 2];
+  const int e = p.tiles[tile].expert, first = p.tiles[tile].first;
+  const int rows = p.tiles[tile].rows;
   const int c = threadIdx.x & 15, m0 = blockIdx.x * 16;
   const int pair = p.order[first + min(c, rows - 1)];
   const T* xp = x + (size_t)(UP ? pair / p.top : pair) * k;
@@ -204,33 +219,176 @@ void expert_rows_t(void* out, const void* x, const void* w, MoePlan p, int m,
 #define EXPERT(NW)                                                      \
   expert_rows_kernel<T, NW, UP><<<grid, NW * 64, 0, stream>>>(          \
       (T*)out, (const T*)x, (const T*)w, p, m, k, act, vec)
-  if (k >= 2048) EXPERT(16);
+  if (k >= 2048) EXPERT(8);
   else EXPERT(4);
 #undef EXPERT
 }
 
+// ---------------------------------------------------------------------------
+// Products of up to 128 pairs of one expert with 256 weight rows, bf16, k a
+// multiple of 64.  Four waves hold 64 pairs x 128 outputs each; two blocks
+// fit a CU, and one computes while the other stores its next tile.  That tile
+// travels through registers during the MFMAs.  16-byte chunks of an LDS row
+// are permuted by the row so that both the stores and the operand loads
+// spread over the banks.  UP: half of the weight rows are an expert's gate
+// rows, half the up rows of the same outputs.
+// ---------------------------------------------------------------------------
+constexpr int BIG_ROWS = 128, BIG_COLS = 256, BIG_K = 64;
+
+template <bool UP>
+__global__ __launch_bounds__(256, 2) void expert_tiles_kernel(
+    bf16* __restrict__ out, const bf16* __restrict__ x,
+    const bf16* __restrict__ w, MoePlan p, int m, int k, int m_tiles,
+    int act) {
+  constexpr int MT = UP ? BIG_COLS / 2 : BIG_COLS;  // outputs of a block
+  constexpr int XI = BIG_ROWS / 32, WI = BIG_COLS / 32;
+  extern __shared__ __attribute__((aligned(16))) bf16 sm[];
+  // an XCD's blocks are neighbours in the list of (weight tile, pair tile)
+  const int total = *p.n_tiles * m_tiles, per = (total + 7) / 8;
+  const int at = blockIdx.x / 8, unit = (blockIdx.x % 8) * per + at;
+  if (at >= per || unit >= total) return;
+  const MoeTile head = p.tiles[unit / m_tiles];
+  const int u = unit - head.tile0 * m_tiles;
+  const MoeTile tile = p.tiles[head.tile0 + u % head.n_tiles];
+  // the last tile of outputs may overlap the one before
+  const int m0 = min(u / head.n_tiles * MT, m - MT);
+
+  const int tid = threadIdx.x, lane = tid & 63;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int c = lane & 15, quad = lane >> 4;
+  const int wr = wave >> 1, wc = wave & 1;
+  // rows of a thread's chunks: r0, r0 + 32, ..
+  const int r0 = tid >> 3, ch = tid & 7;
+  // byte offsets in 32 bits; the weight rows of a thread are 32 apart
+  const char* xb = reinterpret_cast<const char*>(x);
+  unsigned xo[XI];
+#pragma unroll
+  for (int i = 0; i < XI; ++i) {
+    // rows past the end repeat the last one; they are never stored
+    const int pair =
+        p.order[tile.first + min(i * 32 + r0, tile.rows - 1)];
+    xo[i] = ((unsigned)(UP ? pair / p.top : pair) * k + ch * 8) * 2;
+  }
+  const char* wb = reinterpret_cast<const char*>(
+      w + ((size_t)tile.expert * (UP ? 2 : 1) * m + m0) * k);
+  const unsigned wo = ((unsigned)r0 * k + ch * 8) * 2;
+  // up rows lie m after the gate rows of the same outputs
+  auto wskip = [&](int i) {
+    return (size_t)(UP && i * 32 >= MT ? m + i * 32 - MT : i * 32) * k * 2;
+  };
+  const int put = r0 * BIG_K + ((ch ^ (r0 & 7)) << 3);
+  bf16x8 xr[XI], wreg[WI];
+  auto load = [&](int k0) {
+#pragma unroll
+    for (int i = 0; i < XI; ++i)
+      xr[i] = *reinterpret_cast<const bf16x8*>(xb + (xo[i] + k0 * 2));
+#pragma unroll
+    for (int i = 0; i < WI; ++i)
+      wreg[i] = *reinterpret_cast<const bf16x8*>(wb + wskip(i) + (wo + k0 * 2));
+  };
+  auto store = [&](bf16* b) {
+#pragma unroll
+    for (int i = 0; i < XI; ++i)
+      *reinterpret_cast<bf16x8*>(b + i * 32 * BIG_K + put) = xr[i];
+#pragma unroll
+    for (int i = 0; i < WI; ++i)
+      *reinterpret_cast<bf16x8*>(b + (BIG_ROWS + i * 32) * BIG_K + put) =
+          wreg[i];
+  };
+  // first LDS row of this wave's j-th 16 weight rows
+  auto wrow = [&](int j) {
+    return BIG_ROWS + (UP ? (j / 4) * MT + wc * 64 + (j % 4) * 16
+                          : wc * 128 + j * 16);
+  };
+  f32x4 acc[4][8];
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+#pragma unroll
+    for (int j = 0; j < 8; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+
+  const int steps = k / BIG_K;
+  load(0);
+  for (int s = 0; s < steps; ++s) {
+    if (s) __syncthreads();
+    store(sm);
+    if (s + 1 < steps) load((s + 1) * BIG_K);
+    __syncthreads();
+#pragma unroll
+    for (int kk = 0; kk < 2; ++kk) {
+      const int chunk = ((kk * 4 + quad) ^ (c & 7)) << 3;
+      bf16x8 xf[4], wf[8];
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        xf[i] = *reinterpret_cast<const bf16x8*>(
+            sm + (wr * 64 + i * 16 + c) * BIG_K + chunk);
+#pragma unroll
+      for (int j = 0; j < 8; ++j)
+        wf[j] = *reinterpret_cast<const bf16x8*>(
+            sm + (wrow(j) + c) * BIG_K + chunk);
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 8; ++j)
+          acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+              wf[j], xf[i], acc[i][j], 0, 0, 0);
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int row = wr * 64 + i * 16 + c;
+    if (row >= tile.rows) continue;
+    bf16* o = out + (size_t)p.order[tile.first + row] * m;
+#pragma unroll
+    for (int j = 0; j < (UP ? 4 : 8); ++j) {
+      const int col = m0 + (UP ? wc * 64 : wc * 128) + j * 16 + quad * 4;
+      Pack<bf16, 4> v;
+#pragma unroll
+      for (int q = 0; q < 4; ++q)
+        v.v[q] = from_f<bf16>(UP ? gated(acc[i][j][q], acc[i][(j + 4) % 8][q], act)
+                                 : acc[i][j][q]);
+      // m is a multiple of 4
+      if (col < m) *reinterpret_cast<Pack<bf16, 4>*>(o + col) = v;
+    }
+  }
+}
+
+template <bool UP>
+void expert_tiles(void* out, const void* x, const void* w, MoePlan p, int m,
+                  int k, int act, hipStream_t stream) {
+  constexpr size_t smem = (BIG_ROWS + BIG_COLS) * BIG_K * sizeof(bf16);
+  const int m_tiles = (m + (UP ? BIG_COLS / 2 : BIG_COLS) - 1) /
+                      (UP ? BIG_COLS / 2 : BIG_COLS);
+  const long long units = (long long)p.max_tiles * m_tiles;
+  auto kernel = expert_tiles_kernel<UP>;
+  (void)hipFuncSetAttribute((const void*)kernel,
+                            hipFuncAttributeMaxDynamicSharedMemorySize,
+                            (int)smem);
+  kernel<<<(unsigned)((units + 7) / 8 * 8), 256, smem, stream>>>(
+      (bf16*)out, (const bf16*)x, (const bf16*)w, p, m, k, m_tiles, act);
+}
+
 }  // namespace
 
-MoePlan moe_plan(int* buffer, int n, int top, int experts, int bf16_large) {
+MoePlan moe_plan(int* buffer, int n, int top, int experts, int tile_rows) {
   MoePlan p;
   p.pairs = n * top;
   p.top = top;
   p.experts = experts;
-  p.tile_rows = 16;
-  (void)bf16_large;
+  p.tile_rows = tile_rows;
   // every expert's last tile may be short
   const long long tiles = p.pairs / p.tile_rows + experts;
   p.max_tiles = (int)(tiles < p.pairs ? tiles : p.pairs);
   p.chosen = buffer;
   p.order = p.chosen + p.pairs;
   p.n_tiles = p.order + p.pairs;
-  p.tiles = p.n_tiles + 1;
+  p.tiles = reinterpret_cast<MoeTile*>(p.n_tiles + 1);
   return p;
 }
 
-long long moe_plan_ints(int n, int top, int experts) {
+long long moe_plan_ints(int n, int top, int experts, int tile_rows) {
   const long long pairs = (long long)n * top;
-  return 2 * pairs + 1 + 3 * (pairs / 16 + experts);
+  return 2 * pairs + 1 +
+         (pairs / tile_rows + experts) * (sizeof(MoeTile) / sizeof(int));
 }
 
 void launch_moe_route(float* weight, float* z, const void* x,
@@ -251,12 +409,16 @@ void launch_moe_route(float* weight, float* z, const void* x,
 
 void launch_moe_up(void* mid, const void* x, const void* w, MoePlan p,
                    int ff, int k, int act, int f32, hipStream_t stream) {
-  if (f32) expert_rows_t<float, true>(mid, x, w, p, ff, k, act, stream);
+  if (p.tile_rows == BIG_ROWS)
+    expert_tiles<true>(mid, x, w, p, ff, k, act, stream);
+  else if (f32) expert_rows_t<float, true>(mid, x, w, p, ff, k, act, stream);
   else expert_rows_t<bf16, true>(mid, x, w, p, ff, k, act, stream);
 }
 
 void launch_moe_down(void* out, const void* mid, const void* w, MoePlan p,
                      int m, int ff, int f32, hipStream_t stream) {
-  if (f32) expert_rows_t<float, false>(out, mid, w, p, m, ff, 0, stream);
+  if (p.tile_rows == BIG_ROWS)
+    expert_tiles<false>(out, mid, w, p, m, ff, 0, stream);
+  else if (f32) expert_rows_t<float, false>(out, mid, w, p, m, ff, 0, stream);
   else expert_rows_t<bf16, false>(out, mid, w, p, m, ff, 0, stream);
 }

@@ -122,7 +122,10 @@ def _rows(pages, table, slot, first, end, n_cols):
 
 
 def latent_norm_append(pages, kv, kv_w, row_slot, row_pos, table, eps,
-                       q_out=None, q=None, q_w=None) -> None:
+                       q_out=None, q=None, q_w=None, act_out=None, gate=None,
+                       up=None, act=0) -> None:
+    if act_out is not None:
+        gated_act(act_out, gate, up, act)
     if q is not None:
         q_out.copy_(_rms(q, eps) * q_w)
     if kv is None:
@@ -212,7 +215,7 @@ def gated_act(out, gate, up, act) -> None:
     out.copy_(_act(gate.float(), act) * up.float())
 
 
-def moe_route(weight, x, router, top):
+def moe_route(weight, x, router, top, tile_rows=16):
     """Fills the weights [n, top]; returns the plan of the expert products
     (here: the chosen experts [n, top])."""
     z, experts = (x.float() @ router.float().t()).topk(top, -1)
@@ -220,7 +223,7 @@ def moe_route(weight, x, router, top):
     return experts
 
 
-def moe_up(out, x, w, plan, act) -> None:
+def moe_up(out, x, w, plan, act, tile_rows=16) -> None:
     n, top = plan.shape
     for t in range(n):
         for k in range(top):
@@ -228,7 +231,7 @@ def moe_up(out, x, w, plan, act) -> None:
             out[t * top + k] = (_act(gate, act) * up).to(out.dtype)
 
 
-def moe_down(out, mid, w, plan) -> None:
+def moe_down(out, mid, w, plan, tile_rows=16) -> None:
     n, top = plan.shape
     for t in range(n):
         for k in range(top):

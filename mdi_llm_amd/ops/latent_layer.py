@@ -31,6 +31,7 @@ __all__ = ["LatentPlan", "ParallelLayer", "ACTS"]
 
 ACTS = {"silu": 0, "gelu_tanh": 1}
 MAX_EXPANDED = 256      # head sizes of the expanded form
+BIG_TILE = 128          # pairs of one expert in a tile of large batches
 
 
 def _round_up(n: int, k: int) -> int:
@@ -147,6 +148,10 @@ class ParallelLayer:
                 mlp.experts, 2 * mlp.expert_ff, -1)
             self.e_down = mlp.down.weight.detach().view(
                 mlp.experts, -1, mlp.expert_ff)
+            width = self.router.size(1)
+            self.big_tiles = eng.dtype == torch.bfloat16 \
+                and mlp.expert_ff % 64 == 0 and mlp.expert_ff >= 128 \
+                and width % 64 == 0 and width >= 256
 
     # ------------------------------------------------------------------
     def _new(self, *shape, dtype=None) -> torch.Tensor:
@@ -156,18 +161,22 @@ class ParallelLayer:
     def step(self, b, xn: torch.Tensor):
         """The block's sum before the residual multiplier, and the routed
         experts' rows with their weights (None without experts)."""
-        m, ops = self.mixer, self.eng.ops
+        m = self.mixer
         proj = self.eng._linear(xn, self.in_proj)
         y = self._new(b.n, m.out_cols + self.ff)
+        branch = {}
         if self.ff:
-            ops.gated_act(y[:, m.out_cols:], proj[:, self.gate],
-                          proj[:, self.up], self.act)
-        self._attend(b, proj, y[:, :m.out_cols])
+            branch = dict(act_out=y[:, m.out_cols:], gate=proj[:, self.gate],
+                          up=proj[:, self.up], act=self.act)
+        self._attend(b, proj, y[:, :m.out_cols], branch)
         routed = self._experts(b, xn) if self.routed else None
         return self.eng._linear(y, self.out_proj), routed
 
     # -- attention ------------------------------------------------------
-    def _attend(self, b, proj: torch.Tensor, y: torch.Tensor) -> None:
+    def _attend(self, b, proj: torch.Tensor, y: torch.Tensor,
+                branch: dict) -> None:
+        """``branch``: the feed-forward's activation, which shares a launch
+        with the latents' norms."""
         m, e = self.mixer, self.eng
         c, eps = e.cache, e.config.norm_eps
         pages = c.latent[m.source]
@@ -175,7 +184,7 @@ class ParallelLayer:
         kv = proj[:, self.part["dkv"]] if m.owns_latent else None
         e.ops.latent_norm_append(
             pages, kv, self.kv_norm, b.row_slot, b.row_pos, c.table, eps,
-            q_out=cq, q=proj[:, self.part["dq"]], q_w=self.q_norm)
+            q_out=cq, q=proj[:, self.part["dq"]], q_w=self.q_norm, **branch)
         q = e._linear(cq, self.q_up)
         gate = proj[:, self.part["g"]]
         plan = b.latent_plan(m, e.device, e.latent_form)
@@ -191,7 +200,7 @@ class ParallelLayer:
         pages = min(-(-max_ctx // PAGE), (m.window + plan.max_len - 2) // PAGE
                     + 2)
         blocks = plan.seg.size(1) * -(-plan.max_len * m.heads // 64)
-        return max(1, min(-(-512 // blocks), pages, 256))
+        return max(1, min(-(-256 // blocks), pages, 256))
 
     def _absorbed(self, b, plan, q, gate, y, pages) -> None:
         m, e, R = self.mixer, self.eng, self.rpad
@@ -227,10 +236,14 @@ class ParallelLayer:
     # -- experts --------------------------------------------------------
     def _experts(self, b, xn: torch.Tensor):
         ops, n, F = self.eng.ops, b.n, self.expert_ff
+        # pairs (row, choice) per expert decide the tile
+        tile = BIG_TILE if self.big_tiles and \
+            n * self.top >= BIG_TILE // 2 * self.experts and \
+            n * max(xn.size(1), self.top * F) < 1 << 30 else 16
         weight = self._new(n, self.top, dtype=torch.float32)
-        plan = ops.moe_route(weight, xn, self.router, self.top)
+        plan = ops.moe_route(weight, xn, self.router, self.top, tile)
         mid = self._new(n * self.top, F)
-        ops.moe_up(mid, xn, self.e_up, plan, self.act)
+        ops.moe_up(mid, xn, self.e_up, plan, self.act, tile)
         out = self._new(n, self.top, xn.size(1))
-        ops.moe_down(out, mid, self.e_down, plan)
+        ops.moe_down(out, mid, self.e_down, plan, tile)
         return out, weight

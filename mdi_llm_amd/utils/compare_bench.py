@@ -16,10 +16,12 @@ from ..parallel.runner import make_runner
 
 __all__ = ["PAIRS", "compare"]
 
-# hybrid -> existing model of equal width, depth and weight count
+# hybrid -> existing model of equal width, depth and weights per token
 PAIRS = {
     "nerozen-1b": "tiny-llama-1.1b-chat",
     "nerozen-8b": "Meta-Llama-3-8B-Instruct",
+    "resolorn-1b": "tiny-llama-1.1b-chat",
+    "resolorn-8b": "Meta-Llama-3-8B-Instruct",
 }
 SAMPLING = dict(temperature=0.8, top_k=200, seed=1234)
 
@@ -35,6 +37,11 @@ def _stage(cfg: ModelConfig, device, max_seq: int) -> StarterStage:
             p.normal_(0.0, 0.02)
     stage.max_seq_length = min(max_seq, cfg.block_size)
     return stage.eval()
+
+
+def _weights(cfg: ModelConfig) -> int:
+    """Matrix weights that one token uses."""
+    return sum(cfg.layer_weights(i, active=True) for i in range(cfg.n_layer))
 
 
 def _timed(run: Callable[[], None], n: int) -> float:
@@ -55,7 +62,7 @@ def _hybrid(cfg, device, prompt: int, batch: int, steps: int) -> dict:
     r = make_runner(stage, batch, device,
                     n_tokens=max(max_seq, batch * (short + 4 * steps)) + 4096)
     eng, c = r.engine, r.cache
-    out = {"weights": sum(cfg.layer_weights(i) for i in range(cfg.n_layer))}
+    out = {"weights": _weights(cfg)}
     toks = torch.randint(0, cfg.vocab_size, (max_seq,)).tolist()
 
     def prefill():
@@ -95,7 +102,7 @@ def _existing(cfg, device, prompt: int, batch: int, steps: int) -> dict:
     r.reset()
     toks = torch.randint(0, cfg.vocab_size, (stage.max_seq_length,),
                          device=device)
-    out = {"weights": sum(cfg.layer_weights(i) for i in range(cfg.n_layer))}
+    out = {"weights": _weights(cfg)}
 
     def prefill():
         r.tail(r.prefill_head(toks[:prompt], 0)[-1])
