@@ -1,8 +1,10 @@
 """Shared test fixtures: build a complete toy litGPT checkpoint dir
-(model_config.yaml + lit_model.pth + tokenizer.json) on the fly."""
+(model_config.yaml + lit_model.pth + tokenizer.json) on the fly; operations,
+inputs and comparison of the kernel tests; runs of a sequence in portions."""
 
 from pathlib import Path
 
+import pytest
 import torch
 
 
@@ -44,3 +46,56 @@ def make_toy_checkpoint(out_dir: Path, name: str = "nano-test",
     save_checkpoint(out_dir, cfg, m.state_dict())
     make_toy_tokenizer(out_dir)
     return out_dir
+
+
+# -- kernel tests: where an operation runs, and in which precision
+CPU = pytest.param("cpu", torch.float32, id="cpu-f32")
+GPU32 = pytest.param("cuda", torch.float32, id="gpu-f32",
+                     marks=pytest.mark.gpu)
+GPU16 = pytest.param("cuda", torch.bfloat16, id="gpu-bf16",
+                     marks=pytest.mark.gpu)
+everywhere = pytest.mark.parametrize("device,dtype", [CPU, GPU32, GPU16])
+
+def ops_for(device):
+    if device == "cuda":
+        from mdi_llm_amd.ops import require_hip_ops
+
+        return require_hip_ops()
+    from mdi_llm_amd.ops import hybrid_torch
+
+    return hybrid_torch
+
+
+def close(got, want, dtype, scale=None):
+    want = want.double().cpu()
+    got = got.double().cpu()
+    tol = 1e-5 if dtype == torch.float32 else 1.2e-2
+    scale = float(want.abs().max()) if scale is None else scale
+    err = float((got - want).abs().max())
+    assert err <= tol * max(scale, 1e-3), (err, scale)
+
+
+def rand(*shape, seed=0, dtype=torch.float32, device="cpu"):
+    g = torch.Generator().manual_seed(seed)
+    return torch.randn(*shape, generator=g).to(dtype).to(device)
+
+
+def seg(rows, device):
+    return torch.tensor(list(map(list, zip(*rows))), dtype=torch.int32,
+                        device=device)
+
+
+def run_portions(runner, toks, portions, slot=None):
+    """All logits of one sequence cut into the given portions (the last one
+    repeats)."""
+    c = runner.cache
+    slot = c.admit() if slot is None else slot
+    at, out, portions = 0, [], list(portions)
+    while at < len(toks):
+        n = portions.pop(0) if len(portions) > 1 else portions[0]
+        part = toks[at:at + n]
+        out.append(runner.engine.step([(slot, part)],
+                                      [range(len(part))]).float().clone())
+        at += n
+    c.release(slot)
+    return torch.cat(out)

@@ -8,6 +8,7 @@ import pytest
 import torch
 
 import nerozen_oracle as oracle
+from helpers import run_portions
 from nerozen_models import (MODELS, deviation, make_runner, tokens, weights)
 
 CPU = pytest.param("cpu", torch.float32, 2e-5, id="cpu-f32")
@@ -33,22 +34,6 @@ def expected(name, toks):
         cfg, w = model(name)
         _cache[key] = oracle.forward(cfg, w, toks)
     return _cache[key]
-
-
-def run_portions(runner, toks, portions, slot=None):
-    """All logits of one sequence cut into the given portions (the last one
-    repeats)."""
-    c = runner.cache
-    slot = c.admit() if slot is None else slot
-    at, out, portions = 0, [], list(portions)
-    while at < len(toks):
-        n = portions.pop(0) if len(portions) > 1 else portions[0]
-        part = toks[at:at + n]
-        out.append(runner.engine.step([(slot, part)],
-                                      [range(len(part))]).float().clone())
-        at += n
-    c.release(slot)
-    return torch.cat(out)
 
 
 @everywhere

@@ -8,45 +8,10 @@ import pytest
 import torch
 
 import nerozen_oracle as oracle
+from helpers import close, everywhere, ops_for, rand, seg
 from mdi_llm_amd.ops.hybrid_engine import distance_bias
 
-CPU = pytest.param("cpu", torch.float32, id="cpu-f32")
-GPU32 = pytest.param("cuda", torch.float32, id="gpu-f32",
-                     marks=pytest.mark.gpu)
-GPU16 = pytest.param("cuda", torch.bfloat16, id="gpu-bf16",
-                     marks=pytest.mark.gpu)
-everywhere = pytest.mark.parametrize("device,dtype", [CPU, GPU32, GPU16])
-
 PAGE = 64
-
-
-def ops_for(device):
-    if device == "cuda":
-        from mdi_llm_amd.ops import require_hip_ops
-
-        return require_hip_ops()
-    from mdi_llm_amd.ops import hybrid_torch
-
-    return hybrid_torch
-
-
-def close(got, want, dtype, scale=None):
-    want = want.double().cpu()
-    got = got.double().cpu()
-    tol = 1e-5 if dtype == torch.float32 else 1.2e-2
-    scale = float(want.abs().max()) if scale is None else scale
-    err = float((got - want).abs().max())
-    assert err <= tol * max(scale, 1e-3), (err, scale)
-
-
-def rand(*shape, seed=0, dtype=torch.float32, device="cpu"):
-    g = torch.Generator().manual_seed(seed)
-    return torch.randn(*shape, generator=g).to(dtype).to(device)
-
-
-def seg(rows, device):
-    return torch.tensor(list(map(list, zip(*rows))), dtype=torch.int32,
-                        device=device)
 
 
 # ---------------------------------------------------------------------------
