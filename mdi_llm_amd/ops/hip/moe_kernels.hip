@@ -235,11 +235,10 @@ void expert_rows_t(void* out, const void* x, const void* w, MoePlan p, int m,
 // ---------------------------------------------------------------------------
 constexpr int BIG_ROWS = 128, BIG_COLS = 256, BIG_K = 64;
 
-template <bool UP>
+template <bool UP, int ACT>
 __global__ __launch_bounds__(256, 2) void expert_tiles_kernel(
     bf16* __restrict__ out, const bf16* __restrict__ x,
-    const bf16* __restrict__ w, MoePlan p, int m, int k, int m_tiles,
-    int act) {
+    const bf16* __restrict__ w, MoePlan p, int m, int k, int m_tiles) {
   constexpr int MT = UP ? BIG_COLS / 2 : BIG_COLS;  // outputs of a block
   constexpr int XI = BIG_ROWS / 32, WI = BIG_COLS / 32;
   extern __shared__ __attribute__((aligned(16))) bf16 sm[];
@@ -344,7 +343,7 @@ __global__ __launch_bounds__(256, 2) void expert_tiles_kernel(
       Pack<bf16, 4> v;
 #pragma unroll
       for (int q = 0; q < 4; ++q)
-        v.v[q] = from_f<bf16>(UP ? gated(acc[i][j][q], acc[i][(j + 4) % 8][q], act)
+        v.v[q] = from_f<bf16>(UP ? gated(acc[i][j][q], acc[i][(j + 4) % 8][q], ACT)
                                  : acc[i][j][q]);
       // m is a multiple of 4
       if (col < m) *reinterpret_cast<Pack<bf16, 4>*>(o + col) = v;
@@ -352,19 +351,19 @@ __global__ __launch_bounds__(256, 2) void expert_tiles_kernel(
   }
 }
 
-template <bool UP>
+template <bool UP, int ACT>
 void expert_tiles(void* out, const void* x, const void* w, MoePlan p, int m,
-                  int k, int act, hipStream_t stream) {
+                  int k, hipStream_t stream) {
   constexpr size_t smem = (BIG_ROWS + BIG_COLS) * BIG_K * sizeof(bf16);
   const int m_tiles = (m + (UP ? BIG_COLS / 2 : BIG_COLS) - 1) /
                       (UP ? BIG_COLS / 2 : BIG_COLS);
   const long long units = (long long)p.max_tiles * m_tiles;
-  auto kernel = expert_tiles_kernel<UP>;
+  auto kernel = expert_tiles_kernel<UP, ACT>;
   (void)hipFuncSetAttribute((const void*)kernel,
                             hipFuncAttributeMaxDynamicSharedMemorySize,
                             (int)smem);
   kernel<<<(unsigned)((units + 7) / 8 * 8), 256, smem, stream>>>(
-      (bf16*)out, (const bf16*)x, (const bf16*)w, p, m, k, m_tiles, act);
+      (bf16*)out, (const bf16*)x, (const bf16*)w, p, m, k, m_tiles);
 }
 
 }  // namespace
@@ -409,8 +408,10 @@ void launch_moe_route(float* weight, float* z, const void* x,
 
 void launch_moe_up(void* mid, const void* x, const void* w, MoePlan p,
                    int ff, int k, int act, int f32, hipStream_t stream) {
-  if (p.tile_rows == BIG_ROWS)
-    expert_tiles<true>(mid, x, w, p, ff, k, act, stream);
+  if (p.tile_rows == BIG_ROWS && act == 0)
+    expert_tiles<true, 0>(mid, x, w, p, ff, k, stream);
+  else if (p.tile_rows == BIG_ROWS)
+    expert_tiles<true, 1>(mid, x, w, p, ff, k, stream);
   else if (f32) expert_rows_t<float, true>(mid, x, w, p, ff, k, act, stream);
   else expert_rows_t<bf16, true>(mid, x, w, p, ff, k, act, stream);
 }
@@ -418,7 +419,7 @@ void launch_moe_up(void* mid, const void* x, const void* w, MoePlan p,
 void launch_moe_down(void* out, const void* mid, const void* w, MoePlan p,
                      int m, int ff, int f32, hipStream_t stream) {
   if (p.tile_rows == BIG_ROWS)
-    expert_tiles<false>(out, mid, w, p, m, ff, 0, stream);
+    expert_tiles<false, 0>(out, mid, w, p, m, ff, stream);
   else if (f32) expert_rows_t<float, false>(out, mid, w, p, m, ff, 0, stream);
   else expert_rows_t<bf16, false>(out, mid, w, p, m, ff, 0, stream);
 }
