@@ -312,6 +312,7 @@ __global__ __launch_bounds__(256, 2) void expert_tiles_kernel(
     store(sm);
     if (s + 1 < steps) load((s + 1) * BIG_K);
     __syncthreads();
+    // operand loads run a few products ahead of the MFMAs
 #pragma unroll
     for (int kk = 0; kk < 2; ++kk) {
       const int chunk = ((kk * 4 + quad) ^ (c & 7)) << 3;
@@ -325,12 +326,19 @@ __global__ __launch_bounds__(256, 2) void expert_tiles_kernel(
         wf[j] = *reinterpret_cast<const bf16x8*>(
             sm + (wrow(j) + c) * BIG_K + chunk);
 #pragma unroll
-      for (int i = 0; i < 4; ++i)
+      for (int j = 0; j < 8; ++j)
 #pragma unroll
-        for (int j = 0; j < 8; ++j)
+        for (int i = 0; i < 4; ++i)
           acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
               wf[j], xf[i], acc[i][j], 0, 0, 0);
     }
+    __builtin_amdgcn_sched_group_barrier(0x100, 6, 0);
+#pragma unroll
+    for (int g = 0; g < 18; ++g) {
+      __builtin_amdgcn_sched_group_barrier(0x008, 3, 0);
+      __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);
+    }
+    __builtin_amdgcn_sched_group_barrier(0x008, 10, 0);
   }
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
