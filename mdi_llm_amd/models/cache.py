@@ -8,13 +8,13 @@ state per slot.  One page table serves all attention layers of the stage:
 page ``p`` is row ``p`` of every layer's arena.
 
 Layout (what the kernels in ``paged_attn.inc``, ``row_attn.inc`` and
-``hybrid_kernels.hip`` read): K pages ``[pages, kv_heads, 64 * dpad]`` and V pages ``[pages,
-kv_heads, 64 * vpad]`` in MFMA operand order (``k_index``, ``v_index``),
-latent pages ``[pages, 64, rpad]`` with one zero-padded row per token, states
-``[slots, heads, dim, vstride]`` in fp32.  Layers that read one latent share
-its pages (``latent`` is keyed by the layer that makes it).  Nothing needs clearing when
-a page or slot is taken again: keys past a sequence's end are masked, and
-the recurrence starts from zero at position 0.
+``hybrid_kernels.hip`` read): K pages ``[pages, kv_heads, 64 * dpad]`` and V
+pages ``[pages, kv_heads, 64 * vpad]`` in MFMA operand order (``k_index``,
+``v_index``), latent pages ``[pages, 64, rpad]`` with one zero-padded row per
+token, states ``[slots, heads, dim, vstride]`` in fp32.  Layers that read one
+latent share its pages (``latent`` is keyed by the layer that makes it).
+Nothing needs clearing when a page or slot is taken again: keys past a
+sequence's end are masked, and the recurrence starts from zero at position 0.
 """
 
 from __future__ import annotations

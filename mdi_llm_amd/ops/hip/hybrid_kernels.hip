@@ -22,8 +22,7 @@ DEVINL float block_sum(float v, float* red) {
 }
 
 template <typename T, int V, int NT, int KEEP>
-__global__ __launch_bounds__(NT) void residual_norm_kernel(
-    ResidualArgs p) {
+__global__ __launch_bounds__(NT) void residual_norm_kernel(ResidualArgs p) {
   __shared__ float red[NT / 64];
   const size_t row = blockIdx.x;
   const int e = p.e;

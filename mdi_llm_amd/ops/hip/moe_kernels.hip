@@ -24,8 +24,8 @@ DEVINL typename Frag<T>::Row load_steps(const T* row, int at, int k,
 }
 
 // out[row][m]: 16 x 16 tile of x w^T, the contraction split over NW waves in
-// stretches of 64 (a lane's 16 steps of a stretch are contiguous), NM weight
-// rows sets at once.  The sum is left in red[..][row][m] of every wave.
+// stretches of 64 (a lane's 16 steps of a stretch are contiguous), for NM sets
+// of weight rows at once.  Every wave leaves its part in red[wave][set][row][m].
 template <typename T, int NW, int NM>
 DEVINL void tile_product(float (*red)[NM][16][17], const T* x,
                          const T* const (&w)[NM], int k, bool vec) {

@@ -58,7 +58,6 @@ class LatentPlan:
     seg: Optional[torch.Tensor] = None
     rows: Optional[torch.Tensor] = None
     n_rows: int = 0
-    singles: bool = True            # every absorbed entry is one token
     max_len: int = 1
     # expanded: seg [4, s] over the step's rows, context segments [4, s]
     # (start, len, slot, first position) over the gathered rows
@@ -89,7 +88,6 @@ def make_plan(entries: List[Tuple[int, int, int, int]], n_rows: int, m,
             p.ctx_max = max(p.ctx_max, ctx[-1][1])
             p.long_max = max(p.long_max, n)
     p.n_rows = len(rows)
-    p.singles = p.max_len == 1
     if rows == list(range(n_rows)):
         rows = []
     parts = [[x for col in zip(*t) for x in col] for t in (short, long, ctx)]

@@ -317,7 +317,8 @@ class MDIRuntime:
                                   n_samples + (1 if env_serve else 0),
                                   self.device,
                                   expected_s=msg.get("expected_s"))
-        self.comm = RingComm(config.ring_width, seq_len, self.device, n_samples,
+        self.comm = RingComm(config.ring_width, seq_len, self.device,
+                             n_samples,
                              dtype=config.residual_dtype(self.dtype))
         self.runtime = PipelineRuntime(self.runner, msg["rank"],
                                        msg["world"], self.comm, self.device)

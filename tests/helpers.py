@@ -56,6 +56,7 @@ GPU16 = pytest.param("cuda", torch.bfloat16, id="gpu-bf16",
                      marks=pytest.mark.gpu)
 everywhere = pytest.mark.parametrize("device,dtype", [CPU, GPU32, GPU16])
 
+
 def ops_for(device):
     if device == "cuda":
         from mdi_llm_amd.ops import require_hip_ops

@@ -68,7 +68,7 @@ def test_gated_act(cols, skew, act, device, dtype):
     proj = rand(n, 2 * cols + 16, seed=1, dtype=dtype, device=device) * 4
     proj[0, :] *= 10
     out = torch.zeros(n, cols + 8, dtype=dtype, device=device)
-    gate, upper = proj[:, skew:skew + cols], proj[:, skew + cols:skew + 2 * cols]
+    gate, upper = proj[:, skew:skew + 2 * cols].split(cols, 1)
     ops_for(device).gated_act(out[:, 8:], gate, upper, ACTS[act])
     f = getattr(oracle, act)
     want = f(gate.double().cpu()) * upper.double().cpu()
@@ -383,7 +383,7 @@ def test_plan_separates_the_forms():
     entries = [(0, 1, 3, 70), (201, 1, 1, 0), (1, 200, 0, 50)]
     p = make_plan(entries, 202, m, "cpu")
     assert p.seg.t().tolist() == [[0, 1, 3, 70], [1, 1, 1, 0]]
-    assert p.rows.tolist() == [0, 201] and p.n_rows == 2 and p.singles
+    assert p.rows.tolist() == [0, 201] and p.n_rows == 2 and p.max_len == 1
     assert p.long_seg.t().tolist() == [[1, 200, 0, 50]]
     assert p.ctx_seg.t().tolist() == [[0, 232, 0, 18]]
     assert (p.ctx_rows, p.ctx_max, p.long_max) == (232, 232, 200)
