@@ -55,7 +55,7 @@ class ModelConfig:
     norm_class_name: Literal["LayerNorm", "RMSNorm"] = "LayerNorm"
     norm_eps: float = 1e-5
     mlp_class_name: Literal["GptNeoxMLP", "LLaMAMLP", "GemmaMLP", "LLaMAMoE",
-                            "XieluMLP", "GatedMLP"] = "GptNeoxMLP"
+                            "XieluMLP", "GatedMLP", "GeluMLP"] = "GptNeoxMLP"
     gelu_approximate: str = "none"
     intermediate_size: Optional[int] = None
     rope_condense_ratio: int = 1
@@ -73,8 +73,18 @@ class ModelConfig:
     embedding_scale: float = 1.0
     # RMS norm weights are stored as w with norm_offset + w applied
     norm_offset: float = 0.0
+    # a norm ahead of each sublayer (else sublayers read the stream itself)
+    pre_norms: bool = True
     # a second norm on each sublayer's output, before the residual add
     post_norms: bool = False
+    # norms divide each of so many equal parts of a row by its own size
+    norm_groups: int = 1
+    # element-wise factors on what a sublayer adds
+    layer_scale: bool = False
+    # a mixer reads a mix of this token's and the previous token's input
+    token_shift: bool = False
+    # a layer passes on a weighted sum of its result and all earlier ones
+    depth_average: bool = False
     # what a layer adds to the residual stream is multiplied by this
     residual_mult: float = 1.0
 
@@ -105,11 +115,12 @@ class ModelConfig:
     def _sizes_from_layers(self) -> None:
         """Fill the uniform-stack fields from the layer list, so that code
         which only sizes or splits a model need not know about it."""
-        first = self.layers[0]["mixer"]
+        first = next((l["mixer"] for l in self.layers
+                      if "heads" in l["mixer"]), {})
         self.n_layer = len(self.layers)
-        self.n_head = first["heads"]
-        self.n_query_groups = first.get("kv_heads", first["heads"])
-        self.head_size = first["dim"]
+        self.n_head = first.get("heads", 1)
+        self.n_query_groups = first.get("kv_heads", self.n_head)
+        self.head_size = first.get("dim", first.get("vdim", self.n_embd))
         self.intermediate_size = max(
             (l["mlp"]["ff"] if l["mlp"]["kind"] == "dense"
              else l["mlp"]["expert"]["ff"]
@@ -129,21 +140,24 @@ class ModelConfig:
 
         return torch.float32 if self.is_hybrid else dtype
 
-    def shared_latents(self) -> Dict[int, int]:
-        """Layers whose cached latent other layers read (``kv_from``), with
-        the size of a row."""
+    def shared_rows(self) -> Dict[int, int]:
+        """Layers whose cached rows other layers read (``kv_from``), with
+        the size of a row: a latent, or a token's keys and values."""
         rows = {}
         for layer in self.layers or ():
-            src = layer["mixer"].get("kv_from")
-            if src is not None:
-                rows[src] = layer["mixer"]["kv_rank"]
+            m = layer["mixer"]
+            if m.get("kv_from") is not None:
+                rows[m["kv_from"]] = m["kv_rank"] if "kv_rank" in m else \
+                    m["kv_heads"] * (2 * m["dim"] + m["vdim"])
         return dict(sorted(rows.items()))
 
     @property
     def ring_width(self) -> int:
         """Columns of the rows that pass between pipeline stages: the
-        residual stream, then the latents that a later stage may read."""
-        return self.n_embd + sum(self.shared_latents().values())
+        residual stream (with the earlier layers' results, if layers average
+        them), then the cached rows that a later stage may read."""
+        streams = 1 + (self.n_layer if self.depth_average else 0)
+        return streams * self.n_embd + sum(self.shared_rows().values())
 
     def layer_weights(self, i: int, active: bool = False) -> int:
         """Number of matrix weights of layer ``i``; if ``active``, of those
@@ -165,13 +179,25 @@ class ModelConfig:
         elif layer["type"] == "attention":
             rows = (m["heads"] + m["kv_heads"]) * m["dim"] \
                 + m["kv_heads"] * m["vdim"]
+        elif layer["type"] == "diff_attention":
+            rows = 2 * m["heads"] * m["dim"]
+            if m.get("kv_from") is None:
+                rows += m["kv_heads"] * (2 * m["dim"] + m["vdim"])
+        elif layer["type"] == "mamba2":
+            rows = m["heads"] * (m["vdim"] + 1) \
+                + m["heads"] * m["vdim"] + 2 * m["groups"] * m["state"]
+        elif layer["type"] == "rglru":
+            rows = 3 * m["width"]
+            inner = 2 * m["width"] ** 2 // m["blocks"]
         else:
             rows = m["heads"] * (2 * m["dim"] + m["vdim"])
-        rows += m["heads"] * m["vdim"]
+        if "heads" in m:
+            rows += m["heads"] * m["vdim"]
         if mlp and mlp["kind"] == "moe":
             router = mlp["router"]
             used = router["top"] if active else router["experts"]
-            rows += router["experts"] + 3 * used * mlp["expert"]["ff"]
+            rows += router["experts"] + router.get("identity", 0) \
+                + 3 * used * mlp["expert"]["ff"]
             if mlp.get("shared"):
                 rows += 3 * mlp["shared"]["ff"]
         elif mlp:
@@ -322,7 +348,61 @@ def _resolorn(raw: dict) -> dict:
     )
 
 
-native_architectures = {"Nerozen": _nerozen, "Resolorn": _resolorn}
+def _dinuzen(raw: dict) -> dict:
+    """Dinuzen: gated linear recurrences (RG-LRU, Mamba-2) and differential
+    attention in any order, dense or routed feed-forwards, norms on the
+    sublayers' outputs only, token shift, averages over depth."""
+    layers = copy.deepcopy(raw["layers"])
+    for i, layer in enumerate(layers):
+        m, mlp = layer["mixer"], layer["mlp"]
+        if layer["type"] not in ("rglru", "mamba2", "attention"):
+            raise ValueError(f"Dinuzen: unknown mixer {layer['type']!r}")
+        if mlp is not None and mlp["kind"] not in ("dense", "moe"):
+            raise ValueError(
+                f"Dinuzen: unknown feed-forward {mlp['kind']!r}")
+        if mlp is not None and mlp["kind"] == "moe":
+            r = mlp["router"]
+            outputs = r["experts"] + r.get("identity", 0)
+            if not 1 <= r["top"] <= outputs:
+                raise ValueError(f"Dinuzen: layer {i} routes to {r['top']} "
+                                 f"of {outputs} experts")
+        if layer["type"] != "attention":
+            continue
+        layer["type"] = "diff_attention"
+        src = m.get("kv_from")
+        if src is None:
+            continue
+        if not 0 <= src < i or layers[src]["type"] != "diff_attention" \
+                or layers[src]["mixer"].get("kv_from") is not None:
+            raise ValueError(f"Dinuzen: layer {i} reads the keys of layer "
+                             f"{src}, which has none of its own before it")
+        for key in ("heads", "kv_heads", "dim", "vdim", "rot"):
+            if layers[src]["mixer"][key] != m[key]:
+                raise ValueError(f"Dinuzen: layers {i} and {src} share keys "
+                                 f"of unequal {key!r}")
+    return dict(
+        name="Dinuzen",
+        # positions are unlimited; this only bounds what serving allots
+        block_size=32768,
+        vocab_size=raw["vocab"],
+        padded_vocab_size=raw["vocab"],
+        n_embd=raw["width"],
+        layers=layers,
+        norm_class_name="RMSNorm",
+        norm_eps=raw["norm"]["eps"],
+        norm_groups=raw["norm"]["groups"],
+        pre_norms=False,
+        post_norms=True,
+        layer_scale=True,
+        token_shift=True,
+        depth_average=True,
+        parallel_residual=False,
+        mlp_class_name="GeluMLP",
+    )
+
+
+native_architectures = {"Nerozen": _nerozen, "Resolorn": _resolorn,
+                        "Dinuzen": _dinuzen}
 
 
 def is_native_checkpoint(path: Union[str, Path]) -> bool:
@@ -2301,6 +2381,66 @@ configs.extend([
                                       expert=dict(ff=2048),
                                       shared=dict(ff=2048)),
                     block_size=32768),
+])
+
+
+# -- Dinuzen -----------------------------------------------------
+
+
+def _dinuzen_named(name: str, n_layer: int, width: int, vocab: int,
+                   rglru: dict, mamba2: dict, attention: dict, ff: int,
+                   experts: dict, norm_groups: int) -> dict:
+    """A Dinuzen stack in repeats of four layers: RG-LRU, Mamba-2, attention,
+    and attention over the third layer's keys and values; every second layer
+    routes to experts."""
+    layers = []
+    for i in range(n_layer):
+        kind = ("rglru", "mamba2", "attention", "attention")[i % 4]
+        mixer = dict(dict(rglru=rglru, mamba2=mamba2,
+                          attention=attention)[kind])
+        if i % 4 == 3:
+            mixer["kv_from"] = i - 1
+        mlp = dict(experts, kind="moe") if i % 2 else dict(kind="dense",
+                                                           ff=ff)
+        layers.append(dict(type=kind, mixer=mixer, mlp=mlp))
+    conf = _dinuzen(dict(vocab=vocab, width=width, layers=layers,
+                         norm=dict(eps=1e-6, groups=norm_groups)))
+    conf.update(name=name)
+    return conf
+
+
+def _dinuzen_attention(heads: int, kv_heads: int, dim: int, vdim: int,
+                       diff: float) -> dict:
+    return dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim,
+                diff=diff, scale=dim ** -0.5, softcap=50.0,
+                rot=dict(base=10000.0, dims=dim,
+                         scaling=dict(factor=4.0, original=8192, fast=32.0,
+                                      slow=1.0)))
+
+
+configs.extend([
+    _dinuzen_named("dinuzen-nano", 4, 128, 384,
+                   dict(width=160, blocks=5, conv=4),
+                   dict(heads=6, vdim=32, state=48, groups=3, norm_groups=2,
+                        conv=4),
+                   _dinuzen_attention(4, 2, 24, 40, 0.6), 320,
+                   dict(router=dict(experts=6, identity=1, top=2, scale=1.2),
+                        expert=dict(ff=48), shared=dict(ff=72)), 2),
+    # TinyLlama-1.1B and Llama-3-8B widths and weights used per token
+    _dinuzen_named("dinuzen-1b", 22, 2048, 32000,
+                   dict(width=2560, blocks=10, conv=4),
+                   dict(heads=64, vdim=64, state=128, groups=8,
+                        norm_groups=8, conv=4),
+                   _dinuzen_attention(16, 4, 64, 128, 0.7), 8448,
+                   dict(router=dict(experts=32, identity=2, top=6, scale=2.0),
+                        expert=dict(ff=704), shared=dict(ff=1408)), 8),
+    _dinuzen_named("dinuzen-8b", 32, 4096, 128256,
+                   dict(width=5120, blocks=20, conv=4),
+                   dict(heads=64, vdim=128, state=128, groups=8,
+                        norm_groups=8, conv=4),
+                   _dinuzen_attention(32, 8, 64, 128, 0.7), 21504,
+                   dict(router=dict(experts=32, identity=2, top=6, scale=2.0),
+                        expert=dict(ff=2048), shared=dict(ff=2048)), 8),
 ])
 
 

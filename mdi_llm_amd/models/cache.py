@@ -11,10 +11,16 @@ Layout (what the kernels in ``paged_attn.inc``, ``row_attn.inc`` and
 ``hybrid_kernels.hip`` read): K pages ``[pages, kv_heads, 64 * dpad]`` and V
 pages ``[pages, kv_heads, 64 * vpad]`` in MFMA operand order (``k_index``,
 ``v_index``), latent pages ``[pages, 64, rpad]`` with one zero-padded row per
-token, states ``[slots, heads, dim, vstride]`` in fp32.  Layers that read one
-latent share its pages (``latent`` is keyed by the layer that makes it).
+token, states ``[slots, heads, dim, vstride]`` (or ``[slots, channels]``) in
+fp32.  Differential attention has a K page per map and kv head, ``[pages,
+kv_heads * 2, 64 * dpad]``.  Layers that read one latent, or one layer's keys
+and values, share its pages (``latent``, ``k`` and ``v`` are keyed by the layer
+that makes them).  A short convolution's last inputs (``conv``, ``[slots, taps
+- 1, channels]``) and the previous token's row of a layer with token shift
+(``prev``, fp32) are part of a slot as well.
+
 Nothing needs clearing when a page or slot is taken again: keys past a
-sequence's end are masked, and the recurrence starts from zero at position 0.
+sequence's end are masked, and a recurrence, a convolution and a shift start from zeros at position 0.
 """
 
 from __future__ import annotations
@@ -69,7 +75,8 @@ class HybridCache:
     fp8 = False
 
     def __init__(self, mixers, n_slots: int, n_tokens: int,
-                 device: torch.device, dtype: torch.dtype) -> None:
+                 device: torch.device, dtype: torch.dtype,
+                 shift_width: int = 0) -> None:
         self.n_slots = n_slots
         self.n_pages = max(1, -(-n_tokens // PAGE))
         self.spare = n_slots
@@ -79,15 +86,28 @@ class HybridCache:
         self.v: Dict[int, torch.Tensor] = {}
         self.state: Dict[int, torch.Tensor] = {}
         self.latent: Dict[int, torch.Tensor] = {}
+        self.conv: Dict[int, torch.Tensor] = {}
+        self.prev: Dict[int, torch.Tensor] = {}
         for i, m in enumerate(mixers):
-            if m.kind == "attention":
+            if shift_width:
+                self.prev[i] = torch.zeros(n_slots + 1, shift_width,
+                                           device=device,
+                                           dtype=torch.float32)
+            if m.kind in ("rglru", "mamba2"):
+                self.conv[i] = torch.zeros(n_slots + 1, max(1, m.taps - 1),
+                                           m.channels, device=device,
+                                           dtype=dtype)
+            if m.kind in ("attention", "diff_attention"):
+                if m.source in self.k:
+                    continue
                 dpad = _pad_to(m.dim, (32, 64, 128, 256), "attention dim")
                 vpad = _pad_to(m.vdim, (32, 64, 128, 256), "attention vdim")
                 P, G = self.n_pages + 1, m.kv_heads
-                self.k[i] = torch.zeros(P, G, PAGE * dpad, device=device,
-                                        dtype=dtype)
-                self.v[i] = torch.zeros(P, G, PAGE * vpad, device=device,
-                                        dtype=dtype)
+                maps = getattr(m, "maps", 1)
+                self.k[m.source] = torch.zeros(
+                    P, G * maps, PAGE * dpad, device=device, dtype=dtype)
+                self.v[m.source] = torch.zeros(
+                    P, G, PAGE * vpad, device=device, dtype=dtype)
             elif m.kind == "latent_attention":
                 if m.source not in self.latent:
                     rpad = _pad_to(m.rank, (64, 128, 256, 512),
@@ -95,6 +115,10 @@ class HybridCache:
                     self.latent[m.source] = torch.zeros(
                         self.n_pages + 1, PAGE, rpad, device=device,
                         dtype=dtype)
+            elif m.kind == "rglru":
+                self.state[i] = torch.zeros(n_slots + 1, m.width,
+                                            device=device,
+                                            dtype=torch.float32)
             else:
                 vstride = -(-m.vdim // 4) * 4
                 self.state[i] = torch.zeros(
@@ -180,5 +204,6 @@ class HybridCache:
 
     def memory_bytes(self) -> int:
         return sum(t.numel() * t.element_size()
-                   for d in (self.k, self.v, self.state, self.latent)
+                   for d in (self.k, self.v, self.state, self.latent,
+                             self.conv, self.prev)
                    for t in d.values())

@@ -35,7 +35,7 @@ class HGRN2Mixer(nn.Module):
 
     kind = "hgrn2"
 
-    def __init__(self, width: int, spec: dict) -> None:
+    def __init__(self, width: int, spec: dict, index: int) -> None:
         super().__init__()
         self.heads, self.dim, self.vdim = (
             spec["heads"], spec["dim"], spec["vdim"])
@@ -55,8 +55,9 @@ class BiasedAttention(nn.Module):
 
     kind = "attention"
 
-    def __init__(self, width: int, spec: dict) -> None:
+    def __init__(self, width: int, spec: dict, index: int) -> None:
         super().__init__()
+        self.source = index     # model-wide index of the layer's K/V pages
         self.heads, self.kv_heads = spec["heads"], spec["kv_heads"]
         if self.heads % self.kv_heads:
             raise ValueError("heads must be a multiple of kv_heads")
@@ -83,12 +84,115 @@ class BiasedAttention(nn.Module):
         super()._load_from_state_dict(state_dict, prefix, *args, **kwargs)
 
 
+class RGLRUMixer(nn.Module):
+    """Two branches, in_proj rows y | x: x passes a causal convolution and a
+    linear recurrence whose gates are block-diagonal products (gates: the
+    recurrence gate's matrices, then the input gate's); the activated y
+    multiplies what comes out."""
+
+    kind = "rglru"
+
+    def __init__(self, width: int, spec: dict, index: int) -> None:
+        super().__init__()
+        self.width, self.blocks = spec["width"], spec["blocks"]
+        if self.width % self.blocks:
+            raise ValueError("rglru: width must be a multiple of blocks")
+        self.taps, self.channels = spec["conv"], self.width
+        W, part = self.width, self.width // self.blocks
+        self.in_proj = nn.Linear(width, 2 * W, bias=True)
+        self.conv = nn.Parameter(torch.zeros(W, self.taps))
+        self.conv_bias = nn.Parameter(torch.zeros(W))
+        self.gates = nn.Parameter(torch.zeros(2 * self.blocks, part, part))
+        self.gate_bias = nn.Parameter(torch.zeros(2 * self.blocks, part))
+        self.lam = nn.Parameter(torch.zeros(W))
+        self.proj = nn.Linear(W, width, bias=False)
+
+
+class Mamba2Mixer(nn.Module):
+    """State-space duality with a scalar decay per head: in_proj rows are
+    z | x | B | C | dt, of which x, B and C pass a causal convolution."""
+
+    kind = "mamba2"
+
+    def __init__(self, width: int, spec: dict, index: int) -> None:
+        super().__init__()
+        self.heads, self.vdim = spec["heads"], spec["vdim"]
+        self.dim, self.groups = spec["state"], spec["groups"]
+        self.norm_groups, self.taps = spec["norm_groups"], spec["conv"]
+        self.inner = self.heads * self.vdim
+        if self.heads % self.groups or self.inner % self.norm_groups:
+            raise ValueError("mamba2: heads must be a multiple of groups, "
+                             "channels of norm_groups")
+        self.channels = self.inner + 2 * self.groups * self.dim
+        self.in_proj = nn.Linear(
+            width, self.inner + self.channels + self.heads, bias=False)
+        self.conv = nn.Parameter(torch.zeros(self.channels, self.taps))
+        self.conv_bias = nn.Parameter(torch.zeros(self.channels))
+        self.dt_bias = nn.Parameter(torch.zeros(self.heads))
+        self.a_log = nn.Parameter(torch.zeros(self.heads))
+        self.skip = nn.Parameter(torch.zeros(self.heads))
+        self.norm = Scale(self.inner)
+        self.proj = nn.Linear(self.inner, width, bias=False)
+
+
+class DiffAttention(nn.Module):
+    """Differential attention: every head has two attention maps over the
+    same values and gives the first less ``lambda`` times the second.  in_proj
+    rows are q | k | v, queries and keys as (head, map).  A layer with
+    ``kv_from`` has queries only and reads that layer's keys and values.
+    lambda is learned (exp(q1 k1) - exp(q2 k2) + diff, ``lam`` rows q1, k1,
+    q2, k2)."""
+
+    kind = "diff_attention"
+    maps = 2
+
+    def __init__(self, width: int, spec: dict, index: int) -> None:
+        super().__init__()
+        self.heads, self.kv_heads = spec["heads"], spec["kv_heads"]
+        if self.heads % self.kv_heads:
+            raise ValueError("heads must be a multiple of kv_heads")
+        self.dim, self.vdim = spec["dim"], spec["vdim"]
+        self.scale, self.diff = float(spec["scale"]), float(spec["diff"])
+        self.softcap = float(spec.get("softcap") or 0.0)
+        self.rot = dict(spec["rot"])
+        if self.rot["dims"] % 2 or self.rot["dims"] > self.dim:
+            raise ValueError("rotated dimensions come in pairs within a head")
+        self.window, self.keep_first = 1 << 30, 0
+        src = spec.get("kv_from")
+        self.source = index if src is None else src
+        self.owns_kv = src is None
+        rows = self.maps * self.heads * self.dim
+        if self.owns_kv:
+            rows += self.kv_heads * (self.maps * self.dim + self.vdim)
+            self.k_norm = Scale(self.dim)
+        self.in_proj = nn.Linear(width, rows, bias=False)
+        self.q_norm = Scale(self.dim)
+        self.lam = nn.Parameter(torch.zeros(4 * self.dim))
+        self.proj = nn.Linear(self.heads * self.vdim, width, bias=False)
+
+    def map_weight(self) -> float:
+        q1, k1, q2, k2 = self.lam.detach().double().view(4, -1)
+        return float((q1 * k1).sum().exp() - (q2 * k2).sum().exp()
+                     + self.diff)
+
+
 class XieluMLP(nn.Module):
     def __init__(self, width: int, spec: dict) -> None:
         super().__init__()
         self.fc = nn.Linear(width, spec["ff"], bias=False)
         self.proj = nn.Linear(spec["ff"], width, bias=False)
         self.act = nn.Parameter(torch.zeros(2))
+
+
+class GeluMLP(nn.Module):
+    """Up, exact GELU, down."""
+
+    kind = "dense"
+
+    def __init__(self, width: int, spec: dict) -> None:
+        super().__init__()
+        self.fc = nn.Linear(width, spec["ff"], bias=False)
+        self.proj = nn.Linear(spec["ff"], width, bias=False)
 
 
 class LatentAttention(nn.Module):
@@ -143,23 +247,50 @@ class RoutedMLP(nn.Module):
 
     kind = "moe"
     act = "silu"
+    gate_rows = 0           # router rows that are not a choice
 
     def __init__(self, width: int, spec: dict) -> None:
         super().__init__()
         self.experts, self.top = (
             spec["router"]["experts"], spec["router"]["top"])
         self.expert_ff = spec["expert"]["ff"]
+        self.identity = spec["router"].get("identity", 0)
         self.ff = (spec.get("shared") or {}).get("ff", 0)
         self.in_rows = [("shared.gate", self.ff), ("shared.up", self.ff)] \
             if self.ff else []
-        self.router = nn.Linear(width, self.experts, bias=False)
+        self.router = nn.Linear(width, self.experts + self.identity
+                                + self.gate_rows, bias=False)
         self.up = nn.Linear(width, self.experts * 2 * self.expert_ff,
                             bias=False)
         self.down = nn.Linear(self.expert_ff, self.experts * width,
                               bias=False)
 
 
-MIXERS = {m.kind: m for m in (HGRN2Mixer, BiasedAttention)}
+class CorrectedRoutedMLP(RoutedMLP):
+    """Routed experts with weights of their own beside the choice: the
+    softmax over all router outputs plus ``correction`` chooses, without it
+    the weights are made (times ``scale``).  The last ``identity`` outputs
+    stand for the input itself.  The shared expert is gated by the router's
+    last row and has projections of its own (shared_in rows gate | up)."""
+
+    gate_rows = 1
+
+    def __init__(self, width: int, spec: dict) -> None:
+        if not spec.get("shared"):
+            self.gate_rows = 0
+        super().__init__(width, spec)
+        self.scale = float(spec["router"].get("scale", 1.0))
+        self.correction = nn.Parameter(
+            torch.zeros(self.experts + self.identity))
+        if self.ff:
+            self.shared_in = nn.Linear(width, 2 * self.ff, bias=False)
+            self.shared_out = nn.Linear(self.ff, width, bias=False)
+
+
+MIXERS = {m.kind: m for m in (HGRN2Mixer, BiasedAttention, RGLRUMixer,
+                              Mamba2Mixer, DiffAttention)}
+MLPS = {"XieluMLP": {"dense": XieluMLP},
+        "GeluMLP": {"dense": GeluMLP, "moe": CorrectedRoutedMLP}}
 PARALLEL_MIXERS = {m.kind: m for m in (LatentAttention,)}
 PARALLEL_MLPS = {m.kind: m for m in (GatedMLP, RoutedMLP)}
 
@@ -171,14 +302,24 @@ class HybridBlock(nn.Module):
         super().__init__()
         E = config.n_embd
         spec = config.layers[index]
-        self.norm_1 = Scale(E)
-        self.norm_1b = Scale(E) if config.post_norms else None
-        self.mixer = MIXERS[spec["type"]](E, spec["mixer"])
-        self.norm_2 = self.norm_2b = self.mlp = None
+
+        def scale(wanted: bool):
+            return Scale(E) if wanted else None
+
+        self.norm_1 = scale(config.pre_norms)
+        self.norm_1b = scale(config.post_norms)
+        self.ls_1 = scale(config.layer_scale)
+        self.mixer = MIXERS[spec["type"]](E, spec["mixer"], index)
+        self.norm_2 = self.norm_2b = self.ls_2 = self.mlp = None
         if spec["mlp"] is not None:
-            self.norm_2 = Scale(E)
-            self.norm_2b = Scale(E) if config.post_norms else None
-            self.mlp = XieluMLP(E, spec["mlp"])
+            self.norm_2 = scale(config.pre_norms)
+            self.norm_2b = scale(config.post_norms)
+            self.ls_2 = scale(config.layer_scale)
+            mlps = MLPS[config.mlp_class_name]
+            self.mlp = mlps[spec["mlp"]["kind"]](E, spec["mlp"])
+        self.shift = scale(config.token_shift)
+        # coefficients of the embedding and of every result up to this one
+        self.depth = Scale(index + 2) if config.depth_average else None
 
 
 class ParallelBlock(nn.Module):
@@ -233,28 +374,79 @@ def native_tensors(config: ModelConfig) -> Dict[str, Tuple[str, ...]]:
         if config.parallel_residual:
             out.update(_parallel_tensors(spec, src, dst))
             continue
-        norms = ["1", "1b"] if config.post_norms else ["1"]
-        if spec["mlp"] is not None:
-            norms += ["2", "2b"] if config.post_norms else ["2"]
-        for n in norms:
-            out[f"{dst}norm_{n}.weight"] = (f"{src}norm{n}",)
-        mix, mixer = src + "mix.", dst + "mixer."
-        if spec["type"] == "hgrn2":
-            out[mixer + "in_proj.weight"] = (mix + "q", mix + "f", mix + "v")
-            out[mixer + "f_bias"] = (mix + "f.b",)
-            out[mixer + "lower"] = (mix + "lower",)
-            out[mixer + "norm.weight"] = (mix + "norm",)
-        else:
-            out[mixer + "in_proj.weight"] = (mix + "q", mix + "k", mix + "v")
-            out[mixer + "q_norm.weight"] = (mix + "q.norm",)
-            out[mixer + "k_norm.weight"] = (mix + "k.norm",)
-            out[mixer + "rel"] = (mix + "rel",)
-        out[mixer + "proj.weight"] = (mix + "o",)
-        if spec["mlp"] is not None:
-            out[f"{dst}mlp.fc.weight"] = (f"{src}mlp.up",)
-            out[f"{dst}mlp.proj.weight"] = (f"{src}mlp.down",)
-            out[f"{dst}mlp.act"] = (f"{src}mlp.act",)
+        out.update(_block_tensors(config, spec, src, dst))
     return out
+
+
+_MIXER_TENSORS = {
+    "hgrn2": {"in_proj.weight": ("q", "f", "v"), "f_bias": ("f.b",),
+              "lower": ("lower",), "norm.weight": ("norm",)},
+    "attention": {"in_proj.weight": ("q", "k", "v"),
+                  "q_norm.weight": ("q.norm",), "k_norm.weight": ("k.norm",),
+                  "rel": ("rel",)},
+    "rglru": {"in_proj.weight": ("y", "x"), "in_proj.bias": ("y.b", "x.b"),
+              "conv": ("conv",), "conv_bias": ("conv.b",),
+              "gates": ("ra", "ri"), "gate_bias": ("ra.b", "ri.b"),
+              "lam": ("lam",)},
+    "mamba2": {"in_proj.weight": ("in",), "conv": ("conv",),
+               "conv_bias": ("conv.b",), "dt_bias": ("dt_bias",),
+               "a_log": ("A_log",), "skip": ("D",), "norm.weight": ("norm",)},
+    "diff_attention": {"in_proj.weight": ("q", "k", "v"),
+                       "q_norm.weight": ("q.norm",),
+                       "k_norm.weight": ("k.norm",),
+                       "lam": ("lq1", "lk1", "lq2", "lk2")},
+}
+
+
+def _block_tensors(config: ModelConfig, spec: dict, src: str,
+                   dst: str) -> dict:
+    out, mlp = {}, spec["mlp"]
+    for n in ("1",) if mlp is None else ("1", "2"):
+        if config.pre_norms:
+            out[f"{dst}norm_{n}.weight"] = (f"{src}norm{n}",)
+        if config.post_norms:
+            # a block's only norms go without the suffix
+            b = "b" if config.pre_norms else ""
+            out[f"{dst}norm_{n}b.weight"] = (f"{src}norm{n}{b}",)
+        if config.layer_scale:
+            out[f"{dst}ls_{n}.weight"] = (f"{src}ls{n}",)
+    if config.token_shift:
+        out[dst + "shift.weight"] = (src + "shift",)
+    if config.depth_average:
+        out[dst + "depth.weight"] = (src + "dwa",)
+    mix, mixer = src + "mix.", dst + "mixer."
+    for key, names in _MIXER_TENSORS[spec["type"]].items():
+        if spec["mixer"].get("kv_from") is not None:
+            if key == "k_norm.weight":
+                continue
+            names = tuple(n for n in names if n not in ("k", "v"))
+        out[mixer + key] = tuple(mix + n for n in names)
+    out[mixer + "proj.weight"] = (mix + "o",)
+    if mlp is None:
+        return out
+    pre, to = src + "mlp.", dst + "mlp."
+    if mlp["kind"] == "dense":
+        out[to + "fc.weight"] = (pre + "up",)
+        out[to + "proj.weight"] = (pre + "down",)
+        if config.mlp_class_name == "XieluMLP":
+            out[to + "act"] = (pre + "act",)
+        return out
+    out[to + "router.weight"] = (pre + "router",)
+    out[to + "correction"] = (pre + "correction",)
+    out.update(_expert_tensors(mlp, pre, to))
+    if mlp.get("shared"):
+        out[to + "router.weight"] += (pre + "shared.sg",)
+        out[to + "shared_in.weight"] = (pre + "shared.gate",
+                                        pre + "shared.up")
+        out[to + "shared_out.weight"] = (pre + "shared.down",)
+    return out
+
+
+def _expert_tensors(spec: dict, pre: str, to: str) -> dict:
+    n = range(spec["router"]["experts"])
+    return {to + "up.weight": tuple(f"{pre}e{e}.{part}" for e in n
+                                    for part in ("gate", "up")),
+            to + "down.weight": tuple(f"{pre}e{e}.down" for e in n)}
 
 
 def _parallel_tensors(spec: dict, src: str, dst: str) -> dict:
@@ -266,14 +458,11 @@ def _parallel_tensors(spec: dict, src: str, dst: str) -> dict:
         rows += [mlp + "gate", mlp + "up"]
         cols.append(mlp + "down")
     elif kind == "moe":
-        n = range(spec["mlp"]["router"]["experts"])
         if spec["mlp"].get("shared"):
             rows += [mlp + "shared.gate", mlp + "shared.up"]
             cols.append(mlp + "shared.down")
         out[dst + "mlp.router.weight"] = (mlp + "router",)
-        out[dst + "mlp.up.weight"] = tuple(
-            f"{mlp}e{e}.{part}" for e in n for part in ("gate", "up"))
-        out[dst + "mlp.down.weight"] = tuple(f"{mlp}e{e}.down" for e in n)
+        out.update(_expert_tensors(spec["mlp"], mlp, dst + "mlp."))
     mixer = dst + "mixer."
     rows.append(mix + "dq")
     out[mixer + "q_norm.weight"] = (mix + "dq.norm",)

@@ -74,6 +74,42 @@ def build_rope_cache(
     return torch.cos(idx_theta), torch.sin(idx_theta)
 
 
+def scaled_rope_angles(rot: dict) -> Tuple[torch.Tensor, float]:
+    """Angle per position of every pair (float64) and the factor on cos and
+    sin.  ``rot``: ``dims``, ``base`` and, for contexts beyond the trained
+    one, ``scaling`` with the YaRN blend (slow pairs are stretched by
+    ``factor``, fast ones kept; the borders are pairs that turn ``fast`` and
+    ``slow`` times over ``original`` positions)."""
+    n, base = rot["dims"], float(rot["base"])
+    i = torch.arange(n // 2, dtype=torch.float64)
+    theta = base ** (-2.0 * i / n)
+    s = rot.get("scaling")
+    if s is None:
+        return theta, 1.0
+
+    def pair(turns: float) -> float:
+        return n * math.log(s["original"] / (2 * math.pi * turns)) \
+            / (2 * math.log(base))
+
+    lo = max(math.floor(pair(s["fast"])), 0)
+    hi = min(math.ceil(pair(s["slow"])), n - 1)
+    ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+    return (theta * (1.0 - ramp + ramp / s["factor"]),
+            0.1 * math.log(s["factor"]) + 1.0)
+
+
+def build_pair_rope_table(seq_len: int, rot: dict,
+                          device: Optional[torch.device] = None
+                          ) -> torch.Tensor:
+    """[seq_len, dims / 2, 2] cos and sin in fp32, for rotations that pair
+    neighbouring dimensions.  The angles are taken in float64."""
+    theta, mult = scaled_rope_angles(rot)
+    pos = torch.arange(seq_len, dtype=torch.float64)
+    a = torch.outer(pos, theta)
+    return (torch.stack((a.cos(), a.sin()), -1) * mult).float().contiguous() \
+        .to(device)
+
+
 def apply_rope(x: torch.Tensor, cos: torch.Tensor, sin: torch.Tensor) -> torch.Tensor:
     """``x``: (..., T, rope_n_elem); cos/sin: (T, rope_n_elem)."""
     head_size = x.size(-1)

@@ -110,7 +110,8 @@ class StageBase(nn.Module):
             self.kv_pool = HybridCache(
                 [b.mixer for b in self.transformer.h], n_slots,
                 n_tokens or n_slots * self._max_seq_length,
-                device, dtype)
+                device, dtype,
+                self.config.n_embd if self.config.token_shift else 0)
             return
         self.kv_pool = KVCachePool(
             n_slots,

@@ -8,6 +8,10 @@ product for the whole step, and the kernels that look at neighbours in time
 (recurrence, attention) walk the entries as segments.  Steps in which every
 entry is one token are captured as hipGraphs per batch size.
 
+Blocks come in three forms: norms ahead of (and behind) each sublayer, one norm
+for parallel sublayers (``latent_layer``), and norms on the sublayers' outputs
+only, with the options of that form (``_run_output_normed``).
+
 The residual stream, norms, gates, recurrent state and softmax are fp32; the
 weights, matrix products and cached K/V have the stage's dtype (bf16, or
 fp32 throughout).
@@ -29,7 +33,10 @@ import torch.nn.functional as F
 from ..config import ModelConfig
 from ..models.cache import PAGE, HybridCache
 from ..models.sampling import sample as sample_token
+from ..models.model import build_pair_rope_table
 from . import require_hip_ops
+from .experts import RoutedExperts
+from .mixers import RGLRU, Mamba2
 from .latent_layer import LatentPlan, ParallelLayer, make_plan
 
 __all__ = ["HybridEngine", "distance_bias"]
@@ -89,10 +96,13 @@ class Batch:
         return self.plans[key]
 
 
+XIELU, GELU = 1, 2      # activations that a projection can end with
+
+
 class _LayerWeights:
     """One layer's operands: matrices as they are, the rest in fp32."""
 
-    def __init__(self, block) -> None:
+    def __init__(self, eng: "HybridEngine", i: int, block) -> None:
         def f(t):
             return None if t is None else t.detach().float().contiguous()
 
@@ -101,22 +111,51 @@ class _LayerWeights:
 
         self.norm1, self.norm1b = w(block.norm_1), w(block.norm_1b)
         self.norm2, self.norm2b = w(block.norm_2), w(block.norm_2b)
+        # a factor on a sublayer's output joins the weight of its norm
+        for n, ls in (("norm1b", block.ls_1), ("norm2b", block.ls_2)):
+            if ls is not None:
+                setattr(self, n, getattr(self, n) * w(ls))
+        self.shift, self.depth = w(block.shift), w(block.depth)
         m = block.mixer
         self.mixer = m
-        self.in_proj = m.in_proj.weight.detach()
-        self.proj = m.proj.weight.detach()
+        if m.kind in ("rglru", "mamba2"):
+            self.mix = (RGLRU if m.kind == "rglru" else Mamba2)(eng, i, m)
+        else:
+            self.in_proj = m.in_proj.weight.detach()
+            self.proj = m.proj.weight.detach()
         if m.kind == "hgrn2":
             self.f_bias, self.lower = f(m.f_bias), f(m.lower)
             self.norm = f(m.norm.weight)
-        else:
+        elif m.kind == "attention":
             self.q_norm, self.k_norm = f(m.q_norm.weight), f(m.k_norm.weight)
             self.bias = distance_bias(m.rel, m.bias_max)
-        self.mlp = block.mlp is not None
-        if self.mlp:
-            self.fc = block.mlp.fc.weight.detach()
-            self.down = block.mlp.proj.weight.detach()
-            self.act = tuple(F.softplus(block.mlp.act.detach().float())
-                             .tolist())
+            self.rotate, self.two_maps = {}, {}
+        elif m.kind == "diff_attention":
+            self.q_norm = f(m.q_norm.weight)
+            self.k_norm = f(m.k_norm.weight) if m.owns_kv else None
+            self.bias = torch.zeros(m.heads, 1, device=eng.device)
+            self.rotate = dict(rope=eng.rope_table(m.rot))
+            self.two_maps = dict(softcap=m.softcap, map_weight=m.map_weight(),
+                                 out_scale=1.0 - m.diff,
+                                 eps=eng.config.norm_eps)
+        mlp = block.mlp
+        self.mlp = mlp is not None
+        self.experts = self.act = None
+        if not self.mlp:
+            return
+        if mlp.kind == "moe":
+            self.experts = RoutedExperts(eng, mlp)
+            self.shared_ff = mlp.ff
+            if mlp.ff:
+                self.shared_in = mlp.shared_in.weight.detach()
+                self.shared_out = mlp.shared_out.weight.detach()
+            return
+        self.fc = mlp.fc.weight.detach()
+        self.down = mlp.proj.weight.detach()
+        if hasattr(mlp, "act"):
+            self.act = (XIELU, *F.softplus(mlp.act.detach().float()).tolist())
+        else:
+            self.act = (GELU, 0.0, 0.0)
 
 
 class _DecodeStep:
@@ -177,16 +216,18 @@ class HybridEngine:
         self.is_starter = hasattr(stage, "lm_head")
         self.parallel = self.config.parallel_residual
         self.latent_form: Optional[str] = None  # "absorbed" or "expanded"
+        # longest sequence that can occur
+        self.max_ctx = min(cache.n_pages * PAGE, stage.max_seq_length)
+        self._ropes: Dict[str, torch.Tensor] = {}
         if self.parallel:
             self.layers = [ParallelLayer(self, b) for b in stage.transformer.h]
         else:
-            self.layers = [_LayerWeights(b) for b in stage.transformer.h]
+            self.layers = [_LayerWeights(self, i, b)
+                           for i, b in enumerate(stage.transformer.h)]
         for lw in self.layers:
             m = lw.mixer
             if m.kind == "hgrn2" and (m.dim > 256 or m.vdim > 1024):
                 raise ValueError("hgrn2: dim <= 256 and vdim <= 1024")
-        # longest sequence that can occur
-        self.max_ctx = min(cache.n_pages * PAGE, stage.max_seq_length)
         if self.is_starter:
             self.wte = stage.transformer.wte.weight.detach()
             self.final = stage.transformer.ln_f.weight.detach().float()
@@ -197,17 +238,30 @@ class HybridEngine:
         self._steps: Dict[int, _DecodeStep] = {}
 
     def _ring_columns(self, stage) -> None:
-        """Columns of the rows between stages that hold shared latents: those
-        that local layers read from an earlier stage, those made here."""
-        first = stage.first_layer
-        at, self.ring_in, self.ring_out = self.config.n_embd, {}, {}
-        for src, n in self.config.shared_latents().items():
+        """Columns of the rows between stages that hold shared cache rows:
+        those that local layers read from an earlier stage, those made
+        here."""
+        first, cfg = stage.first_layer, self.config
+        self.first_layer = first
+        shared = cfg.shared_rows()
+        at = cfg.ring_width - sum(shared.values())
+        self.ring_in, self.ring_out = {}, {}
+        for src, n in shared.items():
             cols = slice(at, at + n)
             at += n
             if first <= src < first + len(self.layers):
                 self.ring_out[src] = cols
-            elif src in self.cache.latent:
+            elif src in self.cache.latent or src in self.cache.k:
                 self.ring_in[src] = cols
+
+    def rope_table(self, rot: dict) -> torch.Tensor:
+        """cos and sin by position, one table for all layers that rotate
+        alike."""
+        key = repr(sorted(rot.items(), key=str))
+        if key not in self._ropes:
+            self._ropes[key] = build_pair_rope_table(self.max_ctx, rot,
+                                                     self.device)
+        return self._ropes[key]
 
     # ------------------------------------------------------------------
     # building blocks
@@ -237,18 +291,20 @@ class HybridEngine:
             # few rows: the weight stream decides.  Past 16 rows, and for
             # the widest outputs, the library's kernels stream as well,
             # except along a very long K.
-            p, q = act or (0.0, 0.0)
+            kind, p, q = act or (0, 0.0, 0.0)
             out = torch.empty(n, M, dtype=self.dtype, device=self.device)
             if n == 1 and K % 8 == 0:
-                self.ops.gemv(out, w, x, None, None, 4 if act else 0,
+                self.ops.gemv(out, w, x, None, None, kind and kind + 3,
                               rows=4 if M >= 65536 else 1, act_p=p, act_q=q)
                 return out
             if K % 64 == 0 and M < 65536 and (n <= 16 or K >= 16384):
-                self.ops.skinny_gemm(out, w, x, act is not None, p, q)
+                self.ops.skinny_gemm(out, w, x, kind, p, q)
                 return out
         out = F.linear(x, w)
-        if act is not None:
-            self.ops.xielu(out, *act)
+        if act is not None and act[0] == XIELU:
+            self.ops.xielu(out, *act[1:])
+        elif act is not None:
+            self.ops.gelu(out)
         return out
 
     def _hgrn2(self, i: int, lw: _LayerWeights, b: Batch, xn: torch.Tensor):
@@ -277,24 +333,27 @@ class HybridEngine:
                    xn: torch.Tensor):
         m, eps, c = lw.mixer, self.config.norm_eps, self.cache
         proj = self._linear(xn, lw.in_proj)
-        k, v = c.k[i], c.v[i]
-        q = torch.empty(b.n, m.heads, k.size(2) // PAGE, dtype=self.dtype,
-                        device=self.device)
-        self.ops.qk_norm_append(q, k, v, proj, lw.q_norm, lw.k_norm,
-                                b.row_slot, b.row_pos, c.table, m.vdim, eps)
+        k, v = c.k[m.source], c.v[m.source]
+        maps = k.size(1) // m.kv_heads
+        q = torch.empty(b.n, m.heads * maps, k.size(2) // PAGE,
+                        dtype=self.dtype, device=self.device)
+        owns = lw.k_norm is not None    # else an earlier layer's are read
+        self.ops.qk_norm_append(q, k if owns else None, v if owns else None,
+                                proj, lw.q_norm, lw.k_norm, b.row_slot,
+                                b.row_pos, c.table, m.vdim, eps, **lw.rotate)
         y = torch.empty(b.n, m.heads * m.vdim, dtype=self.dtype,
                         device=self.device)
 
         def attend(seg, max_len, splits, part=(None, None)):
             self.ops.paged_attn(y, q, k, v, lw.bias, c.table, seg, max_len,
                                 m.window, m.keep_first, m.scale, splits,
-                                *part)
+                                *part, **lw.two_maps)
 
         if b.singles:
             splits = self._splits(m, b.singles, b.max_ctx)
             part = (None, None)
-            if splits > 1:
-                cells = b.singles * m.heads * splits
+            if splits > 1 or maps > 1:
+                cells = b.singles * m.heads * maps * splits
                 part = (torch.empty(cells * v.size(2) // PAGE, dtype=torch.float32,
                                     device=self.device),
                         torch.empty(cells * 2, dtype=torch.float32,
@@ -304,9 +363,102 @@ class HybridEngine:
             attend(b.seg[:, b.singles:], b.max_len, 0)
         return self._linear(y, lw.proj)
 
+    def _mix(self, i: int, lw: _LayerWeights, b: Batch, xn: torch.Tensor):
+        if lw.mixer.kind in ("rglru", "mamba2"):
+            return lw.mix(b, xn)
+        if lw.mixer.kind == "hgrn2":
+            return self._hgrn2(i, lw, b, xn)
+        return self._attention(i, lw, b, xn)
+
+    # -- blocks with norms on the sublayers' outputs only ---------------
+    def _stream_step(self, b: Optional[Batch], x, y=None, post_w=None,
+                     reader=None, final=False, rows=False, **kw):
+        """x <- embed(tokens) or x + norm(y), with routed experts and the
+        average over depth if asked for; returns what reads the stream next:
+        layer ``reader``'s mixer (its token shift applied), the head
+        (``final``), a feed-forward (``rows``) or nothing."""
+        xn, shift = None, None
+        if reader is not None:
+            shift = self.layers[reader].shift
+        if reader is not None or final or rows:
+            xn = torch.empty(x.shape, dtype=self.dtype, device=self.device)
+        single = b is not None and b.singles == b.seg.size(1)
+        if shift is not None and single:    # the previous row is in the slot
+            kw.update(shift=shift, prev=self.cache.prev[reader],
+                      row_slot=b.row_slot, row_pos=b.row_pos)
+        later = shift is not None and not single
+        self.ops.stream_step(
+            x, y=y, post_w=post_w, xn=None if later else xn,
+            next_w=self.final if final else None,
+            groups=self.config.norm_groups, eps=self.config.norm_eps, **kw)
+        if later:
+            self.ops.token_shift(xn, x, shift, self.cache.prev[reader],
+                                 b.seg, b.max_len)
+        return xn
+
+    def _shared_expert(self, lw: _LayerWeights, xn: torch.Tensor):
+        if not lw.shared_ff:
+            return None
+        h = self._linear(xn, lw.shared_in)
+        mid = torch.empty(xn.size(0), lw.shared_ff, dtype=self.dtype,
+                          device=self.device)
+        self.ops.gated_act(mid, h[:, :lw.shared_ff], h[:, lw.shared_ff:],
+                           lw.experts.act)
+        return self._linear(mid, lw.shared_out)
+
+    def _run_output_normed(self, b: Batch, rows: Optional[torch.Tensor],
+                           final: bool, layers_out: Optional[list] = None):
+        """All local layers.  Returns (rows [n, streams * width], final-normed
+        rows or None); ``rows`` are the stream, then what the layers average:
+        the embedding and every layer's result, where later layers exist."""
+        cfg, first, n = self.config, self.first_layer, b.n
+        L, E = len(self.layers), cfg.n_embd
+        states = coef = None
+        if cfg.depth_average:
+            states = torch.empty(min(first + L + 1, cfg.n_layer), n, E,
+                                 dtype=torch.float32, device=self.device)
+        reader = 0 if L else None
+        if rows is None:
+            x = torch.empty(n, E, dtype=torch.float32, device=self.device)
+            xn = self._stream_step(
+                b, x, reader=reader, final=final and not L, tokens=b.tokens,
+                table=self.wte, scale=cfg.embedding_scale,
+                keep=None if states is None else states[0])
+        else:
+            x = rows[:, :E].contiguous()
+            for j in range(0 if states is None else first + 1):
+                states[j] = rows[:, (j + 1) * E:(j + 2) * E]
+            xn = self._stream_step(b, x, reader=reader, final=final and not L)
+        for i, lw in enumerate(self.layers):
+            last = i + 1 == L
+            end = dict(reader=None if last else i + 1, final=final and last)
+            if states is not None:
+                seen = first + i + 1
+                end.update(hist=states[:seen], coef=lw.depth)
+                if seen < states.size(0):
+                    end.update(keep=states[seen])
+            y = self._mix(i, lw, b, xn)
+            if not lw.mlp:
+                xn = self._stream_step(b, x, y, lw.norm1b, **end)
+            else:
+                xn = self._stream_step(b, x, y, lw.norm1b, rows=True)
+                if lw.experts is not None:
+                    out, weight, plan = lw.experts(xn)
+                    y = self._shared_expert(lw, xn)
+                    end.update(routed=out, routed_w=weight, chosen=plan,
+                               experts=lw.experts.experts)
+                else:
+                    y = self._linear(self._linear(xn, lw.fc, lw.act), lw.down)
+                xn = self._stream_step(b, x, y, lw.norm2b, **end)
+            if layers_out is not None:
+                layers_out.append(x.clone())
+        return (x, states), xn
+
     def _run(self, b: Batch, x: Optional[torch.Tensor], final: bool,
              layers_out: Optional[list] = None):
         """All local layers.  Returns (x, final-normed rows or None)."""
+        if not self.config.pre_norms:
+            return self._run_output_normed(b, x, final, layers_out)
         norms = [lw.norm1 for lw in self.layers[1:]]
         norms.append(self.final if final else None)
         first = self.layers[0].norm1 if self.layers else norms[0]
@@ -324,9 +476,7 @@ class HybridEngine:
                 if layers_out is not None:
                     layers_out.append(x.clone())
                 continue
-            mix = self._hgrn2 if lw.mixer.kind == "hgrn2" else \
-                self._attention
-            y = mix(i, lw, b, xn)
+            y = self._mix(i, lw, b, xn)
             if lw.mlp:
                 xn = self._norm_step(x, y, lw.norm1b, lw.norm2)
                 y = self._linear(self._linear(xn, lw.fc, lw.act), lw.down)
@@ -424,40 +574,64 @@ class HybridEngine:
                x: Optional[torch.Tensor] = None) -> torch.Tensor:
         """Pipeline stages: one sequence's tokens (starter) or the rows of
         the stage before (secondary) -> rows after the local layers, fp32:
-        the residual stream, then the latents that later stages may read."""
+        the residual stream (with the results that later layers average),
+        then the cached rows that later stages may read."""
         rows = None
         if tokens is not None:
             self._check_tokens(tokens)
             n = len(tokens)
         else:
             rows = x.reshape(-1, self.config.ring_width).float()
-            n, x = rows.size(0), rows[:, :self.config.n_embd].clone()
+            n, x = rows.size(0), rows[:, :self.ring_streams()].clone()
         b, _ = self._batch([(slot, n)], tokens)
         for src, cols in self.ring_in.items():
-            self.ops.latent_norm_append(
-                self.cache.latent[src], rows[:, cols].to(self.dtype), None,
-                b.row_slot, b.row_pos, self.cache.table,
-                self.config.norm_eps)
+            self._ring_rows(src, b, rows[:, cols].to(self.dtype).contiguous(),
+                            store=True)
         x = self._run(b, x, False)[0]
-        if self.config.ring_width == self.config.n_embd:
+        if isinstance(x, tuple):        # the stream and what layers average
+            x = x[0] if x[1] is None else torch.cat((x[0], *x[1]), 1)
+        if self.config.ring_width == x.size(1):
             return x
         out = torch.zeros(n, self.config.ring_width, device=self.device) \
             if rows is None else rows.clone()
-        out[:, :self.config.n_embd] = x
+        out[:, :x.size(1)] = x
         for src, cols in self.ring_out.items():
             c = torch.empty(n, cols.stop - cols.start, dtype=self.dtype,
                             device=self.device)
-            self.ops.latent_gather(c, self.cache.latent[src],
-                                   self.cache.table, b.seg, n)
+            self._ring_rows(src, b, c, store=False)
             out[:, cols] = c
         return out
+
+    def ring_streams(self) -> int:
+        """Columns of a ring row ahead of the shared cache rows."""
+        return self.config.ring_width - sum(
+            self.config.shared_rows().values())
+
+    def _ring_rows(self, src: int, b: Batch, rows: torch.Tensor,
+                   store: bool) -> None:
+        """This step's rows of layer ``src``'s latents, or keys and values:
+        into the pages, or out of them."""
+        c, ops = self.cache, self.ops
+        if src in c.k:
+            m = self.config.layers[src]["mixer"]
+            ops.kv_rows(rows, c.k[src], c.v[src], b.row_slot, b.row_pos,
+                        c.table, m["dim"], m["vdim"], store)
+        elif store:
+            ops.latent_norm_append(c.latent[src], rows, None, b.row_slot,
+                                   b.row_pos, c.table, self.config.norm_eps)
+        else:
+            ops.latent_gather(rows, c.latent[src], c.table, b.seg, b.n)
 
     @torch.no_grad()
     def logits(self, x: torch.Tensor) -> torch.Tensor:
         """Rows of the last stage -> logits."""
         x = x.reshape(-1, self.config.ring_width)[:, :self.config.n_embd]
         x = x.float().contiguous()
-        return self._linear(self._norm_step(x, next_w=self.final), self.head)
+        if self.config.pre_norms:
+            xn = self._norm_step(x, next_w=self.final)
+        else:
+            xn = self._stream_step(None, x, final=True)
+        return self._linear(xn, self.head)
 
     # ------------------------------------------------------------------
     # single-token steps (hipGraph per batch size)

@@ -14,7 +14,10 @@ from ..models.cache import PAGE, k_index, v_index
 __all__ = ["residual_norm", "xielu", "hgrn2_step", "hgrn2_scan",
            "qk_norm_append", "paged_attn", "latent_norm_append",
            "latent_gather", "head_proj", "latent_attn", "head_attn",
-           "gated_act", "moe_route", "moe_up", "moe_down", "advance_batch"]
+           "gated_act", "moe_route", "moe_up", "moe_down", "advance_batch",
+           "stream_step", "token_shift", "gelu", "causal_conv", "rglru_step",
+           "rglru_scan", "mamba2_step", "mamba2_scan", "mamba2_out",
+           "kv_rows"]
 
 
 def _rms(x: torch.Tensor, eps: float) -> torch.Tensor:
@@ -71,28 +74,63 @@ def hgrn2_step(out, proj, state, f_bias, lower, norm_w, seg, eps) -> None:
     hgrn2_scan(out, proj, state, f_bias, lower, norm_w, seg, 1, eps)
 
 
+def _rotate(x, rope, pos):
+    """x [n, heads, D]: pairs of neighbours among the first rope dims."""
+    if rope is None:
+        return x
+    c, s = rope[pos].unbind(-1)
+    c, s = c.unsqueeze(1), s.unsqueeze(1)
+    n = 2 * c.size(-1)
+    u, v = x[..., :n:2], x[..., 1:n:2]
+    r = torch.stack((u * c - v * s, v * c + u * s), -1).flatten(-2)
+    return torch.cat((r, x[..., n:]), -1)
+
+
 def qk_norm_append(q_out, kpages, vpages, proj, q_w, k_w, row_slot, row_pos,
-                   table, vdim, eps) -> None:
+                   table, vdim, eps, rope=None) -> None:
     n, H, dpad = q_out.shape
-    G = kpages.size(1)
     D = q_w.numel()
-    q, k, v = proj.split((H * D, G * D, G * vdim), dim=1)
+    pos = row_pos.long()
+    q = _rotate(_rms(proj[:, :H * D].reshape(n, H, D), eps) * q_w, rope, pos)
     q_out.zero_()
-    q_out[..., :D] = (_rms(q.reshape(n, H, D), eps) * q_w).to(q_out.dtype)
+    q_out[..., :D] = q.to(q_out.dtype)
+    if kpages is None:
+        return
+    G, GV = kpages.size(1), vpages.size(1)
+    _, k, v = proj.split((H * D, G * D, GV * vdim), dim=1)
+    k = _rotate(_rms(k.reshape(n, G, D), eps) * k_w, rope, pos)
+    kv_rows(torch.cat((k.to(proj.dtype).flatten(1), v), 1), kpages, vpages,
+            row_slot, row_pos, table, D, vdim, True)
+
+
+def kv_rows(rows, kpages, vpages, row_slot, row_pos, table, dim, vdim,
+            store) -> None:
+    n, G, GV = rows.size(0), kpages.size(1), vpages.size(1)
     pos = row_pos.long()
     page = table[row_slot.long(), pos // PAGE].long().view(n, 1, 1)
-    head = torch.arange(G).view(1, G, 1)
-    at = k_index(dpad)[pos % PAGE, :D].view(n, 1, D)
-    kpages[page, head, at] = (
-        _rms(k.reshape(n, G, D), eps) * k_w).to(kpages.dtype)
-    at = v_index(vpages.size(2) // PAGE)[pos % PAGE, :vdim].view(n, 1, vdim)
-    vpages[page, head, at] = v.reshape(n, G, vdim)
+    at = 0
+    for pages, heads, size, index in (
+            (kpages, G, dim, k_index(kpages.size(2) // PAGE)),
+            (vpages, GV, vdim, v_index(vpages.size(2) // PAGE))):
+        cols = rows[:, at:at + heads * size].view(n, heads, size)
+        at += heads * size
+        where = (page, torch.arange(heads).view(1, -1, 1),
+                 index[pos % PAGE, :size].view(n, 1, size))
+        if store:
+            pages[where] = cols
+        else:
+            cols.copy_(pages[where])
 
 
 def paged_attn(out, q, kpages, vpages, bias, table, seg, max_len, window,
-               keep_first, scale, splits, part_o=None, part_ml=None) -> None:
-    _, H, D = q.shape
-    G = kpages.size(1)
+               keep_first, scale, splits, part_o=None, part_ml=None,
+               softcap=0.0, map_weight=0.0, out_scale=1.0, eps=0.0) -> None:
+    """Two key heads per value head: each query head has two maps, and what
+    is stored is the unit-size difference of their outputs."""
+    D = q.size(2)
+    GV = vpages.size(1)
+    maps = kpages.size(1) // GV
+    H = q.size(1) // maps
     E = out.size(1) // H
     ki, vi = k_index(D), v_index(vpages.size(2) // PAGE)[:, :E]
     far = bias.size(1) - 1
@@ -101,17 +139,25 @@ def paged_attn(out, q, kpages, vpages, bias, table, seg, max_len, window,
         pages = table[slot, : -(-total // PAGE)].long()
         k, v = (t[pages][:, :, at].transpose(0, 1).flatten(1, 2)[:, :total]
                 for t, at in ((kpages, ki), (vpages, vi)))
-        k = k.float().repeat_interleave(H // G, 0)
-        v = v.float().repeat_interleave(H // G, 0)
+        k = k.float().view(GV, maps, total, D).repeat_interleave(H // GV, 0)
+        v = v.float().repeat_interleave(H // GV, 0).unsqueeze(1)
         i = torch.arange(pos0, total).view(-1, 1)
         j = torch.arange(total).view(1, -1)
         d = i - j
         ok = (d >= 0) & ((d < window) | (j < keep_first))
-        s = q[start:start + n].float().transpose(0, 1) @ k.transpose(1, 2)
+        rows = q[start:start + n].float().view(n, H, maps, D)
+        s = rows.permute(1, 2, 0, 3) @ k.transpose(2, 3) * scale
+        if softcap:
+            s = softcap * torch.tanh(s / softcap)
         # the bias table is in log2 units (see the HIP kernel)
-        s = s * scale + bias[:, d.clamp(0, far)] * 0.6931471805599453
+        s = s + bias[:, d.clamp(0, far)].unsqueeze(1) * 0.6931471805599453
         p = s.masked_fill(~ok, float("-inf")).softmax(-1)
-        out[start:start + n] = (p @ v).transpose(0, 1).reshape(n, -1)
+        o = p @ v                                       # [H, maps, n, E]
+        if maps == 2:
+            o = _rms(o[:, 0] - map_weight * o[:, 1], eps) * out_scale
+        else:
+            o = o[:, 0]
+        out[start:start + n] = o.transpose(0, 1).reshape(n, -1).to(out.dtype)
 
 
 def _rows(pages, table, slot, first, end, n_cols):
@@ -215,11 +261,22 @@ def gated_act(out, gate, up, act) -> None:
     out.copy_(_act(gate.float(), act) * up.float())
 
 
-def moe_route(weight, x, router, top, tile_rows=16):
+def moe_route(weight, x, router, top, tile_rows=16, correction=None,
+              scale=1.0, identity=0, gated=False):
     """Fills the weights [n, top]; returns the plan of the expert products
-    (here: the chosen experts [n, top])."""
-    z, experts = (x.float() @ router.float().t()).topk(top, -1)
-    weight.copy_(z.softmax(-1))
+    (here: the chosen outputs [n, top])."""
+    z = x.float() @ router.float().t()
+    if gated:
+        weight[:, top] = torch.sigmoid(z[:, -1])
+        z = z[:, :-1]
+    if correction is None:
+        z, experts = z.topk(top, -1)
+        weight.copy_(z.softmax(-1))
+        return experts
+    s = z.softmax(-1)
+    experts = (s + correction).topk(top, -1).indices
+    s = s.gather(1, experts)
+    weight[:, :top] = s / (s.sum(-1, keepdim=True) + 1e-20) * scale
     return experts
 
 
@@ -227,19 +284,141 @@ def moe_up(out, x, w, plan, act, tile_rows=16) -> None:
     n, top = plan.shape
     for t in range(n):
         for k in range(top):
-            gate, up = (w[plan[t, k]].float() @ x[t].float()).chunk(2)
-            out[t * top + k] = (_act(gate, act) * up).to(out.dtype)
+            if plan[t, k] < w.size(0):
+                gate, up = (w[plan[t, k]].float() @ x[t].float()).chunk(2)
+                out[t * top + k] = (_act(gate, act) * up).to(out.dtype)
 
 
 def moe_down(out, mid, w, plan, tile_rows=16) -> None:
     n, top = plan.shape
     for t in range(n):
         for k in range(top):
-            out[t, k] = (w[plan[t, k]].float()
-                         @ mid[t * top + k].float()).to(out.dtype)
+            if plan[t, k] < w.size(0):
+                out[t, k] = (w[plan[t, k]].float()
+                             @ mid[t * top + k].float()).to(out.dtype)
 
 
 def advance_batch(slots, sampled, pos, tokens, spare) -> None:
     live = slots != spare
     tokens[live] = sampled[live]
     pos[live] += 1
+
+
+def _group_rms(x, groups, eps):
+    return _rms(x.reshape(x.size(0), groups, -1), eps).flatten(1)
+
+
+def stream_step(x, y=None, post_w=None, xn=None, next_w=None, groups=1,
+                eps=1e-6, tokens=None, table=None, scale=1.0, routed=None,
+                routed_w=None, chosen=None, experts=0, hist=None, coef=None,
+                keep=None, shift=None, prev=None, row_slot=None,
+                row_pos=None) -> None:
+    if tokens is not None:
+        x.copy_(table[tokens.long()].float() * scale)
+    elif y is not None or routed is not None:
+        a = torch.zeros_like(x) if y is None else y.float()
+        if routed is not None:
+            n, top, _ = routed.shape
+            if y is not None:
+                a = a * routed_w[:, top:]
+            same = chosen.reshape(-1)[:n * top].view(n, top, 1) >= experts
+            rows = torch.where(same, x.unsqueeze(1), routed.float())
+            a = a + (rows * routed_w[:, :top].unsqueeze(-1)).sum(1)
+        if post_w is not None:
+            a = _group_rms(a, groups, eps) * post_w
+        x += a
+    if keep is not None:
+        keep.copy_(x)
+    if coef is not None:
+        x.copy_((hist * coef[:-1].view(-1, 1, 1)).sum(0) + coef[-1] * x)
+    if xn is None:
+        return
+    if next_w is not None:
+        xn.copy_(_group_rms(x, groups, eps) * next_w)
+    elif shift is not None:
+        slot = row_slot.long()
+        before = torch.where(row_pos.view(-1, 1) > 0, prev[slot], 0.0)
+        xn.copy_(x + (before - x) * shift)
+        prev[slot] = x
+    else:
+        xn.copy_(x)
+
+
+def token_shift(xn, x, shift, prev, seg, max_len) -> None:
+    for start, n, slot, pos0 in _segments(seg):
+        h = x[start:start + n]
+        first = prev[slot] if pos0 else torch.zeros_like(prev[slot])
+        before = torch.cat((first.unsqueeze(0), h[:-1]))
+        xn[start:start + n] = (h + (before - h) * shift).to(xn.dtype)
+        prev[slot] = h[-1]
+
+
+def gelu(z) -> None:
+    z.copy_(torch.nn.functional.gelu(z.float()))
+
+
+def causal_conv(out, x, w, bias, in_bias, state, seg, max_len, act) -> None:
+    back = w.size(0) - 1
+    for start, n, slot, pos0 in _segments(seg):
+        raw = torch.cat((state[slot][:back], x[start:start + n]))
+        rows = raw.float()
+        if in_bias is not None:
+            rows = rows + in_bias
+        rows[:max(0, back - pos0)] = 0.0    # before the sequence's start
+        y = bias + sum(w[k] * rows[k:k + n] for k in range(back + 1))
+        if act:
+            y = torch.nn.functional.silu(y)
+        out[start:start + n] = y.to(out.dtype)
+        if back:
+            state[slot] = raw[-back:]
+
+
+def rglru_scan(out, u, y, y_bias, gates, gate_bias, rate, state, seg,
+               max_len) -> None:
+    B = gates.size(0) // 2
+    z = torch.einsum("nbk,gbmk->gnbm", u.float().unflatten(1, (B, -1)),
+                     gates.float().unflatten(0, (2, B)))
+    z = z + gate_bias.view(2, 1, B, -1)
+    r, i = torch.sigmoid(z).flatten(2)
+    log_a = rate * r
+    a, x = log_a.exp(), (-(2 * log_a).expm1()).sqrt() * i * u.float()
+    g = _act(y.float() + y_bias, 1)
+    for start, n, slot, pos0 in _segments(seg):
+        S = state[slot].clone() if pos0 else torch.zeros_like(state[slot])
+        for t in range(start, start + n):
+            S = a[t] * S + x[t]
+            out[t] = (S * g[t]).to(out.dtype)
+        state[slot] = S
+
+
+def rglru_step(out, u, y, y_bias, gates, gate_bias, rate, state, seg) -> None:
+    rglru_scan(out, u, y, y_bias, gates, gate_bias, rate, state, seg, 1)
+
+
+def mamba2_scan(o, xbc, dt, state, dt_bias, rate, vdim, seg, max_len) -> None:
+    _, H, N, _ = state.shape
+    inner = H * vdim
+    G = (xbc.size(1) - inner) // (2 * N)
+    x, B, C = xbc.float().split((inner, G * N, G * N), 1)
+    B, C = (t.reshape(-1, G, N).repeat_interleave(H // G, 1) for t in (B, C))
+    dt = torch.nn.functional.softplus(dt.float() + dt_bias)
+    decay = (rate * dt).exp()
+    for start, n, slot, pos0 in _segments(seg):
+        S = state[slot] if pos0 else torch.zeros_like(state[slot])
+        for t in range(start, start + n):
+            S = decay[t].view(H, 1, 1) * S
+            S[..., :vdim] += (dt[t].view(H, 1) * B[t]).unsqueeze(-1) \
+                * x[t].view(H, 1, vdim)
+            o[t] = (S[..., :vdim] * C[t].unsqueeze(-1)).sum(1).view(-1)
+        state[slot] = S
+
+
+def mamba2_step(o, xbc, dt, state, dt_bias, rate, vdim, seg) -> None:
+    mamba2_scan(o, xbc, dt, state, dt_bias, rate, vdim, seg, 1)
+
+
+def mamba2_out(out, o, xbc, z, skip, w, groups, eps) -> None:
+    n, inner = o.shape
+    y = o + (xbc[:, :inner].float().view(n, skip.numel(), -1)
+             * skip.view(1, -1, 1)).view(n, inner)
+    out.copy_(_group_rms(y * _act(z.float(), 0), groups, eps) * w)

@@ -26,12 +26,11 @@ from typing import List, Optional, Tuple
 import torch
 
 from ..models.cache import PAGE
+from .experts import ACTS, RoutedExperts
 
-__all__ = ["LatentPlan", "ParallelLayer", "ACTS"]
+__all__ = ["LatentPlan", "ParallelLayer"]
 
-ACTS = {"silu": 0, "gelu_tanh": 1}
 MAX_EXPANDED = 256      # head sizes of the expanded form
-BIG_TILE = 128          # pairs of one expert in a tile of large batches
 
 
 def _round_up(n: int, k: int) -> int:
@@ -137,19 +136,8 @@ class ParallelLayer:
             pre = "shared." if mlp.kind == "moe" else ""
             self.gate, self.up = self.part[pre + "gate"], self.part[pre + "up"]
         self.act = ACTS[mlp.act] if mlp is not None else 0
-        self.routed = mlp is not None and mlp.kind == "moe"
-        if self.routed:
-            self.experts, self.top = mlp.experts, mlp.top
-            self.expert_ff = mlp.expert_ff
-            self.router = mlp.router.weight.detach()
-            self.e_up = mlp.up.weight.detach().view(
-                mlp.experts, 2 * mlp.expert_ff, -1)
-            self.e_down = mlp.down.weight.detach().view(
-                mlp.experts, -1, mlp.expert_ff)
-            width = self.router.size(1)
-            self.big_tiles = eng.dtype == torch.bfloat16 \
-                and mlp.expert_ff % 64 == 0 and mlp.expert_ff >= 128 \
-                and width % 64 == 0 and width >= 256
+        self.experts = RoutedExperts(eng, mlp) \
+            if mlp is not None and mlp.kind == "moe" else None
 
     # ------------------------------------------------------------------
     def _new(self, *shape, dtype=None) -> torch.Tensor:
@@ -167,7 +155,7 @@ class ParallelLayer:
             branch = dict(act_out=y[:, m.out_cols:], gate=proj[:, self.gate],
                           up=proj[:, self.up], act=self.act)
         self._attend(b, proj, y[:, :m.out_cols], branch)
-        routed = self._experts(b, xn) if self.routed else None
+        routed = self.experts(xn)[:2] if self.experts else None
         return self.eng._linear(y, self.out_proj), routed
 
     # -- attention ------------------------------------------------------
@@ -230,18 +218,3 @@ class ParallelLayer:
         kv = e._linear(ctx, self.kv_up)
         e.ops.head_attn(y, q, kv, plan.long_seg, plan.ctx_seg, plan.long_max,
                         m.heads, m.dim, m.vdim, m.window, m.scale, gate)
-
-    # -- experts --------------------------------------------------------
-    def _experts(self, b, xn: torch.Tensor):
-        ops, n, F = self.eng.ops, b.n, self.expert_ff
-        # pairs (row, choice) per expert decide the tile
-        tile = BIG_TILE if self.big_tiles and \
-            n * self.top >= BIG_TILE // 2 * self.experts and \
-            n * max(xn.size(1), self.top * F) < 1 << 30 else 16
-        weight = self._new(n, self.top, dtype=torch.float32)
-        plan = ops.moe_route(weight, xn, self.router, self.top, tile)
-        mid = self._new(n * self.top, F)
-        ops.moe_up(mid, xn, self.e_up, plan, self.act, tile)
-        out = self._new(n, self.top, xn.size(1))
-        ops.moe_down(out, mid, self.e_down, plan, tile)
-        return out, weight

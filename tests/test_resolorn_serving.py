@@ -37,7 +37,7 @@ def test_config_round_trips(tmp_path):
     c = ModelConfig.from_native(cfg)
     assert c.is_hybrid and c.n_layer == 5 and c.padded_vocab_size == 133
     assert c.parallel_residual and c.block_size == 512
-    assert c.shared_latents() == {0: 56, 2: 88}
+    assert c.shared_rows() == {0: 56, 2: 88}
     assert c.ring_width == 72 + 56 + 88
     assert ModelConfig.from_dict(c.to_dict()).to_dict() == c.to_dict()
     c.save(tmp_path / "model_config.yaml")
@@ -54,7 +54,7 @@ def test_registry(name):
     c = ModelConfig.from_name(name)
     assert c.is_hybrid and c.parallel_residual
     assert {l["mlp"]["kind"] for l in c.layers} == {"dense", "moe"}
-    assert len(c.shared_latents()) == c.n_layer // 2
+    assert len(c.shared_rows()) == c.n_layer // 2
 
 
 def test_weight_counts_follow_the_tensors():
