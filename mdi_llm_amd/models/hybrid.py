@@ -177,6 +177,8 @@ class DiffAttention(nn.Module):
 
 
 class XieluMLP(nn.Module):
+    kind = "dense"
+
     def __init__(self, width: int, spec: dict) -> None:
         super().__init__()
         self.fc = nn.Linear(width, spec["ff"], bias=False)

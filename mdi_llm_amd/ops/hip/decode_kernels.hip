@@ -232,11 +232,16 @@ __global__ void layernorm_kernel(bf16* __restrict__ out,
 // kernel + a global round-trip per call): after staging raw x, the block
 // reduces mean/meansq and rewrites LDS with the normalized+weighted value.
 // NORM: 0 none, 1 RMSNorm, 2 LayerNorm.
-// EPI:  0 none, 1 +residual, 2 gelu(tanh), 3 silu, 4 xielu(act_p, act_q).
+// EPI:  0 none, 1 +residual, 2 gelu(tanh), 3 silu, 4 xielu(act_p, act_q),
+// 5 gelu(erf).
 // ---------------------------------------------------------------------------
 DEVINL float gelu_tanh(float v) {
   float c = 0.7978845608028654f * (v + 0.044715f * v * v * v);
   return 0.5f * v * (1.f + tanhf(c));
+}
+
+DEVINL float gelu_erf(float v) {
+  return 0.5f * v * (1.f + erff(0.7071067811865476f * v));
 }
 
 // z/2 plus p z^2 above zero, (1/2 + q)(e^z - 1 - z) below
@@ -499,6 +504,7 @@ __global__ void gemv_direct_kernel(bf16* __restrict__ out,
         if (EPI == 2) a = gelu_tanh(a);
         if (EPI == 3) a = a / (1.f + expf(-a));
         if (EPI == 4) a = xielu(a, act_p, act_q);
+        if (EPI == 5) a = gelu_erf(a);
         out[rw] = f2b(a);
       }
     }
@@ -3264,6 +3270,7 @@ void launch_gemv(void* out, const void* W, const void* x, const void* bias,
     case 14: GEMV_CASE(3, 2); break;
     case 16: GEMV_CASE(4, 0); break;
     case 17: GEMV_CASE(4, 1); break;
+    case 20: GEMV_CASE(5, 0); break;
     default: GEMV_CASE(0, 0);
   }
 #undef GEMV_CASE

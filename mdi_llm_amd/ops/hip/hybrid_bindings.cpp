@@ -143,6 +143,11 @@ void xielu(torch::Tensor z, double p, double q) {
                cur_stream());
 }
 
+void gelu(torch::Tensor z) {
+  launch_gelu(z.data_ptr(), (long long)z.numel(), act_type(z, "z"),
+              cur_stream());
+}
+
 struct Recurrent {
   int heads, dim, vdim, vstride, f32;
   float* state;
@@ -212,57 +217,127 @@ void hgrn2_scan(torch::Tensor out, torch::Tensor proj, torch::Tensor state,
 }
 
 struct Pages {
-  int kv_heads, dpad, vpad;
+  int kv_heads, maps, dpad, vpad;
 };
 
+// one K page per value head, or two (two maps)
 Pages pages(const torch::Tensor& k, const torch::Tensor& v, int f32) {
   check_like(k, f32, "kpages");
   check_like(v, f32, "vpages");
   TORCH_CHECK(k.dim() == 3 && v.dim() == 3 && k.size(0) == v.size(0) &&
-                  k.size(1) == v.size(1) && k.size(2) % (64 * 32) == 0 &&
-                  v.size(2) % (64 * 32) == 0,
-              "pages: expected k [P, G, 64 * dpad] and v [P, G, 64 * vpad]");
-  return Pages{(int)k.size(1), (int)k.size(2) / 64, (int)v.size(2) / 64};
+                  (k.size(1) == v.size(1) || k.size(1) == 2 * v.size(1)) &&
+                  k.size(2) % (64 * 32) == 0 && v.size(2) % (64 * 32) == 0,
+              "pages: expected k [P, G * maps, 64 * dpad] and v [P, G, 64 * "
+              "vpad]");
+  return Pages{(int)v.size(1), (int)(k.size(1) / v.size(1)),
+               (int)k.size(2) / 64, (int)v.size(2) / 64};
 }
 
-void qk_norm_append(torch::Tensor q_out, torch::Tensor kpages,
-                    torch::Tensor vpages, torch::Tensor proj,
-                    torch::Tensor q_w, torch::Tensor k_w,
-                    torch::Tensor row_slot, torch::Tensor row_pos,
-                    torch::Tensor table, int64_t vdim, double eps) {
-  const int f32 = act_type(proj, "proj");
-  const Pages pg = pages(kpages, vpages, f32);
-  check_like(q_out, f32, "q_out");
-  const int n = (int)proj.size(0), dim = (int)q_w.numel();
-  TORCH_CHECK(q_out.dim() == 3 && q_out.size(0) == n &&
-                  q_out.size(2) == pg.dpad && dim <= pg.dpad &&
-                  vdim <= pg.vpad,
-              "q_out must be [n, H, dpad]");
-  const int heads = (int)q_out.size(1);
-  TORCH_CHECK(proj.size(1) ==
-                  (heads + pg.kv_heads) * dim + pg.kv_heads * vdim,
-              "proj columns");
+void set_places(QkAppendArgs& a, const torch::Tensor& row_slot,
+                const torch::Tensor& row_pos, const torch::Tensor& table) {
   TORCH_CHECK(table.dim() == 2, "table must be [slots, pages]");
-  launch_qk_norm_append(
-      q_out.data_ptr(), kpages.data_ptr(), vpages.data_ptr(),
-      proj.data_ptr(), f32_ptr(q_w, dim, "q_w"), f32_ptr(k_w, dim, "k_w"),
-      i32_ptr(row_slot, n, "row_slot"), i32_ptr(row_pos, n, "row_pos"),
-      i32_ptr(table, table.numel(), "table"), (int)table.size(1), n, heads,
-      pg.kv_heads, dim, (int)vdim, pg.dpad, pg.vpad, (float)eps, f32,
-      cur_stream());
+  a.row_slot = i32_ptr(row_slot, a.n, "row_slot");
+  a.row_pos = i32_ptr(row_pos, a.n, "row_pos");
+  a.table = i32_ptr(table, table.numel(), "table");
+  a.table_stride = (int)table.size(1);
+}
+
+void set_pages(QkAppendArgs& a, const torch::Tensor& kpages,
+               const torch::Tensor& vpages, int64_t dim, int64_t vdim,
+               int f32) {
+  const Pages pg = pages(kpages, vpages, f32);
+  a.kpages = kpages.data_ptr();
+  a.vpages = vpages.data_ptr();
+  a.k_heads = pg.kv_heads * pg.maps;
+  a.v_heads = pg.kv_heads;
+  a.dim = (int)dim;
+  a.vdim = (int)vdim;
+  a.dpad = pg.dpad;
+  a.vpad = pg.vpad;
+  TORCH_CHECK(dim > 0 && dim <= pg.dpad && vdim > 0 && vdim <= pg.vpad,
+              "head sizes of the pages");
+}
+
+void qk_norm_append(torch::Tensor q_out, Opt kpages, Opt vpages,
+                    torch::Tensor proj, torch::Tensor q_w, Opt k_w,
+                    torch::Tensor row_slot, torch::Tensor row_pos,
+                    torch::Tensor table, int64_t vdim, double eps, Opt rope) {
+  const int f32 = act_type(proj, "proj");
+  check_like(q_out, f32, "q_out");
+  QkAppendArgs a{};
+  TORCH_CHECK(proj.dim() == 2 && q_out.dim() == 3 &&
+                  q_out.size(0) == proj.size(0) && q_out.size(2) % 32 == 0 &&
+                  q_out.size(2) <= 256,
+              "q_out must be [n, H, dpad]");
+  TORCH_CHECK(!!kpages == !!vpages && !!kpages == !!k_w,
+              "qk_norm_append: bad combination of operands");
+  a.n = (int)proj.size(0);
+  a.heads = (int)q_out.size(1);
+  a.dim = (int)q_w.numel();
+  a.vdim = (int)vdim;
+  a.dpad = (int)q_out.size(2);
+  TORCH_CHECK(a.n > 0 && a.dim > 0 && a.dim <= a.dpad, "q_out columns");
+  if (kpages) {
+    set_pages(a, *kpages, *vpages, a.dim, vdim, f32);
+    TORCH_CHECK(a.dpad == q_out.size(2), "q_out must be [n, H, dpad]");
+    a.k_w = f32_ptr(*k_w, a.dim, "k_w");
+  }
+  TORCH_CHECK(proj.size(1) == (a.heads + a.k_heads) * a.dim + a.v_heads * vdim,
+              "proj columns");
+  if (rope) {
+    // (positions beyond the table are the caller's limit on sequences)
+    TORCH_CHECK(rope->dim() == 3 && rope->size(2) == 2 &&
+                    2 * rope->size(1) <= a.dim,
+                "rope must be [positions, pairs, 2]");
+    TORCH_CHECK(rope->size(0) > 0, "rope positions");
+    a.rope = f32_ptr(*rope, rope->numel(), "rope");
+    a.rot = 2 * (int)rope->size(1);
+  }
+  a.q_out = q_out.data_ptr();
+  a.proj = proj.data_ptr();
+  a.q_w = f32_ptr(q_w, a.dim, "q_w");
+  a.eps = (float)eps;
+  set_places(a, row_slot, row_pos, table);
+  launch_qk_norm_append(a, f32, cur_stream());
+}
+
+void kv_rows(torch::Tensor rows, torch::Tensor kpages, torch::Tensor vpages,
+             torch::Tensor row_slot, torch::Tensor row_pos,
+             torch::Tensor table, int64_t dim, int64_t vdim, bool store) {
+  const int f32 = act_type(rows, "rows");
+  QkAppendArgs a{};
+  set_pages(a, kpages, vpages, dim, vdim, f32);
+  TORCH_CHECK(rows.dim() == 2 && rows.size(0) > 0 &&
+                  rows.size(1) == a.k_heads * dim + a.v_heads * vdim,
+              "kv_rows: columns");
+  a.n = (int)rows.size(0);
+  set_places(a, row_slot, row_pos, table);
+  launch_kv_rows(a, rows.data_ptr(), store ? 1 : 0, f32, cur_stream());
 }
 
 void paged_attn(torch::Tensor out, torch::Tensor q, torch::Tensor kpages,
                 torch::Tensor vpages, torch::Tensor bias,
                 torch::Tensor table, torch::Tensor seg, int64_t max_len,
                 int64_t window, int64_t keep_first, double scale,
-                int64_t splits, Opt part_o, Opt part_ml) {
+                int64_t splits, Opt part_o, Opt part_ml, double softcap,
+                double map_weight, double out_scale, double eps) {
   const int f32 = act_type(q, "q");
   const Pages pg = pages(kpages, vpages, f32);
   check_like(out, f32, "out");
-  TORCH_CHECK(q.dim() == 3 && q.size(2) == pg.dpad, "q must be [n, H, dpad]");
+  TORCH_CHECK(q.dim() == 3 && q.size(2) == pg.dpad &&
+                  q.size(1) % pg.maps == 0,
+              "q must be [n, H * maps, dpad]");
   PagedAttnArgs a{};
-  a.heads = (int)q.size(1);
+  a.maps = pg.maps;
+  a.heads = (int)q.size(1) / pg.maps;
+  TORCH_CHECK(softcap >= 0.0, "softcap");
+  if (softcap > 0.0) {
+    a.cap_in = (float)(scale / softcap);
+    a.cap_log2 = (float)(softcap * 1.4426950408889634);
+  }
+  a.map_weight = (float)map_weight;
+  a.out_scale = (float)out_scale;
+  a.eps = (float)eps;
   a.kv_heads = pg.kv_heads;
   TORCH_CHECK(a.heads % a.kv_heads == 0, "heads per kv head");
   TORCH_CHECK(out.dim() == 2 && out.size(0) == q.size(0) &&
@@ -291,10 +366,12 @@ void paged_attn(torch::Tensor out, torch::Tensor q, torch::Tensor kpages,
   a.splits = (int)splits;
   a.max_len = (int)max_len;
   TORCH_CHECK(splits >= 0 && max_len > 0, "splits and max_len");
-  if (splits > 1) {
-    TORCH_CHECK(max_len == 1, "split keys: one token per segment");
+  TORCH_CHECK(splits <= 1 || max_len == 1,
+              "split keys: one token per segment");
+  if (splits > 1 || (splits == 1 && a.maps > 1)) {
+    TORCH_CHECK(max_len == 1, "two maps: parts hold one token per segment");
     TORCH_CHECK(part_o && part_ml, "split keys need scratch");
-    const int64_t cells = (int64_t)a.seg.n * a.heads * splits;
+    const int64_t cells = (int64_t)a.seg.n * a.heads * a.maps * splits;
     TORCH_CHECK(part_o->numel() >= cells * a.vpad &&
                     part_ml->numel() >= cells * 2,
                 "split scratch too small");
@@ -303,8 +380,10 @@ void paged_attn(torch::Tensor out, torch::Tensor q, torch::Tensor kpages,
     a.part_ml = const_cast<float*>(
         f32_ptr(*part_ml, part_ml->numel(), "part_ml"));
   }
-  const int rc = f32 ? launch_paged_attn_f32(a, cur_stream())
-                     : launch_paged_attn_bf16(a, cur_stream());
+  const auto launch =
+      a.maps == 2 ? (f32 ? launch_diff_attn_f32 : launch_diff_attn_bf16)
+                  : (f32 ? launch_paged_attn_f32 : launch_paged_attn_bf16);
+  const int rc = launch(a, cur_stream());
   TORCH_CHECK(rc == 0, "paged_attn: unsupported padded sizes ", a.dpad, ", ",
               a.vpad);
 }
@@ -580,26 +659,35 @@ MoePlan plan_of(const torch::Tensor& w, const torch::Tensor& plan,
 
 torch::Tensor moe_route(torch::Tensor weight, torch::Tensor x,
                         torch::Tensor router, int64_t top,
-                        int64_t tile_rows) {
+                        int64_t tile_rows, Opt correction, double scale,
+                        int64_t identity, bool gated) {
   const int f32 = act_type(x, "x");
   check_like(router, f32, "router");
   TORCH_CHECK(x.dim() == 2 && router.dim() == 2 &&
                   router.size(1) == x.size(1),
               "moe_route: sizes");
-  const int n = (int)x.size(0), e = (int)router.size(0);
-  TORCH_CHECK(n > 0 && e <= 256 && top >= 1 && top <= e && top <= 64,
-              "moe_route: at most 256 experts, 64 of them for a token");
-  float* wp = const_cast<float*>(f32_ptr(weight, n * top, "weight"));
+  const int n = (int)x.size(0), cols = (int)router.size(0);
+  const int outputs = cols - (gated ? 1 : 0);
+  TORCH_CHECK(n > 0 && outputs <= 256 && top >= 1 && top <= outputs &&
+                  top <= 64,
+              "moe_route: at most 256 outputs, 64 of them for a token");
+  TORCH_CHECK(identity >= 0 && identity < outputs, "moe_route: identity");
+  float* wp = const_cast<float*>(
+      f32_ptr(weight, n * (top + (gated ? 1 : 0)), "weight"));
   check_tile_rows(tile_rows, f32, x.size(1));
+  const int e = outputs - (int)identity;
   torch::Tensor plan =
       torch::empty({moe_plan_ints(n, (int)top, e, (int)tile_rows)},
                    x.options().dtype(torch::kInt32));
   torch::Tensor z =
-      torch::empty({n, e}, x.options().dtype(torch::kFloat32));
+      torch::empty({n, cols}, x.options().dtype(torch::kFloat32));
+  MoePlan p = moe_plan(plan.data_ptr<int>(), n, (int)top, e, (int)tile_rows);
+  p.outputs = outputs;
+  p.gated = gated ? 1 : 0;
+  p.scale = (float)scale;
+  if (correction) p.correction = f32_ptr(*correction, outputs, "correction");
   launch_moe_route(wp, z.data_ptr<float>(), x.data_ptr(), router.data_ptr(),
-                   moe_plan(plan.data_ptr<int>(), n, (int)top, e,
-                            (int)tile_rows),
-                   n, (int)x.size(1), f32, cur_stream());
+                   p, n, (int)x.size(1), f32, cur_stream());
   return plan;
 }
 
@@ -646,7 +734,8 @@ void moe_down(torch::Tensor out, torch::Tensor mid, torch::Tensor w,
 }
 
 void skinny_gemm(torch::Tensor out, torch::Tensor w, torch::Tensor x,
-                 bool act, double act_p, double act_q) {
+                 int64_t act, double act_p, double act_q) {
+  TORCH_CHECK(act >= 0 && act <= 2, "skinny_gemm: act");
   TORCH_CHECK(x.dim() == 2 && w.dim() == 2 && out.dim() == 2, "2-D operands");
   const int n = (int)x.size(0), m = (int)w.size(0), k = (int)x.size(1);
   for (const auto* t : {&out, &w, &x})
@@ -654,9 +743,275 @@ void skinny_gemm(torch::Tensor out, torch::Tensor w, torch::Tensor x,
   TORCH_CHECK(w.size(1) == k && out.size(0) == n && out.size(1) == m,
               "skinny_gemm: sizes");
   const int rc = launch_skinny_gemm(out.data_ptr(), w.data_ptr(),
-                                    x.data_ptr(), n, m, k, act ? 1 : 0,
+                                    x.data_ptr(), n, m, k, (int)act,
                                     (float)act_p, (float)act_q, cur_stream());
   TORCH_CHECK(rc == 0, "skinny_gemm: unsupported n ", n, " or k ", k);
+}
+
+void stream_step(torch::Tensor x, Opt y, Opt post_w, Opt xn, Opt next_w,
+                 int64_t groups, double eps, Opt tokens, Opt table,
+                 double scale, Opt routed, Opt routed_w, Opt chosen,
+                 int64_t experts, Opt hist, Opt coef, Opt keep, Opt shift,
+                 Opt prev, Opt row_slot, Opt row_pos) {
+  TORCH_CHECK(x.dim() == 2 && x.size(0) > 0, "x must be [n, e]");
+  const int64_t n = x.size(0), e = x.size(1);
+  StreamArgs a{};
+  a.x = const_cast<float*>(f32_ptr(x, n * e, "x"));
+  TORCH_CHECK(groups > 0 && e % groups == 0, "stream_step: groups");
+  TORCH_CHECK(!(tokens && (y || routed)) && !!tokens == !!table &&
+                  !!routed == !!routed_w && !!routed == !!chosen &&
+                  !!hist == !!coef && !!shift == !!prev &&
+                  !!shift == !!row_slot && !!shift == !!row_pos &&
+                  !(next_w && shift) && (xn || (!next_w && !shift)),
+              "stream_step: bad combination of operands");
+  const torch::Tensor* act =
+      y ? &*y : routed ? &*routed : xn ? &*xn : table ? &*table : nullptr;
+  const int f32 = act ? act_type(*act, "activation") : 0;
+  if (y) {
+    check_like(*y, f32, "y");
+    TORCH_CHECK(y->numel() == n * e, "y size");
+    a.y = y->data_ptr();
+  }
+  if (xn) {
+    check_like(*xn, f32, "xn");
+    TORCH_CHECK(xn->numel() == n * e, "xn size");
+    a.xn = xn->data_ptr();
+  }
+  if (table) {
+    check_like(*table, f32, "table");
+    TORCH_CHECK(table->dim() == 2 && table->size(1) == e, "table size");
+    a.table = table->data_ptr();
+    a.tokens = i32_ptr(*tokens, n, "tokens");
+  }
+  if (routed) {
+    check_like(*routed, f32, "routed");
+    TORCH_CHECK(routed->dim() == 3 && routed->size(0) == n &&
+                    routed->size(2) == e,
+                "routed must be [n, top, e]");
+    a.top = (int)routed->size(1);
+    a.routed = routed->data_ptr();
+    a.routed_w = f32_ptr(*routed_w, n * (a.top + (y ? 1 : 0)), "routed_w");
+    a.chosen = i32_ptr(*chosen, n * a.top, "chosen");
+    a.experts = (int)experts;
+  }
+  if (post_w) a.post_w = f32_ptr(*post_w, e, "post_w");
+  if (next_w) a.next_w = f32_ptr(*next_w, e, "next_w");
+  if (hist) {
+    TORCH_CHECK(hist->dim() == 3, "hist must be [depth, n, e]");
+    a.depth = (int)hist->size(0);
+    a.hist = f32_ptr(*hist, a.depth * n * e, "hist");
+    a.coef = f32_ptr(*coef, a.depth + 1, "coef");
+  }
+  if (keep) a.keep = const_cast<float*>(f32_ptr(*keep, n * e, "keep"));
+  if (shift) {
+    a.shift = f32_ptr(*shift, e, "shift");
+    TORCH_CHECK(prev->dim() == 2 && prev->size(1) == e,
+                "prev must be [slots, e]");
+    a.prev = const_cast<float*>(f32_ptr(*prev, prev->numel(), "prev"));
+    a.row_slot = i32_ptr(*row_slot, n, "row_slot");
+    a.row_pos = i32_ptr(*row_pos, n, "row_pos");
+  }
+  a.groups = (int)groups;
+  a.n = (int)n;
+  a.e = (int)e;
+  a.scale = (float)scale;
+  a.eps = (float)eps;
+  TORCH_CHECK(launch_stream_step(a, f32, cur_stream()) == 0,
+              "stream_step: row of ", e, " elements");
+}
+
+void token_shift(torch::Tensor xn, torch::Tensor x, torch::Tensor shift,
+                 torch::Tensor prev, torch::Tensor seg, int64_t max_len) {
+  const int f32 = act_type(xn, "xn");
+  TORCH_CHECK(x.dim() == 2 && xn.numel() == x.numel() && x.size(0) > 0,
+              "token_shift: sizes");
+  const int64_t n = x.size(0), e = x.size(1);
+  TORCH_CHECK(prev.dim() == 2 && prev.size(1) == e, "prev must be [slots, e]");
+  TORCH_CHECK(max_len > 0 && max_len <= n, "max_len");
+  launch_token_shift(
+      xn.data_ptr(), f32_ptr(x, n * e, "x"), f32_ptr(shift, e, "shift"),
+      const_cast<float*>(f32_ptr(prev, prev.numel(), "prev")), seg_view(seg),
+      (int)max_len, (int)e, f32, cur_stream());
+}
+
+void causal_conv(torch::Tensor out, torch::Tensor x, torch::Tensor w,
+                 torch::Tensor bias, Opt in_bias, torch::Tensor state,
+                 torch::Tensor seg, int64_t max_len, bool act) {
+  const int f32 = act_type(out, "out");
+  const Rows r = rows_of(x, f32, "x");
+  check_like(state, f32, "state");
+  ConvArgs a{};
+  TORCH_CHECK(w.dim() == 2 && w.size(1) == r.cols && w.size(0) >= 1 &&
+                  w.size(0) <= 16,
+              "causal_conv: w must be [taps, channels], at most 16 taps");
+  a.taps = (int)w.size(0);
+  a.c = r.cols;
+  TORCH_CHECK(out.numel() == (int64_t)r.n * r.cols && state.dim() == 3 &&
+                  state.size(1) == std::max(1, a.taps - 1) &&
+                  state.size(2) == r.cols && max_len > 0 && max_len <= r.n,
+              "causal_conv: sizes");
+  a.out = out.data_ptr();
+  a.x = r.p;
+  a.ld = r.ld;
+  a.w = f32_ptr(w, w.numel(), "w");
+  a.bias = f32_ptr(bias, r.cols, "bias");
+  if (in_bias) a.in_bias = f32_ptr(*in_bias, r.cols, "in_bias");
+  a.state = state.data_ptr();
+  a.seg = seg_view(seg);
+  a.max_len = (int)max_len;
+  a.act = act ? 1 : 0;
+  const int v = f32 ? 4 : 8;
+  a.vec = r.cols % v == 0 && r.ld % v == 0 && (size_t)r.p % 16 == 0;
+  launch_causal_conv(a, f32, cur_stream());
+}
+
+RgLruArgs rglru_args(const torch::Tensor& out, const torch::Tensor& u,
+                     const torch::Tensor& y, const torch::Tensor& y_bias,
+                     const torch::Tensor& gates,
+                     const torch::Tensor& gate_bias,
+                     const torch::Tensor& rate, const torch::Tensor& state,
+                     const torch::Tensor& seg, int f32) {
+  check_like(u, f32, "u");
+  check_like(gates, f32, "gates");
+  const Rows r = rows_of(y, f32, "y");
+  RgLruArgs a{};
+  TORCH_CHECK(u.dim() == 2 && u.size(0) == r.n && u.size(1) == r.cols &&
+                  out.numel() == u.numel(),
+              "rglru: rows");
+  a.n = r.n;
+  a.width = r.cols;
+  TORCH_CHECK(gates.dim() == 3 && gates.size(0) % 2 == 0 &&
+                  gates.size(1) == gates.size(2) &&
+                  gates.size(0) / 2 * gates.size(1) == a.width,
+              "rglru: gates must be [2 * blocks, part, part]");
+  a.blocks = (int)gates.size(0) / 2;
+  TORCH_CHECK(state.dim() == 2 && state.size(1) == a.width,
+              "rglru: state must be [slots, width]");
+  a.out = out.data_ptr();
+  a.u = u.data_ptr();
+  a.y = r.p;
+  a.y_ld = r.ld;
+  a.y_bias = f32_ptr(y_bias, a.width, "y_bias");
+  a.gates = gates.data_ptr();
+  a.gate_bias = f32_ptr(gate_bias, 2 * a.width, "gate_bias");
+  a.rate = f32_ptr(rate, a.width, "rate");
+  a.state = const_cast<float*>(f32_ptr(state, state.numel(), "state"));
+  a.seg = seg_view(seg);
+  return a;
+}
+
+void rglru_step(torch::Tensor out, torch::Tensor u, torch::Tensor y,
+                torch::Tensor y_bias, torch::Tensor gates,
+                torch::Tensor gate_bias, torch::Tensor rate,
+                torch::Tensor state, torch::Tensor seg) {
+  const int f32 = act_type(out, "out");
+  const RgLruArgs a = rglru_args(out, u, y, y_bias, gates, gate_bias, rate,
+                                 state, seg, f32);
+  launch_rglru_step(a, f32, cur_stream());
+}
+
+void rglru_scan(torch::Tensor out, torch::Tensor u, torch::Tensor y,
+                torch::Tensor y_bias, torch::Tensor gates,
+                torch::Tensor gate_bias, torch::Tensor rate,
+                torch::Tensor state, torch::Tensor seg, int64_t max_len) {
+  const int f32 = act_type(out, "out");
+  RgLruArgs a = rglru_args(out, u, y, y_bias, gates, gate_bias, rate, state,
+                           seg, f32);
+  TORCH_CHECK(max_len > 0 && max_len <= a.n, "max_len");
+  a.max_len = (int)max_len;
+  torch::Tensor work = torch::empty({2, a.n, a.width},
+                                    out.options().dtype(torch::kFloat32));
+  a.work = work.data_ptr<float>();
+  launch_rglru_scan(a, f32, cur_stream());
+}
+
+Mamba2Args mamba2_args(const torch::Tensor& o, const torch::Tensor& xbc,
+                       const torch::Tensor& dt, const torch::Tensor& state,
+                       const torch::Tensor& dt_bias,
+                       const torch::Tensor& rate, int64_t vdim,
+                       const torch::Tensor& seg, int f32) {
+  const Rows d = rows_of(dt, f32, "dt");
+  Mamba2Args a{};
+  TORCH_CHECK(state.dim() == 4, "state must be [slots, H, N, vstride]");
+  a.heads = (int)state.size(1);
+  a.dim = (int)state.size(2);
+  a.vstride = (int)state.size(3);
+  a.vdim = (int)vdim;
+  TORCH_CHECK(a.vstride % 4 == 0 && vdim > 0 && vdim <= a.vstride &&
+                  a.dim <= 256 && a.vstride <= 1024 && d.cols == a.heads,
+              "mamba2: sizes");
+  const int64_t inner = (int64_t)a.heads * vdim;
+  TORCH_CHECK(xbc.dim() == 2 && xbc.size(0) == d.n && xbc.size(1) > inner &&
+                  (xbc.size(1) - inner) % (2 * a.dim) == 0,
+              "mamba2: xbc columns");
+  a.groups = (int)((xbc.size(1) - inner) / (2 * a.dim));
+  TORCH_CHECK(a.heads % a.groups == 0, "mamba2: groups");
+  a.o = const_cast<float*>(f32_ptr(o, d.n * inner, "o"));
+  a.xbc = xbc.data_ptr();
+  a.dt = d.p;
+  a.dt_ld = d.ld;
+  a.state = const_cast<float*>(f32_ptr(state, state.numel(), "state"));
+  a.dt_bias = f32_ptr(dt_bias, a.heads, "dt_bias");
+  a.rate = f32_ptr(rate, a.heads, "rate");
+  a.seg = seg_view(seg);
+  return a;
+}
+
+void mamba2_step(torch::Tensor o, torch::Tensor xbc, torch::Tensor dt,
+                 torch::Tensor state, torch::Tensor dt_bias,
+                 torch::Tensor rate, int64_t vdim, torch::Tensor seg) {
+  const int f32 = act_type(xbc, "xbc");
+  launch_mamba2_step(mamba2_args(o, xbc, dt, state, dt_bias, rate, vdim, seg,
+                                 f32), f32, cur_stream());
+}
+
+void mamba2_scan(torch::Tensor o, torch::Tensor xbc, torch::Tensor dt,
+                 torch::Tensor state, torch::Tensor dt_bias,
+                 torch::Tensor rate, int64_t vdim, torch::Tensor seg,
+                 int64_t max_len) {
+  const int f32 = act_type(xbc, "xbc");
+  Mamba2Args a =
+      mamba2_args(o, xbc, dt, state, dt_bias, rate, vdim, seg, f32);
+  TORCH_CHECK(max_len > 0 && max_len <= xbc.size(0), "max_len");
+  a.max_len = (int)max_len;
+  torch::Tensor work = torch::empty(
+      {hgrn2_work_floats((int)xbc.size(0), a.seg.n, a.heads, a.dim)},
+      o.options());
+  a.work = work.data_ptr<float>();
+  TORCH_CHECK(launch_mamba2_scan(a, f32, cur_stream()) == 0,
+              "mamba2_scan: unsupported state ", a.dim);
+}
+
+void mamba2_out(torch::Tensor out, torch::Tensor o, torch::Tensor xbc,
+                torch::Tensor z, torch::Tensor skip, torch::Tensor w,
+                int64_t groups, double eps) {
+  const int f32 = act_type(out, "out");
+  const Rows x = rows_of(xbc, f32, "xbc"), zr = rows_of(z, f32, "z");
+  GatedNormArgs a{};
+  a.n = zr.n;
+  a.inner = zr.cols;
+  const int heads = (int)skip.numel();
+  TORCH_CHECK(x.n == a.n && x.cols >= a.inner && heads > 0 &&
+                  a.inner % heads == 0 && groups > 0 &&
+                  a.inner % groups == 0 &&
+                  out.numel() == (int64_t)a.n * a.inner,
+              "mamba2_out: sizes");
+  a.vdim = a.inner / heads;
+  a.groups = (int)groups;
+  a.out = out.data_ptr();
+  a.o = f32_ptr(o, (int64_t)a.n * a.inner, "o");
+  a.x = x.p;
+  a.z = zr.p;
+  a.xld = x.ld;
+  a.zld = zr.ld;
+  a.skip = f32_ptr(skip, heads, "skip");
+  a.w = f32_ptr(w, a.inner, "w");
+  a.eps = (float)eps;
+  const size_t bytes = f32 ? 16 : 8;
+  a.vec = x.ld % 4 == 0 && zr.ld % 4 == 0 && (size_t)x.p % bytes == 0 &&
+          (size_t)zr.p % bytes == 0;
+  TORCH_CHECK(launch_gated_norm(a, f32, cur_stream()) == 0,
+              "mamba2_out: row of ", a.inner, " elements");
 }
 
 void advance_batch(torch::Tensor slots, torch::Tensor sampled,
@@ -684,6 +1039,50 @@ void bind_hybrid(py::module_& m) {
         py::arg("routed") = none, py::arg("routed_w") = none);
   m.def("xielu", &xielu, "in-place xIELU", py::arg("z"), py::arg("p"),
         py::arg("q"));
+  m.def("gelu", &gelu, "in-place exact GELU", py::arg("z"));
+  m.def("stream_step", &stream_step,
+        "float residual step of blocks with output norms: embed / grouped "
+        "norm + add of a sublayer and routed rows, average over depth, next "
+        "operand",
+        py::arg("x"), py::arg("y") = none, py::arg("post_w") = none,
+        py::arg("xn") = none, py::arg("next_w") = none,
+        py::arg("groups") = 1, py::arg("eps") = 1e-6,
+        py::arg("tokens") = none, py::arg("table") = none,
+        py::arg("scale") = 1.0, py::arg("routed") = none,
+        py::arg("routed_w") = none, py::arg("chosen") = none,
+        py::arg("experts") = 0, py::arg("hist") = none,
+        py::arg("coef") = none, py::arg("keep") = none,
+        py::arg("shift") = none, py::arg("prev") = none,
+        py::arg("row_slot") = none, py::arg("row_pos") = none);
+  m.def("token_shift", &token_shift, "mix with the row before",
+        py::arg("xn"), py::arg("x"), py::arg("shift"), py::arg("prev"),
+        py::arg("seg"), py::arg("max_len"));
+  m.def("causal_conv", &causal_conv, "causal convolution per channel",
+        py::arg("out"), py::arg("x"), py::arg("w"), py::arg("bias"),
+        py::arg("in_bias"), py::arg("state"), py::arg("seg"),
+        py::arg("max_len"), py::arg("act"));
+  m.def("rglru_step", &rglru_step,
+        "RG-LRU gates + recurrence + second branch, one token per segment",
+        py::arg("out"), py::arg("u"), py::arg("y"), py::arg("y_bias"),
+        py::arg("gates"), py::arg("gate_bias"), py::arg("rate"),
+        py::arg("state"), py::arg("seg"));
+  m.def("rglru_scan", &rglru_scan, "RG-LRU over token segments",
+        py::arg("out"), py::arg("u"), py::arg("y"), py::arg("y_bias"),
+        py::arg("gates"), py::arg("gate_bias"), py::arg("rate"),
+        py::arg("state"), py::arg("seg"), py::arg("max_len"));
+  m.def("mamba2_step", &mamba2_step,
+        "Mamba-2 state update + read-out, one token per segment",
+        py::arg("o"), py::arg("xbc"), py::arg("dt"), py::arg("state"),
+        py::arg("dt_bias"), py::arg("rate"), py::arg("vdim"),
+        py::arg("seg"));
+  m.def("mamba2_scan", &mamba2_scan, "Mamba-2 over token segments",
+        py::arg("o"), py::arg("xbc"), py::arg("dt"), py::arg("state"),
+        py::arg("dt_bias"), py::arg("rate"), py::arg("vdim"), py::arg("seg"),
+        py::arg("max_len"));
+  m.def("mamba2_out", &mamba2_out, "skip + gate + grouped norm of the "
+        "read-out", py::arg("out"), py::arg("o"), py::arg("xbc"),
+        py::arg("z"), py::arg("skip"), py::arg("w"), py::arg("groups"),
+        py::arg("eps"));
   m.def("hgrn2_step", &hgrn2_step,
         "HGRN2 gates + state update + read-out + head norm, one token per "
         "segment",
@@ -698,14 +1097,21 @@ void bind_hybrid(py::module_& m) {
         py::arg("kpages"), py::arg("vpages"), py::arg("proj"),
         py::arg("q_w"), py::arg("k_w"), py::arg("row_slot"),
         py::arg("row_pos"), py::arg("table"), py::arg("vdim"),
-        py::arg("eps"));
+        py::arg("eps"), py::arg("rope") = none);
+  m.def("kv_rows", &kv_rows, "cached keys and values <-> flat rows",
+        py::arg("rows"), py::arg("kpages"), py::arg("vpages"),
+        py::arg("row_slot"), py::arg("row_pos"), py::arg("table"),
+        py::arg("dim"), py::arg("vdim"), py::arg("store"));
   m.def("paged_attn", &paged_attn,
-        "paged attention: distance bias, sliding window, kept first tokens",
+        "paged attention: distance bias, sliding window, kept first tokens, "
+        "capped scores, one map or the difference of two",
         py::arg("out"), py::arg("q"), py::arg("kpages"), py::arg("vpages"),
         py::arg("bias"), py::arg("table"), py::arg("seg"),
         py::arg("max_len"), py::arg("window"), py::arg("keep_first"),
         py::arg("scale"), py::arg("splits"), py::arg("part_o") = none,
-        py::arg("part_ml") = none);
+        py::arg("part_ml") = none, py::arg("softcap") = 0.0,
+        py::arg("map_weight") = 0.0, py::arg("out_scale") = 1.0,
+        py::arg("eps") = 0.0);
   m.def("latent_norm_append", &latent_norm_append,
         "norms of the query and key/value latents + paged cache append, and "
         "a gated activation in the same launch",
@@ -738,7 +1144,9 @@ void bind_hybrid(py::module_& m) {
   m.def("moe_route", &moe_route,
         "float router, top experts, pairs ordered by expert",
         py::arg("weight"), py::arg("x"), py::arg("router"), py::arg("top"),
-        py::arg("tile_rows") = 16);
+        py::arg("tile_rows") = 16, py::arg("correction") = none,
+        py::arg("scale") = 1.0, py::arg("identity") = 0,
+        py::arg("gated") = false);
   m.def("moe_up", &moe_up, "experts' gate and up products + activation",
         py::arg("mid"), py::arg("x"), py::arg("w"), py::arg("plan"),
         py::arg("act"), py::arg("tile_rows") = 16);
@@ -746,7 +1154,7 @@ void bind_hybrid(py::module_& m) {
         py::arg("mid"), py::arg("w"), py::arg("plan"),
         py::arg("tile_rows") = 16);
   m.def("skinny_gemm", &skinny_gemm, "projection of up to 32 rows",
-        py::arg("out"), py::arg("w"), py::arg("x"), py::arg("act") = false,
+        py::arg("out"), py::arg("w"), py::arg("x"), py::arg("act") = 0,
         py::arg("act_p") = 0.0, py::arg("act_q") = 0.0);
   m.def("advance_batch", &advance_batch, "decode bookkeeping");
 }

@@ -84,6 +84,14 @@ DEVINL float xielu(float z, float p, float q) {
   return 0.5f * z + (z > 0.f ? p * z * z : (0.5f + q) * (expm1f(z) - z));
 }
 
+DEVINL float gelu_erf(float z) {
+  return 0.5f * z * (1.f + erff(0.7071067811865476f * z));
+}
+
+DEVINL float softplus(float z) {
+  return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)));
+}
+
 DEVINL float sigmoid(float z) { return 1.f / (1.f + expf(-z)); }
 
 DEVINL float gated(float gate, float up, int act) {

@@ -47,6 +47,9 @@ int launch_residual_norm(const ResidualArgs& a, int f32, hipStream_t stream);
 void launch_xielu(void* z, long long n, float p, float q, int f32,
                   hipStream_t stream);
 
+// z <- exact GELU
+void launch_gelu(void* z, long long n, int f32, hipStream_t stream);
+
 // HGRN2 over segments of one token each: gates, state update, read-out and
 // the per-head norm in one launch.  proj [rows, 2*H*D + H*E] = q|f|v.
 void launch_hgrn2_step(void* out, const void* proj, float* state,
@@ -69,16 +72,31 @@ void launch_head_norm(void* out, const float* o, const float* w, SegView seg,
                       int max_len, int heads, int vdim, float eps, int f32,
                       hipStream_t stream);
 
-// Per-head q/k norms, q to a padded buffer, k and v into the paged cache.
-// proj [n, (H+G)*D + G*E] = q|k|v; k pages [P, G, 64 * dpad] and v pages
-// [P, G, 64 * vpad] in the order of PageLayout.
-void launch_qk_norm_append(void* q_out, void* kpages, void* vpages,
-                           const void* proj, const float* q_w,
-                           const float* k_w, const int* row_slot,
-                           const int* row_pos, const int* table,
-                           int table_stride, int n, int heads, int kv_heads,
-                           int dim, int vdim, int dpad, int vpad, float eps,
-                           int f32, hipStream_t stream);
+// Per-head q/k norms (and rotation), q to a padded buffer [n, heads, dpad], k
+// and v into the paged cache.  proj = q|k|v rows; k pages [P, k_heads, 64 *
+// dpad] and v pages [P, v_heads, 64 * vpad] in the order of PageLayout.  No
+// pages: proj = q rows, nothing is stored.
+struct QkAppendArgs {
+  void* q_out;
+  void* kpages;
+  void* vpages;
+  const void* proj;
+  const float* q_w;
+  const float* k_w;
+  const int* row_slot;
+  const int* row_pos;
+  const int* table;
+  const float* rope;  // [positions, rot / 2, 2] or null
+  int table_stride, n, heads, k_heads, v_heads, dim, vdim, dpad, vpad, rot;
+  float eps;
+};
+
+void launch_qk_norm_append(const QkAppendArgs& a, int f32,
+                           hipStream_t stream);
+
+// rows [n, k_heads * dim + v_heads * vdim] <-> pages
+void launch_kv_rows(const QkAppendArgs& a, void* rows, int store, int f32,
+                    hipStream_t stream);
 
 struct PagedAttnArgs {
   void* out;            // [rows, H*vdim]
@@ -96,11 +114,20 @@ struct PagedAttnArgs {
   float scale_log2;
   int splits;           // 0: whole rows per wave; >=1: split the keys
   int max_len;          // longest segment
+  // score <- cap * tanh(score / cap): scale / cap and cap in log2 units
+  float cap_in, cap_log2;  // cap_log2 0: no cap
+  // maps 2: q [rows, H, 2, dpad] and k pages [P, kv_heads * 2, ..], part_o
+  // [n, H, 2, splits, vpad]; out = unit-size (o1 - map_weight * o2) *
+  // out_scale.  Split mode always leaves parts.
+  int maps;
+  float map_weight, out_scale, eps;
 };
 
 // Returns -1 when (dpad, vpad) has no instantiation.
 int launch_paged_attn_bf16(const PagedAttnArgs& a, hipStream_t stream);
 int launch_paged_attn_f32(const PagedAttnArgs& a, hipStream_t stream);
+int launch_diff_attn_bf16(const PagedAttnArgs& a, hipStream_t stream);  // maps 2
+int launch_diff_attn_f32(const PagedAttnArgs& a, hipStream_t stream);
 
 struct RowAttnArgs {
   void* out;              // head h of row r at r * out_row + h * vdim
@@ -194,6 +221,12 @@ struct MoePlan {
   int* n_tiles;
   MoeTile* tiles;
   int pairs, top, experts, tile_rows, max_tiles;
+  // the router: outputs >= experts, those past the experts stand for the row
+  // itself; correction [outputs] or null; gated: one more column of z is a
+  // gate, whose sigmoid is one more weight of each row
+  int outputs, gated;
+  const float* correction;
+  float scale;
 };
 
 // tile_rows: 16, or 128 (bf16, contractions multiples of 64, at least 128
@@ -201,8 +234,8 @@ struct MoePlan {
 MoePlan moe_plan(int* buffer, int n, int top, int experts, int tile_rows);
 long long moe_plan_ints(int n, int top, int experts, int tile_rows);
 
-// z [n, experts] = x router^T in float; weight [n, top] = softmax over the
-// top logits.
+// z [n, outputs + gated] = x router^T in float; chosen outputs and weight [n,
+// top + gated].
 void launch_moe_route(float* weight, float* z, const void* x,
                       const void* router, MoePlan p, int n, int k, int f32,
                       hipStream_t stream);
@@ -220,8 +253,127 @@ void launch_moe_down(void* out, const void* mid, const void* w, MoePlan p,
 void launch_advance_batch(const int* slots, const int* sampled, int* pos,
                           int* tokens, int spare, int n, hipStream_t stream);
 
-// out[n, m] = x[n, :] . w[m, :] in bf16 for up to 32 rows of x, with xIELU
-// if act.  Returns -1 when n or k (a multiple of 64) does not fit.
+// Residual step of blocks with norms on the sublayers' outputs, one row per
+// block.  x [n, e] float:
+//   tokens != null : x = scale * table[token]
+//   y or routed    : a = y (times the last weight, if there are routed rows)
+//                        + weighted routed rows [n, top, e], where a chosen
+//                        output >= experts stands for x itself;
+//                    x += post_w ? groups of rms(a) * post_w : a
+// keep = x; if coef, x = sum_j coef[j] hist[j] + coef[depth] x; then xn is
+//   next_w : groups of rms(x) * next_w
+//   shift  : x + (prev[slot] - x) * shift, and prev[slot] = x
+//   else   : x
+struct StreamArgs {
+  float* x;
+  const void* y;
+  const float* post_w;
+  void* xn;
+  const float* next_w;
+  const int* tokens;
+  const void* table;
+  const void* routed;
+  const float* routed_w;
+  const int* chosen;
+  const float* hist;   // [depth, n, e]
+  const float* coef;   // [depth + 1]
+  float* keep;
+  const float* shift;
+  float* prev;         // [slots, e]
+  const int* row_slot;
+  const int* row_pos;
+  int top, experts, depth, groups, n, e;
+  float scale, eps;
+};
+
+// -1: e is too large
+int launch_stream_step(const StreamArgs& a, int f32, hipStream_t stream);
+
+// xn = x + (the row before - x) * shift over segments; prev [slots, e] is the
+// row before a segment and takes its last one
+void launch_token_shift(void* xn, const float* x, const float* shift,
+                        float* prev, SegView seg, int max_len, int e, int f32,
+                        hipStream_t stream);
+
+// out = act(bias + sum_k w[k] * (x[t - taps + 1 + k] + in_bias)) per channel
+// over segments, zeros before position 0; w [taps, c], x rows ld apart, state
+// [slots, max(1, taps - 1), c] the last rows of x; act: silu.  At most 16
+// taps.
+struct ConvArgs {
+  void* out;
+  const void* x;
+  const float* w;
+  const float* bias;
+  const float* in_bias;  // or null
+  void* state;
+  SegView seg;
+  long long ld;
+  int max_len, c, taps, act;
+  int vec;  // 8 (bf16) or 4 (float) channels per access are aligned
+};
+
+void launch_causal_conv(const ConvArgs& a, int f32, hipStream_t stream);
+
+// RG-LRU: r, i = sigmoid(block-diagonal products of u + gate_bias), a =
+// exp(rate * r), S = a S + sqrt(1 - a^2) i u, out = S * gelu_tanh(y + y_bias).
+// gates [2, blocks, part, part], state [slots, width].
+struct RgLruArgs {
+  void* out;
+  const void* u;      // [rows, width]
+  const void* y;      // rows y_ld apart
+  const float* y_bias;
+  const void* gates;
+  const float* gate_bias;
+  const float* rate;
+  float* state;
+  float* work;        // scan: [2, n, width]
+  SegView seg;
+  long long y_ld;
+  int n, width, blocks, max_len;
+};
+
+void launch_rglru_step(const RgLruArgs& a, int f32, hipStream_t stream);
+void launch_rglru_scan(const RgLruArgs& a, int f32, hipStream_t stream);
+
+// Mamba-2: dt = softplus(dt + dt_bias), S = exp(rate dt) S + dt B x^T, o =
+// S^T C.  xbc [rows, inner + 2 * groups * dim] = x|B|C, dt rows dt_ld apart,
+// state [slots, heads, dim, vstride], o [rows, inner] float.
+struct Mamba2Args {
+  float* o;
+  const void* xbc;
+  const void* dt;
+  float* state;
+  const float* dt_bias;
+  const float* rate;
+  float* work;        // scan: hgrn2_work_floats(...)
+  SegView seg;
+  long long dt_ld;
+  int heads, groups, dim, vdim, vstride, max_len;
+};
+
+void launch_mamba2_step(const Mamba2Args& a, int f32, hipStream_t stream);
+// -1: dim has no instantiation
+int launch_mamba2_scan(const Mamba2Args& a, int f32, hipStream_t stream);
+
+// out = groups of rms((o + skip x) silu(z)) * w; x rows are xld, z rows zld
+// apart, skip [heads].  -1: rows are too long
+struct GatedNormArgs {
+  void* out;
+  const float* o;
+  const void* x;
+  const void* z;
+  const float* skip;
+  const float* w;
+  long long xld, zld;
+  int n, inner, vdim, groups;
+  float eps;
+  int vec;
+};
+
+int launch_gated_norm(const GatedNormArgs& a, int f32, hipStream_t stream);
+
+// out[n, m] = x[n, :] . w[m, :] in bf16 for up to 32 rows of x, with act 1
+// xIELU, 2 exact GELU.  Returns -1 when n or k (a multiple of 64) does not fit.
 int launch_skinny_gemm(void* out, const void* w, const void* x, int n, int m,
                        int k, int act, float act_p, float act_q,
                        hipStream_t stream);

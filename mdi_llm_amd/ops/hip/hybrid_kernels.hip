@@ -2,7 +2,7 @@
 // (gfx950).  All of them take a flat batch of token rows; nothing here knows
 // whether a row belongs to a prompt or to a decode step.
 
-#include "hybrid_common.h"
+#include "matrix_state.h"
 
 // ---------------------------------------------------------------------------
 // Residual + norms, one block of NT threads per row.  Every thread keeps its
@@ -143,189 +143,101 @@ int launch_residual_norm(const ResidualArgs& a, int f32, hipStream_t stream) {
 }
 
 // ---------------------------------------------------------------------------
-// xIELU on a whole GEMM output (single rows have it in the GEMV epilogue)
+// xIELU or exact GELU on a whole GEMM output (single rows have it in the GEMV epilogue)
 // ---------------------------------------------------------------------------
-template <typename T, int V>
-__global__ __launch_bounds__(256) void xielu_kernel(T* __restrict__ z,
-                                                    long long n, float p,
-                                                    float q) {
+template <typename T, int V, bool GELU>
+__global__ __launch_bounds__(256) void act_kernel(T* __restrict__ z,
+                                                  long long n, float p,
+                                                  float q) {
   const long long stride = (long long)gridDim.x * 256 * V;
   for (long long i = ((long long)blockIdx.x * 256 + threadIdx.x) * V; i < n;
        i += stride) {
     Pack<T, V> a = *reinterpret_cast<Pack<T, V>*>(z + i);
 #pragma unroll
-    for (int j = 0; j < V; ++j) a.v[j] = from_f<T>(xielu(to_f(a.v[j]), p, q));
+    for (int j = 0; j < V; ++j) {
+      const float f = to_f(a.v[j]);
+      a.v[j] = from_f<T>(GELU ? gelu_erf(f) : xielu(f, p, q));
+    }
     *reinterpret_cast<Pack<T, V>*>(z + i) = a;
   }
 }
 
-template <typename T, int V>
-static void xielu_t(void* z, long long n, float p, float q,
-                    hipStream_t stream) {
+template <typename T, int V, bool GELU>
+static void act_t(void* z, long long n, float p, float q,
+                  hipStream_t stream) {
   const long long blocks = (n + 256 * V - 1) / (256 * V);
-  xielu_kernel<T, V><<<(int)(blocks < 8192 ? blocks : 8192), 256, 0, stream>>>(
-      (T*)z, n, p, q);
+  act_kernel<T, V, GELU>
+      <<<(int)(blocks < 8192 ? blocks : 8192), 256, 0, stream>>>((T*)z, n, p,
+                                                                 q);
+}
+
+template <bool GELU>
+static void act_any(void* z, long long n, float p, float q, int f32,
+                    hipStream_t stream) {
+  if (f32) {
+    if (n % 4 == 0) act_t<float, 4, GELU>(z, n, p, q, stream);
+    else act_t<float, 1, GELU>(z, n, p, q, stream);
+  } else {
+    if (n % 8 == 0) act_t<bf16, 8, GELU>(z, n, p, q, stream);
+    else act_t<bf16, 1, GELU>(z, n, p, q, stream);
+  }
 }
 
 void launch_xielu(void* z, long long n, float p, float q, int f32,
                   hipStream_t stream) {
-  if (f32) {
-    if (n % 4 == 0) xielu_t<float, 4>(z, n, p, q, stream);
-    else xielu_t<float, 1>(z, n, p, q, stream);
-  } else {
-    if (n % 8 == 0) xielu_t<bf16, 8>(z, n, p, q, stream);
-    else xielu_t<bf16, 1>(z, n, p, q, stream);
-  }
+  act_any<false>(z, n, p, q, f32, stream);
+}
+
+void launch_gelu(void* z, long long n, int f32, hipStream_t stream) {
+  act_any<true>(z, n, 0.f, 0.f, f32, stream);
 }
 
 // ---------------------------------------------------------------------------
-// HGRN2, one token per segment.  One block per (head, segment): the whole
-// [dim, vdim] state of the head passes through registers once (16-byte
-// accesses along vdim), so the block holds all of the head's output and can
-// norm it before it leaves.
+// HGRN2: f is a gate with a lower bound, k = 1 - f (see matrix_state.h).
 // ---------------------------------------------------------------------------
-template <typename T, int NT>
-__global__ __launch_bounds__(NT) void hgrn2_step_kernel(
-    T* __restrict__ out, const T* __restrict__ proj,
-    float* __restrict__ state, const float* __restrict__ f_bias,
-    const float* __restrict__ lower, const float* __restrict__ norm_w,
-    SegView seg, int heads, int dim, int vdim, int vstride, float eps) {
-  extern __shared__ float sm[];
-  __shared__ float red[NT / 64];
-  const int tid = threadIdx.x, h = blockIdx.x, s = blockIdx.y;
-  const int nq = vstride / 4;                 // float4 columns
-  const int lanes = nq < NT ? nq : NT;      // threads along the columns
-  const int groups = NT / lanes;             // row groups
-  float* qs = sm;                             // [dim]
-  float* fs = qs + dim;                       // [dim]
-  float* part = fs + dim;                     // [groups][vstride]
-  const size_t row = seg.start[s];
-  const T* pr = proj + row * (size_t)(heads * (2 * dim + vdim));
-  for (int d = tid; d < dim; d += NT) {
+template <typename T>
+struct Hgrn2Rule {
+  static constexpr bool NORM = true;
+  T* out;
+  const T* proj;
+  const float* f_bias;
+  const float* lower;
+  const float* norm_w;
+  int heads, dim, vdim;
+  DEVINL const T* at(size_t row) const {
+    return proj + row * (size_t)(heads * (2 * dim + vdim));
+  }
+  DEVINL StepFactors factors(size_t row, int h, int d) const {
     const int c = h * dim + d;
-    const float qv = to_f(pr[c]);
-    qs[d] = qv * sigmoid(qv);
-    const float l = lower[c];
-    fs[d] = l + (1.f - l) * sigmoid(to_f(pr[heads * dim + c]) + f_bias[c]);
+    const float q = to_f(at(row)[c]), l = lower[c];
+    const float f = l + (1.f - l) * sigmoid(to_f(at(row)[heads * dim + c]) +
+                                            f_bias[c]);
+    return {q * sigmoid(q), f, 1.f - f};
   }
-  __syncthreads();
-  const T* vr = pr + 2 * heads * dim + h * vdim;
-  float* S = state +
-             ((size_t)seg.slot[s] * heads + h) * (size_t)dim * vstride;
-  const bool fresh = seg.pos0[s] == 0;
-  const int g = tid / lanes;
-  if (g < groups) {
-    for (int c4 = tid % lanes; c4 < nq; c4 += lanes) {
-      float v[4], o[4] = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int j = 0; j < 4; ++j)
-        v[j] = c4 * 4 + j < vdim ? to_f(vr[c4 * 4 + j]) : 0.f;
-#pragma unroll 8
-      for (int d = g; d < dim; d += groups) {
-        float4* p = reinterpret_cast<float4*>(S + (size_t)d * vstride) + c4;
-        float4 a = fresh ? make_float4(0.f, 0.f, 0.f, 0.f) : *p;
-        const float f = fs[d], w = 1.f - f, q = qs[d];
-        a.x = f * a.x + w * v[0];
-        a.y = f * a.y + w * v[1];
-        a.z = f * a.z + w * v[2];
-        a.w = f * a.w + w * v[3];
-        *p = a;
-        o[0] += q * a.x;
-        o[1] += q * a.y;
-        o[2] += q * a.z;
-        o[3] += q * a.w;
-      }
-      *reinterpret_cast<float4*>(part + g * vstride + c4 * 4) =
-          make_float4(o[0], o[1], o[2], o[3]);
-    }
+  DEVINL float value(size_t row, int h, int c) const {
+    return to_f(at(row)[2 * heads * dim + h * vdim + c]);
   }
-  __syncthreads();
-  float ss = 0.f;
-  for (int c = tid; c < vdim; c += NT) {
-    float o = 0.f;
-    for (int k = 0; k < groups; ++k) o += part[k * vstride + c];
-    part[c] = o;  // only this thread reads column c
-    ss += o * o;
+  DEVINL void put(size_t row, int h, int c, float v) const {
+    out[row * (size_t)(heads * vdim) + h * vdim + c] =
+        from_f<T>(v * norm_w[c]);
   }
-  ss = wave_sum(ss);
-  if ((tid & 63) == 0) red[tid >> 6] = ss;
-  __syncthreads();
-  ss = 0.f;
-#pragma unroll
-  for (int k = 0; k < NT / 64; ++k) ss += red[k];
-  const float r = 1.f / sqrtf(ss / vdim + eps);
-  T* o_row = out + row * (size_t)(heads * vdim) + h * vdim;
-  for (int c = tid; c < vdim; c += NT)
-    o_row[c] = from_f<T>(part[c] * r * norm_w[c]);
-}
-
-template <typename T, int NT>
-static void hgrn2_step_t(void* out, const void* proj, float* state,
-                         const float* f_bias, const float* lower,
-                         const float* norm_w, SegView seg, int heads, int dim,
-                         int vdim, int vstride, float eps,
-                         hipStream_t stream) {
-  const int nq = vstride / 4;
-  const int lanes = nq < NT ? nq : NT;
-  const size_t smem =
-      (2 * (size_t)dim + (size_t)(NT / lanes) * vstride) * sizeof(float);
-  hgrn2_step_kernel<T, NT><<<dim3(heads, seg.n), NT, smem, stream>>>(
-      (T*)out, (const T*)proj, state, f_bias, lower, norm_w, seg, heads, dim,
-      vdim, vstride, eps);
-}
+};
 
 void launch_hgrn2_step(void* out, const void* proj, float* state,
                        const float* f_bias, const float* lower,
                        const float* norm_w, SegView seg, int heads, int dim,
                        int vdim, int vstride, float eps, int f32,
                        hipStream_t stream) {
-  // few blocks with a large state each: more waves to keep loads in flight
-  const bool wide = dim * vstride >= 8192 && heads * seg.n <= 512;
-#define STEP(T, NT)                                                       \
-  hgrn2_step_t<T, NT>(out, proj, state, f_bias, lower, norm_w, seg,       \
-                      heads, dim, vdim, vstride, eps, stream)
-  if (f32) {
-    if (wide) STEP(float, 1024);
-    else STEP(float, 256);
-  } else {
-    if (wide) STEP(bf16, 1024);
-    else STEP(bf16, 256);
-  }
+#define STEP(T)                                                              \
+  matrix_step(Hgrn2Rule<T>{(T*)out, (const T*)proj, f_bias, lower, norm_w,   \
+                           heads, dim, vdim},                                \
+              state, seg, heads, dim, vdim, vstride, eps, stream)
+  if (f32) STEP(float);
+  else STEP(bf16);
 #undef STEP
 }
 
-// ---------------------------------------------------------------------------
-// HGRN2 over longer segments, in chunks of 16 tokens.  With S the state at
-// the chunk's start, per channel
-//     R_t = f_first .. f_t          (decay from the start to t)
-//     U_s = f_(s+1) .. f_last       (decay from s to the end)
-// the chunk is three small matrix products,
-//     o_t = (q_t R_t)^T S + sum_(s<=t) P[t][s] v_s
-//     S  <- (f_first .. f_last) S + sum_s (U_s (1 - f_s)) v_s^T
-// with P[t][s] = sum_d q_t (1 - f_s) f_(s+1) .. f_t.  All decays are plain
-// products of gates, so every factor is at most 1 and nothing is divided
-// by; an underflow is a token that is forgotten.  Everything is float and
-// the products run on the float MFMA.
-//
-// The first kernel makes the factors of every (chunk, head) in parallel;
-// the second walks a segment's chunks with a [dim, 16] slice of the state
-// per block, held as MFMA accumulators split over the block's four waves by
-// rows.  An accumulator tile is at the same time the right operand of
-// (q R)^T S once the contraction index is permuted to its layout.
-//
-// Workspace of one (chunk, head), DP = dim padded to 64, 128 or 256:
-//   qr [16][DP] | uk [DP][16] | decay [DP] | P [16][16]
-// Segment s has its chunks from start[s] / 16 + s on, which cannot overlap
-// as long as the segments are in the order of their rows.
-// ---------------------------------------------------------------------------
-using f32x4 = __attribute__((__vector_size__(16))) float;
-
-template <int DP>
-struct ChunkWork {
-  static constexpr int QR = 0, UK = 16 * DP, DECAY = 32 * DP,
-                       P = 33 * DP, SIZE = 33 * DP + 256;
-};
-
+// Factors of a 16-token chunk: all decays are plain products of gates.
 template <typename T, int DP>
 __global__ __launch_bounds__(256) void hgrn2_factors_kernel(
     float* __restrict__ work, const T* __restrict__ proj,
@@ -402,132 +314,6 @@ __global__ __launch_bounds__(256) void hgrn2_factors_kernel(
   }
 }
 
-template <typename T, int TPW>
-__global__ __launch_bounds__(256) void hgrn2_chunks_kernel(
-    float* __restrict__ o, const float* __restrict__ work,
-    const T* __restrict__ proj, float* __restrict__ state, SegView seg,
-    int heads, int dim, int vdim, int vstride) {
-  constexpr int DP = 64 * TPW;
-  using W = ChunkWork<DP>;
-  __shared__ float red[2][4][16][17];
-  const int tid = threadIdx.x, lane = tid & 63;
-  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int c = lane & 15, quad = lane >> 4;
-  // heads vary fastest: the column blocks of a head share an XCD's L2
-  const int s = blockIdx.z, h = blockIdx.x, c0 = blockIdx.y * 16;
-  const int col = c0 + c, d0 = wave * TPW * 16;
-  const int len = seg.len[s], n = (len + 15) / 16;
-  const size_t row0 = seg.start[s];
-  const size_t ld = (size_t)heads * (2 * dim + vdim);
-  const float* w = work + ((row0 / 16 + s) * heads + h) * W::SIZE;
-  const size_t wstep = (size_t)heads * W::SIZE;
-  const T* vp = proj + row0 * ld + 2 * heads * dim + h * vdim +
-                min(col, vdim - 1);
-  float* S = state +
-             ((size_t)seg.slot[s] * heads + h) * (size_t)dim * vstride + col;
-  const bool keep = col < vdim && seg.pos0[s] != 0;
-
-  f32x4 st[TPW];
-#pragma unroll
-  for (int k = 0; k < TPW; ++k)
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int d = d0 + k * 16 + quad * 4 + i;
-      st[k][i] = keep && d < dim ? S[(size_t)d * vstride] : 0.f;
-    }
-
-  // operands of the next chunks on their way (values stay unconverted, so
-  // that nothing waits for them early)
-  constexpr int AHEAD = TPW <= 2 ? 4 : 2;
-  struct Operands {
-    f32x4 qr[TPW], uk[TPW], decay[TPW];
-    float p;
-    T v[4], vw;
-  } ring[AHEAD];
-  auto load = [&](Operands& a, int ch) {
-    const float* wc = w + ch * wstep;
-#pragma unroll
-    for (int k = 0; k < TPW; ++k) {
-      a.qr[k] = *reinterpret_cast<const f32x4*>(
-          wc + W::QR + c * DP + d0 + k * 16 + quad * 4);
-      a.uk[k] = *reinterpret_cast<const f32x4*>(
-          wc + W::UK + (d0 + k * 16 + c) * 16 + quad * 4);
-      a.decay[k] = *reinterpret_cast<const f32x4*>(
-          wc + W::DECAY + d0 + k * 16 + quad * 4);
-    }
-    a.p = wc[W::P + c * 16 + quad * 4 + wave];
-    // rows and columns past the end repeat the last: they meet zero factors
-    // or are not stored
-    auto value = [&](int t) { return vp[(size_t)min(t, len - 1) * ld]; };
-#pragma unroll
-    for (int i = 0; i < 4; ++i) a.v[i] = value(ch * 16 + quad * 4 + i);
-    a.vw = value(ch * 16 + quad * 4 + wave);
-  };
-  auto chunk = [&](const Operands& a, int ch) {
-    // two accumulators: half the dependent chain
-    f32x4 a0{0.f, 0.f, 0.f, 0.f}, a1 = a0;
-    a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(a.p, to_f(a.vw), a0, 0, 0, 0);
-#pragma unroll
-    for (int k = 0; k < TPW; ++k) {
-      a1 = __builtin_amdgcn_mfma_f32_16x16x4f32(a.qr[k][0], st[k][0], a1, 0, 0, 0);
-      a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(a.qr[k][1], st[k][1], a0, 0, 0, 0);
-      a1 = __builtin_amdgcn_mfma_f32_16x16x4f32(a.qr[k][2], st[k][2], a1, 0, 0, 0);
-      a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(a.qr[k][3], st[k][3], a0, 0, 0, 0);
-    }
-#pragma unroll
-    for (int k = 0; k < TPW; ++k) st[k] *= a.decay[k];
-#pragma unroll
-    for (int i = 0; i < 4; ++i)
-#pragma unroll
-      for (int k = 0; k < TPW; ++k)
-        st[k] = __builtin_amdgcn_mfma_f32_16x16x4f32(a.uk[k][i], to_f(a.v[i]),
-                                                     st[k], 0, 0, 0);
-    a0 += a1;
-#pragma unroll
-    for (int i = 0; i < 4; ++i) red[ch & 1][wave][quad * 4 + i][c] = a0[i];
-  };
-  auto emit = [&](int ch) {
-    __syncthreads();  // one per chunk: the other half is written next
-    const int t = tid >> 4, e = tid & 15, tt = ch * 16 + t;
-    if (tt < len && c0 + e < vdim) {
-      float v = 0.f;
-#pragma unroll
-      for (int k = 0; k < 4; ++k) v += red[ch & 1][k][t][e];
-      o[(row0 + tt) * (size_t)(heads * vdim) + h * vdim + c0 + e] = v;
-    }
-  };
-#pragma unroll
-  for (int r = 0; r < AHEAD; ++r) load(ring[r], min(r, n - 1));
-  int base = 0;
-  for (; base + AHEAD <= n; base += AHEAD) {
-#pragma unroll
-    for (int r = 0; r < AHEAD; ++r) {
-      chunk(ring[r], base + r);
-      load(ring[r], min(base + r + AHEAD, n - 1));
-      emit(base + r);
-    }
-  }
-#pragma unroll
-  for (int r = 0; r < AHEAD - 1; ++r)
-    if (base + r < n) {
-      chunk(ring[r], base + r);
-      emit(base + r);
-    }
-  if (col < vdim) {
-#pragma unroll
-    for (int k = 0; k < TPW; ++k)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int d = d0 + k * 16 + quad * 4 + i;
-        if (d < dim) S[(size_t)d * vstride] = st[k][i];
-      }
-  }
-}
-
-static int chunk_dpad(int dim) {
-  return dim <= 64 ? 64 : dim <= 128 ? 128 : dim <= 256 ? 256 : 0;
-}
-
 long long hgrn2_work_floats(int rows, int segments, int heads, int dim) {
   const long long chunks = rows / 16 + segments + 1;
   return chunks * heads * (33 * chunk_dpad(dim) + 256);
@@ -542,9 +328,11 @@ static void hgrn2_scan_sized(float* o, float* work, const void* proj,
   hgrn2_factors_kernel<T, 64 * TPW>
       <<<dim3((max_len + 15) / 16, heads, seg.n), 256, 0, stream>>>(
           work, (const T*)proj, f_bias, lower, seg, heads, dim, vdim);
-  hgrn2_chunks_kernel<T, TPW>
+  matrix_chunks_kernel<T, TPW>
       <<<dim3(heads, (vdim + 15) / 16, seg.n), 256, 0, stream>>>(
-          o, work, (const T*)proj, state, seg, heads, dim, vdim, vstride);
+          o, work, (const T*)proj + 2 * heads * dim,
+          (long long)heads * (2 * dim + vdim), state, seg, heads, dim, vdim,
+          vstride);
 }
 
 template <typename T>
@@ -634,7 +422,8 @@ void launch_head_norm(void* out, const float* o, const float* w, SegView seg,
 // ---------------------------------------------------------------------------
 // q/k head norms + cache append.  q and k: a group of L lanes per (row,
 // head), V channels per lane.  v: pages run along the keys, so a wave takes
-// 64 consecutive rows by V columns.
+// 64 consecutive rows by V columns.  rope [positions, rot / 2, 2], if given,
+// rotates neighbouring channels (2i, 2i + 1) below rot after the norm.
 // ---------------------------------------------------------------------------
 template <typename T, int V, int L>
 __global__ __launch_bounds__(256) void qk_norm_append_kernel(
@@ -642,8 +431,8 @@ __global__ __launch_bounds__(256) void qk_norm_append_kernel(
     const T* __restrict__ proj, const float* __restrict__ q_w,
     const float* __restrict__ k_w, const int* __restrict__ row_slot,
     const int* __restrict__ row_pos, const int* __restrict__ table,
-    int table_stride, int n, int heads, int kv_heads, int dim, int vdim,
-    int dpad, float eps) {
+    int table_stride, int n, int heads, int kv_heads, int dim, long long ld,
+    int dpad, float eps, const float* __restrict__ rope, int rot) {
   constexpr int PER = 256 / L;  // (row, head) pairs per block
   using P = Pack<T, V>;
   const int hk = heads + kv_heads;
@@ -653,8 +442,7 @@ __global__ __launch_bounds__(256) void qk_norm_append_kernel(
   const size_t row = i / hk;
   const int hd = (int)(i - row * hk);
   const bool is_q = hd < heads;
-  const T* src = proj + row * (size_t)(hk * dim + kv_heads * vdim) +
-                 (size_t)hd * dim;
+  const T* src = proj + row * (size_t)ld + (size_t)hd * dim;
   const float* w = is_q ? q_w : k_w;
   T* dst;
   int key = 0;
@@ -686,10 +474,33 @@ __global__ __launch_bounds__(256) void qk_norm_append_kernel(
   for (int k = 0; k < KEEP; ++k) {
     const int d = (k * L + lane) * V;
     if (d >= dpad) break;
-    P b;
+    float f[V];
 #pragma unroll
     for (int j = 0; j < V; ++j)
-      b.v[j] = from_f<T>(d < dim ? to_f(a[k].v[j]) * r * w[d + j] : 0.f);
+      f[j] = d < dim ? to_f(a[k].v[j]) * r * w[d + j] : 0.f;
+    if (rope != nullptr) {
+      const float* cs = rope + (size_t)row_pos[row] * rot;
+      if constexpr (V == 1) {
+        // the partner is the neighbouring lane (rot is even, and so is L)
+        const float other = __shfl_xor(f[0], 1, 64);
+        if (d < rot) {
+          const float c = cs[d & ~1], si = cs[d | 1];
+          f[0] = d & 1 ? f[0] * c + other * si : f[0] * c - other * si;
+        }
+      } else {
+#pragma unroll
+        for (int j = 0; j < V; j += 2)
+          if (d + j < rot) {
+            const float c = cs[d + j], si = cs[d + j + 1];
+            const float u = f[j], v = f[j + 1];
+            f[j] = u * c - v * si;
+            f[j + 1] = v * c + u * si;
+          }
+      }
+    }
+    P b;
+#pragma unroll
+    for (int j = 0; j < V; ++j) b.v[j] = from_f<T>(f[j]);
     if (is_q) {
       *reinterpret_cast<P*>(dst + d) = b;
     } else {
@@ -706,65 +517,97 @@ __global__ __launch_bounds__(256) void qk_norm_append_kernel(
 
 template <typename T, int V>
 __global__ __launch_bounds__(256) void v_append_kernel(
-    T* __restrict__ vpages, const T* __restrict__ proj,
+    T* __restrict__ vpages, const T* __restrict__ values, long long ld,
     const int* __restrict__ row_slot, const int* __restrict__ row_pos,
     const int* __restrict__ table, int table_stride, int n, int heads,
-    int kv_heads, int dim, int vdim, int vpad) {
-  const int chunks = kv_heads * (vdim / V);
+    int vdim, int vpad) {
+  const int chunks = heads * (vdim / V);
   const int ch = blockIdx.y * 4 + (threadIdx.x >> 6);
   const size_t row = (size_t)blockIdx.x * 64 + (threadIdx.x & 63);
   if (ch >= chunks || row >= n) return;
   const int g = ch / (vdim / V), c = (ch % (vdim / V)) * V;
-  const size_t qk = (size_t)(heads + kv_heads) * dim;
   const Pack<T, V> a = *reinterpret_cast<const Pack<T, V>*>(
-      proj + row * (qk + kv_heads * vdim) + qk + (size_t)g * vdim + c);
+      values + row * (size_t)ld + (size_t)g * vdim + c);
   const int pos = row_pos[row];
   const size_t page =
       table[(size_t)row_slot[row] * table_stride + (pos >> 6)];
-  T* dst = vpages + (page * kv_heads + g) * (size_t)(64 * vpad);
+  T* dst = vpages + (page * heads + g) * (size_t)(64 * vpad);
 #pragma unroll
   for (int j = 0; j < V; ++j)
     dst[PageLayout::v(pos & 63, c + j, vpad)] = a.v[j];
 }
 
 template <typename T, int V, int L>
-static void append_t(void* q_out, void* kpages, void* vpages,
-                     const void* proj, const float* q_w, const float* k_w,
-                     const int* row_slot, const int* row_pos,
-                     const int* table, int table_stride, int n, int heads,
-                     int kv_heads, int dim, int vdim, int dpad, int vpad,
-                     float eps, hipStream_t stream) {
-  const long long pairs = (long long)n * (heads + kv_heads);
+static void append_t(const QkAppendArgs& a, hipStream_t stream) {
+  const int k_heads = a.kpages != nullptr ? a.k_heads : 0;
+  const long long pairs = (long long)a.n * (a.heads + k_heads);
+  const long long qk = (long long)(a.heads + k_heads) * a.dim;
+  const long long ld = qk + (k_heads > 0 ? a.v_heads * a.vdim : 0);
   qk_norm_append_kernel<T, V, L>
       <<<(unsigned)((pairs + 256 / L - 1) / (256 / L)), 256, 0, stream>>>(
-          (T*)q_out, (T*)kpages, (const T*)proj, q_w, k_w, row_slot, row_pos,
-          table, table_stride, n, heads, kv_heads, dim, vdim, dpad, eps);
-  const int chunks = kv_heads * (vdim / V);
+          (T*)a.q_out, (T*)a.kpages, (const T*)a.proj, a.q_w, a.k_w,
+          a.row_slot, a.row_pos, a.table, a.table_stride, a.n, a.heads,
+          k_heads, a.dim, ld, a.dpad, a.eps, a.rope, a.rot);
+  if (k_heads == 0) return;
+  const int chunks = a.v_heads * (a.vdim / V);
   v_append_kernel<T, V>
-      <<<dim3((n + 63) / 64, (chunks + 3) / 4), 256, 0, stream>>>(
-          (T*)vpages, (const T*)proj, row_slot, row_pos, table, table_stride,
-          n, heads, kv_heads, dim, vdim, vpad);
+      <<<dim3((a.n + 63) / 64, (chunks + 3) / 4), 256, 0, stream>>>(
+          (T*)a.vpages, (const T*)a.proj + qk, ld, a.row_slot, a.row_pos,
+          a.table, a.table_stride, a.n, a.v_heads, a.vdim, a.vpad);
 }
 
-void launch_qk_norm_append(void* q_out, void* kpages, void* vpages,
-                           const void* proj, const float* q_w,
-                           const float* k_w, const int* row_slot,
-                           const int* row_pos, const int* table,
-                           int table_stride, int n, int heads, int kv_heads,
-                           int dim, int vdim, int dpad, int vpad, float eps,
-                           int f32, hipStream_t stream) {
-#define APPEND(T, V, L)                                                     \
-  append_t<T, V, L>(q_out, kpages, vpages, proj, q_w, k_w, row_slot,        \
-                    row_pos, table, table_stride, n, heads, kv_heads, dim,  \
-                    vdim, dpad, vpad, eps, stream)
+void launch_qk_norm_append(const QkAppendArgs& a, int f32,
+                           hipStream_t stream) {
   if (f32) {
-    if (dim % 4 == 0 && vdim % 4 == 0) APPEND(float, 4, 16);
-    else APPEND(float, 1, 64);
+    if (a.dim % 4 == 0 && a.vdim % 4 == 0) append_t<float, 4, 16>(a, stream);
+    else append_t<float, 1, 64>(a, stream);
   } else {
-    if (dim % 8 == 0 && vdim % 8 == 0) APPEND(bf16, 8, 16);
-    else APPEND(bf16, 1, 64);
+    if (a.dim % 8 == 0 && a.vdim % 8 == 0) append_t<bf16, 8, 16>(a, stream);
+    else append_t<bf16, 1, 64>(a, stream);
   }
-#undef APPEND
+}
+
+// Keys and values of some tokens as flat rows [k heads * dim | v heads *
+// vdim], into the pages or out of them.
+template <typename T, bool STORE>
+__global__ __launch_bounds__(256) void kv_rows_kernel(
+    T* __restrict__ rows, T* __restrict__ kpages, T* __restrict__ vpages,
+    const int* __restrict__ row_slot, const int* __restrict__ row_pos,
+    const int* __restrict__ table, int table_stride, int k_heads, int v_heads,
+    int dim, int vdim, int dpad, int vpad) {
+  const size_t row = blockIdx.x;
+  const int cols = k_heads * dim + v_heads * vdim, pos = row_pos[row];
+  const size_t page =
+      table[(size_t)row_slot[row] * table_stride + (pos >> 6)];
+  for (int i = threadIdx.x; i < cols; i += 256) {
+    T* at;
+    if (i < k_heads * dim) {
+      at = kpages + (page * k_heads + i / dim) * (size_t)(64 * dpad) +
+           PageLayout::k(pos & 63, i % dim, dpad);
+    } else {
+      const int c = i - k_heads * dim;
+      at = vpages + (page * v_heads + c / vdim) * (size_t)(64 * vpad) +
+           PageLayout::v(pos & 63, c % vdim, vpad);
+    }
+    if (STORE) *at = rows[row * cols + i];
+    else rows[row * cols + i] = *at;
+  }
+}
+
+void launch_kv_rows(const QkAppendArgs& a, void* rows, int store, int f32,
+                    hipStream_t stream) {
+#define ROWS(T, ST)                                                         \
+  kv_rows_kernel<T, ST><<<a.n, 256, 0, stream>>>(                           \
+      (T*)rows, (T*)a.kpages, (T*)a.vpages, a.row_slot, a.row_pos, a.table, \
+      a.table_stride, a.k_heads, a.v_heads, a.dim, a.vdim, a.dpad, a.vpad)
+  if (f32) {
+    if (store) ROWS(float, true);
+    else ROWS(float, false);
+  } else {
+    if (store) ROWS(bf16, true);
+    else ROWS(bf16, false);
+  }
+#undef ROWS
 }
 
 // ---------------------------------------------------------------------------

@@ -3,85 +3,12 @@
 // the experts' products over tiles of pairs of one expert.  Nothing comes
 // back to the host, so decode steps can be captured.
 
-#include "mfma_frag.h"
+#include "mfma_tile.h"
 
 namespace {
 
 constexpr int MAX_EXPERTS = 256;
 constexpr int FUSED_ROWS = 64;  // up to here one block chooses and orders
-
-// 8 contraction steps of a row of length k; vec: rows are 16-byte aligned
-template <typename T>
-DEVINL typename Frag<T>::Row load_steps(const T* row, int at, int k,
-                                        bool vec) {
-  using F = Frag<T>;
-  if (vec && at + 8 <= k) return F::load_frag(row + at);
-  typename F::Row r = F::zero();
-#pragma unroll
-  for (int j = 0; j < 8; ++j)
-    if (at + j < k) F::set(r, j, row[at + j]);
-  return r;
-}
-
-// out[row][m]: 16 x 16 tile of x w^T, the contraction split over NW waves in
-// stretches of 64 (a lane's 16 steps of a stretch are contiguous), for NM sets
-// of weight rows at once.  Every wave leaves its part in red[wave][set][row][m].
-template <typename T, int NW, int NM>
-DEVINL void tile_product(float (*red)[NM][16][17], const T* x,
-                         const T* const (&w)[NM], int k, bool vec) {
-  using F = Frag<T>;
-  constexpr int STRIDE = NW * 64, UNR = NM == 1 ? 4 : 2;
-  const int lane = threadIdx.x & 63, c = lane & 15, quad = lane >> 4;
-  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-  f32x4 acc[NM];
-#pragma unroll
-  for (int j = 0; j < NM; ++j) acc[j] = f32x4{0.f, 0.f, 0.f, 0.f};
-  int at = wave * 64;
-  // several stretches of the weight stream in flight
-  for (; vec && at + (UNR - 1) * STRIDE + 64 <= k; at += UNR * STRIDE) {
-    typename F::Row wa[UNR][NM], wb[UNR][NM];
-#pragma unroll
-    for (int u = 0; u < UNR; ++u)
-#pragma unroll
-      for (int j = 0; j < NM; ++j) {
-        wa[u][j] = F::load_frag(w[j] + at + u * STRIDE + quad * 16);
-        wb[u][j] = F::load_frag(w[j] + at + u * STRIDE + quad * 16 + 8);
-      }
-#pragma unroll
-    for (int u = 0; u < UNR; ++u) {
-      const auto xa = F::load_frag(x + at + u * STRIDE + quad * 16);
-      const auto xb = F::load_frag(x + at + u * STRIDE + quad * 16 + 8);
-#pragma unroll
-      for (int j = 0; j < NM; ++j) {
-        acc[j] = F::dot(wa[u][j], xa, acc[j]);
-        acc[j] = F::dot(wb[u][j], xb, acc[j]);
-      }
-    }
-  }
-  for (; at < k; at += STRIDE) {
-    const int s = at + quad * 16;
-    const auto xa = load_steps<T>(x, s, k, vec);
-    const auto xb = load_steps<T>(x, s + 8, k, vec);
-#pragma unroll
-    for (int j = 0; j < NM; ++j) {
-      acc[j] = F::dot(load_steps<T>(w[j], s, k, vec), xa, acc[j]);
-      acc[j] = F::dot(load_steps<T>(w[j], s + 8, k, vec), xb, acc[j]);
-    }
-  }
-#pragma unroll
-  for (int j = 0; j < NM; ++j)
-#pragma unroll
-    for (int i = 0; i < 4; ++i) red[wave][j][c][quad * 4 + i] = acc[j][i];
-  __syncthreads();
-}
-
-template <int NW, int NM>
-DEVINL float tile_sum(const float (*red)[NM][16][17], int j, int row, int m) {
-  float v = 0.f;
-#pragma unroll
-  for (int q = 0; q < NW; ++q) v += red[q][j][row][m];
-  return v;
-}
 
 // ---------------------------------------------------------------------------
 template <typename T, int NW>
@@ -100,30 +27,61 @@ __global__ __launch_bounds__(NW * 64) void router_kernel(
   }
 }
 
-// One wave: the top logits of a row (lower index first among equals) and
-// their softmax.
-DEVINL void choose(float* weight, int* chosen, const float* z, int experts,
-                   int top, int lane) {
-  float v[MAX_EXPERTS / 64];
+// One wave: the choice of a row (lower index first among equals) and its
+// weights.  Without correction the top logits and their softmax; with it the
+// softmax over all outputs plus the correction chooses, and the weights are
+// the chosen scores over their sum, times scale.
+DEVINL void choose(float* weight, int* chosen, const float* z,
+                   const MoePlan& p, int lane) {
+  constexpr int NV = MAX_EXPERTS / 64;
+  const int outputs = p.outputs, top = p.top;
+  float v[NV], score[NV];
 #pragma unroll
-  for (int j = 0; j < MAX_EXPERTS / 64; ++j) {
+  for (int j = 0; j < NV; ++j) {
     const int e = j * 64 + lane;
-    v[j] = e < experts ? z[e] : -__builtin_huge_valf();
+    v[j] = e < outputs ? z[e] : -__builtin_huge_valf();
+  }
+  if (p.correction != nullptr) {
+    float m = v[0], total = 0.f;
+#pragma unroll
+    for (int j = 1; j < NV; ++j) m = fmaxf(m, v[j]);
+    m = wave_max(m);
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      score[j] = expf(v[j] - m);
+      total += score[j];
+    }
+    total = wave_sum(total);
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      const int e = j * 64 + lane;
+      score[j] /= total;
+      if (e < outputs) v[j] = score[j] + p.correction[e];
+    }
   }
   float zmax = 0.f, sum = 0.f, mine = 0.f;
   for (int t = 0; t < top; ++t) {
     float best = v[0];
 #pragma unroll
-    for (int j = 1; j < MAX_EXPERTS / 64; ++j) best = fmaxf(best, v[j]);
+    for (int j = 1; j < NV; ++j) best = fmaxf(best, v[j]);
     best = wave_max(best);
-    int at = experts - 1;  // kept only if a logit is not a number
+    int at = outputs - 1;  // kept only if a logit is not a number
 #pragma unroll
-    for (int j = MAX_EXPERTS / 64 - 1; j >= 0; --j) {
+    for (int j = NV - 1; j >= 0; --j) {
       const unsigned long long hit = __ballot(v[j] == best);
-      if (hit != 0) at = min(j * 64 + __ffsll(hit) - 1, experts - 1);
+      if (hit != 0) at = min(j * 64 + __ffsll(hit) - 1, outputs - 1);
     }
     if (t == 0) zmax = best;
-    const float e = expf(best - zmax);
+    float e;
+    if (p.correction != nullptr) {
+      float s = score[0];
+#pragma unroll
+      for (int j = 1; j < NV; ++j)
+        if (at >> 6 == j) s = score[j];
+      e = __shfl(s, at & 63, 64);
+    } else {
+      e = expf(best - zmax);
+    }
     sum += e;
     // a wave holds up to 64 choices, one per lane
     if (lane == t) {
@@ -131,10 +89,12 @@ DEVINL void choose(float* weight, int* chosen, const float* z, int experts,
       chosen[t] = at;
     }
 #pragma unroll
-    for (int j = 0; j < MAX_EXPERTS / 64; ++j)
+    for (int j = 0; j < NV; ++j)
       if (at == j * 64 + lane) v[j] = -__builtin_huge_valf();
   }
+  if (p.correction != nullptr) sum = (sum + 1e-20f) / p.scale;
   if (lane < top) weight[lane] = mine / sum;
+  if (p.gated && lane == 0) weight[top] = sigmoid(z[outputs]);
 }
 
 __global__ __launch_bounds__(256) void choose_kernel(
@@ -142,11 +102,13 @@ __global__ __launch_bounds__(256) void choose_kernel(
     int n) {
   const int row = blockIdx.x * 4 + (threadIdx.x >> 6);
   if (row >= n) return;
-  choose(weight + (size_t)row * p.top, p.chosen + (size_t)row * p.top,
-         z + (size_t)row * p.experts, p.experts, p.top, threadIdx.x & 63);
+  choose(weight + (size_t)row * (p.top + p.gated),
+         p.chosen + (size_t)row * p.top,
+         z + (size_t)row * (p.outputs + p.gated), p, threadIdx.x & 63);
 }
 
-// One block: the pairs ordered by expert, and the tiles.
+// One block: the pairs ordered by expert, and the tiles.  Pairs of outputs
+// that are not experts are left out.
 __global__ __launch_bounds__(1024) void order_kernel(
     float* __restrict__ weight, const float* __restrict__ z, MoePlan p,
     int n, bool choose_here) {
@@ -154,12 +116,13 @@ __global__ __launch_bounds__(1024) void order_kernel(
   const int tid = threadIdx.x;
   if (choose_here)
     for (int row = tid >> 6; row < n; row += 16)
-      choose(weight + row * p.top, p.chosen + row * p.top,
-             z + row * p.experts, p.experts, p.top, tid & 63);
+      choose(weight + row * (p.top + p.gated), p.chosen + row * p.top,
+             z + row * (p.outputs + p.gated), p, tid & 63);
   if (tid < p.experts) count[tid] = 0;
   __syncthreads();
   // (the block's own global writes are visible to it after the barrier)
-  for (int i = tid; i < p.pairs; i += 1024) atomicAdd(&count[p.chosen[i]], 1);
+  for (int i = tid; i < p.pairs; i += 1024)
+    if (p.chosen[i] < p.experts) atomicAdd(&count[p.chosen[i]], 1);
   __syncthreads();
   if (tid < p.experts) {
     const int shift = 31 - __clz(p.tile_rows);  // a power of two
@@ -178,7 +141,8 @@ __global__ __launch_bounds__(1024) void order_kernel(
   }
   __syncthreads();
   for (int i = tid; i < p.pairs; i += 1024)
-    p.order[atomicAdd(&next[p.chosen[i]], 1)] = i;
+    if (p.chosen[i] < p.experts)
+      p.order[atomicAdd(&next[p.chosen[i]], 1)] = i;
 }
 
 // ---------------------------------------------------------------------------
@@ -377,7 +341,8 @@ void expert_tiles(void* out, const void* x, const void* w, MoePlan p, int m,
 }  // namespace
 
 MoePlan moe_plan(int* buffer, int n, int top, int experts, int tile_rows) {
-  MoePlan p;
+  MoePlan p{};
+  p.outputs = experts;
   p.pairs = n * top;
   p.top = top;
   p.experts = experts;
@@ -401,14 +366,14 @@ long long moe_plan_ints(int n, int top, int experts, int tile_rows) {
 void launch_moe_route(float* weight, float* z, const void* x,
                       const void* router, MoePlan p, int n, int k, int f32,
                       hipStream_t stream) {
-  const dim3 grid((p.experts + 15) / 16, (n + 15) / 16);
+  const int cols = p.outputs + p.gated;
+  const dim3 grid((cols + 15) / 16, (n + 15) / 16);
   if (f32)
     router_kernel<float, 16><<<grid, 1024, 0, stream>>>(
-        z, (const float*)x, (const float*)router, n, p.experts, k,
-        k % 4 == 0);
+        z, (const float*)x, (const float*)router, n, cols, k, k % 4 == 0);
   else
     router_kernel<bf16, 16><<<grid, 1024, 0, stream>>>(
-        z, (const bf16*)x, (const bf16*)router, n, p.experts, k, k % 8 == 0);
+        z, (const bf16*)x, (const bf16*)router, n, cols, k, k % 8 == 0);
   const bool fused = n <= FUSED_ROWS;
   if (!fused) choose_kernel<<<(n + 3) / 4, 256, 0, stream>>>(weight, z, p, n);
   order_kernel<<<1, 1024, 0, stream>>>(weight, z, p, n, fused);

@@ -1,5 +1,5 @@
 #include "paged_attn.inc"
 
 int launch_paged_attn_bf16(const PagedAttnArgs& a, hipStream_t stream) {
-  return launch_dims<bf16>(a, stream);
+  return launch_dims<bf16, 1>(a, stream);
 }

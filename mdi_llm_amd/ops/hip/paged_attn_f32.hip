@@ -1,5 +1,5 @@
 #include "paged_attn.inc"
 
 int launch_paged_attn_f32(const PagedAttnArgs& a, hipStream_t stream) {
-  return launch_dims<float>(a, stream);
+  return launch_dims<float, 1>(a, stream);
 }

@@ -1,0 +1,458 @@
+// Recurrent mixers with a short convolution over ragged batches (gfx950):
+// the convolution, RG-LRU (block-diagonal gates and a scan per channel) and
+// the Mamba-2 rule of the matrix-state kernels.
+
+#include "matrix_state.h"
+#include "mfma_tile.h"
+
+namespace {
+
+constexpr int CONV_TILE = 16;  // tokens of a block, and the most taps
+
+// ---------------------------------------------------------------------------
+// Causal convolution: a thread has V channels of a tile of tokens and keeps
+// the last K - 1 inputs in registers.  K = 0: any number of taps, inputs are
+// read again.  The first tile's block alone reads the slot's inputs, and
+// writes the new ones after that.
+// ---------------------------------------------------------------------------
+template <typename T, int V, int K>
+__global__ __launch_bounds__(256) void causal_conv_kernel(ConvArgs p) {
+  const int s = blockIdx.z, t0 = blockIdx.y * CONV_TILE;
+  const int len = p.seg.len[s];
+  const int c = (blockIdx.x * 256 + threadIdx.x) * V;
+  if (t0 >= len || c >= p.c) return;
+  const int taps = K ? K : p.taps, back = taps - 1;
+  const int keep = max(1, back);  // rows of a slot
+  const int pos0 = p.seg.pos0[s];
+  const size_t row0 = p.seg.start[s];
+  const T* x = (const T*)p.x + row0 * p.ld + c;
+  T* state = (T*)p.state + (size_t)p.seg.slot[s] * keep * p.c + c;
+  using PT = Pack<T, V>;
+  using PF = Pack<float, V>;
+  PF in_bias{};
+  if (p.in_bias != nullptr)
+    in_bias = *reinterpret_cast<const PF*>(p.in_bias + c);
+  const PF bias = *reinterpret_cast<const PF*>(p.bias + c);
+  // raw input of token t of the segment, -back <= t < len
+  auto raw = [&](int t) {
+    return *reinterpret_cast<const PT*>(
+        t >= 0 ? x + (size_t)t * p.ld : state + (size_t)(back + t) * p.c);
+  };
+  auto input = [&](int t) {
+    PF f{};
+    if (pos0 + t >= 0) {  // zeros before the sequence's start
+      const PT r = raw(t);
+#pragma unroll
+      for (int j = 0; j < V; ++j) f.v[j] = to_f(r.v[j]) + in_bias.v[j];
+    }
+    return f;
+  };
+  const int tn = min(CONV_TILE, len - t0);
+  T* out = (T*)p.out + (row0 + t0) * p.c + c;
+  auto put = [&](int t, PF y) {
+    PT o;
+#pragma unroll
+    for (int j = 0; j < V; ++j)
+      o.v[j] = from_f<T>(p.act ? y.v[j] * sigmoid(y.v[j]) : y.v[j]);
+    *reinterpret_cast<PT*>(out + (size_t)t * p.c) = o;
+  };
+  if constexpr (K > 0) {
+    PF w[K], win[K];
+#pragma unroll
+    for (int k = 0; k < K; ++k) {
+      w[k] = *reinterpret_cast<const PF*>(p.w + (size_t)k * p.c + c);
+      if (k < K - 1) win[k] = input(t0 - (K - 1) + k);
+    }
+    for (int t = 0; t < tn; ++t) {
+      win[K - 1] = input(t0 + t);
+      PF y = bias;
+#pragma unroll
+      for (int k = 0; k < K; ++k)
+#pragma unroll
+        for (int j = 0; j < V; ++j) y.v[j] += w[k].v[j] * win[k].v[j];
+      put(t, y);
+#pragma unroll
+      for (int k = 0; k + 1 < K; ++k) win[k] = win[k + 1];
+    }
+  } else {
+    for (int t = 0; t < tn; ++t) {
+      PF y = bias;
+      for (int k = 0; k < taps; ++k) {
+        const PF f = input(t0 + t - back + k);
+        const PF w = *reinterpret_cast<const PF*>(p.w + (size_t)k * p.c + c);
+#pragma unroll
+        for (int j = 0; j < V; ++j) y.v[j] += w.v[j] * f.v[j];
+      }
+      put(t, y);
+    }
+  }
+  // the last inputs; rows move towards the front, so none is lost early
+  if (t0 == 0)
+    for (int k = 0; k < back; ++k)
+      *reinterpret_cast<PT*>(state + (size_t)k * p.c) = raw(len - back + k);
+}
+
+template <typename T, int V>
+void causal_conv_t(const ConvArgs& a, hipStream_t stream) {
+  const dim3 grid((a.c + 256 * V - 1) / (256 * V),
+                  (a.max_len + CONV_TILE - 1) / CONV_TILE, a.seg.n);
+  switch (a.taps) {
+    case 2: causal_conv_kernel<T, V, 2><<<grid, 256, 0, stream>>>(a); break;
+    case 3: causal_conv_kernel<T, V, 3><<<grid, 256, 0, stream>>>(a); break;
+    case 4: causal_conv_kernel<T, V, 4><<<grid, 256, 0, stream>>>(a); break;
+    default: causal_conv_kernel<T, V, 0><<<grid, 256, 0, stream>>>(a);
+  }
+}
+
+// ---------------------------------------------------------------------------
+// RG-LRU
+// ---------------------------------------------------------------------------
+struct Decay {
+  float a, x;  // S <- a S + x
+};
+
+DEVINL Decay rglru_decay(float zr, float zi, float rate, float u) {
+  const float log_a = rate * sigmoid(zr);
+  return {expf(log_a), sqrtf(-expm1f(2.f * log_a)) * sigmoid(zi) * u};
+}
+
+DEVINL float gelu_tanh(float z) { return gated(z, 1.f, 1); }
+
+// Both gates of 64 rows x 16 channels per wave; a and x to work [2, n, width].
+template <typename T>
+__global__ __launch_bounds__(256) void rglru_gates_kernel(RgLruArgs p,
+                                                          bool vec) {
+  using F = Frag<T>;
+  constexpr int RT = 4;
+  const int part = p.width / p.blocks, tiles = (part + 15) / 16;
+  const int lane = threadIdx.x & 63, c = lane & 15, quad = lane >> 4;
+  const int unit =
+      blockIdx.x * 4 + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  if (unit >= tiles * p.blocks) return;
+  const int b = unit / tiles, m0 = unit % tiles * 16;
+  const int r0 = blockIdx.y * RT * 16;
+  const T* w = (const T*)p.gates +
+               ((size_t)b * part + min(m0 + c, part - 1)) * part;
+  const T* wi = w + (size_t)p.width * part;
+  const T* u[RT];
+#pragma unroll
+  for (int t = 0; t < RT; ++t)
+    u[t] = (const T*)p.u + (size_t)min(r0 + t * 16 + c, p.n - 1) * p.width +
+           (size_t)b * part;
+  f32x4 ar[RT], ai[RT];
+#pragma unroll
+  for (int t = 0; t < RT; ++t) ar[t] = ai[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int at = quad * 8; at - quad * 8 < part; at += 32) {
+    const auto fr = load_steps<T>(w, at, part, vec);
+    const auto fi = load_steps<T>(wi, at, part, vec);
+#pragma unroll
+    for (int t = 0; t < RT; ++t) {
+      const auto x = load_steps<T>(u[t], at, part, vec);
+      ar[t] = F::dot(fr, x, ar[t]);
+      ai[t] = F::dot(fi, x, ai[t]);
+    }
+  }
+#pragma unroll
+  for (int t = 0; t < RT; ++t) {
+    const int row = r0 + t * 16 + c;
+    if (row >= p.n) continue;
+    const size_t base = (size_t)row * p.width + (size_t)b * part;
+    f32x4 da, dx;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int m = min(m0 + quad * 4 + i, part - 1), ch = b * part + m;
+      const Decay d = rglru_decay(
+          ar[t][i] + p.gate_bias[ch], ai[t][i] + p.gate_bias[p.width + ch],
+          p.rate[ch], to_f(((const T*)p.u)[base + m]));
+      da[i] = d.a;
+      dx[i] = d.x;
+    }
+    float* oa = p.work + base + m0 + quad * 4;
+    float* ox = oa + (size_t)p.n * p.width;
+    if (part % 4 == 0 && m0 + quad * 4 < part) {
+      *reinterpret_cast<f32x4*>(oa) = da;
+      *reinterpret_cast<f32x4*>(ox) = dx;
+    } else {
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (m0 + quad * 4 + i < part) {
+          oa[i] = da[i];
+          ox[i] = dx[i];
+        }
+    }
+  }
+}
+
+// The recurrence of a segment, 16 channels per block: 16 threads share a
+// channel and take 8 tokens each of a tile of 128, whose maps S -> A S + B are
+// composed through LDS.  The next tile's operands are in flight meanwhile.
+template <typename T>
+__global__ __launch_bounds__(256) void rglru_scan_kernel(RgLruArgs p) {
+  constexpr int TC = 8, SUB = 16, TILE = TC * SUB;
+  __shared__ float ma[2][SUB][17], mx[2][SUB][17];
+  const int s = blockIdx.y, len = p.seg.len[s];
+  const int cl = threadIdx.x & 15, sub = threadIdx.x >> 4;
+  const int c = blockIdx.x * 16 + cl;
+  const bool live = c < p.width;
+  const int cc = min(c, p.width - 1);
+  const size_t row0 = p.seg.start[s];
+  const float* pa = p.work + row0 * p.width + cc;
+  const float* px = pa + (size_t)p.n * p.width;
+  const T* py = (const T*)p.y + row0 * p.y_ld + cc;
+  T* out = (T*)p.out + row0 * p.width + cc;
+  float* state = p.state + (size_t)p.seg.slot[s] * p.width + cc;
+  const float y_bias = p.y_bias[cc];
+  float S = p.seg.pos0[s] != 0 ? *state : 0.f;
+  struct Tile {
+    float a[TC], x[TC];
+    T y[TC];
+  };
+  auto load = [&](Tile& t, int t0) {
+#pragma unroll
+    for (int j = 0; j < TC; ++j) {
+      // tokens past the end repeat the last: their map is replaced below
+      const size_t r = min(t0 + sub * TC + j, len - 1);
+      t.a[j] = pa[r * p.width];
+      t.x[j] = px[r * p.width];
+      t.y[j] = py[r * p.y_ld];
+    }
+  };
+  auto run = [&](Tile& t, int t0, int buf) {
+    float A = 1.f, B = 0.f;
+#pragma unroll
+    for (int j = 0; j < TC; ++j) {
+      if (t0 + sub * TC + j >= len) {
+        t.a[j] = 1.f;
+        t.x[j] = 0.f;
+      }
+      A *= t.a[j];
+      B = t.a[j] * B + t.x[j];
+    }
+    ma[buf][sub][cl] = A;
+    mx[buf][sub][cl] = B;
+    __syncthreads();  // one per tile: the other half is written next
+    float in = S;
+#pragma unroll
+    for (int k = 0; k < SUB; ++k) {
+      if (k == sub) in = S;
+      S = ma[buf][k][cl] * S + mx[buf][k][cl];
+    }
+#pragma unroll
+    for (int j = 0; j < TC; ++j) {
+      in = t.a[j] * in + t.x[j];
+      const int tt = t0 + sub * TC + j;
+      if (live && tt < len)
+        out[(size_t)tt * p.width] =
+            from_f<T>(in * gelu_tanh(to_f(t.y[j]) + y_bias));
+    }
+  };
+  Tile t[2];
+  load(t[0], 0);
+  for (int t0 = 0; t0 < len; t0 += 2 * TILE) {
+    load(t[1], t0 + TILE);
+    run(t[0], t0, 0);
+    if (t0 + TILE >= len) break;
+    load(t[0], t0 + 2 * TILE);
+    run(t[1], t0 + TILE, 1);
+  }
+  if (live && sub == 0) *state = S;
+}
+
+// One token per segment: gates, recurrence and the second branch in one
+// launch; a block has 16 channels of up to 16 segments.
+template <typename T, int NW>
+__global__ __launch_bounds__(NW * 64) void rglru_step_kernel(RgLruArgs p,
+                                                             bool vec) {
+  __shared__ float red[NW][2][16][17];
+  const int part = p.width / p.blocks, tiles = (part + 15) / 16;
+  const int b = blockIdx.x / tiles, m0 = blockIdx.x % tiles * 16;
+  const int s0 = blockIdx.y * 16, c = threadIdx.x & 15;
+  const T* w0 = (const T*)p.gates +
+                ((size_t)b * part + min(m0 + c, part - 1)) * part;
+  const T* const w[2] = {w0, w0 + (size_t)p.width * part};
+  const size_t mine = p.seg.start[min(s0 + c, p.seg.n - 1)];
+  tile_product<T, NW, 2>(red, (const T*)p.u + mine * p.width +
+                                  (size_t)b * part, w, part, vec);
+  for (int i = threadIdx.x; i < 256; i += NW * 64) {
+    const int r = i >> 4, m = m0 + (i & 15), s = s0 + r;
+    if (s >= p.seg.n || m >= part) continue;
+    const int ch = b * part + m;
+    const size_t row = p.seg.start[s];
+    const Decay d = rglru_decay(
+        tile_sum<NW, 2>(red, 0, r, i & 15) + p.gate_bias[ch],
+        tile_sum<NW, 2>(red, 1, r, i & 15) + p.gate_bias[p.width + ch],
+        p.rate[ch], to_f(((const T*)p.u)[row * p.width + ch]));
+    float* state = p.state + (size_t)p.seg.slot[s] * p.width + ch;
+    float S = p.seg.pos0[s] != 0 ? *state : 0.f;
+    S = d.a * S + d.x;
+    *state = S;
+    ((T*)p.out)[row * p.width + ch] = from_f<T>(
+        S * gelu_tanh(to_f(((const T*)p.y)[row * p.y_ld + ch]) +
+                      p.y_bias[ch]));
+  }
+}
+
+template <typename T>
+void rglru_step_t(const RgLruArgs& a, hipStream_t stream) {
+  const int part = a.width / a.blocks;
+  rglru_step_kernel<T, 4>
+      <<<dim3((part + 15) / 16 * a.blocks, (a.seg.n + 15) / 16), 256, 0,
+         stream>>>(a, part % (16 / sizeof(T)) == 0);
+}
+
+template <typename T>
+void rglru_scan_t(const RgLruArgs& a, hipStream_t stream) {
+  const int part = a.width / a.blocks;
+  const int units = (part + 15) / 16 * a.blocks;
+  rglru_gates_kernel<T><<<dim3((units + 3) / 4, (a.n + 63) / 64), 256, 0,
+                          stream>>>(a, part % (16 / sizeof(T)) == 0);
+  rglru_scan_kernel<T><<<dim3((a.width + 15) / 16, a.seg.n), 256, 0,
+                         stream>>>(a);
+}
+
+// ---------------------------------------------------------------------------
+// Mamba-2: one decay per head, keys dt * B, queries C.
+// ---------------------------------------------------------------------------
+template <typename T>
+struct Mamba2Rule {
+  static constexpr bool NORM = false;
+  float* o;
+  const T* xbc;
+  const T* dt;
+  const float* dt_bias;
+  const float* rate;
+  long long dt_ld;
+  int heads, groups, dim, vdim;
+  DEVINL const T* at(size_t row) const {
+    return xbc + row * (size_t)(heads * vdim + 2 * groups * dim);
+  }
+  DEVINL StepFactors factors(size_t row, int h, int d) const {
+    const float t = softplus(to_f(dt[row * dt_ld + h]) + dt_bias[h]);
+    const T* b = at(row) + heads * vdim + h / (heads / groups) * dim;
+    return {to_f(b[groups * dim + d]), expf(rate[h] * t), t * to_f(b[d])};
+  }
+  DEVINL float value(size_t row, int h, int c) const {
+    return to_f(at(row)[h * vdim + c]);
+  }
+  DEVINL void put(size_t row, int h, int c, float v) const {
+    o[row * (size_t)(heads * vdim) + h * vdim + c] = v;
+  }
+};
+
+// Factors of a 16-token chunk (matrix_state.h); decays are exponentials of
+// differences of the running sum of log decays, none above 0.
+template <typename T, int DP>
+__global__ __launch_bounds__(256) void mamba2_factors_kernel(Mamba2Args p) {
+  using W = ChunkWork<DP>;
+  __shared__ float bs[16][DP + 1], cs[16][DP + 1], dts[16], cum[16];
+  const int s = blockIdx.z, h = blockIdx.y, t0 = blockIdx.x * 16;
+  const int tn = min(16, p.seg.len[s] - t0);
+  if (tn <= 0) return;
+  const int tid = threadIdx.x;
+  const size_t row0 = (size_t)p.seg.start[s] + t0;
+  float* w = p.work + (((size_t)p.seg.start[s] / 16 + s + blockIdx.x) *
+                           p.heads + h) * W::SIZE;
+  if (tid < 64) {
+    const int t = tid & 15;
+    float dt = 0.f;  // past the end: nothing decays or is written
+    if (t < tn)
+      dt = softplus(to_f(((const T*)p.dt)[(row0 + t) * p.dt_ld + h]) +
+                    p.dt_bias[h]);
+    float sum = p.rate[h] * dt;
+#pragma unroll
+    for (int off = 1; off < 16; off *= 2) {
+      const float v = __shfl_up(sum, off, 16);
+      if (t >= off) sum += v;
+    }
+    if (tid < 16) {
+      dts[t] = dt;
+      cum[t] = sum;
+    }
+  }
+  const size_t ld = (size_t)p.heads * p.vdim + 2 * p.groups * p.dim;
+  const T* bc = (const T*)p.xbc + row0 * ld + p.heads * p.vdim +
+                h / (p.heads / p.groups) * p.dim;
+  for (int i = tid; i < 16 * DP; i += 256) {
+    const int t = i / DP, d = i % DP;
+    const bool in = t < tn && d < p.dim;
+    bs[t][d] = in ? to_f(bc[t * ld + d]) : 0.f;
+    cs[t][d] = in ? to_f(bc[t * ld + p.groups * p.dim + d]) : 0.f;
+  }
+  __syncthreads();
+  const float total = cum[15];
+  for (int i = tid; i < 16 * DP; i += 256) {
+    const int t = i / DP, d = i % DP;
+    w[W::QR + i] = cs[t][d] * expf(cum[t]);
+    const int ku = i >> 4, tu = i & 15;
+    w[W::UK + i] = bs[tu][ku] * (dts[tu] * expf(total - cum[tu]));
+  }
+  for (int d = tid; d < DP; d += 256) w[W::DECAY + d] = expf(total);
+  const int t = tid >> 4, sp = tid & 15;
+  float acc = 0.f;
+  if (sp <= t) {
+#pragma unroll 8
+    for (int d = 0; d < DP; ++d) acc += cs[t][d] * bs[sp][d];
+    acc *= dts[sp] * expf(cum[t] - cum[sp]);
+  }
+  w[W::P + tid] = acc;
+}
+
+template <typename T, int TPW>
+void mamba2_scan_sized(const Mamba2Args& a, hipStream_t stream) {
+  mamba2_factors_kernel<T, 64 * TPW>
+      <<<dim3((a.max_len + 15) / 16, a.heads, a.seg.n), 256, 0, stream>>>(a);
+  matrix_chunks_kernel<T, TPW>
+      <<<dim3(a.heads, (a.vdim + 15) / 16, a.seg.n), 256, 0, stream>>>(
+          a.o, a.work, (const T*)a.xbc,
+          (long long)a.heads * a.vdim + 2 * a.groups * a.dim, a.state, a.seg,
+          a.heads, a.dim, a.vdim, a.vstride);
+}
+
+template <typename T>
+int mamba2_scan_t(const Mamba2Args& a, hipStream_t stream) {
+  switch (chunk_dpad(a.dim)) {
+    case 64: mamba2_scan_sized<T, 1>(a, stream); return 0;
+    case 128: mamba2_scan_sized<T, 2>(a, stream); return 0;
+    case 256: mamba2_scan_sized<T, 4>(a, stream); return 0;
+  }
+  return -1;
+}
+
+template <typename T>
+void mamba2_step_t(const Mamba2Args& a, hipStream_t stream) {
+  matrix_step(Mamba2Rule<T>{a.o, (const T*)a.xbc, (const T*)a.dt, a.dt_bias,
+                            a.rate, a.dt_ld, a.heads, a.groups, a.dim,
+                            a.vdim},
+              a.state, a.seg, a.heads, a.dim, a.vdim, a.vstride, 0.f, stream);
+}
+
+}  // namespace
+
+void launch_causal_conv(const ConvArgs& a, int f32, hipStream_t stream) {
+  if (f32) {
+    if (a.vec) causal_conv_t<float, 4>(a, stream);
+    else causal_conv_t<float, 1>(a, stream);
+  } else {
+    if (a.vec) causal_conv_t<bf16, 8>(a, stream);
+    else causal_conv_t<bf16, 1>(a, stream);
+  }
+}
+
+void launch_rglru_step(const RgLruArgs& a, int f32, hipStream_t stream) {
+  if (f32) rglru_step_t<float>(a, stream);
+  else rglru_step_t<bf16>(a, stream);
+}
+
+void launch_rglru_scan(const RgLruArgs& a, int f32, hipStream_t stream) {
+  if (f32) rglru_scan_t<float>(a, stream);
+  else rglru_scan_t<bf16>(a, stream);
+}
+
+void launch_mamba2_step(const Mamba2Args& a, int f32, hipStream_t stream) {
+  if (f32) mamba2_step_t<float>(a, stream);
+  else mamba2_step_t<bf16>(a, stream);
+}
+
+int launch_mamba2_scan(const Mamba2Args& a, int f32, hipStream_t stream) {
+  return f32 ? mamba2_scan_t<float>(a, stream) : mamba2_scan_t<bf16>(a, stream);
+}

@@ -29,7 +29,7 @@ DEVINL bf16x8 load_row(const bf16* p) {
 constexpr int NW = 16, STRIDE = NW * 64, UNR = 4;
 
 // NT: tiles of 16 x rows
-template <int NT, bool XIELU>
+template <int NT, int ACT>
 __global__ __launch_bounds__(NW * 64) void skinny_gemm_kernel(
     bf16* __restrict__ out, const bf16* __restrict__ w,
     const bf16* __restrict__ x, int n, int m, int k, float act_p,
@@ -81,7 +81,8 @@ __global__ __launch_bounds__(NW * 64) void skinny_gemm_kernel(
   float v = 0.f;
 #pragma unroll
   for (int q = 0; q < NW; ++q) v += red[q][row >> 4][row & 15][j];
-  if (XIELU) v = xielu(v, act_p, act_q);
+  if (ACT == 1) v = xielu(v, act_p, act_q);
+  if (ACT == 2) v = gelu_erf(v);
   out[(size_t)row * m + m0 + j] = from_f<bf16>(v);
 }
 
@@ -96,11 +97,13 @@ int launch_skinny_gemm(void* out, const void* w, const void* x, int n, int m,
   skinny_gemm_kernel<NT, ACT><<<grid, NW * 64, 0, stream>>>(             \
       (bf16*)out, (const bf16*)w, (const bf16*)x, n, m, k, act_p, act_q)
   if (n <= 16) {
-    if (act) SKINNY(1, true);
-    else SKINNY(1, false);
+    if (act == 2) SKINNY(1, 2);
+    else if (act == 1) SKINNY(1, 1);
+    else SKINNY(1, 0);
   } else {
-    if (act) SKINNY(2, true);
-    else SKINNY(2, false);
+    if (act == 2) SKINNY(2, 2);
+    else if (act == 1) SKINNY(2, 1);
+    else SKINNY(2, 0);
   }
 #undef SKINNY
   return 0;
