@@ -22,6 +22,8 @@ PAIRS = {
     "nerozen-8b": "Meta-Llama-3-8B-Instruct",
     "resolorn-1b": "tiny-llama-1.1b-chat",
     "resolorn-8b": "Meta-Llama-3-8B-Instruct",
+    "dinuzen-1b": "tiny-llama-1.1b-chat",
+    "dinuzen-8b": "Meta-Llama-3-8B-Instruct",
 }
 SAMPLING = dict(temperature=0.8, top_k=200, seed=1234)
 

@@ -73,18 +73,24 @@ def rglru_gates(u, w, pre, blocks):
     return out
 
 
+def decayed_sum(u, r, i, lam):
+    """The recurrence itself, over time."""
+    S, out = torch.zeros_like(u[0]), []
+    for t in range(u.shape[0]):
+        log_a = -8.0 * r[t] * softplus(lam)
+        S = torch.exp(log_a) * S \
+            + torch.sqrt(-torch.expm1(2.0 * log_a)) * i[t] * u[t]
+        out.append(S)
+    return torch.stack(out)
+
+
 def rglru(h, w, pre, m):
     y = gelu_tanh(h @ w[pre + "y"].T + w[pre + "y.b"])
     u = causal_conv(h @ w[pre + "x"].T + w[pre + "x.b"], w[pre + "conv"],
                     w[pre + "conv.b"])
     r, i = rglru_gates(u, w, pre, m["blocks"])
-    S, out = torch.zeros_like(u[0]), []
-    for t in range(h.shape[0]):
-        log_a = -8.0 * r[t] * softplus(w[pre + "lam"])
-        S = torch.exp(log_a) * S \
-            + torch.sqrt(-torch.expm1(2.0 * log_a)) * i[t] * u[t]
-        out.append(S)
-    return (torch.stack(out) * y) @ w[pre + "o"].T
+    S = decayed_sum(u, r, i, w[pre + "lam"])
+    return (S * y) @ w[pre + "o"].T
 
 
 # -- state-space duality ----------------------------------------------------
@@ -142,13 +148,14 @@ def yarn_frequencies(rot):
 def rotate(x, rot):
     """x [T, ..., dim]: pairs (2i, 2i + 1) of the first ``dims``."""
     freqs, mult = yarn_frequencies(rot)
+    at = torch.arange(x.shape[0], dtype=torch.float64)
     out = x.clone()
-    for t in range(x.shape[0]):
-        for i, f in enumerate(freqs):
-            c, s = math.cos(t * f) * mult, math.sin(t * f) * mult
-            u, v = x[t, ..., 2 * i], x[t, ..., 2 * i + 1]
-            out[t, ..., 2 * i] = u * c - v * s
-            out[t, ..., 2 * i + 1] = v * c + u * s
+    for i, f in enumerate(freqs):
+        a = (at * f).view(-1, *[1] * (x.dim() - 2))
+        c, s = torch.cos(a) * mult, torch.sin(a) * mult
+        u, v = x[..., 2 * i], x[..., 2 * i + 1]
+        out[..., 2 * i] = u * c - v * s
+        out[..., 2 * i + 1] = v * c + u * s
     return out
 
 
@@ -176,6 +183,10 @@ def map_weight(w, pre, diff):
                  - torch.exp((w[pre + "lq2"] * w[pre + "lk2"]).sum()) + diff)
 
 
+def difference(a1, a2, lam, diff, eps):
+    return unit(a1 - lam * a2, eps) * (1.0 - diff)
+
+
 def diff_attention(h, kv, w, pre, m, eps):
     """``kv``: this layer's keys and values, or an earlier layer's."""
     T, H, rep = h.shape[0], m["heads"], m["heads"] // m["kv_heads"]
@@ -188,7 +199,7 @@ def diff_attention(h, kv, w, pre, m, eps):
         g = a // rep
         a1, a2 = (attend(q[:, a, j], k[:, g, j], v[:, g], m["scale"], cap)
                   for j in (0, 1))
-        out.append(unit(a1 - lam * a2, eps) * (1.0 - m["diff"]))
+        out.append(difference(a1, a2, lam, m["diff"], eps))
     return torch.cat(out, 1) @ w[pre + "o"].T
 
 
