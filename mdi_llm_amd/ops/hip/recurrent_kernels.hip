@@ -111,74 +111,153 @@ struct Decay {
   float a, x;  // S <- a S + x
 };
 
+// float stages take the library's functions; a bf16 stage the hardware's,
+// which are good to about one unit in the last place of a float
+template <typename T> struct Math {
+  static DEVINL float exp(float x) {
+    return __builtin_amdgcn_exp2f(1.4426950408889634f * x);
+  }
+  static DEVINL float inv(float x) { return __builtin_amdgcn_rcpf(x); }
+  static DEVINL float sqrt(float x) { return __builtin_amdgcn_sqrtf(x); }
+};
+template <> struct Math<float> {
+  static DEVINL float exp(float x) { return expf(x); }
+  static DEVINL float inv(float x) { return 1.f / x; }
+  static DEVINL float sqrt(float x) { return sqrtf(x); }
+};
+
+// a = exp(rate r), and u times the input gate and sqrt(1 - a^2), which is
+// taken from the Taylor series of exp where a is close to 1
+template <typename T>
 DEVINL Decay rglru_decay(float zr, float zi, float rate, float u) {
-  const float log_a = rate * sigmoid(zr);
-  return {expf(log_a), sqrtf(-expm1f(2.f * log_a)) * sigmoid(zi) * u};
+  using M = Math<T>;
+  const float log_a = rate * M::inv(1.f + M::exp(-zr));
+  const float a = M::exp(log_a), y = 2.f * log_a;
+  float e = fmaf(y, 1.f / 720, 1.f / 120);
+  e = fmaf(y, e, 1.f / 24);
+  e = fmaf(y, e, 1.f / 6);
+  e = fmaf(y, e, 0.5f);
+  e = fmaf(y, e, 1.f) * -y;
+  const float rest = y > -0.3f ? e : 1.f - a * a;
+  return {a, M::sqrt(rest) * M::inv(1.f + M::exp(-zi)) * u};
 }
 
-DEVINL float gelu_tanh(float z) { return gated(z, 1.f, 1); }
-
-// Both gates of 64 rows x 16 channels per wave; a and x to work [2, n, width].
+// z (1 + tanh(p(z))) / 2 is z / (1 + exp(-2 p(z)))
 template <typename T>
-__global__ __launch_bounds__(256) void rglru_gates_kernel(RgLruArgs p,
-                                                          bool vec) {
+DEVINL float gelu_tanh(float z) {
+  using M = Math<T>;
+  return z * M::inv(1.f + M::exp(-1.5957691216057308f *
+                                 (z + 0.044715f * z * z * z)));
+}
+
+// Both gates of 64 rows x 32 channels per wave; a and x to work [2, n, width].
+template <typename T, bool VEC>
+__global__ __launch_bounds__(256) void rglru_gates_kernel(RgLruArgs p) {
   using F = Frag<T>;
-  constexpr int RT = 4;
-  const int part = p.width / p.blocks, tiles = (part + 15) / 16;
+  constexpr int RT = 4, CT = 2;
+  const int part = p.width / p.blocks, tiles = (part + CT * 16 - 1) / (CT * 16);
   const int lane = threadIdx.x & 63, c = lane & 15, quad = lane >> 4;
   const int unit =
       blockIdx.x * 4 + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   if (unit >= tiles * p.blocks) return;
-  const int b = unit / tiles, m0 = unit % tiles * 16;
+  const int b = unit / tiles, m0 = unit % tiles * CT * 16;
   const int r0 = blockIdx.y * RT * 16;
-  const T* w = (const T*)p.gates +
-               ((size_t)b * part + min(m0 + c, part - 1)) * part;
-  const T* wi = w + (size_t)p.width * part;
+  const T* w[2][CT];
+#pragma unroll
+  for (int j = 0; j < CT; ++j) {
+    w[0][j] = (const T*)p.gates +
+              ((size_t)b * part + min(m0 + j * 16 + c, part - 1)) * part;
+    w[1][j] = w[0][j] + (size_t)p.width * part;
+  }
   const T* u[RT];
 #pragma unroll
   for (int t = 0; t < RT; ++t)
     u[t] = (const T*)p.u + (size_t)min(r0 + t * 16 + c, p.n - 1) * p.width +
            (size_t)b * part;
-  f32x4 ar[RT], ai[RT];
+  f32x4 acc[2][CT][RT];
 #pragma unroll
-  for (int t = 0; t < RT; ++t) ar[t] = ai[t] = f32x4{0.f, 0.f, 0.f, 0.f};
-  for (int at = quad * 8; at - quad * 8 < part; at += 32) {
-    const auto fr = load_steps<T>(w, at, part, vec);
-    const auto fi = load_steps<T>(wi, at, part, vec);
+  for (int g = 0; g < 2; ++g)
 #pragma unroll
-    for (int t = 0; t < RT; ++t) {
-      const auto x = load_steps<T>(u[t], at, part, vec);
-      ar[t] = F::dot(fr, x, ar[t]);
-      ai[t] = F::dot(fi, x, ai[t]);
-    }
+    for (int j = 0; j < CT; ++j)
+#pragma unroll
+      for (int t = 0; t < RT; ++t) acc[g][j][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+  struct Operands {
+    typename F::Row x[RT], w[2][CT];
+  };
+  auto load = [&](Operands& o, int at) {
+#pragma unroll
+    for (int t = 0; t < RT; ++t) o.x[t] = load_steps<T>(u[t], at, part, VEC);
+#pragma unroll
+    for (int g = 0; g < 2; ++g)
+#pragma unroll
+      for (int j = 0; j < CT; ++j)
+        o.w[g][j] = load_steps<T>(w[g][j], at, part, VEC);
+  };
+  auto dot = [&](const Operands& o) {
+#pragma unroll
+    for (int g = 0; g < 2; ++g)
+#pragma unroll
+      for (int j = 0; j < CT; ++j)
+#pragma unroll
+        for (int t = 0; t < RT; ++t)
+          acc[g][j][t] = F::dot(o.w[g][j], o.x[t], acc[g][j][t]);
+  };
+  const int steps = (part + 31) / 32;
+  Operands o[2];
+  load(o[0], quad * 8);
+  for (int k = 0; k < steps; k += 2) {
+    if (k + 1 < steps) load(o[1], (k + 1) * 32 + quad * 8);
+    dot(o[0]);
+    if (k + 2 < steps) load(o[0], (k + 2) * 32 + quad * 8);
+    if (k + 1 < steps) dot(o[1]);
   }
 #pragma unroll
-  for (int t = 0; t < RT; ++t) {
-    const int row = r0 + t * 16 + c;
-    if (row >= p.n) continue;
-    const size_t base = (size_t)row * p.width + (size_t)b * part;
-    f32x4 da, dx;
+  for (int j = 0; j < CT; ++j) {
+    const int m = m0 + j * 16 + quad * 4;
+    if (m >= part) continue;
+    float br[4], bi[4], rate[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const int m = min(m0 + quad * 4 + i, part - 1), ch = b * part + m;
-      const Decay d = rglru_decay(
-          ar[t][i] + p.gate_bias[ch], ai[t][i] + p.gate_bias[p.width + ch],
-          p.rate[ch], to_f(((const T*)p.u)[base + m]));
-      da[i] = d.a;
-      dx[i] = d.x;
+      const int ch = b * part + min(m + i, part - 1);
+      br[i] = p.gate_bias[ch];
+      bi[i] = p.gate_bias[p.width + ch];
+      rate[i] = p.rate[ch];
     }
-    float* oa = p.work + base + m0 + quad * 4;
-    float* ox = oa + (size_t)p.n * p.width;
-    if (part % 4 == 0 && m0 + quad * 4 < part) {
-      *reinterpret_cast<f32x4*>(oa) = da;
-      *reinterpret_cast<f32x4*>(ox) = dx;
-    } else {
 #pragma unroll
-      for (int i = 0; i < 4; ++i)
-        if (m0 + quad * 4 + i < part) {
-          oa[i] = da[i];
-          ox[i] = dx[i];
-        }
+    for (int t = 0; t < RT; ++t) {
+      const int row = r0 + t * 16 + c;
+      if (row >= p.n) continue;
+      const size_t base = (size_t)row * p.width + (size_t)b * part;
+      f32x4 da, dx;
+      const T* up = (const T*)p.u + base;
+      Pack<T, 4> uu;
+      if (VEC) {
+        uu = *reinterpret_cast<const Pack<T, 4>*>(up + m);
+      } else {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) uu.v[i] = up[min(m + i, part - 1)];
+      }
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const Decay d = rglru_decay<T>(acc[0][j][t][i] + br[i],
+                                       acc[1][j][t][i] + bi[i], rate[i],
+                                       to_f(uu.v[i]));
+        da[i] = d.a;
+        dx[i] = d.x;
+      }
+      float* oa = p.work + base + m;
+      float* ox = oa + (size_t)p.n * p.width;
+      if (VEC) {
+        *reinterpret_cast<f32x4*>(oa) = da;
+        *reinterpret_cast<f32x4*>(ox) = dx;
+      } else {
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          if (m + i < part) {
+            oa[i] = da[i];
+            ox[i] = dx[i];
+          }
+      }
     }
   }
 }
@@ -192,7 +271,9 @@ __global__ __launch_bounds__(256) void rglru_scan_kernel(RgLruArgs p) {
   __shared__ float ma[2][SUB][17], mx[2][SUB][17];
   const int s = blockIdx.y, len = p.seg.len[s];
   const int cl = threadIdx.x & 15, sub = threadIdx.x >> 4;
-  const int c = blockIdx.x * 16 + cl;
+  // blocks of one XCD are neighbours: they share lines in its L2
+  const int c = ((int)(blockIdx.x & 7) * (gridDim.x >> 3) +
+                 (int)(blockIdx.x >> 3)) * 16 + cl;
   const bool live = c < p.width;
   const int cc = min(c, p.width - 1);
   const size_t row0 = p.seg.start[s];
@@ -243,7 +324,7 @@ __global__ __launch_bounds__(256) void rglru_scan_kernel(RgLruArgs p) {
       const int tt = t0 + sub * TC + j;
       if (live && tt < len)
         out[(size_t)tt * p.width] =
-            from_f<T>(in * gelu_tanh(to_f(t.y[j]) + y_bias));
+            from_f<T>(in * gelu_tanh<T>(to_f(t.y[j]) + y_bias));
     }
   };
   Tile t[2];
@@ -278,7 +359,7 @@ __global__ __launch_bounds__(NW * 64) void rglru_step_kernel(RgLruArgs p,
     if (s >= p.seg.n || m >= part) continue;
     const int ch = b * part + m;
     const size_t row = p.seg.start[s];
-    const Decay d = rglru_decay(
+    const Decay d = rglru_decay<T>(
         tile_sum<NW, 2>(red, 0, r, i & 15) + p.gate_bias[ch],
         tile_sum<NW, 2>(red, 1, r, i & 15) + p.gate_bias[p.width + ch],
         p.rate[ch], to_f(((const T*)p.u)[row * p.width + ch]));
@@ -287,7 +368,7 @@ __global__ __launch_bounds__(NW * 64) void rglru_step_kernel(RgLruArgs p,
     S = d.a * S + d.x;
     *state = S;
     ((T*)p.out)[row * p.width + ch] = from_f<T>(
-        S * gelu_tanh(to_f(((const T*)p.y)[row * p.y_ld + ch]) +
+        S * gelu_tanh<T>(to_f(((const T*)p.y)[row * p.y_ld + ch]) +
                       p.y_bias[ch]));
   }
 }
@@ -303,11 +384,14 @@ void rglru_step_t(const RgLruArgs& a, hipStream_t stream) {
 template <typename T>
 void rglru_scan_t(const RgLruArgs& a, hipStream_t stream) {
   const int part = a.width / a.blocks;
-  const int units = (part + 15) / 16 * a.blocks;
-  rglru_gates_kernel<T><<<dim3((units + 3) / 4, (a.n + 63) / 64), 256, 0,
-                          stream>>>(a, part % (16 / sizeof(T)) == 0);
-  rglru_scan_kernel<T><<<dim3((a.width + 15) / 16, a.seg.n), 256, 0,
-                         stream>>>(a);
+  const int units = (part + 31) / 32 * a.blocks;
+  const dim3 grid((units + 3) / 4, (a.n + 63) / 64);
+  if (part % (16 / sizeof(T)) == 0)
+    rglru_gates_kernel<T, true><<<grid, 256, 0, stream>>>(a);
+  else
+    rglru_gates_kernel<T, false><<<grid, 256, 0, stream>>>(a);
+  rglru_scan_kernel<T>
+      <<<dim3((a.width + 127) / 128 * 8, a.seg.n), 256, 0, stream>>>(a);
 }
 
 // ---------------------------------------------------------------------------

@@ -397,13 +397,17 @@ class HybridEngine:
         return xn
 
     def _shared_expert(self, lw: _LayerWeights, xn: torch.Tensor):
-        if not lw.shared_ff:
+        F = lw.shared_ff
+        if not F:
             return None
-        h = self._linear(xn, lw.shared_in)
-        mid = torch.empty(xn.size(0), lw.shared_ff, dtype=self.dtype,
-                          device=self.device)
-        self.ops.gated_act(mid, h[:, :lw.shared_ff], h[:, lw.shared_ff:],
-                           lw.experts.act)
+        mid = torch.empty(xn.size(0), F, dtype=self.dtype, device=self.device)
+        if self.hip and self.dtype == torch.bfloat16 and xn.size(0) == 1 \
+                and 8 <= xn.size(1) <= 32768 and xn.size(1) % 8 == 0:
+            self.ops.gemv_swiglu(mid, lw.shared_in[:F], lw.shared_in[F:], xn,
+                                 False)
+        else:
+            h = self._linear(xn, lw.shared_in)
+            self.ops.gated_act(mid, h[:, :F], h[:, F:], lw.experts.act)
         return self._linear(mid, lw.shared_out)
 
     def _run_output_normed(self, b: Batch, rows: Optional[torch.Tensor],
