@@ -751,8 +751,8 @@ void skinny_gemm(torch::Tensor out, torch::Tensor w, torch::Tensor x,
 void stream_step(torch::Tensor x, Opt y, Opt post_w, Opt xn, Opt next_w,
                  int64_t groups, double eps, Opt tokens, Opt table,
                  double scale, Opt routed, Opt routed_w, Opt chosen,
-                 int64_t experts, Opt hist, Opt coef, Opt keep, Opt shift,
-                 Opt prev, Opt row_slot, Opt row_pos) {
+                 int64_t experts, Opt hist, Opt coef, Opt keep, Opt past,
+                 Opt shift, Opt prev, Opt row_slot, Opt row_pos) {
   TORCH_CHECK(x.dim() == 2 && x.size(0) > 0, "x must be [n, e]");
   const int64_t n = x.size(0), e = x.size(1);
   StreamArgs a{};
@@ -760,7 +760,7 @@ void stream_step(torch::Tensor x, Opt y, Opt post_w, Opt xn, Opt next_w,
   TORCH_CHECK(groups > 0 && e % groups == 0, "stream_step: groups");
   TORCH_CHECK(!(tokens && (y || routed)) && !!tokens == !!table &&
                   !!routed == !!routed_w && !!routed == !!chosen &&
-                  !!hist == !!coef && !!shift == !!prev &&
+                  !!hist == !!coef && !(past && !hist) && !!shift == !!prev &&
                   !!shift == !!row_slot && !!shift == !!row_pos &&
                   !(next_w && shift) && (xn || (!next_w && !shift)),
               "stream_step: bad combination of operands");
@@ -802,6 +802,7 @@ void stream_step(torch::Tensor x, Opt y, Opt post_w, Opt xn, Opt next_w,
     a.hist = f32_ptr(*hist, a.depth * n * e, "hist");
     a.coef = f32_ptr(*coef, a.depth + 1, "coef");
   }
+  if (past) a.past = const_cast<float*>(f32_ptr(*past, n * e, "past"));
   if (keep) a.keep = const_cast<float*>(f32_ptr(*keep, n * e, "keep"));
   if (shift) {
     a.shift = f32_ptr(*shift, e, "shift");
@@ -1052,6 +1053,7 @@ void bind_hybrid(py::module_& m) {
         py::arg("routed_w") = none, py::arg("chosen") = none,
         py::arg("experts") = 0, py::arg("hist") = none,
         py::arg("coef") = none, py::arg("keep") = none,
+        py::arg("past") = none,
         py::arg("shift") = none, py::arg("prev") = none,
         py::arg("row_slot") = none, py::arg("row_pos") = none);
   m.def("token_shift", &token_shift, "mix with the row before",

@@ -277,6 +277,7 @@ struct StreamArgs {
   const int* chosen;
   const float* hist;   // [depth, n, e]
   const float* coef;   // [depth + 1]
+  float* past;         // [n, e]: only the sum over hist, the stream is as it was
   float* keep;
   const float* shift;
   float* prev;         // [slots, e]

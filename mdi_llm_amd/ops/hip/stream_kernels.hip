@@ -2,6 +2,8 @@
 // step with grouped norms, routed rows, the average over depth and the token
 // shift; and the gated group norm behind a state-space read-out.
 
+#include <algorithm>
+
 #include "hybrid_common.h"
 
 namespace {
@@ -29,9 +31,48 @@ DEVINL void group_scales(const float (&ss)[KEEP], float* part, float* inv,
   __syncthreads();
 }
 
+constexpr int PAST_COLS = 128;  // vectors of a block below
+
+// The weighted sum of earlier results by blocks of their own, beside the
+// blocks of the rows: NT / PAST_COLS threads share a column.
+template <int V, int NT>
+DEVINL void past_sum(const StreamArgs& p, float* part, int block) {
+  using PF = Pack<float, V>;
+  constexpr int SPLIT = NT / PAST_COLS;
+  const int col = threadIdx.x % PAST_COLS, first = threadIdx.x / PAST_COLS;
+  const size_t total = (size_t)p.n * p.e;
+  const size_t at = ((size_t)block * PAST_COLS + col) * V;
+  PF sum{};
+  if (at < total) {
+#pragma unroll 8
+    for (int d = first; d < p.depth; d += SPLIT) {
+      const float f = p.coef[d];
+      const PF v = *reinterpret_cast<const PF*>(p.hist + d * total + at);
+#pragma unroll
+      for (int j = 0; j < V; ++j) sum.v[j] += f * v.v[j];
+    }
+  }
+#pragma unroll
+  for (int j = 0; j < V; ++j)
+    part[(first * V + j) * PAST_COLS + col] = sum.v[j];
+  __syncthreads();
+  if (first == 0 && at < total) {
+#pragma unroll
+    for (int j = 0; j < V; ++j)
+#pragma unroll
+      for (int k = 1; k < SPLIT; ++k)
+        sum.v[j] += part[(k * V + j) * PAST_COLS + col];
+    *reinterpret_cast<PF*>(p.past + at) = sum;
+  }
+}
+
 template <typename T, int V, int NT, int KEEP>
 __global__ __launch_bounds__(NT) void stream_step_kernel(StreamArgs p) {
   extern __shared__ float part[];
+  if ((int)blockIdx.x >= p.n) {
+    past_sum<V, NT>(p, part, blockIdx.x - p.n);
+    return;
+  }
   const int e = p.e, per = e / V / p.groups;
   float* inv = part + e / V;
   const size_t row = blockIdx.x;
@@ -106,7 +147,7 @@ __global__ __launch_bounds__(NT) void stream_step_kernel(StreamArgs p) {
   if (p.keep != nullptr) {
     EACH(i) *reinterpret_cast<PF*>(p.keep + row * e + i) = a[k];
   }
-  if (p.coef != nullptr) {
+  if (p.coef != nullptr && p.past == nullptr) {
     const float own = p.coef[p.depth];
     EACH(i) {
 #pragma unroll
@@ -186,9 +227,15 @@ __global__ __launch_bounds__(NT) void stream_step_kernel(StreamArgs p) {
 template <typename T, int V>
 int stream_step_t(const StreamArgs& a, hipStream_t stream) {
   const int e = a.e;
-  const size_t smem = (e / V + a.groups) * sizeof(float);
+  size_t smem = (e / V + a.groups) * sizeof(float);
+  int blocks = a.n;
+  if (a.past != nullptr) {
+    const size_t vectors = (size_t)a.n * e / V;
+    blocks += (int)((vectors + PAST_COLS - 1) / PAST_COLS);
+    smem = std::max(smem, 1024 * V * sizeof(float));
+  }
 #define RUN(V, NT, KEEP) \
-  stream_step_kernel<T, V, NT, KEEP><<<a.n, NT, smem, stream>>>(a)
+  stream_step_kernel<T, V, NT, KEEP><<<blocks, NT, smem, stream>>>(a)
   ROW_SHAPES(V, a.n <= 256)
 #undef RUN
 }

@@ -96,6 +96,7 @@ class Batch:
         return self.plans[key]
 
 
+FEW_ROWS = 64           # rows whose residual steps are bound by latency
 XIELU, GELU = 1, 2      # activations that a projection can end with
 
 
@@ -116,6 +117,9 @@ class _LayerWeights:
             if ls is not None:
                 setattr(self, n, getattr(self, n) * w(ls))
         self.shift, self.depth = w(block.shift), w(block.depth)
+        if self.depth is not None:  # for a sum over earlier results
+            self.depth_end = torch.stack((torch.ones_like(self.depth[-1]),
+                                          self.depth[-1]))
         m = block.mixer
         self.mixer = m
         if m.kind in ("rglru", "mamba2"):
@@ -417,7 +421,7 @@ class HybridEngine:
         the embedding and every layer's result, where later layers exist."""
         cfg, first, n = self.config, self.first_layer, b.n
         L, E = len(self.layers), cfg.n_embd
-        states = coef = None
+        states = None
         if cfg.depth_average:
             states = torch.empty(min(first + L + 1, cfg.n_layer), n, E,
                                  dtype=torch.float32, device=self.device)
@@ -445,7 +449,14 @@ class HybridEngine:
             if not lw.mlp:
                 xn = self._stream_step(b, x, y, lw.norm1b, **end)
             else:
-                xn = self._stream_step(b, x, y, lw.norm1b, rows=True)
+                ahead = {}
+                if states is not None and n <= FEW_ROWS:
+                    # other blocks of this launch sum up what is there
+                    ahead.update(hist=end["hist"], coef=lw.depth,
+                                 past=torch.empty_like(x))
+                    end.update(hist=ahead["past"].unsqueeze(0),
+                               coef=lw.depth_end)
+                xn = self._stream_step(b, x, y, lw.norm1b, rows=True, **ahead)
                 if lw.experts is not None:
                     out, weight, plan = lw.experts(xn)
                     y = self._shared_expert(lw, xn)

@@ -311,7 +311,7 @@ def _group_rms(x, groups, eps):
 def stream_step(x, y=None, post_w=None, xn=None, next_w=None, groups=1,
                 eps=1e-6, tokens=None, table=None, scale=1.0, routed=None,
                 routed_w=None, chosen=None, experts=0, hist=None, coef=None,
-                keep=None, shift=None, prev=None, row_slot=None,
+                keep=None, past=None, shift=None, prev=None, row_slot=None,
                 row_pos=None) -> None:
     if tokens is not None:
         x.copy_(table[tokens.long()].float() * scale)
@@ -329,7 +329,9 @@ def stream_step(x, y=None, post_w=None, xn=None, next_w=None, groups=1,
         x += a
     if keep is not None:
         keep.copy_(x)
-    if coef is not None:
+    if past is not None:
+        past.copy_((hist * coef[:-1].view(-1, 1, 1)).sum(0))
+    elif coef is not None:
         x.copy_((hist * coef[:-1].view(-1, 1, 1)).sum(0) + coef[-1] * x)
     if xn is None:
         return

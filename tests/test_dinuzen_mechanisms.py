@@ -65,6 +65,14 @@ def test_average_over_depth(e, groups, depth, device, dtype):
     w = rand(e, seed=3, device=device)
     hist = rand(depth + 1, n, e, seed=4, device=device)
     coef = rand(depth + 1, seed=5, device=device)
+    # ahead of time, beside another step that only adds
+    z, x0 = torch.zeros_like(y), x.clone()
+    past = torch.full((n, e), 5.0, device=device)
+    ops.stream_step(x, z, w, groups=groups, eps=eps, hist=hist[:depth],
+                    coef=coef, past=past)
+    assert torch.equal(x, x0)
+    close(past, oracle.depth_average(list(f64(hist[:depth])),
+                                     f64(coef[:-1])), torch.float32)
     xn = torch.empty(n, e, dtype=dtype, device=device)
     own = f64(x) + oracle.group_norm(f64(y), f64(w), groups, eps)
     want = oracle.depth_average(list(f64(hist[:depth])) + [own], f64(coef))
