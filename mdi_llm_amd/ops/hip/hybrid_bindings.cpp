@@ -293,6 +293,8 @@ void qk_norm_append(torch::Tensor q_out, Opt kpages, Opt vpages,
     a.rope = f32_ptr(*rope, rope->numel(), "rope");
     a.rot = 2 * (int)rope->size(1);
   }
+  TORCH_CHECK((int64_t)a.n * (a.heads + a.k_heads) < (int64_t)1 << 31,
+              "qk_norm_append: rows");
   a.q_out = q_out.data_ptr();
   a.proj = proj.data_ptr();
   a.q_w = f32_ptr(q_w, a.dim, "q_w");

@@ -439,8 +439,10 @@ __global__ __launch_bounds__(256) void qk_norm_append_kernel(
   const long long i = (long long)blockIdx.x * PER + threadIdx.x / L;
   if (i >= (long long)n * hk) return;
   const int lane = threadIdx.x % L;
-  const size_t row = i / hk;
-  const int hd = (int)(i - row * hk);
+  // (fewer pairs than 2^31: the host checks)
+  const unsigned r32 = (unsigned)i / (unsigned)hk;
+  const size_t row = r32;
+  const int hd = (int)((unsigned)i - r32 * hk);
   const bool is_q = hd < heads;
   const T* src = proj + row * (size_t)ld + (size_t)hd * dim;
   const float* w = is_q ? q_w : k_w;
@@ -562,7 +564,10 @@ void launch_qk_norm_append(const QkAppendArgs& a, int f32,
     if (a.dim % 4 == 0 && a.vdim % 4 == 0) append_t<float, 4, 16>(a, stream);
     else append_t<float, 1, 64>(a, stream);
   } else {
-    if (a.dim % 8 == 0 && a.vdim % 8 == 0) append_t<bf16, 8, 16>(a, stream);
+    if (a.dim % 8 == 0 && a.vdim % 8 == 0 && a.dpad <= 64)
+      append_t<bf16, 8, 8>(a, stream);
+    else if (a.dim % 8 == 0 && a.vdim % 8 == 0)
+      append_t<bf16, 8, 16>(a, stream);
     else append_t<bf16, 1, 64>(a, stream);
   }
 }
