@@ -20,7 +20,8 @@ that makes them).  A short convolution's last inputs (``conv``, ``[slots, taps
 (``prev``, fp32) are part of a slot as well.
 
 Nothing needs clearing when a page or slot is taken again: keys past a
-sequence's end are masked, and a recurrence, a convolution and a shift start from zeros at position 0.
+sequence's end are masked, and a recurrence, a convolution and a shift start
+from zeros at position 0.
 """
 
 from __future__ import annotations
