@@ -55,7 +55,8 @@ class ModelConfig:
     norm_class_name: Literal["LayerNorm", "RMSNorm"] = "LayerNorm"
     norm_eps: float = 1e-5
     mlp_class_name: Literal["GptNeoxMLP", "LLaMAMLP", "GemmaMLP", "LLaMAMoE",
-                            "XieluMLP", "GatedMLP", "GeluMLP"] = "GptNeoxMLP"
+                            "XieluMLP", "GatedMLP", "GeluMLP",
+                            "SquaredReluMLP"] = "GptNeoxMLP"
     gelu_approximate: str = "none"
     intermediate_size: Optional[int] = None
     rope_condense_ratio: int = 1
@@ -68,7 +69,8 @@ class ModelConfig:
     pos_embedding: Literal["rope", "learned"] = "rope"
     # -- stacks whose layers differ (models/hybrid.py) --
     # one entry per layer: {"type": mixer, "mixer": {sizes and constants},
-    # "mlp": {"kind", sizes} or None}; None means n_layer equal blocks
+    # "mlp": {"kind", sizes} or None}; None means n_layer equal blocks.  An
+    # entry with "weights_of" uses that layer's parameters (its own cache)
     layers: Optional[list] = None
     embedding_scale: float = 1.0
     # RMS norm weights are stored as w with norm_offset + w applied
@@ -87,6 +89,8 @@ class ModelConfig:
     depth_average: bool = False
     # what a layer adds to the residual stream is multiplied by this
     residual_mult: float = 1.0
+    # ... and the logits by this
+    logit_scale: float = 1.0
 
     def __post_init__(self) -> None:
         if self.layers is not None:
@@ -115,8 +119,9 @@ class ModelConfig:
     def _sizes_from_layers(self) -> None:
         """Fill the uniform-stack fields from the layer list, so that code
         which only sizes or splits a model need not know about it."""
-        first = next((l["mixer"] for l in self.layers
-                      if "heads" in l["mixer"]), {})
+        mixers = [part for l in self.layers
+                  for part in (l["mixer"], l["mixer"].get("left", {}))]
+        first = next((m for m in mixers if "heads" in m), {})
         self.n_layer = len(self.layers)
         self.n_head = first.get("heads", 1)
         self.n_query_groups = first.get("kv_heads", self.n_head)
@@ -159,6 +164,11 @@ class ModelConfig:
         streams = 1 + (self.n_layer if self.depth_average else 0)
         return streams * self.n_embd + sum(self.shared_rows().values())
 
+    def weights_of(self, i: int) -> int:
+        """The layer whose parameters layer ``i`` uses."""
+        return (self.layers[i].get("weights_of", i)
+                if self.layers is not None else i)
+
     def layer_weights(self, i: int, active: bool = False) -> int:
         """Number of matrix weights of layer ``i``; if ``active``, of those
         that one token uses."""
@@ -189,6 +199,13 @@ class ModelConfig:
         elif layer["type"] == "rglru":
             rows = 3 * m["width"]
             inner = 2 * m["width"] ** 2 // m["blocks"]
+        elif layer["type"] == "paired":
+            a = m["left"]
+            rows = (a["heads"] + a["kv_heads"]) * a["dim"] \
+                + (2 * a["heads"] + a["kv_heads"]) * a["vdim"] \
+                + 4 * m["right"]["width"]
+        elif layer["type"] == "mlstm":
+            rows = 2 * m["heads"] * (m["dim"] + m["vdim"] + 1)
         else:
             rows = m["heads"] * (2 * m["dim"] + m["vdim"])
         if "heads" in m:
@@ -401,8 +418,56 @@ def _dinuzen(raw: dict) -> dict:
     )
 
 
+def _sosutar(raw: dict) -> dict:
+    """Sosutar: matrix memories with exponential gates (mLSTM), and pairs of
+    gated attention and a minimal gated recurrence (minGRU) that read one
+    input; learned positions, layer scale, squared-ReLU feed-forwards; layers
+    may use an earlier layer's parameters."""
+    layers = copy.deepcopy(raw["layers"])
+    for i, layer in enumerate(layers):
+        if layer["type"] not in ("mlstm", "parallel"):
+            raise ValueError(f"Sosutar: unknown mixer {layer['type']!r}")
+        if layer["mlp"] is not None and layer["mlp"]["kind"] != "dense":
+            raise ValueError(
+                f"Sosutar: unknown feed-forward {layer['mlp']['kind']!r}")
+        if layer["type"] == "parallel":
+            layer["type"] = "paired"
+            layer["mixer"]["left"]["type"] = "gated_attention"
+            layer["mixer"]["right"]["type"] = "mingru"
+    for i, layer in enumerate(layers):
+        src, hops = layer.pop("weights_of", None), 0
+        if src is None:
+            continue
+        # of a layer that shares itself: the one with the tensors
+        while raw["layers"][src].get("weights_of") is not None:
+            src, hops = raw["layers"][src]["weights_of"], hops + 1
+            if hops > len(layers):
+                raise ValueError(f"Sosutar: layer {i} has no weights")
+        if any(layers[src][key] != layer[key]
+               for key in ("type", "mixer", "mlp")):
+            raise ValueError(f"Sosutar: layers {i} and {src} share weights "
+                             "but differ")
+        layer["weights_of"] = src
+    return dict(
+        name="Sosutar",
+        block_size=raw["max_positions"],
+        vocab_size=raw["vocab"],
+        padded_vocab_size=raw["vocab"],
+        n_embd=raw["width"],
+        layers=layers,
+        embedding_scale=raw["embedding"]["scale"],
+        pos_embedding="learned",
+        norm_class_name="RMSNorm",
+        norm_eps=raw["norm"]["eps"],
+        layer_scale=True,
+        logit_scale=raw["logit_scale"],
+        parallel_residual=False,
+        mlp_class_name="SquaredReluMLP",
+    )
+
+
 native_architectures = {"Nerozen": _nerozen, "Resolorn": _resolorn,
-                        "Dinuzen": _dinuzen}
+                        "Dinuzen": _dinuzen, "Sosutar": _sosutar}
 
 
 def is_native_checkpoint(path: Union[str, Path]) -> bool:
@@ -2441,6 +2506,55 @@ configs.extend([
                    _dinuzen_attention(32, 8, 64, 128, 0.7), 21504,
                    dict(router=dict(experts=32, identity=2, top=6, scale=2.0),
                         expert=dict(ff=2048), shared=dict(ff=2048)), 8),
+])
+
+
+# -- Sosutar -----------------------------------------------------
+
+
+def _sosutar_named(name: str, n_layer: int, width: int, vocab: int, ff: int,
+                   mlstm: dict, left: dict, right: dict, every: int,
+                   block_size: int, again: tuple = ()) -> dict:
+    """A Sosutar stack with a pair of attention and recurrence in every
+    ``every``-th layer and a matrix memory in the others; layers ``again``
+    use the parameters of the layer before."""
+    layers = []
+    for i in range(n_layer):
+        pair = i % every == every - 1
+        mixer = dict(left=dict(left), right=dict(right)) if pair \
+            else dict(mlstm)
+        layers.append(dict(type="parallel" if pair else "mlstm", mixer=mixer,
+                           mlp=dict(kind="dense", ff=ff)))
+        if i in again:
+            layers[i]["weights_of"] = i - 1
+    conf = _sosutar(dict(vocab=vocab, width=width, layers=layers,
+                         embedding=dict(scale=1.0), norm=dict(eps=1e-6),
+                         logit_scale=1.0, max_positions=block_size))
+    conf.update(name=name)
+    return conf
+
+
+def _sosutar_attention(heads: int, kv_heads: int, dim: int, size: int,
+                       every: int = 8192) -> dict:
+    return dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim,
+                scale=dim ** -0.5, mask=dict(size=size),
+                q_temp=dict(coef=0.1, every=every))
+
+
+configs.extend([
+    _sosutar_named("sosutar-nano", 5, 128, 384, 320,
+                   dict(heads=4, dim=24, vdim=40, gate_cap=10.0),
+                   _sosutar_attention(6, 2, 32, 72, 50), dict(width=160),
+                   every=3, block_size=1024, again=(1,)),
+    # TinyLlama-1.1B and Llama-3-8B widths and weights
+    _sosutar_named("sosutar-1b", 22, 2048, 32000, 5632,
+                   dict(heads=16, dim=128, vdim=128, gate_cap=15.0),
+                   _sosutar_attention(32, 4, 64, 1024), dict(width=2048),
+                   every=4, block_size=32768),
+    _sosutar_named("sosutar-8b", 32, 4096, 128256, 16384,
+                   dict(heads=32, dim=128, vdim=128, gate_cap=15.0),
+                   _sosutar_attention(32, 8, 128, 2048), dict(width=4096),
+                   every=4, block_size=32768),
 ])
 
 

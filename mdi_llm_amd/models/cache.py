@@ -15,7 +15,9 @@ token, states ``[slots, heads, dim, vstride]`` (or ``[slots, channels]``) in
 fp32.  Differential attention has a K page per map and kv head, ``[pages,
 kv_heads * 2, 64 * dpad]``.  Layers that read one latent, or one layer's keys
 and values, share its pages (``latent``, ``k`` and ``v`` are keyed by the layer
-that makes them).  A short convolution's last inputs (``conv``, ``[slots, taps
+that makes them).  A matrix memory with exponential gates keeps its
+normaliser as one more column and the exponent of both in ``peak`` (``[slots,
+heads]``, fp32).  A short convolution's last inputs (``conv``, ``[slots, taps
 - 1, channels]``) and the previous token's row of a layer with token shift
 (``prev``, fp32) are part of a slot as well.
 
@@ -89,7 +91,11 @@ class HybridCache:
         self.latent: Dict[int, torch.Tensor] = {}
         self.conv: Dict[int, torch.Tensor] = {}
         self.prev: Dict[int, torch.Tensor] = {}
-        for i, m in enumerate(mixers):
+        self.peak: Dict[int, torch.Tensor] = {}
+        # (a mixer that is made of parts caches what they cache)
+        parts = [(i, p) for i, m in enumerate(mixers)
+                 for p in getattr(m, "parts", (m,))]
+        for i, m in parts:
             if shift_width:
                 self.prev[i] = torch.zeros(n_slots + 1, shift_width,
                                            device=device,
@@ -98,7 +104,7 @@ class HybridCache:
                 self.conv[i] = torch.zeros(n_slots + 1, max(1, m.taps - 1),
                                            m.channels, device=device,
                                            dtype=dtype)
-            if m.kind in ("attention", "diff_attention"):
+            if m.kind in ("attention", "diff_attention", "gated_attention"):
                 if m.source in self.k:
                     continue
                 dpad = _pad_to(m.dim, (32, 64, 128, 256), "attention dim")
@@ -116,12 +122,18 @@ class HybridCache:
                     self.latent[m.source] = torch.zeros(
                         self.n_pages + 1, PAGE, rpad, device=device,
                         dtype=dtype)
-            elif m.kind == "rglru":
+            elif m.kind in ("rglru", "mingru"):
                 self.state[i] = torch.zeros(n_slots + 1, m.width,
                                             device=device,
                                             dtype=torch.float32)
             else:
-                vstride = -(-m.vdim // 4) * 4
+                cols = m.vdim
+                if m.kind == "mlstm":
+                    cols += 1
+                    self.peak[i] = torch.zeros(n_slots + 1, m.heads,
+                                               device=device,
+                                               dtype=torch.float32)
+                vstride = -(-cols // 4) * 4
                 self.state[i] = torch.zeros(
                     n_slots + 1, m.heads, m.dim, vstride, device=device,
                     dtype=torch.float32)
@@ -206,5 +218,5 @@ class HybridCache:
     def memory_bytes(self) -> int:
         return sum(t.numel() * t.element_size()
                    for d in (self.k, self.v, self.state, self.latent,
-                             self.conv, self.prev)
+                             self.conv, self.prev, self.peak)
                    for t in d.values())

@@ -18,7 +18,7 @@ import torch.nn as nn
 
 from ..config import ModelConfig
 
-__all__ = ["HybridBlock", "ParallelBlock", "make_block",
+__all__ = ["HybridBlock", "ParallelBlock", "make_block", "make_blocks",
            "native_state_dict", "native_tensors"]
 
 
@@ -176,6 +176,91 @@ class DiffAttention(nn.Module):
                      + self.diff)
 
 
+class MLSTMMixer(nn.Module):
+    """Matrix memory per head with exponential input and forget gates, both
+    capped: in_proj rows are q | k | v | output gate | input gate logits |
+    forget gate logits."""
+
+    kind = "mlstm"
+
+    def __init__(self, width: int, spec: dict, index: int) -> None:
+        super().__init__()
+        self.heads, self.dim, self.vdim = (
+            spec["heads"], spec["dim"], spec["vdim"])
+        self.gate_cap = float(spec["gate_cap"])
+        H = self.heads
+        self.in_proj = nn.Linear(
+            width, 2 * H * (self.dim + self.vdim + 1), bias=False)
+        self.gate_bias = nn.Parameter(torch.zeros(2 * H))
+        self.norm = Scale(H * self.vdim)
+        self.proj = nn.Linear(H * self.vdim, width, bias=False)
+
+
+class GatedAttention(nn.Module):
+    """Windowed attention with norms over all query and all key channels,
+    queries that warm up with their position, values of unit size, a fixed
+    slope by distance, a sink in the softmax and an element-wise output gate.
+    Part of a ``PairedMixer``: in_rows are its rows of the pair's in_proj."""
+
+    kind = "gated_attention"
+
+    def __init__(self, width: int, spec: dict, index: int) -> None:
+        super().__init__()
+        self.source = index     # model-wide index of the layer's K/V pages
+        self.heads, self.kv_heads = spec["heads"], spec["kv_heads"]
+        if self.heads % self.kv_heads:
+            raise ValueError("heads must be a multiple of kv_heads")
+        self.dim, self.vdim = spec["dim"], spec["vdim"]
+        self.scale = float(spec["scale"])
+        self.q_temp = spec.get("q_temp")
+        self.window = int((spec.get("mask") or {}).get("size", 1 << 30))
+        self.keep_first = 0
+        q, k = self.heads * self.dim, self.kv_heads * self.dim
+        self.inner = self.heads * self.vdim
+        self.in_rows = q + k + self.kv_heads * self.vdim + self.inner
+        self.q_norm, self.k_norm = Scale(q), Scale(k)
+        self.sink = nn.Parameter(torch.zeros(self.heads))
+        self.proj = nn.Linear(self.inner, width, bias=False)
+
+
+class MinGRU(nn.Module):
+    """Gated recurrence per channel whose gates read the current token only.
+    Part of a ``PairedMixer``: its rows of in_proj are gate z | input | output
+    gate, of which the first two have a bias."""
+
+    kind = "mingru"
+
+    def __init__(self, width: int, spec: dict, index: int) -> None:
+        super().__init__()
+        self.width = self.inner = spec["width"]
+        self.in_rows = 3 * self.width
+        self.bias = nn.Parameter(torch.zeros(2 * self.width))
+        self.proj = nn.Linear(self.width, width, bias=False)
+
+
+PARTS = {m.kind: m for m in (GatedAttention, MinGRU)}
+
+
+class PairedMixer(nn.Module):
+    """Two mixers side by side over one input, whose outputs are normed and
+    averaged.  in_proj rows: the left part's, then the right part's."""
+
+    kind = "paired"
+
+    def __init__(self, width: int, spec: dict, index: int) -> None:
+        super().__init__()
+        self.left, self.right = (
+            PARTS[spec[side]["type"]](width, spec[side], index)
+            for side in ("left", "right"))
+        self.in_proj = nn.Linear(
+            width, self.left.in_rows + self.right.in_rows, bias=False)
+        self.left_norm, self.right_norm = Scale(width), Scale(width)
+
+    @property
+    def parts(self):
+        return self.left, self.right
+
+
 class XieluMLP(nn.Module):
     kind = "dense"
 
@@ -195,6 +280,10 @@ class GeluMLP(nn.Module):
         super().__init__()
         self.fc = nn.Linear(width, spec["ff"], bias=False)
         self.proj = nn.Linear(spec["ff"], width, bias=False)
+
+
+class SquaredReluMLP(GeluMLP):
+    """Up, squared ReLU, down."""
 
 
 class LatentAttention(nn.Module):
@@ -290,9 +379,11 @@ class CorrectedRoutedMLP(RoutedMLP):
 
 
 MIXERS = {m.kind: m for m in (HGRN2Mixer, BiasedAttention, RGLRUMixer,
-                              Mamba2Mixer, DiffAttention)}
+                              Mamba2Mixer, DiffAttention, MLSTMMixer,
+                              PairedMixer)}
 MLPS = {"XieluMLP": {"dense": XieluMLP},
-        "GeluMLP": {"dense": GeluMLP, "moe": CorrectedRoutedMLP}}
+        "GeluMLP": {"dense": GeluMLP, "moe": CorrectedRoutedMLP},
+        "SquaredReluMLP": {"dense": SquaredReluMLP}}
 PARALLEL_MIXERS = {m.kind: m for m in (LatentAttention,)}
 PARALLEL_MLPS = {m.kind: m for m in (GatedMLP, RoutedMLP)}
 
@@ -351,6 +442,27 @@ class ParallelBlock(nn.Module):
         return mlp + self.mixer.in_rows + self.mixer.gate_rows
 
 
+def make_blocks(config: ModelConfig, first: int, n: int) -> nn.ModuleList:
+    """Layers ``first`` .. of the model.  Those that use another layer's
+    weights hold its parameters, as long as it is one of them; else they have
+    a copy."""
+    blocks = nn.ModuleList(make_block(config, first + i) for i in range(n))
+    seen: Dict[int, nn.Module] = {}
+    for i, block in enumerate(blocks):
+        owner = seen.setdefault(config.weights_of(first + i), block)
+        if owner is not block:
+            _share(block, owner)
+    return blocks
+
+
+def _share(block: nn.Module, owner: nn.Module) -> None:
+    for name in owner._parameters:
+        block._parameters[name] = owner._parameters[name]
+    for name, part in owner._modules.items():
+        if part is not None:
+            _share(block._modules[name], part)
+
+
 def make_block(config: ModelConfig, index: int) -> nn.Module:
     cls = ParallelBlock if config.parallel_residual else HybridBlock
     return cls(config, index)
@@ -372,7 +484,7 @@ def native_tensors(config: ModelConfig) -> Dict[str, Tuple[str, ...]]:
     if config.pos_embedding == "learned":
         out["transformer.wpe.weight"] = ("pos",)
     for i, spec in enumerate(config.layers):
-        src, dst = f"l{i}.", f"transformer.h.{i}."
+        src, dst = f"l{config.weights_of(i)}.", f"transformer.h.{i}."
         if config.parallel_residual:
             out.update(_parallel_tensors(spec, src, dst))
             continue
@@ -397,6 +509,18 @@ _MIXER_TENSORS = {
                        "q_norm.weight": ("q.norm",),
                        "k_norm.weight": ("k.norm",),
                        "lam": ("lq1", "lk1", "lq2", "lk2")},
+    "mlstm": {"in_proj.weight": ("q", "k", "v", "g", "i", "f"),
+              "gate_bias": ("i.b", "f.b"), "norm.weight": ("norm",)},
+    "paired": {"in_proj.weight": ("left.q", "left.k", "left.v", "left.g",
+                                  "right.z", "right.x", "right.g"),
+               "left.q_norm.weight": ("left.q.norm",),
+               "left.k_norm.weight": ("left.k.norm",),
+               "left.sink": ("left.sink",),
+               "left.proj.weight": ("left.o",),
+               "right.bias": ("right.z.b", "right.x.b"),
+               "right.proj.weight": ("right.o",),
+               "left_norm.weight": ("left.out",),
+               "right_norm.weight": ("right.out",)},
 }
 
 
@@ -423,7 +547,8 @@ def _block_tensors(config: ModelConfig, spec: dict, src: str,
                 continue
             names = tuple(n for n in names if n not in ("k", "v"))
         out[mixer + key] = tuple(mix + n for n in names)
-    out[mixer + "proj.weight"] = (mix + "o",)
+    if spec["type"] != "paired":    # (whose parts have one each)
+        out[mixer + "proj.weight"] = (mix + "o",)
     if mlp is None:
         return out
     pre, to = src + "mlp.", dst + "mlp."
@@ -482,9 +607,12 @@ def _parallel_tensors(spec: dict, src: str, dst: str) -> dict:
 def native_state_dict(config: ModelConfig, get) -> dict:
     """State dict in the framework's layout; ``get(name)`` reads one tensor
     (so that a file is read tensor by tensor)."""
-    sd = {}
+    sd, made = {}, {}
     for key, names in native_tensors(config).items():
-        parts = [get(n) for n in names]
-        dim = 1 if key.endswith(".out_proj.weight") else 0
-        sd[key] = parts[0] if len(parts) == 1 else torch.cat(parts, dim)
+        if names not in made:   # (layers may use the same tensors)
+            parts = [get(n) for n in names]
+            dim = 1 if key.endswith(".out_proj.weight") else 0
+            made[names] = parts[0] if len(parts) == 1 \
+                else torch.cat(parts, dim)
+        sd[key] = made[names]
     return sd

@@ -24,7 +24,7 @@ import torch.nn as nn
 
 from ..config import ModelConfig
 from .cache import HybridCache
-from .hybrid import Scale, make_block
+from .hybrid import Scale, make_blocks
 from .model import Block, KVCachePool, build_rope_cache, norm_class
 
 __all__ = ["StageBase", "StarterStage", "SecondaryStage", "build_stage"]
@@ -44,9 +44,11 @@ class StageBase(nn.Module):
         self._build_rope()
 
     def _make_blocks(self) -> nn.ModuleList:
-        cls = make_block if self.config.is_hybrid else Block
+        if self.config.is_hybrid:
+            return make_blocks(self.config, self.first_layer,
+                               self.n_local_layers)
         return nn.ModuleList(
-            cls(self.config, self.first_layer + i)
+            Block(self.config, self.first_layer + i)
             for i in range(self.n_local_layers)
         )
 

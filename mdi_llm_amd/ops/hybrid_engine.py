@@ -36,7 +36,7 @@ from ..models.sampling import sample as sample_token
 from ..models.model import build_pair_rope_table
 from . import require_hip_ops
 from .experts import RoutedExperts
-from .mixers import RGLRU, Mamba2
+from .mixers import MIXERS
 from .latent_layer import LatentPlan, ParallelLayer, make_plan
 
 __all__ = ["HybridEngine", "distance_bias"]
@@ -97,7 +97,7 @@ class Batch:
 
 
 FEW_ROWS = 64           # rows whose residual steps are bound by latency
-XIELU, GELU = 1, 2      # activations that a projection can end with
+XIELU, GELU, RELU2 = 1, 2, 3    # activations that a projection can end with
 
 
 class _LayerWeights:
@@ -112,18 +112,27 @@ class _LayerWeights:
 
         self.norm1, self.norm1b = w(block.norm_1), w(block.norm_1b)
         self.norm2, self.norm2b = w(block.norm_2), w(block.norm_2b)
+        m = block.mixer
+        self.norm1c = None      # of a second output beside the first
+        if m.kind == "paired":
+            self.norm1b = 0.5 * w(m.left_norm)
+            self.norm1c = 0.5 * w(m.right_norm)
         # a factor on a sublayer's output joins the weight of its norm
-        for n, ls in (("norm1b", block.ls_1), ("norm2b", block.ls_2)):
-            if ls is not None:
-                setattr(self, n, getattr(self, n) * w(ls))
+        self.gain1, self.gain2 = w(block.ls_1), w(block.ls_2)
+        if self.norm1b is not None and self.gain1 is not None:
+            self.norm1b = self.norm1b * self.gain1
+            if self.norm1c is not None:
+                self.norm1c = self.norm1c * self.gain1
+            self.gain1 = None
+        if self.norm2b is not None and self.gain2 is not None:
+            self.norm2b, self.gain2 = self.norm2b * self.gain2, None
         self.shift, self.depth = w(block.shift), w(block.depth)
         if self.depth is not None:  # for a sum over earlier results
             self.depth_end = torch.stack((torch.ones_like(self.depth[-1]),
                                           self.depth[-1]))
-        m = block.mixer
-        self.mixer = m
-        if m.kind in ("rglru", "mamba2"):
-            self.mix = (RGLRU if m.kind == "rglru" else Mamba2)(eng, i, m)
+        self.mixer, self.mix = m, None
+        if m.kind in MIXERS:
+            self.mix = MIXERS[m.kind](eng, i, m)
         else:
             self.in_proj = m.in_proj.weight.detach()
             self.proj = m.proj.weight.detach()
@@ -159,7 +168,8 @@ class _LayerWeights:
         if hasattr(mlp, "act"):
             self.act = (XIELU, *F.softplus(mlp.act.detach().float()).tolist())
         else:
-            self.act = (GELU, 0.0, 0.0)
+            squared = eng.config.mlp_class_name == "SquaredReluMLP"
+            self.act = (RELU2 if squared else GELU, 0.0, 0.0)
 
 
 class _DecodeStep:
@@ -222,7 +232,7 @@ class HybridEngine:
         self.latent_form: Optional[str] = None  # "absorbed" or "expanded"
         # longest sequence that can occur
         self.max_ctx = min(cache.n_pages * PAGE, stage.max_seq_length)
-        self._ropes: Dict[str, torch.Tensor] = {}
+        self._tables: Dict[str, torch.Tensor] = {}  # by position
         if self.parallel:
             self.layers = [ParallelLayer(self, b) for b in stage.transformer.h]
         else:
@@ -234,7 +244,9 @@ class HybridEngine:
                 raise ValueError("hgrn2: dim <= 256 and vdim <= 1024")
         if self.is_starter:
             self.wte = stage.transformer.wte.weight.detach()
-            self.final = stage.transformer.ln_f.weight.detach().float()
+            # (a factor on the logits joins the last norm's weight)
+            self.final = stage.transformer.ln_f.weight.detach().float() \
+                * self.config.logit_scale
             self.head = stage.lm_head.weight.detach()
             wpe = getattr(stage.transformer, "wpe", None)
             self.wpe = None if wpe is None else wpe.weight.detach()
@@ -262,19 +274,35 @@ class HybridEngine:
         """cos and sin by position, one table for all layers that rotate
         alike."""
         key = repr(sorted(rot.items(), key=str))
-        if key not in self._ropes:
-            self._ropes[key] = build_pair_rope_table(self.max_ctx, rot,
-                                                     self.device)
-        return self._ropes[key]
+        if key not in self._tables:
+            self._tables[key] = build_pair_rope_table(self.max_ctx, rot,
+                                                      self.device)
+        return self._tables[key]
+
+    def query_scale_table(self, every, coef: float) -> torch.Tensor:
+        """Factors on queries that grow with the logarithm of the position,
+        a step every ``every`` tokens."""
+        key = repr(("query scale", every, coef))
+        if key not in self._tables:
+            p = torch.arange(1, self.max_ctx + 1, dtype=torch.float64)
+            f = 1.0 + coef * torch.log(torch.floor(p / every) + 1.0)
+            self._tables[key] = f.float().to(self.device)
+        return self._tables[key]
 
     # ------------------------------------------------------------------
     # building blocks
     # ------------------------------------------------------------------
     def _norm_step(self, x, y=None, post_w=None, next_w=None, tokens=None,
-                   row_pos=None, routed=None):
+                   row_pos=None, routed=None, gain=None, post_w2=None):
         """x <- embed(tokens) or x + post-norm(y) (+ routed experts); the
-        next pre-norm."""
+        next pre-norm.  ``gain``: factors on y without a norm; a pair of
+        outputs in y has two post-norms."""
         xn, extra = None, {}
+        if isinstance(y, tuple):
+            y, y2 = y
+            extra.update(y2=y2, post_w2=post_w2)
+        if gain is not None:
+            extra.update(gain=gain)
         if tokens is not None and self.wpe is not None:
             extra.update(pos_table=self.wpe, row_pos=row_pos)
         if routed is not None:
@@ -307,8 +335,10 @@ class HybridEngine:
         out = F.linear(x, w)
         if act is not None and act[0] == XIELU:
             self.ops.xielu(out, *act[1:])
-        elif act is not None:
+        elif act is not None and act[0] == GELU:
             self.ops.gelu(out)
+        elif act is not None:
+            self.ops.relu2(out)
         return out
 
     def _hgrn2(self, i: int, lw: _LayerWeights, b: Batch, xn: torch.Tensor):
@@ -345,13 +375,22 @@ class HybridEngine:
         self.ops.qk_norm_append(q, k if owns else None, v if owns else None,
                                 proj, lw.q_norm, lw.k_norm, b.row_slot,
                                 b.row_pos, c.table, m.vdim, eps, **lw.rotate)
+        return self._linear(self.attend(m, b, q, lw.bias, **lw.two_maps),
+                            lw.proj)
+
+    def attend(self, m, b: Batch, q: torch.Tensor, bias=None, **kw):
+        """Heads' outputs [n, heads * vdim] of padded queries over the cached
+        keys and values, this step's included."""
+        c = self.cache
+        k, v = c.k[m.source], c.v[m.source]
+        maps = k.size(1) // m.kv_heads
         y = torch.empty(b.n, m.heads * m.vdim, dtype=self.dtype,
                         device=self.device)
 
         def attend(seg, max_len, splits, part=(None, None)):
-            self.ops.paged_attn(y, q, k, v, lw.bias, c.table, seg, max_len,
+            self.ops.paged_attn(y, q, k, v, bias, c.table, seg, max_len,
                                 m.window, m.keep_first, m.scale, splits,
-                                *part, **lw.two_maps)
+                                *part, **kw)
 
         if b.singles:
             splits = self._splits(m, b.singles, b.max_ctx)
@@ -365,10 +404,10 @@ class HybridEngine:
             attend(b.seg[:, :b.singles], 1, splits, part)
         if b.singles < b.seg.size(1):
             attend(b.seg[:, b.singles:], b.max_len, 0)
-        return self._linear(y, lw.proj)
+        return y
 
     def _mix(self, i: int, lw: _LayerWeights, b: Batch, xn: torch.Tensor):
-        if lw.mixer.kind in ("rglru", "mamba2"):
+        if lw.mix is not None:
             return lw.mix(b, xn)
         if lw.mixer.kind == "hgrn2":
             return self._hgrn2(i, lw, b, xn)
@@ -493,11 +532,13 @@ class HybridEngine:
                 continue
             y = self._mix(i, lw, b, xn)
             if lw.mlp:
-                xn = self._norm_step(x, y, lw.norm1b, lw.norm2)
+                xn = self._norm_step(x, y, lw.norm1b, lw.norm2,
+                                     gain=lw.gain1, post_w2=lw.norm1c)
                 y = self._linear(self._linear(xn, lw.fc, lw.act), lw.down)
-                xn = self._norm_step(x, y, lw.norm2b, after)
+                xn = self._norm_step(x, y, lw.norm2b, after, gain=lw.gain2)
             else:
-                xn = self._norm_step(x, y, lw.norm1b, after)
+                xn = self._norm_step(x, y, lw.norm1b, after, gain=lw.gain1,
+                                     post_w2=lw.norm1c)
             if layers_out is not None:
                 layers_out.append(x.clone())
         return x, xn

@@ -17,7 +17,8 @@ __all__ = ["residual_norm", "xielu", "hgrn2_step", "hgrn2_scan",
            "gated_act", "moe_route", "moe_up", "moe_down", "advance_batch",
            "stream_step", "token_shift", "gelu", "causal_conv", "rglru_step",
            "rglru_scan", "mamba2_step", "mamba2_scan", "mamba2_out",
-           "kv_rows"]
+           "kv_rows", "row_norm_append", "relu2", "mlstm_step", "mlstm_scan",
+           "mingru_step", "mingru_scan"]
 
 
 def _rms(x: torch.Tensor, eps: float) -> torch.Tensor:
@@ -27,14 +28,18 @@ def _rms(x: torch.Tensor, eps: float) -> torch.Tensor:
 
 def residual_norm(x, y=None, post_w=None, xn=None, next_w=None, tokens=None,
                   table=None, scale=1.0, offset=0.0, eps=1e-6, mult=1.0,
-                  pos_table=None, row_pos=None, routed=None,
-                  routed_w=None) -> None:
+                  pos_table=None, row_pos=None, routed=None, routed_w=None,
+                  gain=None, y2=None, post_w2=None) -> None:
     if tokens is not None:
         x.copy_(table[tokens.long()].float() * scale)
         if pos_table is not None:
             x += pos_table[row_pos.long()].float()
     elif y is not None:
         a = y.float() if post_w is None else _rms(y, eps) * (offset + post_w)
+        if gain is not None:
+            a = a * gain
+        if y2 is not None:
+            a = a + _rms(y2, eps) * (offset + post_w2)
         if routed is not None:
             a = a + (routed.float() * routed_w.unsqueeze(-1)).sum(1)
         x += a * mult
@@ -122,9 +127,28 @@ def kv_rows(rows, kpages, vpages, row_slot, row_pos, table, dim, vdim,
             cols.copy_(pages[where])
 
 
+def row_norm_append(q_out, kpages, vpages, proj, q_w, k_w, row_slot, row_pos,
+                    table, vdim, eps, q_scale=None, unit_values=True) -> None:
+    n, H, _ = q_out.shape
+    G, D = kpages.size(1), q_w.numel() // H
+    pos = row_pos.long()
+    q, k, v = proj.split((H * D, G * D, G * vdim), dim=1)
+    q = _rms(q, eps) * q_w
+    if q_scale is not None:
+        q = q * q_scale[pos].unsqueeze(1)
+    q_out.zero_()
+    q_out[..., :D] = q.view(n, H, D).to(q_out.dtype)
+    k = _rms(k, eps) * k_w
+    if unit_values:
+        v = _rms(v.reshape(n, G, vdim), eps).flatten(1)
+    kv_rows(torch.cat((k, v), 1).to(proj.dtype), kpages, vpages, row_slot,
+            row_pos, table, D, vdim, True)
+
+
 def paged_attn(out, q, kpages, vpages, bias, table, seg, max_len, window,
                keep_first, scale, splits, part_o=None, part_ml=None,
-               softcap=0.0, map_weight=0.0, out_scale=1.0, eps=0.0) -> None:
+               softcap=0.0, map_weight=0.0, out_scale=1.0, eps=0.0,
+               slopes=None, sink=None, gate=None) -> None:
     """Two key heads per value head: each query head has two maps, and what
     is stored is the unit-size difference of their outputs."""
     D = q.size(2)
@@ -133,7 +157,6 @@ def paged_attn(out, q, kpages, vpages, bias, table, seg, max_len, window,
     H = q.size(1) // maps
     E = out.size(1) // H
     ki, vi = k_index(D), v_index(vpages.size(2) // PAGE)[:, :E]
-    far = bias.size(1) - 1
     for start, n, slot, pos0 in _segments(seg):
         total = pos0 + n
         pages = table[slot, : -(-total // PAGE)].long()
@@ -149,15 +172,25 @@ def paged_attn(out, q, kpages, vpages, bias, table, seg, max_len, window,
         s = rows.permute(1, 2, 0, 3) @ k.transpose(2, 3) * scale
         if softcap:
             s = softcap * torch.tanh(s / softcap)
-        # the bias table is in log2 units (see the HIP kernel)
-        s = s + bias[:, d.clamp(0, far)].unsqueeze(1) * 0.6931471805599453
-        p = s.masked_fill(~ok, float("-inf")).softmax(-1)
+        # bias table and slopes are in log2 units (see the HIP kernel)
+        b = bias[:, d.clamp(0, bias.size(1) - 1)] if slopes is None \
+            else -slopes.view(-1, 1, 1) * d
+        s = s + b.unsqueeze(1) * 0.6931471805599453
+        s = s.masked_fill(~ok, float("-inf"))
+        if sink is None:
+            p = s.softmax(-1)
+        else:
+            extra = sink.view(-1, 1, 1, 1).expand(-1, maps, n, 1)
+            p = torch.cat((s, extra), -1).softmax(-1)[..., :-1]
         o = p @ v                                       # [H, maps, n, E]
         if maps == 2:
             o = _rms(o[:, 0] - map_weight * o[:, 1], eps) * out_scale
         else:
             o = o[:, 0]
-        out[start:start + n] = o.transpose(0, 1).reshape(n, -1).to(out.dtype)
+        o = o.transpose(0, 1).reshape(n, -1)
+        if gate is not None:
+            o = o * torch.sigmoid(gate[start:start + n].float())
+        out[start:start + n] = o.to(out.dtype)
 
 
 def _rows(pages, table, slot, first, end, n_cols):
@@ -359,6 +392,10 @@ def gelu(z) -> None:
     z.copy_(torch.nn.functional.gelu(z.float()))
 
 
+def relu2(z) -> None:
+    z.copy_(z.float().clamp(min=0.0).square())
+
+
 def causal_conv(out, x, w, bias, in_bias, state, seg, max_len, act) -> None:
     back = w.size(0) - 1
     for start, n, slot, pos0 in _segments(seg):
@@ -424,3 +461,54 @@ def mamba2_out(out, o, xbc, z, skip, w, groups, eps) -> None:
     y = o + (xbc[:, :inner].float().view(n, skip.numel(), -1)
              * skip.view(1, -1, 1)).view(n, inner)
     out.copy_(_group_rms(y * _act(z.float(), 0), groups, eps) * w)
+
+
+def mlstm_scan(out, proj, state, peak, gate_bias, norm_w, cap, q_scale, eps,
+               seg, max_len) -> None:
+    """The normaliser is the state's column behind the values."""
+    _, H, D, _ = state.shape
+    E = norm_w.numel() // H
+    q, k, v, g, gates = proj.float().split(
+        (H * D, H * D, H * E, H * E, 2 * H), 1)
+    i, f = (cap * torch.tanh((gates + gate_bias) / cap)).split(H, 1)
+    f = torch.nn.functional.logsigmoid(f)
+    q = (q * q_scale).view(-1, H, D, 1)
+    v = torch.cat((v.view(-1, H, E), torch.ones(len(v), H, 1)), -1)
+    for start, n, slot, pos0 in _segments(seg):
+        S, m = state[slot], peak[slot]
+        if pos0 == 0:
+            S, m = torch.zeros_like(S), torch.zeros_like(m)
+        for t in range(start, start + n):
+            new = torch.maximum(f[t] + m, i[t])
+            S = torch.exp(f[t] + m - new).view(H, 1, 1) * S
+            S[..., :E + 1] += torch.exp(i[t] - new).view(H, 1, 1) \
+                * k[t].view(H, D, 1) * v[t].view(H, 1, E + 1)
+            m = new
+            r = (S[..., :E + 1] * q[t]).sum(1)
+            size = torch.maximum(r[:, E:].abs(), torch.exp(-m).view(H, 1))
+            r = _rms(r[:, :E] / (size + 1e-6), eps).view(-1) * norm_w
+            out[t] = (r * torch.sigmoid(g[t])).to(out.dtype)
+        state[slot], peak[slot] = S, m
+
+
+def mlstm_step(*args) -> None:
+    mlstm_scan(*args, 1)
+
+
+def mingru_scan(out, proj, bias, state, seg, max_len) -> None:
+    W = state.size(1)
+    z, u, g = proj.float().split(W, 1)
+    z = torch.sigmoid(z + bias[:W])
+    u = u + bias[W:]
+    c = torch.where(u >= 0, u + 0.5, torch.sigmoid(u))
+    g = torch.nn.functional.silu(g)
+    for start, n, slot, pos0 in _segments(seg):
+        S = state[slot].clone() if pos0 else torch.zeros_like(state[slot])
+        for t in range(start, start + n):
+            S = (1.0 - z[t]) * S + z[t] * c[t]
+            out[t] = (S * g[t]).to(out.dtype)
+        state[slot] = S
+
+
+def mingru_step(out, proj, bias, state, seg) -> None:
+    mingru_scan(out, proj, bias, state, seg, 1)
