@@ -83,7 +83,8 @@ void gemv(torch::Tensor out, torch::Tensor W, torch::Tensor x,
   }
   TORCH_CHECK(K % 8 == 0, "K must be a multiple of 8");
   TORCH_CHECK(epilogue != 4 || norm_kind != 2, "xielu: no LayerNorm form");
-  TORCH_CHECK(epilogue != 5 || norm_kind == 0, "gelu(erf): no norm");
+  TORCH_CHECK((epilogue != 5 && epilogue != 6) || norm_kind == 0,
+              "gelu(erf), squared relu: no norm");
   const void* bp = nullptr;
   const void* rp = nullptr;
   const void* nwp = nullptr;

@@ -13,7 +13,7 @@ void launch_layernorm(void* out, const void* x, const void* w, const void* b,
                       int n, float eps, hipStream_t stream);
 
 // epilogue: 0 none, 1 +res, 2 gelu(tanh), 3 silu, 4 xielu(act_p, act_q)
-// 5 gelu(erf) (4 has no LayerNorm form, 5 no norm)
+// 5 gelu(erf), 6 squared relu (4 has no LayerNorm form, 5 and 6 no norm)
 // norm_kind: 0 none, 1 fused RMSNorm on x, 2 fused LayerNorm on x
 // rows: output rows per wave (1/2/4); 0 = auto by M
 // eidx/estride (optional): W += eidx[0]*estride at replay time — selects

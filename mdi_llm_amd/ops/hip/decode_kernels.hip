@@ -233,7 +233,7 @@ __global__ void layernorm_kernel(bf16* __restrict__ out,
 // reduces mean/meansq and rewrites LDS with the normalized+weighted value.
 // NORM: 0 none, 1 RMSNorm, 2 LayerNorm.
 // EPI:  0 none, 1 +residual, 2 gelu(tanh), 3 silu, 4 xielu(act_p, act_q),
-// 5 gelu(erf).
+// 5 gelu(erf), 6 squared relu.
 // ---------------------------------------------------------------------------
 DEVINL float gelu_tanh(float v) {
   float c = 0.7978845608028654f * (v + 0.044715f * v * v * v);
@@ -505,6 +505,7 @@ __global__ void gemv_direct_kernel(bf16* __restrict__ out,
         if (EPI == 3) a = a / (1.f + expf(-a));
         if (EPI == 4) a = xielu(a, act_p, act_q);
         if (EPI == 5) a = gelu_erf(a);
+        if (EPI == 6) a = fmaxf(a, 0.f) * fmaxf(a, 0.f);
         out[rw] = f2b(a);
       }
     }
@@ -3271,6 +3272,7 @@ void launch_gemv(void* out, const void* W, const void* x, const void* bias,
     case 16: GEMV_CASE(4, 0); break;
     case 17: GEMV_CASE(4, 1); break;
     case 20: GEMV_CASE(5, 0); break;
+    case 24: GEMV_CASE(6, 0); break;
     default: GEMV_CASE(0, 0);
   }
 #undef GEMV_CASE

@@ -79,7 +79,7 @@ int row_type(const torch::Tensor& t, const char* name) {
 void residual_norm(torch::Tensor x, Opt y, Opt post_w, Opt xn, Opt next_w,
                    Opt tokens, Opt table, double scale, double offset,
                    double eps, double mult, Opt pos_table, Opt row_pos,
-                   Opt routed, Opt routed_w) {
+                   Opt routed, Opt routed_w, Opt gain, Opt y2, Opt post_w2) {
   TORCH_CHECK(x.dim() == 2 && x.size(0) > 0, "x must be [n, e]");
   const int n = (int)x.size(0), e = (int)x.size(1);
   float* xp = const_cast<float*>(f32_ptr(x, (int64_t)n * e, "x"));
@@ -103,7 +103,17 @@ void residual_norm(torch::Tensor x, Opt y, Opt post_w, Opt xn, Opt next_w,
   TORCH_CHECK(!!pos_table == !!row_pos && (!pos_table || tokens) &&
                   !!routed == !!routed_w && (!routed || y),
               "residual_norm: bad combination of operands");
+  TORCH_CHECK(!(gain && (post_w || !y)) && !!y2 == !!post_w2 &&
+                  (!y2 || (y && post_w)),
+              "residual_norm: bad combination of operands");
   ResidualArgs a{};
+  if (gain) a.gain = f32_ptr(*gain, e, "gain");
+  if (y2) {
+    check_like(*y2, f32, "y2");
+    TORCH_CHECK(y2->numel() == x.numel(), "y2 size");
+    a.y2 = y2->data_ptr();
+    a.post_w2 = f32_ptr(*post_w2, e, "post_w2");
+  }
   if (pos_table) {
     check_like(*pos_table, f32, "pos_table");
     TORCH_CHECK(pos_table->dim() == 2 && pos_table->size(1) == e,
@@ -146,6 +156,11 @@ void xielu(torch::Tensor z, double p, double q) {
 void gelu(torch::Tensor z) {
   launch_gelu(z.data_ptr(), (long long)z.numel(), act_type(z, "z"),
               cur_stream());
+}
+
+void relu2(torch::Tensor z) {
+  launch_relu2(z.data_ptr(), (long long)z.numel(), act_type(z, "z"),
+               cur_stream());
 }
 
 struct Recurrent {
@@ -303,6 +318,45 @@ void qk_norm_append(torch::Tensor q_out, Opt kpages, Opt vpages,
   launch_qk_norm_append(a, f32, cur_stream());
 }
 
+void row_norm_append(torch::Tensor q_out, torch::Tensor kpages,
+                     torch::Tensor vpages, torch::Tensor proj,
+                     torch::Tensor q_w, torch::Tensor k_w,
+                     torch::Tensor row_slot, torch::Tensor row_pos,
+                     torch::Tensor table, int64_t vdim, double eps,
+                     Opt q_scale, bool unit_values) {
+  const int f32 = act_type(q_out, "q_out");
+  const Rows r = rows_of(proj, f32, "proj");
+  RowAppendArgs a{};
+  TORCH_CHECK(q_out.dim() == 3 && q_out.size(0) == r.n && q_out.size(1) > 0 &&
+                  q_out.size(2) <= 256 && q_w.numel() % q_out.size(1) == 0,
+              "q_out must be [n, H, dpad]");
+  a.qk.n = r.n;
+  a.qk.heads = (int)q_out.size(1);
+  const int64_t dim = q_w.numel() / a.qk.heads;
+  set_pages(a.qk, kpages, vpages, dim, vdim, f32);
+  TORCH_CHECK(a.qk.dpad == q_out.size(2) && a.qk.k_heads == a.qk.v_heads &&
+                  a.qk.vpad <= 256,
+              "row_norm_append: pages");
+  TORCH_CHECK(r.cols == (a.qk.heads + a.qk.k_heads) * dim +
+                            a.qk.v_heads * vdim,
+              "proj columns");
+  a.qk.q_out = q_out.data_ptr();
+  a.qk.proj = r.p;
+  a.qk.q_w = f32_ptr(q_w, a.qk.heads * dim, "q_w");
+  a.qk.k_w = f32_ptr(k_w, a.qk.k_heads * dim, "k_w");
+  a.qk.eps = (float)eps;
+  set_places(a.qk, row_slot, row_pos, table);
+  // (positions beyond the table are the caller's limit on sequences)
+  if (q_scale) a.q_scale = f32_ptr(*q_scale, q_scale->numel(), "q_scale");
+  a.ld = r.ld;
+  a.unit_values = unit_values ? 1 : 0;
+  const int v = f32 ? 4 : 8;
+  a.vec = dim % v == 0 && vdim % v == 0 && r.ld % v == 0 &&
+          (size_t)r.p % 16 == 0;
+  TORCH_CHECK(launch_row_norm_append(a, f32, cur_stream()) == 0,
+              "row_norm_append: values of ", vdim);
+}
+
 void kv_rows(torch::Tensor rows, torch::Tensor kpages, torch::Tensor vpages,
              torch::Tensor row_slot, torch::Tensor row_pos,
              torch::Tensor table, int64_t dim, int64_t vdim, bool store) {
@@ -318,11 +372,12 @@ void kv_rows(torch::Tensor rows, torch::Tensor kpages, torch::Tensor vpages,
 }
 
 void paged_attn(torch::Tensor out, torch::Tensor q, torch::Tensor kpages,
-                torch::Tensor vpages, torch::Tensor bias,
-                torch::Tensor table, torch::Tensor seg, int64_t max_len,
-                int64_t window, int64_t keep_first, double scale,
-                int64_t splits, Opt part_o, Opt part_ml, double softcap,
-                double map_weight, double out_scale, double eps) {
+                torch::Tensor vpages, Opt bias, torch::Tensor table,
+                torch::Tensor seg, int64_t max_len, int64_t window,
+                int64_t keep_first, double scale, int64_t splits, Opt part_o,
+                Opt part_ml, double softcap, double map_weight,
+                double out_scale, double eps, Opt slopes, Opt sink,
+                Opt gate) {
   const int f32 = act_type(q, "q");
   const Pages pg = pages(kpages, vpages, f32);
   check_like(out, f32, "out");
@@ -349,10 +404,26 @@ void paged_attn(torch::Tensor out, torch::Tensor q, torch::Tensor kpages,
   a.dpad = pg.dpad;
   a.vpad = pg.vpad;
   TORCH_CHECK(a.vdim <= a.vpad, "vdim");
-  TORCH_CHECK(bias.dim() == 2 && bias.size(0) == a.heads && bias.size(1) > 0,
-              "bias must be [H, n]");
-  a.bias = f32_ptr(bias, bias.numel(), "bias");
-  a.bias_len = (int)bias.size(1);
+  TORCH_CHECK(!!bias != !!slopes, "paged_attn: a bias table or slopes");
+  TORCH_CHECK(a.maps == 1 || !(slopes || sink || gate),
+              "paged_attn: slopes, sink and gate go with one map");
+  if (bias) {
+    TORCH_CHECK(bias->dim() == 2 && bias->size(0) == a.heads &&
+                    bias->size(1) > 0,
+                "bias must be [H, n]");
+    a.bias = f32_ptr(*bias, bias->numel(), "bias");
+    a.bias_len = (int)bias->size(1);
+  } else {
+    a.slopes = f32_ptr(*slopes, a.heads, "slopes");
+  }
+  if (sink) a.sink = f32_ptr(*sink, a.heads, "sink");
+  if (gate) {
+    const Rows g = rows_of(*gate, f32, "gate");
+    TORCH_CHECK(g.n == out.size(0) && g.cols == out.size(1),
+                "gate must be [n, H*vdim]");
+    a.gate = g.p;
+    a.gate_ld = g.ld;
+  }
   TORCH_CHECK(table.dim() == 2, "table must be [slots, pages]");
   a.table = i32_ptr(table, table.numel(), "table");
   a.table_stride = (int)table.size(1);
@@ -384,7 +455,8 @@ void paged_attn(torch::Tensor out, torch::Tensor q, torch::Tensor kpages,
   }
   const auto launch =
       a.maps == 2 ? (f32 ? launch_diff_attn_f32 : launch_diff_attn_bf16)
-                  : (f32 ? launch_paged_attn_f32 : launch_paged_attn_bf16);
+      : slopes ? (f32 ? launch_slope_attn_f32 : launch_slope_attn_bf16)
+               : (f32 ? launch_paged_attn_f32 : launch_paged_attn_bf16);
   const int rc = launch(a, cur_stream());
   TORCH_CHECK(rc == 0, "paged_attn: unsupported padded sizes ", a.dpad, ", ",
               a.vpad);
@@ -737,7 +809,7 @@ void moe_down(torch::Tensor out, torch::Tensor mid, torch::Tensor w,
 
 void skinny_gemm(torch::Tensor out, torch::Tensor w, torch::Tensor x,
                  int64_t act, double act_p, double act_q) {
-  TORCH_CHECK(act >= 0 && act <= 2, "skinny_gemm: act");
+  TORCH_CHECK(act >= 0 && act <= 3, "skinny_gemm: act");
   TORCH_CHECK(x.dim() == 2 && w.dim() == 2 && out.dim() == 2, "2-D operands");
   const int n = (int)x.size(0), m = (int)w.size(0), k = (int)x.size(1);
   for (const auto* t : {&out, &w, &x})
@@ -985,6 +1057,105 @@ void mamba2_scan(torch::Tensor o, torch::Tensor xbc, torch::Tensor dt,
               "mamba2_scan: unsupported state ", a.dim);
 }
 
+MLstmArgs mlstm_args(const torch::Tensor& out, const torch::Tensor& proj,
+                     const torch::Tensor& state, const torch::Tensor& peak,
+                     const torch::Tensor& gate_bias,
+                     const torch::Tensor& norm_w, double cap, double q_scale,
+                     double eps, const torch::Tensor& seg, int f32) {
+  check_like(proj, f32, "proj");
+  MLstmArgs a{};
+  TORCH_CHECK(state.dim() == 4 && proj.dim() == 2 && proj.size(0) > 0,
+              "mlstm: state must be [slots, H, dim, vstride]");
+  a.n = (int)proj.size(0);
+  a.heads = (int)state.size(1);
+  a.dim = (int)state.size(2);
+  a.vstride = (int)state.size(3);
+  TORCH_CHECK(norm_w.numel() % a.heads == 0, "mlstm: norm_w");
+  a.vdim = (int)(norm_w.numel() / a.heads);
+  TORCH_CHECK(a.vstride % 4 == 0 && a.vdim > 0 && a.vdim < a.vstride &&
+                  a.dim <= 256 && a.vstride <= 1024 && cap > 0.0,
+              "mlstm: sizes");
+  TORCH_CHECK(proj.size(1) == 2LL * a.heads * (a.dim + a.vdim + 1) &&
+                  out.numel() == (int64_t)a.n * a.heads * a.vdim &&
+                  (int64_t)a.n * a.heads < (int64_t)1 << 31,
+              "mlstm: rows");
+  TORCH_CHECK(peak.dim() == 2 && peak.size(0) == state.size(0) &&
+                  peak.size(1) == a.heads,
+              "mlstm: peak must be [slots, H]");
+  a.out = out.data_ptr();
+  a.proj = proj.data_ptr();
+  a.state = const_cast<float*>(f32_ptr(state, state.numel(), "state"));
+  a.peak = const_cast<float*>(f32_ptr(peak, peak.numel(), "peak"));
+  a.gate_bias = f32_ptr(gate_bias, 2 * a.heads, "gate_bias");
+  a.norm_w = f32_ptr(norm_w, a.heads * a.vdim, "norm_w");
+  a.cap = (float)cap;
+  a.q_scale = (float)q_scale;
+  a.eps = (float)eps;
+  a.seg = seg_view(seg);
+  return a;
+}
+
+void mlstm_step(torch::Tensor out, torch::Tensor proj, torch::Tensor state,
+                torch::Tensor peak, torch::Tensor gate_bias,
+                torch::Tensor norm_w, double cap, double q_scale, double eps,
+                torch::Tensor seg) {
+  const int f32 = act_type(out, "out");
+  launch_mlstm_step(mlstm_args(out, proj, state, peak, gate_bias, norm_w, cap,
+                               q_scale, eps, seg, f32),
+                    f32, cur_stream());
+}
+
+void mlstm_scan(torch::Tensor out, torch::Tensor proj, torch::Tensor state,
+                torch::Tensor peak, torch::Tensor gate_bias,
+                torch::Tensor norm_w, double cap, double q_scale, double eps,
+                torch::Tensor seg, int64_t max_len) {
+  const int f32 = act_type(out, "out");
+  MLstmArgs a = mlstm_args(out, proj, state, peak, gate_bias, norm_w, cap,
+                           q_scale, eps, seg, f32);
+  TORCH_CHECK(max_len > 0 && max_len <= a.n, "max_len");
+  a.max_len = (int)max_len;
+  torch::Tensor work = torch::empty(
+      {mlstm_work_floats(a.n, a.seg.n, a.heads, a.dim, a.vdim)},
+      state.options());
+  a.work = work.data_ptr<float>();
+  TORCH_CHECK(launch_mlstm_scan(a, f32, cur_stream()) == 0,
+              "mlstm_scan: unsupported dim ", a.dim);
+}
+
+MinGruArgs mingru_args(const torch::Tensor& out, const torch::Tensor& proj,
+                       const torch::Tensor& bias, const torch::Tensor& state,
+                       const torch::Tensor& seg, int f32) {
+  const Rows r = rows_of(proj, f32, "proj");
+  MinGruArgs a{};
+  TORCH_CHECK(state.dim() == 2 && r.cols == 3 * state.size(1) &&
+                  out.numel() == (int64_t)r.n * state.size(1),
+              "mingru: proj must be [n, 3 * width], state [slots, width]");
+  a.width = (int)state.size(1);
+  a.out = out.data_ptr();
+  a.proj = r.p;
+  a.ld = r.ld;
+  a.bias = f32_ptr(bias, 2 * a.width, "bias");
+  a.state = const_cast<float*>(f32_ptr(state, state.numel(), "state"));
+  a.seg = seg_view(seg);
+  return a;
+}
+
+void mingru_step(torch::Tensor out, torch::Tensor proj, torch::Tensor bias,
+                 torch::Tensor state, torch::Tensor seg) {
+  const int f32 = act_type(out, "out");
+  launch_mingru_step(mingru_args(out, proj, bias, state, seg, f32), f32,
+                     cur_stream());
+}
+
+void mingru_scan(torch::Tensor out, torch::Tensor proj, torch::Tensor bias,
+                 torch::Tensor state, torch::Tensor seg, int64_t max_len) {
+  const int f32 = act_type(out, "out");
+  MinGruArgs a = mingru_args(out, proj, bias, state, seg, f32);
+  TORCH_CHECK(max_len > 0 && max_len <= proj.size(0), "max_len");
+  a.max_len = (int)max_len;
+  launch_mingru_scan(a, f32, cur_stream());
+}
+
 void mamba2_out(torch::Tensor out, torch::Tensor o, torch::Tensor xbc,
                 torch::Tensor z, torch::Tensor skip, torch::Tensor w,
                 int64_t groups, double eps) {
@@ -1039,7 +1210,10 @@ void bind_hybrid(py::module_& m) {
         py::arg("scale") = 1.0, py::arg("offset") = 0.0,
         py::arg("eps") = 1e-6, py::arg("mult") = 1.0,
         py::arg("pos_table") = none, py::arg("row_pos") = none,
-        py::arg("routed") = none, py::arg("routed_w") = none);
+        py::arg("routed") = none, py::arg("routed_w") = none,
+        py::arg("gain") = none, py::arg("y2") = none,
+        py::arg("post_w2") = none);
+  m.def("relu2", &relu2, "in-place squared ReLU", py::arg("z"));
   m.def("xielu", &xielu, "in-place xIELU", py::arg("z"), py::arg("p"),
         py::arg("q"));
   m.def("gelu", &gelu, "in-place exact GELU", py::arg("z"));
@@ -1087,6 +1261,24 @@ void bind_hybrid(py::module_& m) {
         "read-out", py::arg("out"), py::arg("o"), py::arg("xbc"),
         py::arg("z"), py::arg("skip"), py::arg("w"), py::arg("groups"),
         py::arg("eps"));
+  m.def("mlstm_step", &mlstm_step,
+        "mLSTM gates + state update + normalised, gated read-out, one token "
+        "per segment",
+        py::arg("out"), py::arg("proj"), py::arg("state"), py::arg("peak"),
+        py::arg("gate_bias"), py::arg("norm_w"), py::arg("cap"),
+        py::arg("q_scale"), py::arg("eps"), py::arg("seg"));
+  m.def("mlstm_scan", &mlstm_scan, "mLSTM over token segments",
+        py::arg("out"), py::arg("proj"), py::arg("state"), py::arg("peak"),
+        py::arg("gate_bias"), py::arg("norm_w"), py::arg("cap"),
+        py::arg("q_scale"), py::arg("eps"), py::arg("seg"),
+        py::arg("max_len"));
+  m.def("mingru_step", &mingru_step,
+        "minGRU gates + recurrence + output gate, one token per segment",
+        py::arg("out"), py::arg("proj"), py::arg("bias"), py::arg("state"),
+        py::arg("seg"));
+  m.def("mingru_scan", &mingru_scan, "minGRU over token segments",
+        py::arg("out"), py::arg("proj"), py::arg("bias"), py::arg("state"),
+        py::arg("seg"), py::arg("max_len"));
   m.def("hgrn2_step", &hgrn2_step,
         "HGRN2 gates + state update + read-out + head norm, one token per "
         "segment",
@@ -1102,20 +1294,29 @@ void bind_hybrid(py::module_& m) {
         py::arg("q_w"), py::arg("k_w"), py::arg("row_slot"),
         py::arg("row_pos"), py::arg("table"), py::arg("vdim"),
         py::arg("eps"), py::arg("rope") = none);
+  m.def("row_norm_append", &row_norm_append,
+        "q/k RMS norms over whole rows, query scale by position, values of "
+        "unit size + paged cache append",
+        py::arg("q_out"), py::arg("kpages"), py::arg("vpages"),
+        py::arg("proj"), py::arg("q_w"), py::arg("k_w"), py::arg("row_slot"),
+        py::arg("row_pos"), py::arg("table"), py::arg("vdim"), py::arg("eps"),
+        py::arg("q_scale") = none, py::arg("unit_values") = true);
   m.def("kv_rows", &kv_rows, "cached keys and values <-> flat rows",
         py::arg("rows"), py::arg("kpages"), py::arg("vpages"),
         py::arg("row_slot"), py::arg("row_pos"), py::arg("table"),
         py::arg("dim"), py::arg("vdim"), py::arg("store"));
   m.def("paged_attn", &paged_attn,
-        "paged attention: distance bias, sliding window, kept first tokens, "
-        "capped scores, one map or the difference of two",
+        "paged attention: distance bias or slopes, sliding window, kept "
+        "first tokens, capped scores, sink, output gate, one map or the "
+        "difference of two",
         py::arg("out"), py::arg("q"), py::arg("kpages"), py::arg("vpages"),
         py::arg("bias"), py::arg("table"), py::arg("seg"),
         py::arg("max_len"), py::arg("window"), py::arg("keep_first"),
         py::arg("scale"), py::arg("splits"), py::arg("part_o") = none,
         py::arg("part_ml") = none, py::arg("softcap") = 0.0,
         py::arg("map_weight") = 0.0, py::arg("out_scale") = 1.0,
-        py::arg("eps") = 0.0);
+        py::arg("eps") = 0.0, py::arg("slopes") = none,
+        py::arg("sink") = none, py::arg("gate") = none);
   m.def("latent_norm_append", &latent_norm_append,
         "norms of the query and key/value latents + paged cache append, and "
         "a gated activation in the same launch",

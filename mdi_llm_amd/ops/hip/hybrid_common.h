@@ -88,6 +88,11 @@ DEVINL float gelu_erf(float z) {
   return 0.5f * z * (1.f + erff(0.7071067811865476f * z));
 }
 
+DEVINL float relu2(float z) {
+  const float p = fmaxf(z, 0.f);
+  return p * p;
+}
+
 DEVINL float softplus(float z) {
   return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)));
 }

@@ -20,13 +20,18 @@ struct SegView {
 // Residual + norm step, one row per block.  x [n, e] float:
 //   tokens != null : x = scale * table[token]
 //                    (+ pos_table[row_pos] if there is one)
-//   y != null      : x += mult * (post_w ? rms(y) * (offset + post_w) : y,
-//                    plus the weighted routed rows [n, top, e] if any)
+//   y != null      : x += mult * (post_w ? rms(y) * (offset + post_w) : y
+//                    (times gain, if there is one), plus a second output
+//                    rms(y2) * (offset + post_w2) and the weighted routed
+//                    rows [n, top, e] if any); post_w if y2
 // then, if next_w, xn = rms(x) * (offset + next_w).
 struct ResidualArgs {
   float* x;
   const void* y;
   const float* post_w;
+  const float* gain;
+  const void* y2;
+  const float* post_w2;
   void* xn;
   const float* next_w;
   const int* tokens;
@@ -49,6 +54,9 @@ void launch_xielu(void* z, long long n, float p, float q, int f32,
 
 // z <- exact GELU
 void launch_gelu(void* z, long long n, int f32, hipStream_t stream);
+
+// z <- max(z, 0)^2
+void launch_relu2(void* z, long long n, int f32, hipStream_t stream);
 
 // HGRN2 over segments of one token each: gates, state update, read-out and
 // the per-head norm in one launch.  proj [rows, 2*H*D + H*E] = q|f|v.
@@ -98,6 +106,22 @@ void launch_qk_norm_append(const QkAppendArgs& a, int f32,
 void launch_kv_rows(const QkAppendArgs& a, void* rows, int store, int f32,
                     hipStream_t stream);
 
+// The same for norms over a whole row of queries and of keys (q_w [heads *
+// dim], k_w [k_heads * dim]), queries times q_scale[position] if it is there,
+// values divided by their head's root mean square if unit_values.  rope is
+// not used; proj rows are ld apart; vec: 8 (bf16) or 4 (float) channels per
+// access are aligned and stay within a head.
+struct RowAppendArgs {
+  QkAppendArgs qk;
+  const float* q_scale;
+  long long ld;
+  int unit_values, vec;
+};
+
+// -1: no room for the values' tile
+int launch_row_norm_append(const RowAppendArgs& a, int f32,
+                           hipStream_t stream);
+
 struct PagedAttnArgs {
   void* out;            // [rows, H*vdim]
   const void* q;        // [rows, H, dpad]
@@ -121,6 +145,11 @@ struct PagedAttnArgs {
   // out_scale.  Split mode always leaves parts.
   int maps;
   float map_weight, out_scale, eps;
+  // one map only:
+  const float* slopes;  // [H] in log2 units, taken off per distance; no bias
+  const float* sink;    // [H] score of one more term of the softmax
+  const void* gate;     // out *= sigmoid(gate[row * gate_ld + h * vdim + ..])
+  long long gate_ld;
 };
 
 // Returns -1 when (dpad, vpad) has no instantiation.
@@ -128,6 +157,8 @@ int launch_paged_attn_bf16(const PagedAttnArgs& a, hipStream_t stream);
 int launch_paged_attn_f32(const PagedAttnArgs& a, hipStream_t stream);
 int launch_diff_attn_bf16(const PagedAttnArgs& a, hipStream_t stream);  // maps 2
 int launch_diff_attn_f32(const PagedAttnArgs& a, hipStream_t stream);
+int launch_slope_attn_bf16(const PagedAttnArgs& a, hipStream_t stream);  // slopes
+int launch_slope_attn_f32(const PagedAttnArgs& a, hipStream_t stream);
 
 struct RowAttnArgs {
   void* out;              // head h of row r at r * out_row + h * vdim
@@ -356,6 +387,47 @@ void launch_mamba2_step(const Mamba2Args& a, int f32, hipStream_t stream);
 // -1: dim has no instantiation
 int launch_mamba2_scan(const Mamba2Args& a, int f32, hipStream_t stream);
 
+// mLSTM: per head, with log gates i = cap tanh(z_i / cap) and f =
+// logsigmoid(cap tanh(z_f / cap)), m' = max(f + m, i), S = exp(f + m - m') S +
+// exp(i - m') k v^T and the same for the normaliser n with v = 1; o = S^T q /
+// (max(|n . q|, exp(-m')) + 1e-6), brought to unit size, times norm_w and
+// sigmoid(g).  proj rows = q|k|v|g|z_i|z_f, gate_bias [2 H], state [slots, H,
+// dim, vstride] with n in column vdim, peak [slots, H] = m, norm_w [H * vdim].
+struct MLstmArgs {
+  void* out;            // [rows, H * vdim]
+  const void* proj;
+  float* state;
+  float* peak;
+  const float* gate_bias;
+  const float* norm_w;
+  float* work;          // scan: mlstm_work(...) floats
+  SegView seg;
+  int n, heads, dim, vdim, vstride, max_len;
+  float cap, q_scale, eps;
+};
+
+void launch_mlstm_step(const MLstmArgs& a, int f32, hipStream_t stream);
+long long mlstm_work_floats(int rows, int segments, int heads, int dim,
+                            int vdim);
+// segments in the order of their rows; -1: dim has no instantiation
+int launch_mlstm_scan(const MLstmArgs& a, int f32, hipStream_t stream);
+
+// minGRU: z = sigmoid(. + bias), c = u + 1/2 or sigmoid(u) below 0 with u = .
+// + bias, S = (1 - z) S + z c, out = S silu(g).  proj rows = z|u|g, ld apart,
+// bias [2 * width], state [slots, width].
+struct MinGruArgs {
+  void* out;
+  const void* proj;
+  const float* bias;
+  float* state;
+  SegView seg;
+  long long ld;
+  int width, max_len;
+};
+
+void launch_mingru_step(const MinGruArgs& a, int f32, hipStream_t stream);
+void launch_mingru_scan(const MinGruArgs& a, int f32, hipStream_t stream);
+
 // out = groups of rms((o + skip x) silu(z)) * w; x rows are xld, z rows zld
 // apart, skip [heads].  -1: rows are too long
 struct GatedNormArgs {
@@ -374,7 +446,7 @@ struct GatedNormArgs {
 int launch_gated_norm(const GatedNormArgs& a, int f32, hipStream_t stream);
 
 // out[n, m] = x[n, :] . w[m, :] in bf16 for up to 32 rows of x, with act 1
-// xIELU, 2 exact GELU.  Returns -1 when n or k (a multiple of 64) does not fit.
+// xIELU, 2 exact GELU, 3 squared ReLU.  Returns -1 when n or k (a multiple of 64) does not fit.
 int launch_skinny_gemm(void* out, const void* w, const void* x, int n, int m,
                        int k, int act, float act_p, float act_q,
                        hipStream_t stream);

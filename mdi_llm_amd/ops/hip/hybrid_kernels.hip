@@ -58,7 +58,29 @@ __global__ __launch_bounds__(NT) void residual_norm_kernel(ResidualArgs p) {
       y += row * e;
       PT b[KEEP];
       EACH(i) b[k] = *reinterpret_cast<const PT*>(y + i);
-      if (p.post_w != nullptr) {
+      if (p.y2 != nullptr) {
+        const T* y2 = (const T*)p.y2 + row * e;
+        PT b2[KEEP];
+        EACH(i) b2[k] = *reinterpret_cast<const PT*>(y2 + i);
+        float s = 0.f, s2 = 0.f;
+        EACH(i) {
+#pragma unroll
+          for (int j = 0; j < V; ++j) {
+            s += to_f(b[k].v[j]) * to_f(b[k].v[j]);
+            s2 += to_f(b2[k].v[j]) * to_f(b2[k].v[j]);
+          }
+        }
+        const float r = p.mult / sqrtf(block_sum<NT>(s, red) / e + eps);
+        const float r2 = p.mult / sqrtf(block_sum<NT>(s2, red) / e + eps);
+        EACH(i) {
+          const PF w = *reinterpret_cast<const PF*>(p.post_w + i);
+          const PF w2 = *reinterpret_cast<const PF*>(p.post_w2 + i);
+#pragma unroll
+          for (int j = 0; j < V; ++j)
+            a[k].v[j] += to_f(b[k].v[j]) * r * (offset + w.v[j]) +
+                         to_f(b2[k].v[j]) * r2 * (offset + w2.v[j]);
+        }
+      } else if (p.post_w != nullptr) {
         PF w[KEEP];
         EACH(i) w[k] = *reinterpret_cast<const PF*>(p.post_w + i);
         float s = 0.f;
@@ -72,6 +94,13 @@ __global__ __launch_bounds__(NT) void residual_norm_kernel(ResidualArgs p) {
           for (int j = 0; j < V; ++j)
             a[k].v[j] +=
                 to_f(b[k].v[j]) * r * (offset + w[k].v[j]) * p.mult;
+        }
+      } else if (p.gain != nullptr) {
+        EACH(i) {
+          const PF w = *reinterpret_cast<const PF*>(p.gain + i);
+#pragma unroll
+          for (int j = 0; j < V; ++j)
+            a[k].v[j] += to_f(b[k].v[j]) * w.v[j] * p.mult;
         }
       } else {
         EACH(i) {
@@ -143,9 +172,10 @@ int launch_residual_norm(const ResidualArgs& a, int f32, hipStream_t stream) {
 }
 
 // ---------------------------------------------------------------------------
-// xIELU or exact GELU on a whole GEMM output (single rows have it in the GEMV epilogue)
+// xIELU (1), exact GELU (2) or squared ReLU (3) on a whole GEMM output (single
+// rows have it in the GEMV epilogue)
 // ---------------------------------------------------------------------------
-template <typename T, int V, bool GELU>
+template <typename T, int V, int ACT>
 __global__ __launch_bounds__(256) void act_kernel(T* __restrict__ z,
                                                   long long n, float p,
                                                   float q) {
@@ -156,40 +186,46 @@ __global__ __launch_bounds__(256) void act_kernel(T* __restrict__ z,
 #pragma unroll
     for (int j = 0; j < V; ++j) {
       const float f = to_f(a.v[j]);
-      a.v[j] = from_f<T>(GELU ? gelu_erf(f) : xielu(f, p, q));
+      a.v[j] = from_f<T>(ACT == 3   ? relu2(f)
+                         : ACT == 2 ? gelu_erf(f)
+                                    : xielu(f, p, q));
     }
     *reinterpret_cast<Pack<T, V>*>(z + i) = a;
   }
 }
 
-template <typename T, int V, bool GELU>
+template <typename T, int V, int ACT>
 static void act_t(void* z, long long n, float p, float q,
                   hipStream_t stream) {
   const long long blocks = (n + 256 * V - 1) / (256 * V);
-  act_kernel<T, V, GELU>
+  act_kernel<T, V, ACT>
       <<<(int)(blocks < 8192 ? blocks : 8192), 256, 0, stream>>>((T*)z, n, p,
                                                                  q);
 }
 
-template <bool GELU>
+template <int ACT>
 static void act_any(void* z, long long n, float p, float q, int f32,
                     hipStream_t stream) {
   if (f32) {
-    if (n % 4 == 0) act_t<float, 4, GELU>(z, n, p, q, stream);
-    else act_t<float, 1, GELU>(z, n, p, q, stream);
+    if (n % 4 == 0) act_t<float, 4, ACT>(z, n, p, q, stream);
+    else act_t<float, 1, ACT>(z, n, p, q, stream);
   } else {
-    if (n % 8 == 0) act_t<bf16, 8, GELU>(z, n, p, q, stream);
-    else act_t<bf16, 1, GELU>(z, n, p, q, stream);
+    if (n % 8 == 0) act_t<bf16, 8, ACT>(z, n, p, q, stream);
+    else act_t<bf16, 1, ACT>(z, n, p, q, stream);
   }
 }
 
 void launch_xielu(void* z, long long n, float p, float q, int f32,
                   hipStream_t stream) {
-  act_any<false>(z, n, p, q, f32, stream);
+  act_any<1>(z, n, p, q, f32, stream);
 }
 
 void launch_gelu(void* z, long long n, int f32, hipStream_t stream) {
-  act_any<true>(z, n, 0.f, 0.f, f32, stream);
+  act_any<2>(z, n, 0.f, 0.f, f32, stream);
+}
+
+void launch_relu2(void* z, long long n, int f32, hipStream_t stream) {
+  act_any<3>(z, n, 0.f, 0.f, f32, stream);
 }
 
 // ---------------------------------------------------------------------------
@@ -197,7 +233,7 @@ void launch_gelu(void* z, long long n, int f32, hipStream_t stream) {
 // ---------------------------------------------------------------------------
 template <typename T>
 struct Hgrn2Rule {
-  static constexpr bool NORM = true;
+  static constexpr bool NORM = true, NORMALISER = false;
   T* out;
   const T* proj;
   const float* f_bias;
@@ -315,8 +351,7 @@ __global__ __launch_bounds__(256) void hgrn2_factors_kernel(
 }
 
 long long hgrn2_work_floats(int rows, int segments, int heads, int dim) {
-  const long long chunks = rows / 16 + segments + 1;
-  return chunks * heads * (33 * chunk_dpad(dim) + 256);
+  return chunk_work_floats(rows, segments, heads, dim);
 }
 
 template <typename T, int TPW>
@@ -570,6 +605,158 @@ void launch_qk_norm_append(const QkAppendArgs& a, int f32,
       append_t<bf16, 8, 16>(a, stream);
     else append_t<bf16, 1, 64>(a, stream);
   }
+}
+
+// ---------------------------------------------------------------------------
+// Norms over all query and all key channels of a row + cache append: one block
+// per row.  VALUES: the row's values as well, a wave per head; for prompts the
+// kernel below takes 64 rows of a head, so that it writes runs of keys.
+// ---------------------------------------------------------------------------
+template <typename T, int V, int NT, bool VALUES>
+__global__ __launch_bounds__(NT) void row_norm_append_kernel(RowAppendArgs p) {
+  __shared__ float red[NT / 64];
+  using P = Pack<T, V>;
+  const QkAppendArgs& a = p.qk;
+  const size_t row = blockIdx.x;
+  const int tid = threadIdx.x, nq = a.heads * a.dim, nk = a.k_heads * a.dim;
+  const T* src = (const T*)a.proj + row * (size_t)p.ld;
+  const int pos = a.row_pos[row];
+  const size_t page =
+      a.table[(size_t)a.row_slot[row] * a.table_stride + (pos >> 6)];
+  float sq = 0.f, sk = 0.f;
+  for (int i = tid * V; i < nq + nk; i += NT * V) {
+    const P b = *reinterpret_cast<const P*>(src + i);
+    float s = 0.f;
+#pragma unroll
+    for (int j = 0; j < V; ++j) s += to_f(b.v[j]) * to_f(b.v[j]);
+    if (i < nq) sq += s;
+    else sk += s;
+  }
+  const float heat = p.q_scale != nullptr ? p.q_scale[pos] : 1.f;
+  const float rq = heat / sqrtf(block_sum<NT>(sq, red) / nq + a.eps);
+  const float rk = 1.f / sqrtf(block_sum<NT>(sk, red) / nk + a.eps);
+  const int per = a.dpad / V, total = (a.heads + a.k_heads) * per;
+  for (int i = tid; i < total; i += NT) {
+    const int h = i / per, d = (i - h * per) * V;
+    const bool is_q = h < a.heads;
+    const int c = h * a.dim + d;    // channel of the row, and of its weights
+    P b{};
+    if (d < a.dim) {
+      b = *reinterpret_cast<const P*>(src + c);
+      const float* w = is_q ? a.q_w + c : a.k_w + (c - nq);
+      const float r = is_q ? rq : rk;
+#pragma unroll
+      for (int j = 0; j < V; ++j)
+        b.v[j] = from_f<T>(to_f(b.v[j]) * r * w[j]);
+    }
+    if (is_q) {
+      *reinterpret_cast<P*>((T*)a.q_out + (row * a.heads + h) * a.dpad + d) =
+          b;
+    } else {
+      T* dst = (T*)a.kpages +
+               (page * a.k_heads + (h - a.heads)) * (size_t)(64 * a.dpad);
+      constexpr int RUN = V < 4 ? V : 4;
+#pragma unroll
+      for (int j = 0; j < V; j += RUN)
+        *reinterpret_cast<Pack<T, RUN>*>(
+            dst + PageLayout::k(pos & 63, d + j, a.dpad)) =
+            *reinterpret_cast<const Pack<T, RUN>*>(b.v + j);
+    }
+  }
+  if constexpr (VALUES) {
+    const int lane = tid & 63;
+    for (int g = tid >> 6; g < a.v_heads; g += NT / 64) {
+      const T* v = src + nq + nk + g * a.vdim;
+      T* dst = (T*)a.vpages + (page * a.v_heads + g) * (size_t)(64 * a.vpad);
+      float f[4], s = 0.f;  // (vdim is at most 256)
+#pragma unroll
+      for (int k = 0; k < 4; ++k) {
+        const int c = k * 64 + lane;
+        f[k] = c < a.vdim ? to_f(v[c]) : 0.f;
+        s += f[k] * f[k];
+      }
+      float r = 1.f;
+      if (p.unit_values) r = 1.f / sqrtf(wave_sum(s) / a.vdim + a.eps);
+#pragma unroll
+      for (int k = 0; k < 4; ++k) {
+        const int c = k * 64 + lane;
+        if (c < a.vdim)
+          dst[PageLayout::v(pos & 63, c, a.vpad)] = from_f<T>(f[k] * r);
+      }
+    }
+  }
+}
+
+// 64 rows of one value head per block, through LDS
+template <typename T, int V>
+__global__ __launch_bounds__(256) void unit_v_append_kernel(RowAppendArgs p) {
+  extern __shared__ __attribute__((aligned(16))) char sm_raw[];
+  const QkAppendArgs& a = p.qk;
+  T* sm = reinterpret_cast<T*>(sm_raw);
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int g = blockIdx.y, ld = a.vdim + 2;  // (an odd number of banks)
+  const size_t row0 = (size_t)blockIdx.x * 64;
+  const int rows = min(64, a.n - (int)row0);
+  const T* src = (const T*)a.proj + (a.heads + a.k_heads) * a.dim + g * a.vdim;
+  using P = Pack<T, V>;
+  // four lanes a row
+  const int r = tid >> 2, part = tid & 3;
+  float s = 0.f;
+  if (r < rows)
+    for (int c = part * V; c < a.vdim; c += 4 * V) {
+      const P b = *reinterpret_cast<const P*>(src + (row0 + r) * p.ld + c);
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        s += to_f(b.v[j]) * to_f(b.v[j]);
+        sm[r * ld + c + j] = b.v[j];
+      }
+    }
+  s += __shfl_xor(s, 1, 64);
+  s += __shfl_xor(s, 2, 64);
+  __shared__ float inv[64];
+  if (part == 0)
+    inv[r] = p.unit_values ? 1.f / sqrtf(s / a.vdim + a.eps) : 1.f;
+  __syncthreads();
+  if (lane >= rows) return;
+  const size_t row = row0 + lane;
+  const int pos = a.row_pos[row];
+  const size_t page =
+      a.table[(size_t)a.row_slot[row] * a.table_stride + (pos >> 6)];
+  T* dst = (T*)a.vpages + (page * a.v_heads + g) * (size_t)(64 * a.vpad);
+  for (int c = wave; c < a.vdim; c += 4)
+    dst[PageLayout::v(pos & 63, c, a.vpad)] =
+        from_f<T>(to_f(sm[lane * ld + c]) * inv[lane]);
+}
+
+template <typename T, int V>
+static int row_append_t(const RowAppendArgs& a, hipStream_t stream) {
+  const QkAppendArgs& q = a.qk;
+  if (q.n <= 64) {
+    if ((q.heads + q.k_heads) * q.dim > 512 * V)
+      row_norm_append_kernel<T, V, 1024, true><<<q.n, 1024, 0, stream>>>(a);
+    else
+      row_norm_append_kernel<T, V, 256, true><<<q.n, 256, 0, stream>>>(a);
+    return 0;
+  }
+  row_norm_append_kernel<T, V, 256, false><<<q.n, 256, 0, stream>>>(a);
+  const size_t smem = 64 * (q.vdim + 2) * sizeof(T);
+  auto kernel = unit_v_append_kernel<T, V>;
+  if (smem > 60000 &&
+      hipFuncSetAttribute((const void*)kernel,
+                          hipFuncAttributeMaxDynamicSharedMemorySize,
+                          (int)smem) != hipSuccess)
+    return -1;
+  kernel<<<dim3((q.n + 63) / 64, q.v_heads), 256, smem, stream>>>(a);
+  return 0;
+}
+
+int launch_row_norm_append(const RowAppendArgs& a, int f32,
+                           hipStream_t stream) {
+  if (f32)
+    return a.vec ? row_append_t<float, 4>(a, stream)
+                 : row_append_t<float, 1>(a, stream);
+  return a.vec ? row_append_t<bf16, 8>(a, stream)
+               : row_append_t<bf16, 1>(a, stream);
 }
 
 // Keys and values of some tokens as flat rows [k heads * dim | v heads *

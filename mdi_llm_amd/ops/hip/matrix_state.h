@@ -18,7 +18,10 @@ struct StepFactors {
 // state of the head passes through registers once (16-byte accesses along
 // vdim), so the block holds all of the head's output and can norm it before
 // it leaves.  Rule has factors(row, h, d), value(row, h, c), put(row, h, c, v)
-// and NORM: whether what put gets is the output of unit size.
+// and NORM: whether what put gets is the output of unit size.  A rule with
+// NORMALISER has one more column whose values are 1; before the unit size the
+// output is divided by size(what that column reads out), and enter and leave
+// frame the step of a slot's head.
 // ---------------------------------------------------------------------------
 template <int NT, typename Rule>
 __global__ __launch_bounds__(NT) void matrix_step_kernel(
@@ -35,6 +38,8 @@ __global__ __launch_bounds__(NT) void matrix_step_kernel(
   float* ks = fs + dim;                       // [dim]
   float* part = ks + dim;                     // [groups][vstride]
   const size_t row = seg.start[s];
+  if constexpr (Rule::NORMALISER)
+    rule.enter(row, h, seg.slot[s], seg.pos0[s] == 0);
   for (int d = tid; d < dim; d += NT) {
     const StepFactors x = rule.factors(row, h, d);
     qs[d] = x.q;
@@ -51,7 +56,9 @@ __global__ __launch_bounds__(NT) void matrix_step_kernel(
       float v[4], o[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int j = 0; j < 4; ++j)
-        v[j] = c4 * 4 + j < vdim ? rule.value(row, h, c4 * 4 + j) : 0.f;
+        v[j] = c4 * 4 + j < vdim ? rule.value(row, h, c4 * 4 + j)
+               : Rule::NORMALISER && c4 * 4 + j == vdim ? 1.f
+                                                        : 0.f;
 #pragma unroll 8
       for (int d = g; d < dim; d += groups) {
         float4* p = reinterpret_cast<float4*>(S + (size_t)d * vstride) + c4;
@@ -79,7 +86,13 @@ __global__ __launch_bounds__(NT) void matrix_step_kernel(
     part[c] = o;  // only this thread reads column c
     ss += o * o;
   }
-  float r = 1.f;
+  float r = 1.f, inv = 1.f;
+  if constexpr (Rule::NORMALISER) {
+    float n = 0.f;
+    for (int k = 0; k < groups; ++k) n += part[k * vstride + vdim];
+    inv = 1.f / rule.size(n);
+    if (tid == 0) rule.leave(h, seg.slot[s]);
+  }
   if constexpr (Rule::NORM) {
     ss = wave_sum(ss);
     if ((tid & 63) == 0) red[tid >> 6] = ss;
@@ -87,7 +100,7 @@ __global__ __launch_bounds__(NT) void matrix_step_kernel(
     ss = 0.f;
 #pragma unroll
     for (int k = 0; k < NT / 64; ++k) ss += red[k];
-    r = 1.f / sqrtf(ss / vdim + eps);
+    r = inv / sqrtf(ss * inv * inv / vdim + eps);
   }
   for (int c = tid; c < vdim; c += NT) rule.put(row, h, c, part[c] * r);
 }
@@ -133,6 +146,9 @@ void matrix_step(const Rule& rule, float* state, SegView seg, int heads,
 //   qr [16][DP] | uk [DP][16] | decay [DP] | P [16][16]
 // Segment s has its chunks from start[s] / 16 + s on, which cannot overlap
 // as long as the segments are in the order of their rows.
+//
+// ONES: one more column whose values are 1; its read-out goes to ones_out
+// [rows, heads].
 // ---------------------------------------------------------------------------
 template <int DP>
 struct ChunkWork {
@@ -140,11 +156,12 @@ struct ChunkWork {
                        P = 33 * DP, SIZE = 33 * DP + 256;
 };
 
-template <typename T, int TPW>
+template <typename T, int TPW, bool ONES = false>
 __global__ __launch_bounds__(256) void matrix_chunks_kernel(
     float* __restrict__ o, const float* __restrict__ work,
     const T* __restrict__ values, long long ld, float* __restrict__ state,
-    SegView seg, int heads, int dim, int vdim, int vstride) {
+    SegView seg, int heads, int dim, int vdim, int vstride,
+    float* __restrict__ ones_out = nullptr) {
   constexpr int DP = 64 * TPW;
   using W = ChunkWork<DP>;
   __shared__ float red[2][4][16][17];
@@ -162,7 +179,10 @@ __global__ __launch_bounds__(256) void matrix_chunks_kernel(
   const T* vp = values + row0 * ld + h * vdim + min(col, vdim - 1);
   float* S = state +
              ((size_t)seg.slot[s] * heads + h) * (size_t)dim * vstride + col;
-  const bool keep = col < vdim && seg.pos0[s] != 0;
+  const int cols = vdim + (ONES ? 1 : 0);
+  const bool keep = col < cols && seg.pos0[s] != 0;
+  // (decided where a value is used, so that nothing waits for its load)
+  auto number = [&](T v) { return ONES && col >= vdim ? 1.f : to_f(v); };
 
   f32x4 st[TPW];
 #pragma unroll
@@ -203,7 +223,7 @@ __global__ __launch_bounds__(256) void matrix_chunks_kernel(
   auto chunk = [&](const Operands& a, int ch) {
     // two accumulators: half the dependent chain
     f32x4 a0{0.f, 0.f, 0.f, 0.f}, a1 = a0;
-    a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(a.p, to_f(a.vw), a0, 0, 0, 0);
+    a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(a.p, number(a.vw), a0, 0, 0, 0);
 #pragma unroll
     for (int k = 0; k < TPW; ++k) {
       a1 = __builtin_amdgcn_mfma_f32_16x16x4f32(a.qr[k][0], st[k][0], a1, 0, 0, 0);
@@ -217,8 +237,8 @@ __global__ __launch_bounds__(256) void matrix_chunks_kernel(
     for (int i = 0; i < 4; ++i)
 #pragma unroll
       for (int k = 0; k < TPW; ++k)
-        st[k] = __builtin_amdgcn_mfma_f32_16x16x4f32(a.uk[k][i], to_f(a.v[i]),
-                                                     st[k], 0, 0, 0);
+        st[k] = __builtin_amdgcn_mfma_f32_16x16x4f32(
+            a.uk[k][i], number(a.v[i]), st[k], 0, 0, 0);
     a0 += a1;
 #pragma unroll
     for (int i = 0; i < 4; ++i) red[ch & 1][wave][quad * 4 + i][c] = a0[i];
@@ -226,11 +246,14 @@ __global__ __launch_bounds__(256) void matrix_chunks_kernel(
   auto emit = [&](int ch) {
     __syncthreads();  // one per chunk: the other half is written next
     const int t = tid >> 4, e = tid & 15, tt = ch * 16 + t;
-    if (tt < len && c0 + e < vdim) {
+    if (tt < len && c0 + e < cols) {
       float v = 0.f;
 #pragma unroll
       for (int k = 0; k < 4; ++k) v += red[ch & 1][k][t][e];
-      o[(row0 + tt) * (size_t)(heads * vdim) + h * vdim + c0 + e] = v;
+      if (ONES && c0 + e == vdim)
+        ones_out[(row0 + tt) * heads + h] = v;
+      else
+        o[(row0 + tt) * (size_t)(heads * vdim) + h * vdim + c0 + e] = v;
     }
   };
 #pragma unroll
@@ -250,7 +273,7 @@ __global__ __launch_bounds__(256) void matrix_chunks_kernel(
       chunk(ring[r], base + r);
       emit(base + r);
     }
-  if (col < vdim) {
+  if (col < cols) {
 #pragma unroll
     for (int k = 0; k < TPW; ++k)
 #pragma unroll
@@ -263,4 +286,10 @@ __global__ __launch_bounds__(256) void matrix_chunks_kernel(
 
 inline int chunk_dpad(int dim) {
   return dim <= 64 ? 64 : dim <= 128 ? 128 : dim <= 256 ? 256 : 0;
+}
+
+inline long long chunk_work_floats(int rows, int segments, int heads,
+                                   int dim) {
+  const long long chunks = rows / 16 + segments + 1;
+  return chunks * heads * (33 * chunk_dpad(dim) + 256);
 }

@@ -1,6 +1,6 @@
-// Recurrent mixers with a short convolution over ragged batches (gfx950):
-// the convolution, RG-LRU (block-diagonal gates and a scan per channel) and
-// the Mamba-2 rule of the matrix-state kernels.
+// Recurrent mixers over ragged batches (gfx950): the short convolution, the
+// scan per channel with RG-LRU (block-diagonal gates) and minGRU, and the
+// Mamba-2 rule of the matrix-state kernels.
 
 #include "matrix_state.h"
 #include "mfma_tile.h"
@@ -262,52 +262,44 @@ __global__ __launch_bounds__(256) void rglru_gates_kernel(RgLruArgs p) {
   }
 }
 
-// The recurrence of a segment, 16 channels per block: 16 threads share a
-// channel and take 8 tokens each of a tile of 128, whose maps S -> A S + B are
-// composed through LDS.  The next tile's operands are in flight meanwhile.
-template <typename T>
-__global__ __launch_bounds__(256) void rglru_scan_kernel(RgLruArgs p) {
+// A recurrence S <- a S + x over a segment, 16 channels per block: 16 threads
+// share a channel and take 8 tokens each of a tile of 128, whose maps S -> A S
+// + B are composed through LDS.  The next tile's operands are in flight
+// meanwhile.  Rule has In (a token's operands), enter(c), load(row, c),
+// map(in) and put(row, c, S, in).
+template <typename Rule>
+__global__ __launch_bounds__(256) void channel_scan_kernel(
+    Rule rule, float* __restrict__ states, SegView seg, int width) {
   constexpr int TC = 8, SUB = 16, TILE = TC * SUB;
   __shared__ float ma[2][SUB][17], mx[2][SUB][17];
-  const int s = blockIdx.y, len = p.seg.len[s];
+  const int s = blockIdx.y, len = seg.len[s];
   const int cl = threadIdx.x & 15, sub = threadIdx.x >> 4;
   // blocks of one XCD are neighbours: they share lines in its L2
   const int c = ((int)(blockIdx.x & 7) * (gridDim.x >> 3) +
                  (int)(blockIdx.x >> 3)) * 16 + cl;
-  const bool live = c < p.width;
-  const int cc = min(c, p.width - 1);
-  const size_t row0 = p.seg.start[s];
-  const float* pa = p.work + row0 * p.width + cc;
-  const float* px = pa + (size_t)p.n * p.width;
-  const T* py = (const T*)p.y + row0 * p.y_ld + cc;
-  T* out = (T*)p.out + row0 * p.width + cc;
-  float* state = p.state + (size_t)p.seg.slot[s] * p.width + cc;
-  const float y_bias = p.y_bias[cc];
-  float S = p.seg.pos0[s] != 0 ? *state : 0.f;
+  const bool live = c < width;
+  const int cc = min(c, width - 1);
+  const size_t row0 = seg.start[s];
+  float* state = states + (size_t)seg.slot[s] * width + cc;
+  rule.enter(cc);
+  float S = seg.pos0[s] != 0 ? *state : 0.f;
   struct Tile {
-    float a[TC], x[TC];
-    T y[TC];
+    typename Rule::In in[TC];
   };
   auto load = [&](Tile& t, int t0) {
 #pragma unroll
-    for (int j = 0; j < TC; ++j) {
+    for (int j = 0; j < TC; ++j)
       // tokens past the end repeat the last: their map is replaced below
-      const size_t r = min(t0 + sub * TC + j, len - 1);
-      t.a[j] = pa[r * p.width];
-      t.x[j] = px[r * p.width];
-      t.y[j] = py[r * p.y_ld];
-    }
+      t.in[j] = rule.load(row0 + min(t0 + sub * TC + j, len - 1), cc);
   };
   auto run = [&](Tile& t, int t0, int buf) {
     float A = 1.f, B = 0.f;
+    Decay d[TC];
 #pragma unroll
     for (int j = 0; j < TC; ++j) {
-      if (t0 + sub * TC + j >= len) {
-        t.a[j] = 1.f;
-        t.x[j] = 0.f;
-      }
-      A *= t.a[j];
-      B = t.a[j] * B + t.x[j];
+      d[j] = t0 + sub * TC + j < len ? rule.map(t.in[j]) : Decay{1.f, 0.f};
+      A *= d[j].a;
+      B = d[j].a * B + d[j].x;
     }
     ma[buf][sub][cl] = A;
     mx[buf][sub][cl] = B;
@@ -320,11 +312,9 @@ __global__ __launch_bounds__(256) void rglru_scan_kernel(RgLruArgs p) {
     }
 #pragma unroll
     for (int j = 0; j < TC; ++j) {
-      in = t.a[j] * in + t.x[j];
+      in = d[j].a * in + d[j].x;
       const int tt = t0 + sub * TC + j;
-      if (live && tt < len)
-        out[(size_t)tt * p.width] =
-            from_f<T>(in * gelu_tanh<T>(to_f(t.y[j]) + y_bias));
+      if (live && tt < len) rule.put(row0 + tt, cc, in, t.in[j]);
     }
   };
   Tile t[2];
@@ -338,6 +328,38 @@ __global__ __launch_bounds__(256) void rglru_scan_kernel(RgLruArgs p) {
   }
   if (live && sub == 0) *state = S;
 }
+
+template <typename Rule>
+void channel_scan(const Rule& rule, float* state, SegView seg, int width,
+                  hipStream_t stream) {
+  channel_scan_kernel<Rule><<<dim3((width + 127) / 128 * 8, seg.n), 256, 0,
+                              stream>>>(rule, state, seg, width);
+}
+
+template <typename T>
+struct RgLruScan {
+  struct In {
+    float a, x;
+    T y;
+  };
+  T* out;
+  const float* a;
+  const float* x;
+  const T* y;
+  const float* bias;
+  long long y_ld;
+  int width;
+  float y_bias;
+  DEVINL void enter(int c) { y_bias = bias[c]; }
+  DEVINL In load(size_t row, int c) const {
+    const size_t at = row * width + c;
+    return {a[at], x[at], y[row * y_ld + c]};
+  }
+  DEVINL Decay map(const In& i) const { return {i.a, i.x}; }
+  DEVINL void put(size_t row, int c, float S, const In& i) const {
+    out[row * width + c] = from_f<T>(S * gelu_tanh<T>(to_f(i.y) + y_bias));
+  }
+};
 
 // One token per segment: gates, recurrence and the second branch in one
 // launch; a block has 16 channels of up to 16 segments.
@@ -390,8 +412,74 @@ void rglru_scan_t(const RgLruArgs& a, hipStream_t stream) {
     rglru_gates_kernel<T, true><<<grid, 256, 0, stream>>>(a);
   else
     rglru_gates_kernel<T, false><<<grid, 256, 0, stream>>>(a);
-  rglru_scan_kernel<T>
-      <<<dim3((a.width + 127) / 128 * 8, a.seg.n), 256, 0, stream>>>(a);
+  channel_scan(RgLruScan<T>{(T*)a.out, a.work,
+                            a.work + (size_t)a.n * a.width, (const T*)a.y,
+                            a.y_bias, a.y_ld, a.width, 0.f},
+               a.state, a.seg, a.width, stream);
+}
+
+// ---------------------------------------------------------------------------
+// minGRU: all gates are functions of the token's own projections
+// ---------------------------------------------------------------------------
+template <typename T>
+struct MinGruScan {
+  using M = Math<T>;
+  struct In {
+    T z, u, g;
+  };
+  T* out;
+  const T* proj;
+  const float* bias;
+  long long ld;
+  int width;
+  float bz, bu;
+  static DEVINL float gate(float v) { return M::inv(1.f + M::exp(-v)); }
+  DEVINL void enter(int c) {
+    bz = bias[c];
+    bu = bias[width + c];
+  }
+  DEVINL In load(size_t row, int c) const {
+    const T* p = proj + row * ld + c;
+    return {p[0], p[width], p[2 * width]};
+  }
+  DEVINL Decay map(const In& i) const {
+    // 1 - z from its own side: exact where z is close to 1
+    const float v = to_f(i.z) + bz, u = to_f(i.u) + bu;
+    const float c = u >= 0.f ? u + 0.5f : gate(u);
+    return {gate(-v), gate(v) * c};
+  }
+  DEVINL void put(size_t row, int c, float S, const In& i) const {
+    const float g = to_f(i.g);
+    out[row * width + c] = from_f<T>(S * g * gate(g));
+  }
+};
+
+template <typename T>
+MinGruScan<T> mingru_rule(const MinGruArgs& a) {
+  return {(T*)a.out, (const T*)a.proj, a.bias, a.ld, a.width, 0.f, 0.f};
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void mingru_step_kernel(MinGruScan<T> rule,
+                                                          float* states,
+                                                          SegView seg) {
+  const int c = blockIdx.x * 256 + threadIdx.x, s = blockIdx.y;
+  if (c >= rule.width) return;
+  const size_t row = seg.start[s];
+  float* state = states + (size_t)seg.slot[s] * rule.width + c;
+  rule.enter(c);
+  const typename MinGruScan<T>::In in = rule.load(row, c);
+  const float S = seg.pos0[s] != 0 ? *state : 0.f;
+  const Decay d = rule.map(in);
+  const float next = d.a * S + d.x;
+  *state = next;
+  rule.put(row, c, next, in);
+}
+
+template <typename T>
+void mingru_step_t(const MinGruArgs& a, hipStream_t stream) {
+  mingru_step_kernel<T><<<dim3((a.width + 255) / 256, a.seg.n), 256, 0,
+                          stream>>>(mingru_rule<T>(a), a.state, a.seg);
 }
 
 // ---------------------------------------------------------------------------
@@ -399,7 +487,7 @@ void rglru_scan_t(const RgLruArgs& a, hipStream_t stream) {
 // ---------------------------------------------------------------------------
 template <typename T>
 struct Mamba2Rule {
-  static constexpr bool NORM = false;
+  static constexpr bool NORM = false, NORMALISER = false;
   float* o;
   const T* xbc;
   const T* dt;
@@ -530,6 +618,18 @@ void launch_rglru_step(const RgLruArgs& a, int f32, hipStream_t stream) {
 void launch_rglru_scan(const RgLruArgs& a, int f32, hipStream_t stream) {
   if (f32) rglru_scan_t<float>(a, stream);
   else rglru_scan_t<bf16>(a, stream);
+}
+
+void launch_mingru_step(const MinGruArgs& a, int f32, hipStream_t stream) {
+  if (f32) mingru_step_t<float>(a, stream);
+  else mingru_step_t<bf16>(a, stream);
+}
+
+void launch_mingru_scan(const MinGruArgs& a, int f32, hipStream_t stream) {
+  if (f32)
+    channel_scan(mingru_rule<float>(a), a.state, a.seg, a.width, stream);
+  else
+    channel_scan(mingru_rule<bf16>(a), a.state, a.seg, a.width, stream);
 }
 
 void launch_mamba2_step(const Mamba2Args& a, int f32, hipStream_t stream) {

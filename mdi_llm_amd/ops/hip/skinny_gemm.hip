@@ -83,6 +83,7 @@ __global__ __launch_bounds__(NW * 64) void skinny_gemm_kernel(
   for (int q = 0; q < NW; ++q) v += red[q][row >> 4][row & 15][j];
   if (ACT == 1) v = xielu(v, act_p, act_q);
   if (ACT == 2) v = gelu_erf(v);
+  if (ACT == 3) v = relu2(v);
   out[(size_t)row * m + m0 + j] = from_f<bf16>(v);
 }
 
@@ -97,11 +98,13 @@ int launch_skinny_gemm(void* out, const void* w, const void* x, int n, int m,
   skinny_gemm_kernel<NT, ACT><<<grid, NW * 64, 0, stream>>>(             \
       (bf16*)out, (const bf16*)w, (const bf16*)x, n, m, k, act_p, act_q)
   if (n <= 16) {
-    if (act == 2) SKINNY(1, 2);
+    if (act == 3) SKINNY(1, 3);
+    else if (act == 2) SKINNY(1, 2);
     else if (act == 1) SKINNY(1, 1);
     else SKINNY(1, 0);
   } else {
-    if (act == 2) SKINNY(2, 2);
+    if (act == 3) SKINNY(2, 3);
+    else if (act == 2) SKINNY(2, 2);
     else if (act == 1) SKINNY(2, 1);
     else SKINNY(2, 0);
   }

@@ -32,10 +32,11 @@ OFFLOAD_ARCH = os.environ.get("PYTORCH_ROCM_ARCH", "gfx950").split(";")[0]
 KERNEL_SOURCES = ["decode_kernels.hip", "hybrid_kernels.hip",
                   "paged_attn_bf16.hip", "paged_attn_f32.hip",
                   "diff_attn_bf16.hip", "diff_attn_f32.hip",
+                  "slope_attn_bf16.hip", "slope_attn_f32.hip",
                   "row_attn_bf16.hip", "row_attn_f32.hip",
                   "latent_kernels.hip", "moe_kernels.hip",
-                  "recurrent_kernels.hip", "stream_kernels.hip",
-                  "skinny_gemm.hip"]
+                  "recurrent_kernels.hip", "mlstm_kernels.hip",
+                  "stream_kernels.hip", "skinny_gemm.hip"]
 HEADERS = [HIP_DIR / h for h in ("decode_kernels.h", "hybrid_kernels.h",
                                  "hybrid_common.h", "mfma_frag.h",
                                  "mfma_tile.h", "matrix_state.h",
