@@ -48,7 +48,8 @@ def parse_args():
     ap.add_argument("--no-graphs", action="store_true")
     ap.add_argument("--hybrid", nargs="*", default=None,
                     choices=["nerozen-1b", "nerozen-8b", "resolorn-1b",
-                             "resolorn-8b", "dinuzen-1b", "dinuzen-8b"],
+                             "resolorn-8b", "dinuzen-1b", "dinuzen-8b",
+                             "sosutar-1b", "sosutar-8b"],
                     metavar="MODEL",
                     help="instead of the headline workload: prefill and "
                          "decode throughput of these hybrid stacks (default "

@@ -147,8 +147,9 @@ void matrix_step(const Rule& rule, float* state, SegView seg, int heads,
 // Segment s has its chunks from start[s] / 16 + s on, which cannot overlap
 // as long as the segments are in the order of their rows.
 //
-// ONES: one more column whose values are 1; its read-out goes to ones_out
-// [rows, heads].
+// SUMS: one more column whose values are 1, which is a vector per head and
+// needs no products: sums [chunk, heads, DP] has sum_s U_s k_s of each chunk,
+// in whose place the head's last block leaves the column at the chunk's start.
 // ---------------------------------------------------------------------------
 template <int DP>
 struct ChunkWork {
@@ -156,12 +157,53 @@ struct ChunkWork {
                        P = 33 * DP, SIZE = 33 * DP + 256;
 };
 
-template <typename T, int TPW, bool ONES = false>
+template <int DP>
+DEVINL void running_sums(float* __restrict__ sums, const float* __restrict__ w,
+                         float* __restrict__ column, bool fresh, int chunks,
+                         int heads, int dim, int vstride) {
+  constexpr int AHEAD = 8;
+  const int d = threadIdx.x;
+  if (d >= DP) return;
+  const size_t step = (size_t)heads * DP;
+  const size_t wstep = (size_t)heads * ChunkWork<DP>::SIZE;
+  sums += d;
+  w += ChunkWork<DP>::DECAY + d;
+  float n = !fresh && d < dim ? column[(size_t)d * vstride] : 0.f;
+  float u[2][AHEAD], f[2][AHEAD];
+  auto load = [&](int b, int c0) {
+#pragma unroll
+    for (int j = 0; j < AHEAD; ++j) {
+      const int c = min(c0 + j, chunks - 1);
+      u[b][j] = sums[c * step];
+      f[b][j] = w[c * wstep];
+    }
+  };
+  auto run = [&](int b, int c0) {
+#pragma unroll
+    for (int j = 0; j < AHEAD; ++j)
+      if (c0 + j < chunks) {
+        sums[(c0 + j) * step] = n;
+        n = f[b][j] * n + u[b][j];
+      }
+  };
+  // (a chunk is loaded before its place is written: loads run ahead, and what
+  // they repeat past the end is not used)
+  load(0, 0);
+  for (int c0 = 0; c0 < chunks; c0 += 2 * AHEAD) {
+    load(1, c0 + AHEAD);
+    run(0, c0);
+    load(0, c0 + 2 * AHEAD);
+    run(1, c0 + AHEAD);
+  }
+  if (d < dim) column[(size_t)d * vstride] = n;
+}
+
+template <typename T, int TPW, bool SUMS = false>
 __global__ __launch_bounds__(256) void matrix_chunks_kernel(
     float* __restrict__ o, const float* __restrict__ work,
     const T* __restrict__ values, long long ld, float* __restrict__ state,
     SegView seg, int heads, int dim, int vdim, int vstride,
-    float* __restrict__ ones_out = nullptr) {
+    float* __restrict__ sums = nullptr) {
   constexpr int DP = 64 * TPW;
   using W = ChunkWork<DP>;
   __shared__ float red[2][4][16][17];
@@ -175,14 +217,21 @@ __global__ __launch_bounds__(256) void matrix_chunks_kernel(
   const size_t row0 = seg.start[s];
   const float* w = work + ((row0 / 16 + s) * heads + h) * W::SIZE;
   const size_t wstep = (size_t)heads * W::SIZE;
+  if constexpr (SUMS) {
+    if (blockIdx.y + 1 == gridDim.y) {
+      running_sums<DP>(
+          sums + ((row0 / 16 + s) * heads + h) * DP, w,
+          state + ((size_t)seg.slot[s] * heads + h) * (size_t)dim * vstride +
+              vdim,
+          seg.pos0[s] == 0, n, heads, dim, vstride);
+      return;
+    }
+  }
   // values: head h of row r at r * ld + h * vdim
   const T* vp = values + row0 * ld + h * vdim + min(col, vdim - 1);
   float* S = state +
              ((size_t)seg.slot[s] * heads + h) * (size_t)dim * vstride + col;
-  const int cols = vdim + (ONES ? 1 : 0);
-  const bool keep = col < cols && seg.pos0[s] != 0;
-  // (decided where a value is used, so that nothing waits for its load)
-  auto number = [&](T v) { return ONES && col >= vdim ? 1.f : to_f(v); };
+  const bool keep = col < vdim && seg.pos0[s] != 0;
 
   f32x4 st[TPW];
 #pragma unroll
@@ -223,7 +272,7 @@ __global__ __launch_bounds__(256) void matrix_chunks_kernel(
   auto chunk = [&](const Operands& a, int ch) {
     // two accumulators: half the dependent chain
     f32x4 a0{0.f, 0.f, 0.f, 0.f}, a1 = a0;
-    a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(a.p, number(a.vw), a0, 0, 0, 0);
+    a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(a.p, to_f(a.vw), a0, 0, 0, 0);
 #pragma unroll
     for (int k = 0; k < TPW; ++k) {
       a1 = __builtin_amdgcn_mfma_f32_16x16x4f32(a.qr[k][0], st[k][0], a1, 0, 0, 0);
@@ -237,8 +286,8 @@ __global__ __launch_bounds__(256) void matrix_chunks_kernel(
     for (int i = 0; i < 4; ++i)
 #pragma unroll
       for (int k = 0; k < TPW; ++k)
-        st[k] = __builtin_amdgcn_mfma_f32_16x16x4f32(
-            a.uk[k][i], number(a.v[i]), st[k], 0, 0, 0);
+        st[k] = __builtin_amdgcn_mfma_f32_16x16x4f32(a.uk[k][i], to_f(a.v[i]),
+                                                     st[k], 0, 0, 0);
     a0 += a1;
 #pragma unroll
     for (int i = 0; i < 4; ++i) red[ch & 1][wave][quad * 4 + i][c] = a0[i];
@@ -246,14 +295,11 @@ __global__ __launch_bounds__(256) void matrix_chunks_kernel(
   auto emit = [&](int ch) {
     __syncthreads();  // one per chunk: the other half is written next
     const int t = tid >> 4, e = tid & 15, tt = ch * 16 + t;
-    if (tt < len && c0 + e < cols) {
+    if (tt < len && c0 + e < vdim) {
       float v = 0.f;
 #pragma unroll
       for (int k = 0; k < 4; ++k) v += red[ch & 1][k][t][e];
-      if (ONES && c0 + e == vdim)
-        ones_out[(row0 + tt) * heads + h] = v;
-      else
-        o[(row0 + tt) * (size_t)(heads * vdim) + h * vdim + c0 + e] = v;
+      o[(row0 + tt) * (size_t)(heads * vdim) + h * vdim + c0 + e] = v;
     }
   };
 #pragma unroll
@@ -273,7 +319,7 @@ __global__ __launch_bounds__(256) void matrix_chunks_kernel(
       chunk(ring[r], base + r);
       emit(base + r);
     }
-  if (col < cols) {
+  if (col < vdim) {
 #pragma unroll
     for (int k = 0; k < TPW; ++k)
 #pragma unroll
@@ -292,4 +338,9 @@ inline long long chunk_work_floats(int rows, int segments, int heads,
                                    int dim) {
   const long long chunks = rows / 16 + segments + 1;
   return chunks * heads * (33 * chunk_dpad(dim) + 256);
+}
+
+inline long long chunk_sums_floats(int rows, int segments, int heads,
+                                   int dim) {
+  return (long long)(rows / 16 + segments + 1) * heads * chunk_dpad(dim);
 }

@@ -75,23 +75,25 @@ void step_t(const MLstmArgs& a, hipStream_t stream) {
               stream);
 }
 
-// Workspace of a scan: chunk factors, the raw read-out, and by head and row
-// the log gates, m after each token, and what the normaliser reads out; m
-// before each segment.
+// Workspace of a scan: chunk factors and sums, the raw read-out; by head and
+// row the log gates, m after each token, and the normaliser's read-out as
+// n . q = from * (n at the chunk's start . q) + own; m before each segment.
 struct ScanWork {
-  float *chunks, *o, *i, *f, *m, *n, *start;
+  float *chunks, *sums, *o, *i, *f, *m, *from, *own, *start;
 };
 
 ScanWork scan_work(const MLstmArgs& a) {
   const size_t cells = (size_t)a.n * a.heads;
   ScanWork w;
   w.chunks = a.work;
-  w.o = w.chunks + chunk_work_floats(a.n, a.seg.n, a.heads, a.dim);
+  w.sums = w.chunks + chunk_work_floats(a.n, a.seg.n, a.heads, a.dim);
+  w.o = w.sums + chunk_sums_floats(a.n, a.seg.n, a.heads, a.dim);
   w.i = w.o + cells * a.vdim;
   w.f = w.i + cells;
   w.m = w.f + cells;
-  w.n = w.m + cells;
-  w.start = w.n + cells;
+  w.from = w.m + cells;
+  w.own = w.from + cells;
+  w.start = w.own + cells;
   return w;
 }
 
@@ -171,8 +173,9 @@ __global__ __launch_bounds__(256) void mlstm_factors_kernel(MLstmArgs p,
   if (tn <= 0) return;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const size_t row0 = (size_t)p.seg.start[s] + t0, at = (size_t)h * p.n + row0;
-  float* w = sw.chunks + (((size_t)p.seg.start[s] / 16 + s + blockIdx.x) *
-                              p.heads + h) * W::SIZE;
+  const size_t chunk =
+      ((size_t)p.seg.start[s] / 16 + s + blockIdx.x) * p.heads + h;
+  float* w = sw.chunks + chunk * W::SIZE;
   const long long ld = 2LL * p.heads * (p.dim + p.vdim + 1);
   const T* q = (const T*)p.proj + row0 * ld + h * p.dim;
   const T* k = q + p.heads * p.dim;
@@ -204,6 +207,7 @@ __global__ __launch_bounds__(256) void mlstm_factors_kernel(MLstmArgs p,
     lm[t] = m;
     const float total = __shfl(sum, 15, 16), end = __shfl(m, 15, 16);
     from[t] = t < tn ? expf(sum + m0 - m) * p.q_scale : 0.f;
+    if (t < tn) sw.from[at + t] = from[t];
     to[t] = expf(i + (total - sum) - end);
   }
   for (int i = tid; i < 16 * DP; i += 256) {
@@ -218,59 +222,100 @@ __global__ __launch_bounds__(256) void mlstm_factors_kernel(MLstmArgs p,
         t < tn && d < p.dim ? to_f(q[t * ld + d]) * from[t] : 0.f;
     w[W::UK + i] = to_f(ks[i & 15][i >> 4]) * to[i & 15];
   }
-  for (int d = tid; d < DP; d += 256) w[W::DECAY + d] = decay;
+  for (int d = tid; d < DP; d += 256) {
+    w[W::DECAY + d] = decay;
+    float sum = 0.f;
+#pragma unroll
+    for (int t = 0; t < 16; ++t) sum += to_f(ks[t][d]) * to[t];
+    sw.sums[chunk * DP + d] = sum;
+  }
   const int t = tid >> 4, sp = tid & 15;
   float dot = 0.f;
 #pragma unroll
   for (int j = 0; j < 4; ++j) dot += red[j][t][sp];
-  w[W::P + tid] = sp <= t && t < tn
-                      ? dot * p.q_scale *
-                            expf(li[sp] + (cum[t] - cum[sp]) - lm[t])
-                      : 0.f;
+  const float weight =
+      sp <= t && t < tn ? dot * p.q_scale *
+                              expf(li[sp] + (cum[t] - cum[sp]) - lm[t])
+                        : 0.f;
+  w[W::P + tid] = weight;
+  const float own = row16_sum(weight);
+  if (sp == 0 && t < tn) sw.own[at + t] = own;
 }
 
-// one wave per (row, head): V columns per access
-template <typename T, int V>
+// Normalised, of unit size, gated: a wave has ROWS neighbouring rows of a head
+// (all of one chunk), V columns per access.
+template <typename T, int V, int KEEP, int ROWS>
 __global__ __launch_bounds__(256) void mlstm_out_kernel(MLstmArgs p,
-                                                        ScanWork w) {
-  constexpr int KEEP = 16 / V;
-  const int s = blockIdx.y, lane = threadIdx.x & 63;
-  const unsigned cell = blockIdx.x * 4u + (threadIdx.x >> 6);
-  if (cell >= (unsigned)p.seg.len[s] * (unsigned)p.heads) return;
-  const int h = cell % p.heads;
-  const size_t row = (size_t)p.seg.start[s] + cell / p.heads;
+                                                        ScanWork w,
+                                                        int dpad) {
+  const int s = blockIdx.y, lane = threadIdx.x & 63, len = p.seg.len[s];
+  const unsigned unit = blockIdx.x * 4u + (threadIdx.x >> 6);
+  const int h = unit % p.heads, t0 = unit / p.heads * ROWS;
+  if (t0 >= len) return;
+  const size_t row0 = p.seg.start[s];
   const int col0 = h * p.vdim, inner = p.heads * p.vdim;
-  const float* o = w.o + row * inner + col0;
-  const T* g = (const T*)p.proj +
-               row * (size_t)(2 * p.heads * (p.dim + p.vdim + 1)) +
-               2 * p.heads * p.dim + inner + col0;
-  const float n = w.n[row * p.heads + h], m = w.m[(size_t)h * p.n + row];
-  Pack<float, V> a[KEEP];
-  Pack<T, V> b[KEEP];
-  float ss = 0.f;
+  const size_t ld = 2 * p.heads * (size_t)(p.dim + p.vdim + 1);
+  const float* sum = w.sums + ((row0 / 16 + s + t0 / 16) * p.heads + h) * dpad;
+  Pack<float, V> a[ROWS][KEEP];
+  Pack<T, V> b[ROWS][KEEP];
+  float n[ROWS], from[ROWS], own[ROWS], m[ROWS];
 #pragma unroll
-  for (int k = 0; k < KEEP; ++k) {
-    const int c = (k * 64 + lane) * V;
-    if (c >= p.vdim) break;
-    a[k] = *reinterpret_cast<const Pack<float, V>*>(o + c);
-    b[k] = *reinterpret_cast<const Pack<T, V>*>(g + c);
+  for (int r = 0; r < ROWS; ++r) {
+    // rows past the end repeat the last one; they are not stored
+    const size_t row = row0 + min(t0 + r, len - 1);
+    const size_t at = (size_t)h * p.n + row;
+    const T* proj = (const T*)p.proj + row * ld;
+    const float* o = w.o + row * inner + col0;
+    const T* g = proj + 2 * p.heads * p.dim + inner + col0;
 #pragma unroll
-    for (int j = 0; j < V; ++j) ss += a[k].v[j] * a[k].v[j];
+    for (int k = 0; k < KEEP; ++k) {
+      const int c = (k * 64 + lane) * V;
+      if (c >= p.vdim) break;
+      a[r][k] = *reinterpret_cast<const Pack<float, V>*>(o + c);
+      b[r][k] = *reinterpret_cast<const Pack<T, V>*>(g + c);
+    }
+    n[r] = 0.f;
+    for (int d = lane; d < p.dim; d += 64)
+      n[r] += to_f(proj[h * p.dim + d]) * sum[d];
+    from[r] = w.from[at];
+    own[r] = w.own[at];
+    m[r] = w.m[at];
   }
-  const float inv = 1.f / (fmaxf(fabsf(n), expf(-m)) + 1e-6f);
-  const float r = inv / sqrtf(wave_sum(ss) * inv * inv / p.vdim + p.eps);
-  T* out = (T*)p.out + row * inner + col0;
 #pragma unroll
-  for (int k = 0; k < KEEP; ++k) {
-    const int c = (k * 64 + lane) * V;
-    if (c >= p.vdim) break;
-    Pack<T, V> y;
+  for (int r = 0; r < ROWS; ++r) {
+    float ss = 0.f;
 #pragma unroll
-    for (int j = 0; j < V; ++j)
-      y.v[j] = from_f<T>(a[k].v[j] * r * p.norm_w[col0 + c + j] *
-                         sigmoid(to_f(b[k].v[j])));
-    *reinterpret_cast<Pack<T, V>*>(out + c) = y;
+    for (int k = 0; k < KEEP; ++k) {
+      if ((k * 64 + lane) * V >= p.vdim) break;
+#pragma unroll
+      for (int j = 0; j < V; ++j) ss += a[r][k].v[j] * a[r][k].v[j];
+    }
+    const float q = from[r] * wave_sum(n[r]) + own[r];
+    const float inv = 1.f / (fmaxf(fabsf(q), expf(-m[r])) + 1e-6f);
+    const float f = inv / sqrtf(wave_sum(ss) * inv * inv / p.vdim + p.eps);
+    if (t0 + r >= len) break;
+    T* out = (T*)p.out + (row0 + t0 + r) * inner + col0;
+#pragma unroll
+    for (int k = 0; k < KEEP; ++k) {
+      const int c = (k * 64 + lane) * V;
+      if (c >= p.vdim) break;
+      Pack<T, V> y;
+#pragma unroll
+      for (int j = 0; j < V; ++j)
+        y.v[j] = from_f<T>(a[r][k].v[j] * f * p.norm_w[col0 + c + j] *
+                           sigmoid(to_f(b[r][k].v[j])));
+      *reinterpret_cast<Pack<T, V>*>(out + c) = y;
+    }
   }
+}
+
+template <typename T, int V, int KEEP, int ROWS>
+void out_sized(const MLstmArgs& a, const ScanWork& w, hipStream_t stream) {
+  const long long units =
+      (long long)((a.max_len + ROWS - 1) / ROWS) * a.heads;
+  mlstm_out_kernel<T, V, KEEP, ROWS>
+      <<<dim3((unsigned)((units + 3) / 4), a.seg.n), 256, 0, stream>>>(
+          a, w, chunk_dpad(a.dim));
 }
 
 template <typename T, int TPW>
@@ -284,15 +329,17 @@ void scan_sized(const MLstmArgs& a, hipStream_t stream) {
       <<<dim3((a.max_len + 15) / 16, a.heads, a.seg.n), 256, 0, stream>>>(
           a, w, a.dim % n == 0 && ld % n == 0);
   matrix_chunks_kernel<T, TPW, true>
-      <<<dim3(a.heads, (a.vdim + 16) / 16, a.seg.n), 256, 0, stream>>>(
+      <<<dim3(a.heads, (a.vdim + 15) / 16 + 1, a.seg.n), 256, 0, stream>>>(
           w.o, w.chunks, (const T*)a.proj + 2 * a.heads * a.dim, ld, a.state,
-          a.seg, a.heads, a.dim, a.vdim, a.vstride, w.n);
-  const dim3 grid((unsigned)(((long long)a.max_len * a.heads + 3) / 4),
-                  a.seg.n);
-  if (a.vdim % 2 == 0)
-    mlstm_out_kernel<T, 2><<<grid, 256, 0, stream>>>(a, w);
-  else
-    mlstm_out_kernel<T, 1><<<grid, 256, 0, stream>>>(a, w);
+          a.seg, a.heads, a.dim, a.vdim, a.vstride, w.sums);
+  if (a.vdim % 2 != 0) {
+    if (a.vdim <= 64) out_sized<T, 1, 1, 4>(a, w, stream);
+    else out_sized<T, 1, 16, 1>(a, w, stream);
+  } else {
+    if (a.vdim <= 128) out_sized<T, 2, 1, 4>(a, w, stream);
+    else if (a.vdim <= 256) out_sized<T, 2, 2, 4>(a, w, stream);
+    else out_sized<T, 2, 8, 1>(a, w, stream);
+  }
 }
 
 template <typename T>
@@ -315,7 +362,8 @@ void launch_mlstm_step(const MLstmArgs& a, int f32, hipStream_t stream) {
 long long mlstm_work_floats(int rows, int segments, int heads, int dim,
                             int vdim) {
   return chunk_work_floats(rows, segments, heads, dim) +
-         (long long)rows * heads * (vdim + 4) + (long long)segments * heads;
+         chunk_sums_floats(rows, segments, heads, dim) +
+         (long long)rows * heads * (vdim + 5) + (long long)segments * heads;
 }
 
 int launch_mlstm_scan(const MLstmArgs& a, int f32, hipStream_t stream) {

@@ -24,6 +24,9 @@ PAIRS = {
     "resolorn-8b": "Meta-Llama-3-8B-Instruct",
     "dinuzen-1b": "tiny-llama-1.1b-chat",
     "dinuzen-8b": "Meta-Llama-3-8B-Instruct",
+    # the closest one: matrix states and windowed attention
+    "sosutar-1b": "nerozen-1b",
+    "sosutar-8b": "nerozen-8b",
 }
 SAMPLING = dict(temperature=0.8, top_k=200, seed=1234)
 
@@ -127,8 +130,9 @@ def compare(name: str, prompt: int = 4096, batch: int = 32,
     """Measure ``name`` and its counterpart; tokens/s by phase."""
     device = torch.device("cuda:0")
     res = {}
-    for model, run in ((name, _hybrid), (PAIRS[name], _existing)):
+    for model in (name, PAIRS[name]):
         cfg = ModelConfig.from_name(model)
+        run = _hybrid if cfg.is_hybrid else _existing
         # the counterpart's position limit does not bound its kernels
         cfg.block_size = max(cfg.block_size, prompt + 64)
         res[model] = {k: round(v, 1) if k != "weights" else v
