@@ -46,12 +46,13 @@ def errors(got, want):
 
 
 def agrees(got, want, dtype):
-    """Norms of a few elements, or of what nearly cancels, enlarge the
-    rounding of single positions."""
+    """Norms of a few elements, or of what nearly cancels (a first token's
+    q . k), enlarge the rounding of single positions."""
     e = errors(got, want).sort().values
     n = e.numel()
     most, worst = (4e-5, 1e-3) if dtype == torch.float32 else (0.06, 0.25)
-    return float(e[-1]) < worst and float(e[int(0.85 * (n - 1))]) < most
+    return float(e[-1]) < worst and (
+        n < 8 or float(e[int(0.85 * (n - 1))]) < most)
 
 
 def runner(name, device, dtype, **kw):
