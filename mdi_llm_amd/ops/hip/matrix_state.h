@@ -30,14 +30,28 @@ __global__ __launch_bounds__(NT) void matrix_step_kernel(
   extern __shared__ float sm[];
   __shared__ float red[NT / 64];
   const int tid = threadIdx.x, h = blockIdx.x, s = blockIdx.y;
-  const int nq = vstride / 4;                 // float4 columns
-  const int lanes = nq < NT ? nq : NT;      // threads along the columns
-  const int groups = NT / lanes;             // row groups
+  const int nq = vstride / 4;                 // float4 columns, at most NT
+  const int groups = NT / nq;                 // row groups
   float* qs = sm;                             // [dim]
   float* fs = qs + dim;                       // [dim]
   float* ks = fs + dim;                       // [dim]
   float* part = ks + dim;                     // [groups][vstride]
   const size_t row = seg.start[s];
+  float* S = state +
+             ((size_t)seg.slot[s] * heads + h) * (size_t)dim * vstride;
+  const bool fresh = seg.pos0[s] == 0;
+  // a thread has one column of a row group; its first rows are on their way
+  // while the factors are made
+  constexpr int AHEAD = 8;
+  const int g = tid / nq, c4 = tid % nq;
+  float4 ahead[AHEAD];
+  if (g < groups && !fresh) {
+#pragma unroll
+    for (int j = 0; j < AHEAD; ++j)
+      if (g + j * groups < dim)
+        ahead[j] = *(reinterpret_cast<const float4*>(
+                         S + (size_t)(g + j * groups) * vstride) + c4);
+  }
   if constexpr (Rule::NORMALISER)
     rule.enter(row, h, seg.slot[s], seg.pos0[s] == 0);
   for (int d = tid; d < dim; d += NT) {
@@ -47,36 +61,35 @@ __global__ __launch_bounds__(NT) void matrix_step_kernel(
     ks[d] = x.k;
   }
   __syncthreads();
-  float* S = state +
-             ((size_t)seg.slot[s] * heads + h) * (size_t)dim * vstride;
-  const bool fresh = seg.pos0[s] == 0;
-  const int g = tid / lanes;
   if (g < groups) {
-    for (int c4 = tid % lanes; c4 < nq; c4 += lanes) {
-      float v[4], o[4] = {0.f, 0.f, 0.f, 0.f};
+    float v[4], o[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        v[j] = c4 * 4 + j < vdim ? rule.value(row, h, c4 * 4 + j)
-               : Rule::NORMALISER && c4 * 4 + j == vdim ? 1.f
-                                                        : 0.f;
+    for (int j = 0; j < 4; ++j)
+      v[j] = c4 * 4 + j < vdim ? rule.value(row, h, c4 * 4 + j)
+             : Rule::NORMALISER && c4 * 4 + j == vdim ? 1.f
+                                                      : 0.f;
+    auto update = [&](int d, float4 a) {
+      if (fresh) a = make_float4(0.f, 0.f, 0.f, 0.f);
+      const float f = fs[d], w = ks[d], q = qs[d];
+      a.x = f * a.x + w * v[0];
+      a.y = f * a.y + w * v[1];
+      a.z = f * a.z + w * v[2];
+      a.w = f * a.w + w * v[3];
+      *(reinterpret_cast<float4*>(S + (size_t)d * vstride) + c4) = a;
+      o[0] += q * a.x;
+      o[1] += q * a.y;
+      o[2] += q * a.z;
+      o[3] += q * a.w;
+    };
+#pragma unroll
+    for (int j = 0; j < AHEAD; ++j)
+      if (g + j * groups < dim) update(g + j * groups, ahead[j]);
 #pragma unroll 8
-      for (int d = g; d < dim; d += groups) {
-        float4* p = reinterpret_cast<float4*>(S + (size_t)d * vstride) + c4;
-        float4 a = fresh ? make_float4(0.f, 0.f, 0.f, 0.f) : *p;
-        const float f = fs[d], w = ks[d], q = qs[d];
-        a.x = f * a.x + w * v[0];
-        a.y = f * a.y + w * v[1];
-        a.z = f * a.z + w * v[2];
-        a.w = f * a.w + w * v[3];
-        *p = a;
-        o[0] += q * a.x;
-        o[1] += q * a.y;
-        o[2] += q * a.z;
-        o[3] += q * a.w;
-      }
-      *reinterpret_cast<float4*>(part + g * vstride + c4 * 4) =
-          make_float4(o[0], o[1], o[2], o[3]);
-    }
+    for (int d = g + AHEAD * groups; d < dim; d += groups)
+      update(d, *(reinterpret_cast<const float4*>(S + (size_t)d * vstride) +
+                  c4));
+    *reinterpret_cast<float4*>(part + g * vstride + c4 * 4) =
+        make_float4(o[0], o[1], o[2], o[3]);
   }
   __syncthreads();
   float ss = 0.f;
@@ -112,9 +125,9 @@ void matrix_step(const Rule& rule, float* state, SegView seg, int heads,
   // few blocks with a large state each: more waves to keep loads in flight
   const int nt =
       dim * vstride >= 8192 && heads * seg.n <= 512 ? 1024 : 256;
-  const int nq = vstride / 4, lanes = nq < nt ? nq : nt;
   const size_t smem =
-      (3 * (size_t)dim + (size_t)(nt / lanes) * vstride) * sizeof(float);
+      (3 * (size_t)dim + (size_t)(nt / (vstride / 4)) * vstride) *
+      sizeof(float);
   const dim3 grid(heads, seg.n);
   if (nt == 1024)
     matrix_step_kernel<1024, Rule><<<grid, 1024, smem, stream>>>(

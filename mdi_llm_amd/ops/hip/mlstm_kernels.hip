@@ -244,10 +244,9 @@ __global__ __launch_bounds__(256) void mlstm_factors_kernel(MLstmArgs p,
 
 // Normalised, of unit size, gated: a wave has ROWS neighbouring rows of a head
 // (all of one chunk), V columns per access.
-template <typename T, int V, int KEEP, int ROWS>
+template <typename T, int TPW, int V, int KEEP, int ROWS>
 __global__ __launch_bounds__(256) void mlstm_out_kernel(MLstmArgs p,
-                                                        ScanWork w,
-                                                        int dpad) {
+                                                        ScanWork w) {
   const int s = blockIdx.y, lane = threadIdx.x & 63, len = p.seg.len[s];
   const unsigned unit = blockIdx.x * 4u + (threadIdx.x >> 6);
   const int h = unit % p.heads, t0 = unit / p.heads * ROWS;
@@ -255,10 +254,15 @@ __global__ __launch_bounds__(256) void mlstm_out_kernel(MLstmArgs p,
   const size_t row0 = p.seg.start[s];
   const int col0 = h * p.vdim, inner = p.heads * p.vdim;
   const size_t ld = 2 * p.heads * (size_t)(p.dim + p.vdim + 1);
-  const float* sum = w.sums + ((row0 / 16 + s + t0 / 16) * p.heads + h) * dpad;
+  const float* sum =
+      w.sums + ((row0 / 16 + s + t0 / 16) * p.heads + h) * (64 * TPW);
+  // all loads ahead of the first use
   Pack<float, V> a[ROWS][KEEP];
   Pack<T, V> b[ROWS][KEEP];
-  float n[ROWS], from[ROWS], own[ROWS], m[ROWS];
+  T q[ROWS][TPW];
+  float u[TPW], from[ROWS], own[ROWS], m[ROWS];
+#pragma unroll
+  for (int k = 0; k < TPW; ++k) u[k] = sum[k * 64 + lane];  // 0 past dim
 #pragma unroll
   for (int r = 0; r < ROWS; ++r) {
     // rows past the end repeat the last one; they are not stored
@@ -274,24 +278,26 @@ __global__ __launch_bounds__(256) void mlstm_out_kernel(MLstmArgs p,
       a[r][k] = *reinterpret_cast<const Pack<float, V>*>(o + c);
       b[r][k] = *reinterpret_cast<const Pack<T, V>*>(g + c);
     }
-    n[r] = 0.f;
-    for (int d = lane; d < p.dim; d += 64)
-      n[r] += to_f(proj[h * p.dim + d]) * sum[d];
+#pragma unroll
+    for (int k = 0; k < TPW; ++k)
+      q[r][k] = proj[h * p.dim + min(k * 64 + lane, p.dim - 1)];
     from[r] = w.from[at];
     own[r] = w.own[at];
     m[r] = w.m[at];
   }
 #pragma unroll
   for (int r = 0; r < ROWS; ++r) {
-    float ss = 0.f;
+    float ss = 0.f, dot = 0.f;
+#pragma unroll
+    for (int k = 0; k < TPW; ++k) dot += to_f(q[r][k]) * u[k];
 #pragma unroll
     for (int k = 0; k < KEEP; ++k) {
       if ((k * 64 + lane) * V >= p.vdim) break;
 #pragma unroll
       for (int j = 0; j < V; ++j) ss += a[r][k].v[j] * a[r][k].v[j];
     }
-    const float q = from[r] * wave_sum(n[r]) + own[r];
-    const float inv = 1.f / (fmaxf(fabsf(q), expf(-m[r])) + 1e-6f);
+    const float n = from[r] * wave_sum(dot) + own[r];
+    const float inv = 1.f / (fmaxf(fabsf(n), expf(-m[r])) + 1e-6f);
     const float f = inv / sqrtf(wave_sum(ss) * inv * inv / p.vdim + p.eps);
     if (t0 + r >= len) break;
     T* out = (T*)p.out + (row0 + t0 + r) * inner + col0;
@@ -309,13 +315,12 @@ __global__ __launch_bounds__(256) void mlstm_out_kernel(MLstmArgs p,
   }
 }
 
-template <typename T, int V, int KEEP, int ROWS>
+template <typename T, int TPW, int V, int KEEP, int ROWS>
 void out_sized(const MLstmArgs& a, const ScanWork& w, hipStream_t stream) {
   const long long units =
       (long long)((a.max_len + ROWS - 1) / ROWS) * a.heads;
-  mlstm_out_kernel<T, V, KEEP, ROWS>
-      <<<dim3((unsigned)((units + 3) / 4), a.seg.n), 256, 0, stream>>>(
-          a, w, chunk_dpad(a.dim));
+  mlstm_out_kernel<T, TPW, V, KEEP, ROWS>
+      <<<dim3((unsigned)((units + 3) / 4), a.seg.n), 256, 0, stream>>>(a, w);
 }
 
 template <typename T, int TPW>
@@ -333,12 +338,12 @@ void scan_sized(const MLstmArgs& a, hipStream_t stream) {
           w.o, w.chunks, (const T*)a.proj + 2 * a.heads * a.dim, ld, a.state,
           a.seg, a.heads, a.dim, a.vdim, a.vstride, w.sums);
   if (a.vdim % 2 != 0) {
-    if (a.vdim <= 64) out_sized<T, 1, 1, 4>(a, w, stream);
-    else out_sized<T, 1, 16, 1>(a, w, stream);
+    if (a.vdim <= 64) out_sized<T, TPW, 1, 1, 4>(a, w, stream);
+    else out_sized<T, TPW, 1, 16, 1>(a, w, stream);
   } else {
-    if (a.vdim <= 128) out_sized<T, 2, 1, 4>(a, w, stream);
-    else if (a.vdim <= 256) out_sized<T, 2, 2, 4>(a, w, stream);
-    else out_sized<T, 2, 8, 1>(a, w, stream);
+    if (a.vdim <= 128) out_sized<T, TPW, 2, 1, 4>(a, w, stream);
+    else if (a.vdim <= 256) out_sized<T, TPW, 2, 2, 4>(a, w, stream);
+    else out_sized<T, TPW, 2, 8, 1>(a, w, stream);
   }
 }
 
