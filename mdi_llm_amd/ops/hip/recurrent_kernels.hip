@@ -262,15 +262,15 @@ __global__ __launch_bounds__(256) void rglru_gates_kernel(RgLruArgs p) {
   }
 }
 
-// A recurrence S <- a S + x over a segment, 16 channels per block: 16 threads
-// share a channel and take 8 tokens each of a tile of 128, whose maps S -> A S
-// + B are composed through LDS.  The next tile's operands are in flight
-// meanwhile.  Rule has In (a token's operands), enter(c), load(row, c),
-// map(in) and put(row, c, S, in).
+// A recurrence S <- a S + x over a segment, 16 channels per block: SUB threads
+// share a channel and take TC tokens each of a tile, whose maps S -> A S + B are
+// composed through LDS.  The next tile's operands are in flight meanwhile.
+// Rule has TC, SUB, In (a token's operands), enter(c), load(row, c), map(in) and
+// put(row, c, S, in).
 template <typename Rule>
-__global__ __launch_bounds__(256) void channel_scan_kernel(
+__global__ __launch_bounds__(Rule::SUB * 16) void channel_scan_kernel(
     Rule rule, float* __restrict__ states, SegView seg, int width) {
-  constexpr int TC = 8, SUB = 16, TILE = TC * SUB;
+  constexpr int TC = Rule::TC, SUB = Rule::SUB, TILE = TC * SUB;
   __shared__ float ma[2][SUB][17], mx[2][SUB][17];
   const int s = blockIdx.y, len = seg.len[s];
   const int cl = threadIdx.x & 15, sub = threadIdx.x >> 4;
@@ -332,12 +332,14 @@ __global__ __launch_bounds__(256) void channel_scan_kernel(
 template <typename Rule>
 void channel_scan(const Rule& rule, float* state, SegView seg, int width,
                   hipStream_t stream) {
-  channel_scan_kernel<Rule><<<dim3((width + 127) / 128 * 8, seg.n), 256, 0,
-                              stream>>>(rule, state, seg, width);
+  channel_scan_kernel<Rule>
+      <<<dim3((width + 127) / 128 * 8, seg.n), Rule::SUB * 16, 0, stream>>>(
+          rule, state, seg, width);
 }
 
 template <typename T>
 struct RgLruScan {
+  static constexpr int TC = 8, SUB = 16;
   struct In {
     float a, x;
     T y;
@@ -423,6 +425,7 @@ void rglru_scan_t(const RgLruArgs& a, hipStream_t stream) {
 // ---------------------------------------------------------------------------
 template <typename T>
 struct MinGruScan {
+  static constexpr int TC = 8, SUB = 32;
   using M = Math<T>;
   struct In {
     T z, u, g;
@@ -443,10 +446,11 @@ struct MinGruScan {
     return {p[0], p[width], p[2 * width]};
   }
   DEVINL Decay map(const In& i) const {
-    // 1 - z from its own side: exact where z is close to 1
-    const float v = to_f(i.z) + bz, u = to_f(i.u) + bu;
+    // z = 1 / (1 + e) and 1 - z = e / (1 + e), for any z
+    const float e = M::exp(fminf(-(to_f(i.z) + bz), 80.f));
+    const float z = M::inv(1.f + e), u = to_f(i.u) + bu;
     const float c = u >= 0.f ? u + 0.5f : gate(u);
-    return {gate(-v), gate(v) * c};
+    return {e * z, z * c};
   }
   DEVINL void put(size_t row, int c, float S, const In& i) const {
     const float g = to_f(i.g);
