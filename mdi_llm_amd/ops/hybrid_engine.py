@@ -8,9 +8,10 @@ product for the whole step, and the kernels that look at neighbours in time
 (recurrence, attention) walk the entries as segments.  Steps in which every
 entry is one token are captured as hipGraphs per batch size.
 
-Blocks come in three forms: norms ahead of (and behind) each sublayer, one norm
-for parallel sublayers (``latent_layer``), and norms on the sublayers' outputs
-only, with the options of that form (``_run_output_normed``).
+Blocks come in three forms: norms ahead of (and behind) each sublayer, or ahead
+and behind the two parts of a mixer (``mixers.Paired``); one norm for parallel
+sublayers (``latent_layer``); and norms on the sublayers' outputs only, with the
+options of that form (``_run_output_normed``).
 
 The residual stream, norms, gates, recurrent state and softmax are fp32; the
 weights, matrix products and cached K/V have the stage's dtype (bf16, or

@@ -171,7 +171,7 @@ def test_ring_pipeline_matches_standalone(world, device, tmp_path):
     go through host memory."""
     from mdi_llm_amd.parallel.runtime import PipelineRuntime, SamplingParams
 
-    cfg, w = model("odd")
+    cfg, w = model("mixed")
     save(tmp_path, cfg, w)
     prompts = [tokens(cfg, n, n) for n in (70, 5, 33)]
     torch.save(prompts, tmp_path / "prompts.pt")
@@ -191,7 +191,7 @@ def test_ring_pipeline_matches_standalone(world, device, tmp_path):
 def checkpoint(tmp_path_factory):
     d = tmp_path_factory.mktemp("sosutar") / "toy"
     tok = make_toy_tokenizer(d)
-    cfg = dict(MODELS["odd"],
+    cfg = dict(MODELS["mixed"],
                vocab=max(json.loads(tok.read_text())["model"]["vocab"]
                          .values()) + 1)
     save(d, cfg, weights(cfg))
@@ -258,7 +258,7 @@ def test_trace_replay(device, tmp_path):
     """Requests that pause, end and give back what they hold."""
     from mdi_llm_amd.trace import load_runner, replay
 
-    cfg, w = model("odd")
+    cfg, w = model("mixed")
     save(tmp_path / "m", cfg, w)
     a, b, c = (tokens(cfg, n, n) for n in (90, 10, 70))
     steps = [
