@@ -224,9 +224,10 @@ class GatedAttention(nn.Module):
 
 
 class MinGRU(nn.Module):
-    """Gated recurrence per channel whose gates read the current token only.
-    Part of a ``PairedMixer``: its rows of in_proj are gate z | input | output
-    gate, of which the first two have a bias."""
+    """Recurrence per channel that blends its state with a candidate; blend
+    and candidate depend on the token alone.  Part of a ``PairedMixer``: its
+    rows of in_proj are blend z | input | output gate, of which the first two
+    have a bias."""
 
     kind = "mingru"
 
@@ -242,8 +243,8 @@ PARTS = {m.kind: m for m in (GatedAttention, MinGRU)}
 
 
 class PairedMixer(nn.Module):
-    """Two mixers side by side over one input, whose outputs are normed and
-    averaged.  in_proj rows: the left part's, then the right part's."""
+    """A pair of mixers over one input, the mean of whose normed outputs is
+    the result.  in_proj rows: the left part's, then the right part's."""
 
     kind = "paired"
 

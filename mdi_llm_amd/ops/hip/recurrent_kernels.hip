@@ -421,7 +421,7 @@ void rglru_scan_t(const RgLruArgs& a, hipStream_t stream) {
 }
 
 // ---------------------------------------------------------------------------
-// minGRU: all gates are functions of the token's own projections
+// minGRU: the maps come from the projections alone
 // ---------------------------------------------------------------------------
 template <typename T>
 struct MinGruScan {

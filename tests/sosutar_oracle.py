@@ -107,7 +107,7 @@ def gated_attention(h, w, pre, m, eps):
     return y @ w[pre + "o"].T
 
 
-# -- recurrence whose gates read the current token only ----------------------
+# -- blend of a state and a candidate, per channel ---------------------------
 def candidate(u):
     return torch.where(u >= 0, u + 0.5, sigmoid(u))
 

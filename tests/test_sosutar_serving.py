@@ -4,6 +4,7 @@ pipeline stages, command lines and trace replay."""
 import copy
 import io
 import json
+import re
 import subprocess
 import sys
 from pathlib import Path
@@ -204,7 +205,9 @@ def test_sample_cli(checkpoint, device):
              "--n-tokens", "6", "--device", device, "--sequence-length",
              "512"])
     assert r.returncode == 0, r.stderr[-2000:]
-    assert "sample 2" in r.stdout and "18 tokens" in r.stdout
+    # (a random model may draw the end token)
+    n = int(re.search(r"(\d+) tokens in", r.stdout)[1])
+    assert "sample 2" in r.stdout and 3 <= n <= 18
     assert f"backend={'hip' if device == 'cuda' else 'torch'}" in r.stdout
 
 
