@@ -400,7 +400,7 @@ struct MLstmArgs {
   float* peak;
   const float* gate_bias;
   const float* norm_w;
-  float* work;          // scan: mlstm_work(...) floats
+  float* work;          // scan: mlstm_work_floats(...)
   SegView seg;
   int n, heads, dim, vdim, vstride, max_len;
   float cap, q_scale, eps;
